@@ -21,7 +21,8 @@ HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # points that the oracle pins (RoPE, kf_expf, RMSNorm).
 # -fno-slp-vectorize: keeps the dequant chain in plain v_fma/v_sub (the packed-f32 forms the SLP pass picks cost more issue
 # slots, need s_nop hazard padding and 40 % more registers on this kernel)
-HIP_FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fno-slp-vectorize", "-Wall", "-Wno-unused-function"]
+# -packed-fp32-ops: no v_pk_add_f32 / v_pk_mul_f32 / v_pk_fma_f32 (some of their forms have given wrong results on this part); the two halves of an f32x2 fma are two v_fma_f32, same bits
+HIP_FLAGS = ["--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fno-slp-vectorize", "-Wall", "-Wno-unused-function"]
 # MFMA results that the VALU works on next (attention scores, the epilogues of the token-batch GEMMs): with the default AGPR form of the MFMA destination the
 # compiler moves every such value AGPR -> VGPR (v_accvgpr_read) and zero-fills accumulators through v_accvgpr_write -- 160 of the ~330 vector instructions of a
 # key tile in the attention backward.  The VGPR form has none of them (and the files below stay inside 256 VGPRs where it matters).
