@@ -1,0 +1,127 @@
+/*
+ * kf_rb.h -- C ABI of libkf_hip.so, continued: the ROW-BATCH operators.  A row batch is the next tokens of several sequences side by side (prompts of unequal
+ * length without padding, or one token of each), every row with its own position and state slot.  The operators work on a 32-bit residual stream, take the kind of
+ * every mechanism (activation, chunk size, rotation, gate, scale, experts ...) as a parameter and exist in two storages: KF_BF16 (bf16 operands, 32-bit accumulation)
+ * and KF_F32 (true 32-bit throughout).  Conventions of kf_abi.h apply: device pointers, a stream of one ctx, 0 or a negative code, no allocation.
+ *
+ * Padding: the widths a product runs over are padded with zeros to multiples of KF_RB_PAD in weights and activations alike, weight rows too: tile kernels need no tails.
+ */
+#ifndef KF_RB_H
+#define KF_RB_H
+#include "kf_abi.h"
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+#define KF_RB_PAD 64
+#define KF_RB_DECODE_MAX 64 /* rows of a decode batch the streaming products serve; larger batches take the tile kernels */
+
+/* activations: relu(z); z sigmoid(z); 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) */
+enum kf_rb_act { KF_RB_RELU = 0, KF_RB_SILU = 1, KF_RB_GELU_TANH = 2 };
+
+/* what a product's epilogue does with row dot d[t][m]:
+ *   STORE      y[t][m] = d             (y in the batch's storage)
+ *   STORE_F32  y[t][m] = d             (fp32)
+ *   RESIDUAL   y[t][m] = alpha res[t][m] + d   (fp32)
+ *   GATED      y[t][f] = act(d[t][gate f]) * d[t][up f]; the weight holds gate and up interleaved in blocks of 16 rows (16 gate, 16 up, ...), m counts both */
+enum kf_rb_epilogue { KF_RB_STORE = 0, KF_RB_STORE_F32 = 1, KF_RB_RESIDUAL = 2, KF_RB_GATED = 3 };
+
+/* the routed (row, choice) pairs of a batch, grouped by expert; pair p = row * top + choice */
+typedef struct kf_rb_experts {
+    int32_t n_expert, top;
+    int32_t tile;               /* pairs per tile of the list (every tile belongs to one expert) */
+    int32_t n_tile;             /* tiles the list has room for: kf_rb_list_tiles() */
+    const int32_t* tile_expert; /* [n_tile] the tile's expert, -1: empty (a run of them at the end) */
+    const int32_t* list;        /* [n_tile][tile] pairs, -1: none */
+    const int32_t* ids;         /* [rows * top] chosen expert of every pair, -1: inactive row */
+    const float* weight;        /* [rows * top] */
+    int64_t w_stride;           /* elements from one expert's matrix to the next */
+} kf_rb_experts;
+
+/* how a product meets the experts:
+ *   ALL   no experts
+ *   UP    pair p reads row p / top of x and writes row p of y; GATED only: y is scaled by the pair's weight before it is stored
+ *   DOWN  pair p reads row p of x and writes row p of y (fp32, STORE_F32)
+ *   SUM   row t: RESIDUAL with d = the sum over its pairs of (expert's matrix . row p of x) -- decode batches only */
+enum kf_rb_experts_mode { KF_RB_ALL = 0, KF_RB_UP = 1, KF_RB_DOWN = 2, KF_RB_SUM = 3 };
+
+typedef struct kf_rb_product {
+    const void* w;   /* [m][k] row-major (x n_expert) */
+    const void* x;   /* rows ldx apart */
+    void* y;         /* rows ldy apart */
+    const float* res;
+    int64_t ldx, ldy, ldr;
+    int32_t type;    /* KF_BF16 | KF_F32: w, x and a STORE / GATED y */
+    int32_t m, k, n; /* m, k: multiples of KF_RB_PAD; n: token rows of the batch.  bf16 with experts: tiles of 16, 32, 48 or 64 pairs (n <= KF_RB_DECODE_MAX), 64 or 128
+                        (more rows); fp32: 64 */
+    int32_t epilogue, act, mode;
+    float alpha;
+    const kf_rb_experts* experts;
+} kf_rb_product;
+int kf_rb_linear(kf_ctx* ctx, const kf_rb_product* p);
+
+/* load time: a bf16 matrix src [rows][cols] into a padded one of storage `type` with rows ld apart (columns cols .. ld - 1 are left alone: allocate zeroed).
+ * half < 0: row r goes to row r; half 0 / 1: to row 32 (r / 16) + 16 half + r % 16, the gate / up halves of a GATED product's weight */
+int kf_rb_pack(kf_ctx* ctx, int type, const kf_bf16* src, int rows, int cols, void* dst, int64_t ld, int half);
+
+/* tokens -> rows of the table: x fp32 [n][ldx] and h (storage `type`) [n][ldx]; columns dim .. ldx - 1 are written as zeros.  table rows are ldx apart too. */
+int kf_rb_embed(kf_ctx* ctx, int type, const void* table, int vocab, int dim, int64_t ldx, const int32_t* tokens, int n, float* x, void* h);
+/* a decode batch: row s is slot s of a state array d_state [n][4] = {token, pos, parked, status}, token = d_forced[s][pos] when that is >= 0.  Also writes the rows'
+ * meta (below); a parked slot, or one whose position is outside [0, max_pos), becomes an inactive row (the latter with status bit 64). */
+int kf_rb_embed_state(kf_ctx* ctx, int type, const void* table, int vocab, int dim, int64_t ldx, int32_t* d_state, const int32_t* d_forced, int forced_stride, int max_pos,
+                      int n, float* x, void* h, int32_t* meta);
+
+/* RMS norm of fp32 rows, z / sqrt(mean(z^2) + eps) * w over `dim` columns: x_out (fp32, may be NULL) and h_out (storage `type`) both ld apart, pad columns zero.
+ *   plain:   z = row t of z
+ *   experts: z = alpha res[t] + sum over the row's `top` pairs of z[t * top + j]      (res != NULL)
+ *   rows != NULL: output row t comes from row rows[t] */
+int kf_rb_norm(kf_ctx* ctx, int type, const float* z, const float* res, float alpha, int top, const void* w, float eps, int dim, int64_t ld, int n, const int32_t* rows,
+               float* x_out, void* h_out);
+
+/* a row's meta: {position (< 0: inactive), slot, position of the sequence's first row in this batch, position of its last row in this batch} */
+#define KF_RB_META 4
+/* a sequence's rows: {first row, rows, position of the first row, slot} */
+
+/* one attention layer over a row batch.  raw [rows][ldraw] holds q (n_head * dim columns), then k (n_kv * dim), then the output gate (n_head * dim, gated != 0).
+ * The values ARE the projected keys (before norm and rotation); q and k are RMS-normed per head, then the first rot_dims dimensions of each head rotated (i with
+ * i + rot_dims / 2) by the angles of `rope`; score = q . k * scale; position i sees j <= i with floor(i / chunk) == floor(j / chunk) (chunk 0: every j <= i).
+ * out [rows][ldout] (columns n_head * dim) = softmax(scores) . v  (* sigmoid(gate)).
+ * The state: k (normed, rotated) and v rows of slot s, position j at cache[s * slot_stride + (j % cache_rows) * n_kv * dim]; cache_rows >= min(chunk, positions). */
+typedef struct kf_rb_attention {
+    void* raw;
+    void* out;
+    void* k_new;            /* [rows][n_kv * dim] scratch: the batch's normed, rotated keys (prefill form) */
+    void *k_cache, *v_cache;
+    const void *q_norm, *k_norm; /* [dim], NULL: no norm */
+    const float* rope;      /* [max_pos][rot_dims / 2][2] (cos, sin) */
+    void* scratch;          /* decode form, kf_rb_attention_scratch() bytes */
+    int64_t ldraw, ldout, slot_stride;
+    int32_t type, n_head, n_kv, dim, rot_dims, chunk, cache_rows, gated;
+    float scale, eps;
+} kf_rb_attention;
+/* rows of n_seq sequences, longest max_n rows: seqs [n_seq][4], meta [n_rows][4] on the device */
+int kf_rb_attention_prefill(kf_ctx* ctx, const kf_rb_attention* a, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n);
+/* one row per slot; max_pos bounds the positions of the active rows (launch geometry) */
+int kf_rb_attention_decode(kf_ctx* ctx, const kf_rb_attention* a, const int32_t* meta, int n_rows, int max_pos);
+size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim);
+/* host: (cos, sin) of pos * f_i, f_i = base^(-2 i / dims), i < dims / 2.  factor != 1: wavelengths above original / low are stretched by factor, those below
+ * original / high kept, between the two the blend (1 - s) f / factor + s f with s = (original / wavelength - low) / (high - low). */
+int kf_rb_rope_table_host(float* h_table, int n_pos, int dims, double base, double factor, double low, double high, double original);
+
+/* router: logits fp32 [n][ld] (+ bias [n_expert] in the batch's storage, may be NULL) -> the `top` largest of every row (ties: the lower expert) and the softmax over them;
+ * rows whose meta position is < 0 (meta != NULL) choose nothing.  Then the pairs grouped by expert into the list.  experts: the arrays it points to are written. */
+int kf_rb_route(kf_ctx* ctx, int type, const float* logits, int64_t ld, const void* bias, int n, const int32_t* meta, const kf_rb_experts* experts);
+int kf_rb_list_tiles(int n, int top, int n_expert, int tile);
+
+/* greedy pick over fp32 logits [n][ld], first maximum; row s advances slot s: d_tokens_out[s][pos] = id, d_state[s] = {id, pos + 1}.  Inactive rows (meta) are left
+ * alone.  scratch: kf_rb_pick_scratch(n) bytes. */
+int kf_rb_pick(kf_ctx* ctx, const float* logits, int64_t ld, int vocab, int n, const int32_t* meta, int32_t* d_state, int32_t* d_tokens_out, int tokens_stride, void* scratch);
+size_t kf_rb_pick_scratch(int n);
+/* fp32 logits row -> bf16 (what kf_sample reads) */
+int kf_rb_to_bf16(kf_ctx* ctx, const float* src, kf_bf16* dst, size_t n);
+
+#ifdef __cplusplus
+}
+#endif
+#endif

@@ -6,14 +6,14 @@
 Both are written next to this file so they travel with the source tree.  No JIT cache.
 """
 import os
+import re
 import subprocess
 import sys
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 HOST = os.path.join(HERE, "host")
-HIP_SOURCES = ["kf_gemv.hip", "kf_gemv_canon.hip", "kf_gemm.hip", "kf_gemm2.hip", "kf_gemm3.hip", "kf_attn.hip", "kf_engine.hip", "kf_xengine.hip", "kf_xengine_q1.hip", "kf_attn_prefill.hip", "kf_ops.hip", "kf_lut.hip", "kf_loss.hip", "kf_norm_bwd.hip", "kf_linear_bwd.hip", "kf_embed_bwd.hip", "kf_attn_bwd_mfma.hip", "kf_awq.hip", "kf_tp.hip", "kf_abi.hip"]
-HIP_DEPS = ["kf_device.h", "kf_kernels.h", "kf_gemm_common.h", "kf_gemv_blocks.h", "kf_attn_common.h", "kf_engine_common.h", "kf_xengine_kernel.h"]
+HIP_SOURCES = ["kf_gemv.hip", "kf_gemv_canon.hip", "kf_gemm.hip", "kf_gemm2.hip", "kf_gemm3.hip", "kf_attn.hip", "kf_engine.hip", "kf_xengine.hip", "kf_xengine_q1.hip", "kf_attn_prefill.hip", "kf_ops.hip", "kf_lut.hip", "kf_loss.hip", "kf_norm_bwd.hip", "kf_linear_bwd.hip", "kf_embed_bwd.hip", "kf_attn_bwd_mfma.hip", "kf_awq.hip", "kf_tp.hip", "kf_rb_ops.hip", "kf_rb_linear.hip", "kf_rb_gemm.hip", "kf_rb_attn.hip", "kf_abi.hip"]
 LIB_HIP = os.path.join(HERE, "libkf_hip.so")
 LIB_HOST = os.path.join(HERE, "libkf_host.so")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
@@ -36,15 +36,26 @@ def _stale(target, deps):
     return any(os.path.getmtime(d) > t for d in deps)
 
 
-def build_hip(force=False, verbose=False):
-    srcs = [os.path.join(CSRC, s) for s in HIP_SOURCES]
-    deps = srcs + [os.path.join(CSRC, d) for d in HIP_DEPS] + [os.path.join(HERE, "..", "include", "kf_abi.h")]
+def _includes(path, seen=None):
+    """path and every in-tree file it #includes, directly or not"""
+    seen = set() if seen is None else seen
+    path = os.path.normpath(path)
+    if path in seen or not os.path.exists(path):
+        return seen
+    seen.add(path)
+    with open(path) as f:
+        for m in re.finditer(r'^\s*#include "([^"]+)"', f.read(), re.M):
+            _includes(os.path.join(os.path.dirname(path), m.group(1)), seen)
+    return seen
+
+
+def _compile(sources, force, verbose):
+    """objects of the named csrc/ files, compiled where stale"""
     objs, cmds = [], []
-    for s in srcs:
+    for s in [os.path.join(CSRC, s) for s in sources]:
         o = s[:-4] + ".o"
         objs.append(o)
-        extra = [os.path.join(CSRC, "kf_gemv.hip")] if os.path.basename(s) == "kf_gemv_canon.hip" else []   # it #includes kf_gemv.hip
-        if force or _stale(o, [s] + extra + deps[len(srcs):]):
+        if force or _stale(o, _includes(s)):
             cmds.append([HIPCC] + HIP_FLAGS + HIP_FILE_FLAGS.get(os.path.basename(s), []) + ["-c", s, "-o", o])
     if cmds:   # independent translation units: a few at a time (the container has 8 CPUs; one hipcc peaks near 2 GB)
         from concurrent.futures import ThreadPoolExecutor
@@ -55,6 +66,11 @@ def build_hip(force=False, verbose=False):
             subprocess.check_call(cmd)
         with ThreadPoolExecutor(max_workers=int(os.environ.get("KF_BUILD_JOBS", "6"))) as ex:
             list(ex.map(run, cmds))
+    return objs
+
+
+def build_hip(force=False, verbose=False):
+    objs = _compile(HIP_SOURCES, force, verbose)
     if force or _stale(LIB_HIP, objs):
         cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_HIP] + objs
         if verbose:
@@ -63,17 +79,55 @@ def build_hip(force=False, verbose=False):
     return LIB_HIP
 
 
+HOST_SOURCES = ["kf_host.cpp", "kf_safetensors.cpp", "kf_train.cpp", "kf_seq.cpp", "kf_tizusun.cpp"]
+
+
+def _host_cmd(out, libdir, opt):
+    return ["g++"] + opt + ["-std=c++17", "-fPIC", "-shared", "-Wall", "-o", out] + [os.path.join(HOST, s) for s in HOST_SOURCES] + ["-L" + libdir, "-lkf_hip", "-Wl,-rpath,$ORIGIN"]
+
+
+def _host_deps(libhip):
+    deps = set()
+    for s in HOST_SOURCES:
+        _includes(os.path.join(HOST, s), deps)
+    return sorted(deps) + [libhip]
+
+
 def build_host(force=False, verbose=False):
-    src = os.path.join(HOST, "kf_host.cpp")
-    src2 = os.path.join(HOST, "kf_safetensors.cpp")
-    src3 = os.path.join(HOST, "kf_train.cpp")
-    deps = [src, src2, src3, os.path.join(HOST, "kf_safetensors.hpp"), os.path.join(HOST, "kf_host.hpp"), os.path.join(HERE, "..", "include", "kf_abi.h"), LIB_HIP]
-    if force or _stale(LIB_HOST, deps):
-        cmd = ["g++", "-O2", "-std=c++17", "-fPIC", "-shared", "-Wall", "-o", LIB_HOST, src, src2, src3, "-L" + HERE, "-lkf_hip", "-Wl,-rpath,$ORIGIN"]
+    if force or _stale(LIB_HOST, _host_deps(LIB_HIP)):
+        cmd = _host_cmd(LIB_HOST, HERE, ["-O2"])
         if verbose:
             print(" ".join(cmd))
         subprocess.check_call(cmd)
     return LIB_HOST
+
+
+# What one family of models launches.  A fresh checkout that only serves such a model (bin/trace_run) compiles these files and no others: seconds instead of minutes.
+PARTS = {"rows": ["kf_rb_ops.hip", "kf_rb_linear.hip", "kf_rb_gemm.hip", "kf_rb_attn.hip", "kf_ops.hip", "kf_abi.hip"]}
+
+
+def build_part(part, verbose=False):
+    """The two libraries with the device code of one part, in a directory of their own (koifish_amd/part_<part>/): the launchers of every other kernel are bound to a stub
+    that reports KF_UNSUPPORTED_DATATYPE.  Returns the directory (what KF_LIB_DIR takes)."""
+    out = os.path.join(HERE, "part_" + part)
+    os.makedirs(out, exist_ok=True)
+    hip, host = os.path.join(out, "libkf_hip.so"), os.path.join(out, "libkf_host.so")
+    objs = _compile(PARTS[part], False, verbose)
+    if _stale(hip, objs):
+        def symbols(flag):
+            return {l.split()[-1] for o in objs for l in subprocess.check_output(["nm", flag, o]).decode().splitlines() if l.split()}
+        absent = sorted(s for s in symbols("--undefined-only") - symbols("--defined-only") if s.startswith("_ZN2kf"))
+        stub = os.path.join(out, "absent.c")
+        with open(stub, "w") as f:
+            f.write("/* launchers of kernels this build leaves out */\nint kf_part_absent(void) { return -1000; }\n")
+        subprocess.check_call(["gcc", "-O1", "-fPIC", "-fvisibility=hidden", "-c", stub, "-o", stub[:-2] + ".o"])
+        cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", hip] + objs + [stub[:-2] + ".o"] + ["-Wl,--defsym=%s=kf_part_absent" % s for s in absent]
+        if verbose:
+            print(" ".join(cmd[:12]), "...", flush=True)
+        subprocess.check_call(cmd)
+    if _stale(host, _host_deps(hip)):
+        subprocess.check_call(_host_cmd(host, out, ["-O2"]))
+    return out
 
 
 def build_host_asan(verbose=False):
@@ -81,13 +135,8 @@ def build_host_asan(verbose=False):
     files.  Written to libkf_host_asan.so; tests/test_host_asan_cpu.py runs the checkpoint tests under it (LD_PRELOAD of libasan, KF_HOST_LIB).
     Never for the GPU box: sanitizers run on the CPU build only."""
     out = os.path.join(HERE, "libkf_host_asan.so")
-    src = os.path.join(HOST, "kf_host.cpp")
-    src2 = os.path.join(HOST, "kf_safetensors.cpp")
-    src3 = os.path.join(HOST, "kf_train.cpp")
-    deps = [src, src2, src3, os.path.join(HOST, "kf_safetensors.hpp"), os.path.join(HOST, "kf_host.hpp"), os.path.join(HERE, "..", "include", "kf_abi.h"), LIB_HIP]
-    if _stale(out, deps):
-        cmd = ["g++", "-O1", "-g", "-fno-omit-frame-pointer", "-fsanitize=address,undefined", "-fno-sanitize-recover=undefined", "-std=c++17", "-fPIC", "-shared", "-Wall",
-               "-o", out, src, src2, src3, "-L" + HERE, "-lkf_hip", "-Wl,-rpath,$ORIGIN"]
+    if _stale(out, _host_deps(LIB_HIP)):
+        cmd = _host_cmd(out, HERE, ["-O1", "-g", "-fno-omit-frame-pointer", "-fsanitize=address,undefined", "-fno-sanitize-recover=undefined"])
         if verbose:
             print(" ".join(cmd))
         subprocess.check_call(cmd)

@@ -1,0 +1,604 @@
+// kf_rb_attn.hip -- attention of a row batch (kf_rb.h): per-head RMS norm + partial rotation of q and k, values = the projected keys, chunked causal mask, free scale,
+// sigmoid output gate, a ring of cache rows per slot.
+//
+// bf16, dim a multiple of 8 up to 256: MFMA flash form, the register / LDS scheme of kf_attn_prefill.hip (S^T = K Q^T by v_mfma_f32_32x32x16_bf16, a column = one (token,
+// query head) pair per lane pair, P split into a bf16 pair for the P.V product, V^T fragments by ds_read_b64_tr_b16), with
+//   * columns flattened over (token, head): any number of query heads per kv-head;
+//   * keys and values of the batch's own tokens read from the batch, older ones from the slot's ring: a prompt is attended to before its rows overwrite the ring;
+//   * only the tiles between a wave's first chunk start and its last position.
+// A decode row is one workgroup per (kv-head, key range): q and the new key are prepared in LDS, each of its four waves walks its own 32-key tiles (staged into LDS of its
+// own, no barrier in the walk) and the four partial softmaxes meet at the end.
+// fp32 storage (and other head sizes): a plain form, one wave per (row, head), 32-bit throughout.
+#include <algorithm>
+
+#include "kf_ctx.h"
+#include "kf_rb_common.h"
+
+namespace kf {
+
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x4_t __attribute__((ext_vector_type(4)));
+typedef float f32x16_t __attribute__((ext_vector_type(16)));
+
+constexpr float RB_LOG2E = 1.44269502162933349609375f;
+__device__ __forceinline__ float rb_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ int rb_first_key(int pos, int chunk) { return chunk > 0 ? pos - pos % chunk : 0; }
+
+// one head (dim elements at src) normed and rotated by one wave into dst; buf: dim floats of LDS of this wave
+template <class T>
+__device__ __forceinline__ void rb_prep_head(const T* __restrict__ src, T* dst, const T* __restrict__ w, const float* __restrict__ rope, int rot, int dim, int pos, float eps, float* buf,
+                                             int lane) {
+    float ss = 0.f;
+    for (int i = lane; i < dim; i += 64) {
+        const float v = rb_ld(src + i);
+        buf[i] = v;
+        ss = fmaf(v, v, ss);
+    }
+    ss = wave_sum(ss);
+    const float rs = w ? 1.0f / sqrtf(ss / (float)dim + eps) : 1.0f;
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    const int half = rot >> 1;
+    for (int i = lane; i < half; i += 64) {
+        const float u = buf[i] * rs * (w ? rb_ld(w + i) : 1.f), v = buf[i + half] * rs * (w ? rb_ld(w + i + half) : 1.f);
+        const float2 cs = *reinterpret_cast<const float2*>(rope + ((size_t)pos * half + i) * 2);
+        rb_st(dst + i, u * cs.x - v * cs.y);
+        rb_st(dst + i + half, v * cs.x + u * cs.y);
+    }
+    for (int i = rot + lane; i < dim; i += 64) rb_st(dst + i, buf[i] * rs * (w ? rb_ld(w + i) : 1.f));
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// ---- q in place, k -> k_new (prefill) or, STORE: k and v into the slot's ring (decode)
+template <class T, bool STORE>
+__global__ void __launch_bounds__(256) rb_prep_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta) {
+    extern __shared__ float s_buf[];
+    const int r = blockIdx.x, wid = threadIdx.x >> 6, lane = threadIdx.x & 63, u = blockIdx.y * 4 + wid;
+    const int pos = meta[KF_RB_META * r];
+    if (pos < 0 || u >= a.n_head + a.n_kv) return; /* no barrier below */
+    T* raw = reinterpret_cast<T*>(a.raw) + (size_t)r * a.ldraw;
+    float* buf = s_buf + wid * a.dim;
+    if (u < a.n_head) {
+        T* q = raw + (size_t)u * a.dim;
+        rb_prep_head(q, q, reinterpret_cast<const T*>(a.q_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, buf, lane);
+        return;
+    }
+    const int g = u - a.n_head, kvd = a.n_kv * a.dim;
+    const T* k = raw + (size_t)u * a.dim;
+    T* dst;
+    if constexpr (STORE) {
+        const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * kvd + (size_t)g * a.dim;
+        dst = reinterpret_cast<T*>(a.k_cache) + at;
+        T* v = reinterpret_cast<T*>(a.v_cache) + at;
+        for (int i = lane; i < a.dim; i += 64) v[i] = k[i];
+    } else {
+        dst = reinterpret_cast<T*>(a.k_new) + (size_t)r * kvd + (size_t)g * a.dim;
+    }
+    rb_prep_head(k, dst, reinterpret_cast<const T*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, buf, lane);
+}
+// ---- the batch's last cache_rows keys / values of every sequence into its slot's ring
+template <class T>
+__global__ void __launch_bounds__(256) rb_store_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta) {
+    const int r = blockIdx.x, pos = meta[KF_RB_META * r], last = meta[KF_RB_META * r + 3];
+    if (pos < 0 || pos <= last - a.cache_rows) return;
+    const int kvd = a.n_kv * a.dim;
+    const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * kvd;
+    const T* k = reinterpret_cast<const T*>(a.k_new) + (size_t)r * kvd;
+    const T* v = reinterpret_cast<const T*>(a.raw) + (size_t)r * a.ldraw + (size_t)a.n_head * a.dim;
+    T *kc = reinterpret_cast<T*>(a.k_cache) + at, *vc = reinterpret_cast<T*>(a.v_cache) + at;
+    for (int i = threadIdx.x; i < kvd; i += blockDim.x) kc[i] = k[i], vc[i] = v[i];
+}
+
+// ---- the plain form: one wave per (row, head); scores of 64 keys at a time, one key per lane, then the values with one dimension per lane.
+// ring_only: every key up to the row's own is in the ring already (decode)
+template <class T>
+__global__ void __launch_bounds__(64) rb_attn_plain_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta, int ring_only) {
+    extern __shared__ float s_q[]; /* [dim] */
+    __shared__ float s_p[64];
+    __shared__ const T* s_v[64];
+    const int r = blockIdx.x, n = blockIdx.y, lane = threadIdx.x;
+    const int pos = meta[KF_RB_META * r], slot = meta[KF_RB_META * r + 1], pos0 = ring_only ? pos + 1 : meta[KF_RB_META * r + 2];
+    if (pos < 0) return;
+    const int g = n / (a.n_head / a.n_kv), kvd = a.n_kv * a.dim;
+    const T* raw = reinterpret_cast<const T*>(a.raw);
+    for (int i = lane; i < a.dim; i += 64) s_q[i] = rb_ld(raw + (size_t)r * a.ldraw + (size_t)n * a.dim + i);
+    __syncthreads();
+    constexpr int ND = 8; /* dims per lane: dim <= 512 */
+    float o[ND];
+#pragma unroll
+    for (int j = 0; j < ND; j++) o[j] = 0.f;
+    float M = -__builtin_inff(), l = 0.f;
+    for (int k0 = rb_first_key(pos, a.chunk); k0 <= pos; k0 += 64) {
+        const int key = k0 + lane;
+        float s = -__builtin_inff();
+        const T* v = nullptr;
+        if (key <= pos) {
+            const T* k;
+            if (key >= pos0) {
+                const size_t row = (size_t)r - (pos - key);
+                k = reinterpret_cast<const T*>(a.k_new) + row * kvd + (size_t)g * a.dim;
+                v = raw + row * a.ldraw + (size_t)(a.n_head + g) * a.dim;
+            } else {
+                const size_t at = (size_t)slot * a.slot_stride + (size_t)(key % a.cache_rows) * kvd + (size_t)g * a.dim;
+                k = reinterpret_cast<const T*>(a.k_cache) + at, v = reinterpret_cast<const T*>(a.v_cache) + at;
+            }
+            float d = 0.f;
+            for (int i = 0; i < a.dim; i++) d = fmaf(s_q[i], rb_ld(k + i), d);
+            s = d * a.scale;
+        }
+        const float mt = wave_max(s), Mn = fmaxf(M, mt);
+        const float alpha = expf(M - Mn), p = expf(s - Mn); /* masked: 0 */
+        l = l * alpha + wave_sum(p);
+        M = Mn;
+        __syncthreads();
+        s_p[lane] = p, s_v[lane] = v;
+        __syncthreads();
+        const int nk = pos - k0 + 1 < 64 ? pos - k0 + 1 : 64;
+#pragma unroll
+        for (int j = 0; j < ND; j++) o[j] *= alpha;
+        for (int i = 0; i < nk; i++) {
+            const float pi = s_p[i];
+            const T* vi = s_v[i];
+#pragma unroll
+            for (int j = 0; j < ND; j++) {
+                const int d = lane + 64 * j;
+                if (d < a.dim) o[j] = fmaf(pi, rb_ld(vi + d), o[j]);
+            }
+        }
+    }
+    const T* gate = raw + (size_t)r * a.ldraw + (size_t)(a.n_head + a.n_kv + n) * a.dim;
+    T* out = reinterpret_cast<T*>(a.out) + (size_t)r * a.ldout + (size_t)n * a.dim;
+#pragma unroll
+    for (int j = 0; j < ND; j++) {
+        const int d = lane + 64 * j;
+        if (d < a.dim) rb_st(out + d, o[j] / l * (a.gated ? rb_sigmoid(rb_ld(gate + d)) : 1.f));
+    }
+}
+
+// ---- MFMA form: one 32-key tile against a wave's 32 columns
+constexpr int RB_VPAD = 32; /* V row padding, elements: the 4 rows of a transposing read land on distinct bank groups */
+template <int HD>
+struct RbTile {
+    static constexpr int NS = HD / 16, NDB = HD / 32, KS = HD + 8, VS = HD + RB_VPAD;
+    f32x16_t o[NDB];
+    float M, l;
+    __device__ __forceinline__ void init() {
+#pragma unroll
+        for (int db = 0; db < NDB; db++)
+#pragma unroll
+            for (int i = 0; i < 16; i++) o[db][i] = 0.f;
+        M = -__builtin_inff(), l = 0.f;
+    }
+    // keys k0 .. k0 + 31 staged at kb [32][KS], vb [32][VS]; the column sees keys lo .. hi (every: the whole tile is visible to every column of the wave)
+    __device__ __forceinline__ void step(const uint16_t* kb, const uint16_t* vb, const u32x4 (&qf)[NS], float sc2, int k0, int lo, int hi, bool every, int lane) {
+        const int r = lane & 31, h = lane >> 5;
+        f32x16_t st;
+#pragma unroll
+        for (int i = 0; i < 16; i++) st[i] = 0.f;
+#pragma unroll
+        for (int s = 0; s < NS; s++) {
+            const u32x4 A = *reinterpret_cast<const u32x4*>(kb + r * KS + 16 * s + 8 * h);
+            st = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, A), __builtin_bit_cast(bf16x8_t, qf[s]), st, 0, 0, 0);
+        }
+        float mt = -__builtin_inff();
+#pragma unroll
+        for (int i = 0; i < 16; i++) {
+            const int key = k0 + 4 * h + (i & 3) + 8 * (i >> 2);
+            st[i] = every || (key >= lo && key <= hi) ? st[i] * sc2 : -__builtin_inff();
+            mt = fmaxf(mt, st[i]);
+        }
+        mt = xmax32(mt);
+        if (mt > M) {
+            const float alpha = rb_exp2(M - mt);
+            l *= alpha;
+#pragma unroll
+            for (int db = 0; db < NDB; db++)
+#pragma unroll
+                for (int i = 0; i < 16; i++) o[db][i] *= alpha;
+            M = mt;
+        }
+        const float Mref = M == -__builtin_inff() ? 0.f : M; /* a column that has seen nothing: p = 0 */
+        uint32_t ph[8], pl[8];
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            const float p0 = rb_exp2(st[2 * i] - Mref), p1 = rb_exp2(st[2 * i + 1] - Mref);
+            l += p0;
+            l += p1;
+            ph[i] = pack_bf16x2(p0, p1);
+            pl[i] = pack_bf16x2(p0 - bf_lo(ph[i]), p1 - bf_hi(ph[i]));
+        }
+#pragma unroll
+        for (int s2 = 0; s2 < 2; s2++) {
+            const u32x4 B = u32x4{ph[4 * s2], ph[4 * s2 + 1], ph[4 * s2 + 2], ph[4 * s2 + 3]}, B2 = u32x4{pl[4 * s2], pl[4 * s2 + 1], pl[4 * s2 + 2], pl[4 * s2 + 3]};
+#pragma unroll
+            for (int db = 0; db < NDB; db++) {
+                const uint16_t* vp = vb + (16 * s2 + 4 * h + ((lane & 15) >> 2)) * VS + db * 32 + (lane & 16) + 4 * (lane & 3);
+                const bf16x4_t x = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) bf16x4_t*)(vp));
+                const bf16x4_t y = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) bf16x4_t*)(vp + 8 * VS));
+                const bf16x8_t A = bf16x8_t{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+                o[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(A, __builtin_bit_cast(bf16x8_t, B), o[db], 0, 0, 0);
+                o[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(A, __builtin_bit_cast(bf16x8_t, B2), o[db], 0, 0, 0);
+            }
+        }
+    }
+};
+
+// where key `key` of a sequence lies: the batch's own rows from pos0 on, the ring before
+struct RbKeys {
+    const uint16_t *k_new, *v_new; /* the sequence's first batch row, this kv-head */
+    const uint16_t *k_ring, *v_ring;
+    long long ldk, ldv;            /* batch row strides; a ring row is ldk apart too */
+    int pos0, ring;
+    __device__ __forceinline__ void at(int key, const uint16_t*& k, const uint16_t*& v) const {
+        if (key >= pos0) {
+            k = k_new + (size_t)(key - pos0) * ldk, v = v_new + (size_t)(key - pos0) * ldv;
+        } else {
+            const size_t o = (size_t)(key % ring) * ldk;
+            k = k_ring + o, v = v_ring + o;
+        }
+    }
+};
+
+// q, k_new prepared.  grid (column blocks of the longest sequence, n_kv, sequences); 128 columns per workgroup, 32 per wave, two LDS tiles
+template <int HD>
+__global__ void __launch_bounds__(256, HD <= 128 ? 2 : 1) rb_attn_prefill_kernel(const kf_rb_attention a, const int32_t* __restrict__ seqs) {
+    using Tile = RbTile<HD>;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+    constexpr int KS = Tile::KS, VS = Tile::VS, CH = HD / 8, CPT = (32 * CH + 255) / 256;
+    uint16_t* ks = reinterpret_cast<uint16_t*>(smem_raw); /* 2 x [32][KS] */
+    uint16_t* vs = ks + 2 * 32 * KS;                      /* 2 x [32][VS] */
+    const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3];
+    const int GQ = a.n_head / a.n_kv, ncol = n * GQ, g = blockIdx.y, bx = (int)gridDim.x - 1 - (int)blockIdx.x;
+    if (bx * 128 >= ncol) return; /* workgroup-uniform */
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5, kvd = a.n_kv * a.dim;
+    const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw;
+    RbKeys kv;
+    kv.k_new = reinterpret_cast<const uint16_t*>(a.k_new) + (size_t)row0 * kvd + (size_t)g * a.dim, kv.v_new = raw + (size_t)(a.n_head + g) * a.dim;
+    kv.k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
+    kv.v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
+    kv.ldk = kvd, kv.ldv = a.ldraw, kv.pos0 = pos0, kv.ring = a.cache_rows;
+    // this lane pair's column; columns past the end repeat the last one and are not stored
+    int c = bx * 128 + wid * 32 + r;
+    const bool col_ok = c < ncol;
+    c = col_ok ? c : ncol - 1;
+    const int tok = c / GQ, head = g * GQ + (c - tok * GQ), pos = pos0 + tok, lo = rb_first_key(pos, a.chunk);
+    // the wave's and the workgroup's key ranges
+    auto tok_of = [&](int cc) { return (cc < ncol ? cc : ncol - 1) / GQ; };
+    const int w0 = pos0 + tok_of(bx * 128 + wid * 32), w1 = pos0 + tok_of(bx * 128 + wid * 32 + 31);
+    const int wlo = rb_first_key(w0, a.chunk), wlo1 = rb_first_key(w1, a.chunk);
+    const int klo = rb_first_key(pos0 + tok_of(bx * 128), a.chunk), khi = pos0 + tok_of(bx * 128 + 127);
+    u32x4 qf[Tile::NS];
+    {
+        const uint16_t* q = raw + (size_t)tok * a.ldraw + (size_t)head * a.dim;
+#pragma unroll
+        for (int s = 0; s < Tile::NS; s++) {
+            qf[s] = u32x4{0, 0, 0, 0};
+            if (16 * s + 8 * h < a.dim) qf[s] = *reinterpret_cast<const u32x4*>(q + 16 * s + 8 * h);
+        }
+    }
+    u32x4 kr[CPT], vr[CPT];
+    auto tload = [&](int k0) {
+#pragma unroll
+        for (int i = 0; i < CPT; i++) {
+            const int ch = tid + 256 * i, key = ch / CH, d = (ch - key * CH) * 8;
+            kr[i] = vr[i] = u32x4{0, 0, 0, 0};
+            if (key < 32 && d < a.dim) {
+                const int kk = k0 + key < khi ? k0 + key : khi; /* past the last key: masked, never read past it */
+                const uint16_t *kp, *vp;
+                kv.at(kk, kp, vp);
+                kr[i] = *reinterpret_cast<const u32x4*>(kp + d), vr[i] = *reinterpret_cast<const u32x4*>(vp + d);
+            }
+        }
+    };
+    auto tstore = [&](int b) {
+#pragma unroll
+        for (int i = 0; i < CPT; i++) {
+            const int ch = tid + 256 * i, key = ch / CH, d = (ch - key * CH) * 8;
+            if (key < 32) {
+                *reinterpret_cast<u32x4*>(ks + (b * 32 + key) * KS + d) = kr[i];
+                *reinterpret_cast<u32x4*>(vs + (b * 32 + key) * VS + d) = vr[i];
+            }
+        }
+    };
+    Tile T;
+    T.init();
+    const float sc2 = a.scale * RB_LOG2E;
+    tload(klo);
+    tstore(0);
+    __syncthreads();
+    int b = 0;
+    for (int k0 = klo; k0 <= khi; k0 += 32, b ^= 1) {
+        const bool more = k0 + 32 <= khi;
+        if (more) tload(k0 + 32);
+        if (k0 + 31 >= wlo && k0 <= w1) /* wave-uniform */
+            T.step(ks + b * 32 * KS, vs + b * 32 * VS, qf, sc2, k0, lo, pos, k0 >= wlo1 && k0 + 31 <= w0, lane);
+        if (more) tstore(b ^ 1);
+        __syncthreads();
+    }
+    const float l = xsum32(T.l);
+    if (!col_ok) return;
+    const float inv = 1.0f / l;
+    const uint16_t* gate = raw + (size_t)tok * a.ldraw + (size_t)(a.n_head + a.n_kv + head) * a.dim;
+    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)(row0 + tok) * a.ldout + (size_t)head * a.dim;
+#pragma unroll
+    for (int db = 0; db < Tile::NDB; db++)
+#pragma unroll
+        for (int q = 0; q < 4; q++) {
+            const int d = 32 * db + 8 * q + 4 * h;
+            if (d >= a.dim) continue;
+            f32x4 v = f32x4{T.o[db][4 * q] * inv, T.o[db][4 * q + 1] * inv, T.o[db][4 * q + 2] * inv, T.o[db][4 * q + 3] * inv};
+            if (a.gated) {
+                const f32x4 gv = rb_ld4(gate + d);
+#pragma unroll
+                for (int j = 0; j < 4; j++) v[j] *= rb_sigmoid(gv[j]);
+            }
+            rb_st4(out + d, v);
+        }
+}
+
+// decode: grid (n_kv * column blocks of 32 query heads, key ranges of `span` keys, rows).  raw is not prepared: q and k are normed and rotated here, the workgroup whose
+// range holds the row's position puts the new key and value into the ring.
+template <int HD>
+__global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta, int span, int n_range) {
+    using Tile = RbTile<HD>;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+    constexpr int KS = Tile::KS, VS = Tile::VS, CH = HD / 8, WAVE_EL = 32 * (KS + VS), NREG = Tile::NDB * 16;
+    const int rr = blockIdx.z, pos = meta[KF_RB_META * rr], slot = meta[KF_RB_META * rr + 1];
+    if (pos < 0) return; /* workgroup-uniform, like the next */
+    const int first = rb_first_key(pos, a.chunk), k_lo = first + (int)blockIdx.y * span, k_hi = k_lo + span - 1 < pos ? k_lo + span - 1 : pos;
+    if (k_lo > pos) return;
+    const int GQ = a.n_head / a.n_kv, ncb = (GQ + 31) / 32, g = blockIdx.x / ncb, cb = blockIdx.x % ncb, col0 = cb * 32, ncol = GQ - col0 < 32 ? GQ - col0 : 32;
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5, kvd = a.n_kv * a.dim;
+    uint16_t* s_q = reinterpret_cast<uint16_t*>(smem_raw);                  /* [32][KS] */
+    float* s_buf = reinterpret_cast<float*>(smem_raw + 32 * KS * 2);        /* [4][HD] */
+    uint16_t* s_kv = reinterpret_cast<uint16_t*>(smem_raw + 32 * KS * 2 + 16 * HD); /* [4 waves][32][KS] + [32][VS] */
+    const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)rr * a.ldraw;
+    const size_t base = (size_t)slot * a.slot_stride + (size_t)g * a.dim;
+    uint16_t *kc = reinterpret_cast<uint16_t*>(a.k_cache) + base, *vc = reinterpret_cast<uint16_t*>(a.v_cache) + base;
+    for (int i = tid; i < 32 * KS / 8; i += 256) reinterpret_cast<u32x4*>(s_q)[i] = u32x4{0, 0, 0, 0};
+    __syncthreads();
+    for (int u = wid; u <= ncol; u += 4) {
+        if (u < ncol) {
+            rb_prep_head(raw + (size_t)(g * GQ + col0 + u) * a.dim, s_q + u * KS, reinterpret_cast<const uint16_t*>(a.q_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
+        } else if (k_hi == pos) {
+            const uint16_t* k = raw + (size_t)(a.n_head + g) * a.dim;
+            const size_t at = (size_t)(pos % a.cache_rows) * kvd;
+            for (int i = lane; i < a.dim; i += 64) vc[at + i] = k[i];
+            rb_prep_head(k, kc + at, reinterpret_cast<const uint16_t*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
+        }
+    }
+    __threadfence_block();
+    __syncthreads();
+    u32x4 qf[Tile::NS];
+#pragma unroll
+    for (int s = 0; s < Tile::NS; s++) qf[s] = *reinterpret_cast<const u32x4*>(s_q + r * KS + 16 * s + 8 * h);
+    uint16_t *ks = s_kv + (size_t)wid * WAVE_EL, *vs = ks + 32 * KS;
+    Tile T;
+    T.init();
+    const float sc2 = a.scale * RB_LOG2E;
+    constexpr int CPT = CH / 2; /* chunks per lane of a 32-row tile */
+    for (int k0 = k_lo + wid * 32; k0 <= k_hi; k0 += 128) {
+        u32x4 kr[CPT], vr[CPT];
+#pragma unroll
+        for (int i = 0; i < CPT; i++) {
+            const int ch = lane + 64 * i, key = ch / CH, d = (ch - key * CH) * 8;
+            kr[i] = vr[i] = u32x4{0, 0, 0, 0};
+            if (d < a.dim) {
+                const int kk = k0 + key < k_hi ? k0 + key : k_hi;
+                const size_t at = (size_t)(kk % a.cache_rows) * kvd + d;
+                kr[i] = *reinterpret_cast<const u32x4*>(kc + at), vr[i] = *reinterpret_cast<const u32x4*>(vc + at);
+            }
+        }
+        __builtin_amdgcn_wave_barrier();
+#pragma unroll
+        for (int i = 0; i < CPT; i++) {
+            const int ch = lane + 64 * i, key = ch / CH, d = (ch - key * CH) * 8;
+            *reinterpret_cast<u32x4*>(ks + key * KS + d) = kr[i];
+            *reinterpret_cast<u32x4*>(vs + key * VS + d) = vr[i];
+        }
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); /* the tile is this wave's own: its LDS accesses are in order, only the compiler has to be told */
+        __builtin_amdgcn_wave_barrier();
+        __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+        T.step(ks, vs, qf, sc2, k0, k_lo, k_hi, k0 + 31 <= k_hi, lane);
+    }
+    // the four waves' partial softmaxes: registers lane-major per wave, every wave finishes a quarter of them
+    __syncthreads();
+    float* ex = reinterpret_cast<float*>(s_kv); /* [4][NREG + 2][64] */
+    static_assert((NREG + 2) * 64 * 4 <= WAVE_EL * 2 + 4096, "merge area");
+#pragma unroll
+    for (int db = 0; db < Tile::NDB; db++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) ex[((size_t)wid * (NREG + 2) + db * 16 + i) * 64 + lane] = T.o[db][i];
+    ex[((size_t)wid * (NREG + 2) + NREG) * 64 + lane] = T.M;
+    ex[((size_t)wid * (NREG + 2) + NREG + 1) * 64 + lane] = xsum32(T.l);
+    __syncthreads();
+    float f[4], M = -__builtin_inff(), L = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; w++) M = fmaxf(M, ex[((size_t)w * (NREG + 2) + NREG) * 64 + lane]); /* wave 0 has seen a key: finite */
+#pragma unroll
+    for (int w = 0; w < 4; w++) {
+        f[w] = rb_exp2(ex[((size_t)w * (NREG + 2) + NREG) * 64 + lane] - M);
+        L += f[w] * ex[((size_t)w * (NREG + 2) + NREG + 1) * 64 + lane];
+    }
+    if (r >= ncol) return;
+    const int head = g * GQ + col0 + r;
+    const uint16_t* gate = raw + (size_t)(a.n_head + a.n_kv + head) * a.dim;
+    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)rr * a.ldout + (size_t)head * a.dim;
+    float* part = reinterpret_cast<float*>(a.scratch) + (((size_t)rr * a.n_head + head) * n_range + blockIdx.y) * (a.dim + 2);
+    const float inv = 1.0f / L;
+    for (int q = wid; q < Tile::NDB * 4; q += 4) { /* a quad of registers = four consecutive d */
+        const int d = 8 * q + 4 * h;
+        if (d >= a.dim) continue;
+        f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int w = 0; w < 4; w++)
+#pragma unroll
+            for (int j = 0; j < 4; j++) v[j] = fmaf(f[w], ex[((size_t)w * (NREG + 2) + 4 * q + j) * 64 + lane], v[j]);
+        if (n_range > 1) {
+#pragma unroll
+            for (int j = 0; j < 4; j++) part[2 + d + j] = v[j];
+        } else {
+            const f32x4 gv = a.gated ? rb_ld4(gate + d) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int j = 0; j < 4; j++) v[j] *= a.gated ? inv * rb_sigmoid(gv[j]) : inv;
+            rb_st4(out + d, v);
+        }
+    }
+    if (n_range > 1 && wid == 0 && h == 0) part[0] = M, part[1] = L;
+}
+__global__ void __launch_bounds__(64) rb_attn_combine_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta, int span, int n_range) {
+    const int rr = blockIdx.y, head = blockIdx.x, lane = threadIdx.x, pos = meta[KF_RB_META * rr];
+    if (pos < 0) return;
+    const int used = (pos - rb_first_key(pos, a.chunk)) / span + 1;
+    const float* part = reinterpret_cast<const float*>(a.scratch) + ((size_t)rr * a.n_head + head) * n_range * (a.dim + 2);
+    float M = -__builtin_inff(), L = 0.f;
+    for (int s = 0; s < used; s++) M = fmaxf(M, part[(size_t)s * (a.dim + 2)]);
+    for (int s = 0; s < used; s++) L += rb_exp2(part[(size_t)s * (a.dim + 2)] - M) * part[(size_t)s * (a.dim + 2) + 1];
+    const uint16_t* gate = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)rr * a.ldraw + (size_t)(a.n_head + a.n_kv + head) * a.dim;
+    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)rr * a.ldout + (size_t)head * a.dim;
+    for (int d = lane; d < a.dim; d += 64) {
+        float v = 0.f;
+        for (int s = 0; s < used; s++) v = fmaf(rb_exp2(part[(size_t)s * (a.dim + 2)] - M), part[(size_t)s * (a.dim + 2) + 2 + d], v);
+        out[d] = f2bf(v / L * (a.gated ? rb_sigmoid(bf2f(gate[d])) : 1.f));
+    }
+}
+
+constexpr int RB_MAX_RANGES = 32;
+static void decode_ranges(int n_rows, int n_kv, int keys, int& span, int& n_range) {
+    n_range = (keys + 255) / 256; /* a range is at least two tiles per wave */
+    const int want = (1024 + n_rows * n_kv - 1) / (n_rows * n_kv);
+    n_range = std::max(1, std::min(n_range, std::min(want, RB_MAX_RANGES)));
+    span = ((keys + n_range - 1) / n_range + 127) / 128 * 128;
+    n_range = (keys + span - 1) / span;
+}
+template <class K>
+static int big_lds(K kernel, size_t smem, int& done) {
+    if (done || smem <= 64 * 1024) return KF_OK;
+    if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) != hipSuccess) return KF_HIP_CHECK;
+    done = 1;
+    return KF_OK;
+}
+template <int HD>
+static int prefill_go(hipStream_t st, const kf_rb_attention& a, const int32_t* seqs, int n_seq, int max_n) {
+    constexpr size_t smem = 2 * 2 * 32 * (size_t)(RbTile<HD>::KS + RbTile<HD>::VS);
+    static int done = 0;
+    if (big_lds(rb_attn_prefill_kernel<HD>, smem, done)) return KF_HIP_CHECK;
+    const int GQ = a.n_head / a.n_kv;
+    hipLaunchKernelGGL(rb_attn_prefill_kernel<HD>, dim3((unsigned)(((long long)max_n * GQ + 127) / 128), a.n_kv, n_seq), dim3(256), smem, st, a, seqs);
+    return KF_OK;
+}
+template <int HD>
+static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n_rows, int span, int n_range) {
+    constexpr size_t tiles = 4 * 2 * 32 * (size_t)(RbTile<HD>::KS + RbTile<HD>::VS), merge = 4 * (size_t)(RbTile<HD>::NDB * 16 + 2) * 256;
+    constexpr size_t smem = 32 * RbTile<HD>::KS * 2 + 16 * HD + (tiles > merge ? tiles : merge);
+    static_assert(smem <= 160 * 1024, "LDS");
+    static int done = 0;
+    if (big_lds(rb_attn_decode_kernel<HD>, smem, done)) return KF_HIP_CHECK;
+    const int ncb = (a.n_head / a.n_kv + 31) / 32;
+    hipLaunchKernelGGL(rb_attn_decode_kernel<HD>, dim3(a.n_kv * ncb, n_range, n_rows), dim3(256), smem, st, a, meta, span, n_range);
+    if (n_range > 1) hipLaunchKernelGGL(rb_attn_combine_kernel, dim3(a.n_head, n_rows), dim3(64), 0, st, a, meta, span, n_range);
+    return KF_OK;
+}
+static bool mfma_served(const kf_rb_attention& a) {
+    return a.type == KF_BF16 && a.dim % 8 == 0 && a.dim <= 256 && a.ldraw % 8 == 0 && a.ldout % 4 == 0 && a.slot_stride % 8 == 0;
+}
+#define RB_BY_DIM(call)                       \
+    (a.dim <= 32    ? call(32)                \
+     : a.dim <= 64  ? call(64)                \
+     : a.dim <= 96  ? call(96)                \
+     : a.dim <= 128 ? call(128)               \
+     : a.dim <= 192 ? call(192)               \
+                    : call(256))
+
+template <class T>
+static void prep_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n, bool store) {
+    const dim3 grid(n, (a.n_head + a.n_kv + 3) / 4);
+    const size_t smem = 4 * (size_t)a.dim * sizeof(float);
+    if (store) hipLaunchKernelGGL((rb_prep_kernel<T, true>), grid, dim3(256), smem, st, a, meta);
+    else hipLaunchKernelGGL((rb_prep_kernel<T, false>), grid, dim3(256), smem, st, a, meta);
+}
+template <class T>
+static void plain_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n, int ring_only) {
+    hipLaunchKernelGGL(rb_attn_plain_kernel<T>, dim3(n, a.n_head), dim3(64), (size_t)a.dim * sizeof(float), st, a, meta, ring_only);
+}
+template <class T>
+static void store_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n) {
+    const int kvd = a.n_kv * a.dim;
+    hipLaunchKernelGGL(rb_store_kernel<T>, dim3(n), dim3(kvd >= 256 ? 256 : 64), 0, st, a, meta);
+}
+
+}  // namespace kf
+
+using namespace kf;
+static int check_attention(const kf_rb_attention* a, const int32_t* meta, int n, const char* who) {
+    if (!a || !meta || n < 1 || !a->raw || !a->out || !a->k_cache || !a->v_cache || !a->rope) return abi_fail(KF_INVALID_ARGS, "%s: null pointer", who);
+    if (a->type != KF_BF16 && a->type != KF_F32) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: storage %d", who, a->type);
+    if (a->n_head < 1 || a->n_kv < 1 || a->n_head % a->n_kv || a->dim < 1 || a->rot_dims < 0 || a->rot_dims > a->dim || (a->rot_dims & 1) || a->chunk < 0 || a->cache_rows < 1)
+        return abi_fail(KF_INVALID_ARGS, "%s: %d / %d heads of %d, %d rotated, chunk %d, %d cache rows", who, a->n_head, a->n_kv, a->dim, a->rot_dims, a->chunk, a->cache_rows);
+    if (a->dim > 512) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: head size %d (served: up to 512)", who, a->dim);
+    const int64_t cols = (int64_t)(a->gated ? 2 : 1) * a->n_head * a->dim + (int64_t)a->n_kv * a->dim;
+    if (a->ldraw < cols || a->ldout < (int64_t)a->n_head * a->dim || a->slot_stride < (int64_t)a->cache_rows * a->n_kv * a->dim) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
+    if (!al16(a->raw) || !al16(a->out) || !al16(a->k_cache) || !al16(a->v_cache)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
+    return KF_OK;
+}
+extern "C" {
+
+size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim) { return n_rows < 1 || n_head < 1 || dim < 1 ? 0 : (size_t)n_rows * n_head * RB_MAX_RANGES * (dim + 2) * sizeof(float); }
+
+int kf_rb_attention_prefill(kf_ctx* c, const kf_rb_attention* ap, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n) {
+    CHKCTX(c);
+    const int rc = check_attention(ap, meta, n_rows, "kf_rb_attention_prefill");
+    if (rc) return rc;
+    if (!seqs || n_seq < 1 || max_n < 1 || max_n > n_rows || !ap->k_new || !al16(ap->k_new)) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_prefill: bad arguments");
+    const kf_rb_attention& a = *ap;
+    hipStream_t st = c->stream;
+    int r = KF_OK;
+    if (a.type == KF_BF16) {
+        prep_go<uint16_t>(st, a, meta, n_rows, false);
+        if (mfma_served(a)) {
+#define RB_CALL(HD) prefill_go<HD>(st, a, seqs, n_seq, max_n)
+            r = RB_BY_DIM(RB_CALL);
+#undef RB_CALL
+        } else {
+            plain_go<uint16_t>(st, a, meta, n_rows, 0);
+        }
+        store_go<uint16_t>(st, a, meta, n_rows);
+    } else {
+        prep_go<float>(st, a, meta, n_rows, false);
+        plain_go<float>(st, a, meta, n_rows, 0);
+        store_go<float>(st, a, meta, n_rows);
+    }
+    if (r != KF_OK || hipGetLastError() != hipSuccess) return abi_fail(KF_HIP_CHECK, "kf_rb_attention_prefill: launch failed");
+    return KF_OK;
+}
+int kf_rb_attention_decode(kf_ctx* c, const kf_rb_attention* ap, const int32_t* meta, int n_rows, int max_pos) {
+    CHKCTX(c);
+    const int rc = check_attention(ap, meta, n_rows, "kf_rb_attention_decode");
+    if (rc) return rc;
+    if (max_pos < 0) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: max_pos %d", max_pos);
+    const kf_rb_attention& a = *ap;
+    hipStream_t st = c->stream;
+    int r = KF_OK;
+    if (mfma_served(a)) {
+        int keys = max_pos + 1, span, n_range;
+        if (a.chunk > 0 && keys > a.chunk) keys = a.chunk;
+        decode_ranges(n_rows, a.n_kv * ((a.n_head / a.n_kv + 31) / 32), keys, span, n_range);
+        if (n_range > 1 && !a.scratch) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: null scratch");
+#define RB_CALL(HD) decode_go<HD>(st, a, meta, n_rows, span, n_range)
+        r = RB_BY_DIM(RB_CALL);
+#undef RB_CALL
+    } else if (a.type == KF_BF16) {
+        prep_go<uint16_t>(st, a, meta, n_rows, true);
+        plain_go<uint16_t>(st, a, meta, n_rows, 1);
+    } else {
+        prep_go<float>(st, a, meta, n_rows, true);
+        plain_go<float>(st, a, meta, n_rows, 1);
+    }
+    if (r != KF_OK || hipGetLastError() != hipSuccess) return abi_fail(KF_HIP_CHECK, "kf_rb_attention_decode: launch failed");
+    return KF_OK;
+}
+
+}  // extern "C"

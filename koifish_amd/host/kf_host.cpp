@@ -1,9 +1,12 @@
 // kf_host.cpp -- see kf_host.hpp.  Plain C++17, no HIP headers; every device action is a kf_* ABI call.
 #include "kf_host.hpp"
 
+#include <algorithm>
 #include <cassert>
 #include <cstdio>
 #include <cstring>
+
+#include "kf_seq.hpp"
 
 namespace koifish {
 
@@ -55,6 +58,25 @@ int KVCache::Init(kf_ctx* c, int nl, int ms, int kvd) {
 void* KVCache::Get(CTYPE type, int layer, int pos) const {
     floatX* base = ToX(type == KV_KEY ? key : val);
     return base + ((size_t)layer * max_seq_len + pos) * kv_dim;
+}
+
+int KVCache::InitRings(kf_ctx* c, const std::vector<Ring>& layers, int n_slots, int type) {
+    rings = layers, n_slot = n_slots, n_layer = (int)layers.size(), elem = type == KF_F32 ? 4 : 2;
+    size_t n = 0;
+    for (Ring& r : rings) {
+        r.begin = n;
+        n += ((size_t)r.rows * r.dim * n_slots + 127) & ~(size_t)127;
+    }
+    for (hGTensor* t : {&key, &val}) {
+        *t = std::make_shared<GTensor>();
+        (*t)->type = type == KF_F32 ? typNUMBER::F32 : typNUMBER::BF16, (*t)->szData = n * elem;
+        KF_TRY((*t)->Alloc(c, n * elem));
+        KF_TRY(kf_memset(c, (*t)->data, 0, n * elem));
+    }
+    return KF_OK;
+}
+void* KVCache::Ring0(CTYPE type, int layer) const {
+    return reinterpret_cast<uint8_t*>((type == KV_KEY ? key : val)->data) + rings[layer].begin * elem;
 }
 
 // ------------------------------------------------------------------------------------------------ neurons
@@ -340,6 +362,10 @@ int Fish::EnsureLinearScratch(const kf_weight& w, int nTok) {
 int Fish::EnsureEngine() {
     if (engine_state != 0) return engine_state > 0 ? KF_OK : KF_ENGINE_NOT_SERVED;
     engine_state = -1;
+    if (Seq()) {
+        engine_why = std::string(Arch()) + ": the persistent engine walks Qwen3 layers";
+        return KF_ENGINE_NOT_SERVED;
+    }
     std::vector<kf_engine_layer> L(config.nLayer);
     for (int l = 0; l < config.nLayer; l++) {
         SelfAttention* a = attn[l].get();
@@ -462,6 +488,7 @@ int Fish::EngineCheck() {
 // ------------------------------------------------------------------------------------------------ tensor parallel
 int Fish::TPInit(int rank, int world, int vocab_row0) {
     if (world < 2 || world > 8 || rank < 0 || rank >= world) return KF_INVALID_ARGS;
+    if (Seq()) return KF_UNSUPPORTED_DATATYPE;
     std::memset(&tp.comm, 0, sizeof(tp.comm));
     tp.rank = rank, tp.world = world, tp.vocab_row0 = vocab_row0;
     tp.comm.rank = rank, tp.comm.world = world, tp.comm.n_max = config.nEmbed, tp.comm.per_step = 2u * (uint32_t)config.nLayer + 1u;
@@ -611,7 +638,7 @@ kf_graph* Fish::GraphFor(int pos) {
         graph_mode = true;
         const int save = fuse_level;
         fuse_level = 1;
-        if (kf_graph_begin(ctx) != KF_OK) return nullptr;
+        if (Warm(pos_bound()) != KF_OK || kf_graph_begin(ctx) != KF_OK) return nullptr;
         int rc = EnqueueStep(pos_bound());
         kf_graph* g = nullptr;
         int rc2 = kf_graph_end(ctx, &g);
@@ -806,6 +833,7 @@ int Fish::Generate(const int* prompt, int n_prompt, int n_new, int* out, bool us
 XcdReplicas::~XcdReplicas() {
     if (!hFish) return;
     kf_ctx* ctx = hFish->ctx;
+    if (slots) kf_sync(ctx);
     if (engine) {
         kf_sync(ctx);
         kf_xengine_destroy(engine);
@@ -907,11 +935,81 @@ int XcdReplicas::MakeEngine(bool allocate) {
     return KF_OK;
 }
 int XcdReplicas::Build(Fish* f, int n_seq_) {
-    if (!f || n_seq_ < 1 || n_seq_ > KF_XENGINE_MAX_SEQ) return KF_INVALID_ARGS;
+    if (!f || n_seq_ < 1) return KF_INVALID_ARGS;
+    if (SeqFish* sf = f->Seq()) {
+        const std::string miss = sf->Missing();
+        if (!miss.empty()) {
+            why = "tensor '" + miss + "' has not been set";
+            return KF_INVALID_ARGS;
+        }
+        hFish = f, n_seq = n_seq_;
+        kf_ctx* ctx = f->ctx;
+        const size_t ids = (size_t)n_seq * f->config.n_ctx * 4;
+        KF_TRY(kf_malloc(ctx, (size_t)n_seq * 16, (void**)&d_state));
+        KF_TRY(kf_malloc(ctx, ids, (void**)&d_forced));
+        KF_TRY(kf_malloc(ctx, ids, (void**)&d_tokens_out));
+        KF_TRY(kf_memset(ctx, d_state, 0, (size_t)n_seq * 16));
+        KF_TRY(kf_memset(ctx, d_forced, 0xff, ids));
+        KF_TRY(kf_memset(ctx, d_tokens_out, 0, ids));
+        slots = std::make_unique<SeqSlots>();
+        slots->d_state = d_state, slots->d_forced = d_forced, slots->d_tokens_out = d_tokens_out;
+        return sf->InitSlots(*slots, n_seq);
+    }
+    if (n_seq_ > KF_XENGINE_MAX_SEQ) return KF_INVALID_ARGS;
     hFish = f, n_seq = n_seq_;
     return MakeEngine(true);
 }
+int XcdReplicas::StepAll(int n, bool pick) {
+    if (slots) return hFish->Seq()->StepSlots(*slots, n, pick, true);
+    return kf_xengine_steps(hFish->ctx, engine, ToX(x), d_state, n, pick ? 1 : 0);
+}
+int XcdReplicas::Draw(int s) {  // state {token, pos} -> {id, pos + 1}, ids out [pos] = id
+    const MODEL_CARD& c = hFish->config;
+    if (slots) return hFish->Seq()->Draw(*slots, s, samp_params, d_rng + s);
+    return (samp_params.true_topk ? kf_sample_topk : kf_sample)(hFish->ctx, ToX(logits) + (size_t)s * c.vocab, c.vocab, samp_params.top_k, samp_params.temperature, samp_params.top_p, d_rng + s,
+                                                                nullptr, d_state + 4 * s, d_tokens_out + (size_t)s * c.n_ctx, d_forced + (size_t)s * c.n_ctx, c.n_ctx);
+}
+int XcdReplicas::Acquire() {
+    if (!slots) return KF_INVALID_ARGS;
+    for (int s = 0; s < n_seq; s++)
+        if (!slots->taken[s]) {
+            slots->taken[s] = 1;
+            return s;
+        }
+    return KF_INVALID_ARGS;
+}
+int XcdReplicas::Release(int seq) {
+    if (!slots || seq < 0 || seq >= n_seq || !slots->taken[seq]) return KF_INVALID_ARGS;
+    slots->taken[seq] = 0, slots->pos[seq] = 0; /* the rings need no clearing: a row is read only after the sequence that owns the slot has written it */
+    return KF_OK;
+}
+int XcdReplicas::Run(const SeqSpan* spans, int n_span, const int32_t* want, int n_want, float* out) {
+    if (!slots || !spans || n_span < 1 || (n_want && (!want || !out))) return KF_INVALID_ARGS;
+    SeqFish* f = hFish->Seq();
+    kf_ctx* ctx = f->ctx;
+    bool decode = true;
+    for (int i = 0; i < n_span; i++) decode = decode && spans[i].n == 1 && spans[i].pos0 > 0;
+    if (!decode) return f->Spans(*slots, spans, n_span, want, n_want, out, false);
+    std::vector<int32_t> state((size_t)4 * n_seq, 0);
+    for (int s = 0; s < n_seq; s++) state[4 * s + 2] = 1;
+    std::vector<char> parked(n_seq, 1);
+    for (int i = 0; i < n_span; i++) {
+        const SeqSpan& p = spans[i];
+        if (p.slot < 0 || p.slot >= n_seq || !parked[p.slot] || !p.tokens || p.pos0 >= f->card.n_ctx || p.tokens[0] < 0 || p.tokens[0] >= f->card.vocab) return KF_INVALID_ARGS;
+        parked[p.slot] = 0, slots->pos[p.slot] = p.pos0;
+        state[4 * p.slot] = p.tokens[0], state[4 * p.slot + 1] = p.pos0, state[4 * p.slot + 2] = 0;
+    }
+    for (int i = 0; i < n_want; i++)
+        if (want[2 * i] < 0 || want[2 * i] >= n_span || want[2 * i + 1] != 0) return KF_INVALID_ARGS;
+    slots->parked = parked;
+    KF_TRY(kf_h2d(ctx, d_state, state.data(), state.size() * 4));
+    KF_TRY(StepAll(1, false));
+    for (int i = 0; i < n_want; i++)
+        KF_TRY(kf_d2h(ctx, out + (size_t)i * f->card.vocab, reinterpret_cast<float*>(slots->dec.logits->data) + (size_t)spans[want[2 * i]].slot * f->seq_head.m, (size_t)f->card.vocab * 4));
+    return kf_sync(ctx);
+}
 int XcdReplicas::Fresh() {
+    if (slots) return KF_OK;
     if (engine && built_gen == hFish->weights_gen) return KF_OK;
     kf_ctx* ctx = hFish->ctx;
     if (engine) {
@@ -929,6 +1027,7 @@ int XcdReplicas::SetForced(int seq, const int32_t* ids, int n) {
 int XcdReplicas::SetState(int seq, int token, int pos) {
     if (seq < 0 || seq >= n_seq || pos < 0 || pos >= hFish->config.n_ctx || token < 0 || token >= hFish->config.vocab) return KF_INVALID_ARGS;
     KF_TRY(kf_memset32(hFish->ctx, d_state + 4 * seq + 3, 0, 1)); /* the status word of the re-aimed sequence */
+    if (slots) slots->pos[seq] = pos;
     return kf_set_state(hFish->ctx, d_state + 4 * seq, token, pos);
 }
 // CHAT_SAMPLER for Chat (greedy by default): one rng word per sequence, seeded per request
@@ -945,6 +1044,7 @@ int XcdReplicas::SetSampler(const CHAT_SAMPLER& sp) {
 // sequence's cache rows and skipped it (kf_abi.h: d_state [n_seq][4] = {token, pos, parked, status}).
 int XcdReplicas::Park(int seq, bool on) {
     if (seq < 0 || seq >= n_seq) return KF_INVALID_ARGS;
+    if (slots) slots->parked[seq] = on;
     return kf_memset32(hFish->ctx, d_state + 4 * seq + 2, on ? 1 : 0, 1); /* on the stream, no host sync: the queue flips these between launches */
 }
 int XcdReplicas::Status(int seq, int32_t* out4) {
@@ -958,6 +1058,10 @@ int XcdReplicas::Prefill(int seq, const int* tokens, int n) {
     if (seq < 0 || seq >= n_seq || !tokens || n < 1 || n >= c.n_ctx) return KF_INVALID_ARGS;
     kf_ctx* ctx = hFish->ctx;
     KF_TRY(Fresh());
+    if (slots) {
+        const SeqSpan sp{seq, 0, n, tokens};
+        return hFish->Seq()->Spans(*slots, &sp, 1, nullptr, 0, nullptr, true);
+    }
     {   /* the sequence's cache has the model's own layout ([layer][row][kv_dim]): for the length of the call the model's cache IS the sequence's, the rows land where they stay */
         struct Aim {
             KVCache& kc;
@@ -986,6 +1090,11 @@ int XcdReplicas::PrefillBatch(const int* slots, const int32_t* tokens, const int
         for (int t = 0; t < lens[i]; t++)
             if (tokens[(size_t)i * stride + t] < 0 || tokens[(size_t)i * stride + t] >= c.vocab) return KF_INVALID_ARGS;
         T = lens[i] > T ? lens[i] : T;
+    }
+    if (this->slots) {
+        std::vector<SeqSpan> sp;
+        for (int i = 0; i < S; i++) sp.push_back(SeqSpan{slots[i], 0, lens[i], tokens + (size_t)i * stride});
+        return f->Seq()->Spans(*this->slots, sp.data(), S, nullptr, 0, nullptr, true);
     }
     /* rows of a prompt behind its end (padding up to the batch's longest): finite values that nobody reads before a decode step rewrites them */
     const int R = S * T, C = c.nEmbed;
@@ -1056,7 +1165,7 @@ int XcdReplicas::RunSteps(int n) {
     KF_TRY(Fresh());
     for (int i = 0; i < n;) {
         const int m = n - i < steps_per_launch ? n - i : steps_per_launch;
-        KF_TRY(kf_xengine_steps(hFish->ctx, engine, ToX(x), d_state, m, 1));
+        KF_TRY(StepAll(m, true));
         i += m, steps_run += m;
     }
     return KF_OK;
@@ -1079,11 +1188,6 @@ int XcdReplicas::Chat(const int32_t* prompts, const int32_t* prompt_len, int n_r
         for (int r = 0; r < n_req; r++)
             if (max_new_each[r] < 1 || max_new_each[r] > max_new) return KF_INVALID_ARGS;
     const bool sampled = !samp_params.greedy();
-    auto draw = [&](int s) -> int {  // the slot's next id from its logits: state {token, pos} -> {id, pos + 1}, ids out [pos] = id
-        return (samp_params.true_topk ? kf_sample_topk : kf_sample)(hFish->ctx, ToX(logits) + (size_t)s * c.vocab, c.vocab, samp_params.top_k, samp_params.temperature,
-                                                                     samp_params.top_p, d_rng + s, nullptr, d_state + 4 * s, d_tokens_out + (size_t)s * c.n_ctx,
-                                                                     d_forced + (size_t)s * c.n_ctx, c.n_ctx);
-    };
     for (int r = 0; r < n_req; r++)
         if (prompt_len[r] < 1 || prompt_len[r] > stride || prompt_len[r] >= c.n_ctx) return KF_INVALID_ARGS;
     kf_ctx* ctx = hFish->ctx;
@@ -1138,7 +1242,7 @@ int XcdReplicas::Chat(const int32_t* prompts, const int32_t* prompt_len, int n_r
                         const uint64_t seed = samp_params.seed + (uint64_t)q.req;
                         KF_TRY(kf_set_state(ctx, reinterpret_cast<int32_t*>(d_rng + s), (int)(uint32_t)seed, (int)(uint32_t)(seed >> 32))); /* two words on the stream */
                         KF_TRY(kf_set_state(ctx, d_state + 4 * s, prompts[(size_t)q.req * stride + q.len - 1], q.len - 1));
-                        KF_TRY(draw(s));
+                        KF_TRY(Draw(s));
                     }
                     if (eos >= 0) {
                         int32_t first;
@@ -1154,10 +1258,10 @@ int XcdReplicas::Chat(const int32_t* prompts, const int32_t* prompt_len, int n_r
             for (int s = 0; s < n_seq; s++)
                 if (slot[s].req >= 0) active++, k = slot[s].want - slot[s].have < k ? slot[s].want - slot[s].have : k;
             if (!active) continue;
-            KF_TRY(kf_xengine_steps(ctx, engine, ToX(x), d_state, k, sampled ? 0 : 1));
+            KF_TRY(StepAll(k, !sampled));
             if (sampled)
                 for (int s = 0; s < n_seq; s++)
-                    if (slot[s].req >= 0) KF_TRY(draw(s));
+                    if (slot[s].req >= 0) KF_TRY(Draw(s));
             st[0]++, st[1] += k, steps_run += k;
             for (int s = 0; s < n_seq; s++) {
                 Slot& q = slot[s];
@@ -1204,7 +1308,7 @@ XcdTP::~XcdTP() {
 int XcdTP::Build(Fish** fs, int world) {
     if (!fs || world < 1) return KF_INVALID_ARGS;
     for (int r = 0; r < world; r++)
-        if (!fs[r]) return KF_INVALID_ARGS;
+        if (!fs[r] || fs[r]->Seq()) return KF_INVALID_ARGS;
     ranks.assign(fs, fs + world);
     Fish* f0 = fs[0];
     kf_ctx* ctx = f0->ctx;
@@ -1350,13 +1454,15 @@ void kfh_destroy(void* h) { delete reinterpret_cast<Fish*>(h); }
 const char* kfh_host_error(void) { return g_host_err.c_str(); } /* why the last kfh_create failed */
 void* kfh_ctx(void* h) { return reinterpret_cast<Fish*>(h)->ctx; }
 int kfh_set_fuse_level(void* h, int lvl) {
-    reinterpret_cast<Fish*>(h)->fuse_level = lvl;
+    Fish* f = reinterpret_cast<Fish*>(h);
+    if (f->Seq()) return lvl == 1 ? KF_OK : KF_INVALID_ARGS; /* one form of the step */
+    f->fuse_level = lvl;
     return KF_OK;
 }
 // sparse forward: h_hot[ffn] (1 = hot, CS_Picker::hot) for one layer's FFN, NULL = dense again.  The mask becomes a device row list here (load time).
 int kfh_set_hot(void* h, int layer, const int32_t* h_hot, int n) {
     Fish* f = reinterpret_cast<Fish*>(h);
-    if (layer < 0 || layer >= f->config.nLayer) return KF_INVALID_ARGS;
+    if (layer < 0 || layer >= (int)f->ffn.size()) return KF_INVALID_ARGS;
     FFN* m = f->ffn[layer].get();
     if (h_hot && n != f->config.n_ff) return KF_INVALID_ARGS; /* arguments first: a rejected call changes nothing */
     f->DropEngineTable(); /* the engine's layer table (and the captured graphs) hold the masks: rebuilt on the next step; the resident bf16 copies and the measured delays do not
@@ -1380,7 +1486,7 @@ int kfh_set_hot(void* h, int layer, const int32_t* h_hot, int n) {
 }
 int kfh_n_hot(void* h, int layer) {
     Fish* f = reinterpret_cast<Fish*>(h);
-    return (layer < 0 || layer >= f->config.nLayer) ? KF_INVALID_ARGS : f->ffn[layer]->n_hot;
+    return (layer < 0 || layer >= (int)f->ffn.size()) ? KF_INVALID_ARGS : f->ffn[layer]->n_hot;
 }
 // the persistent decode engine: on (default) / off; captured step graphs are dropped so that the next step is captured the new way
 int kfh_set_engine(void* h, int on) {
@@ -1499,7 +1605,7 @@ int kfh_engine_check(void* h) {
 
 static SLP* slot_of(Fish* f, int layer, int slot) {
     if (layer < 0) return slot == 1 ? &f->head.proj : nullptr;
-    if (layer >= f->config.nLayer) return nullptr;
+    if (layer >= (int)f->attn.size()) return nullptr;
     SelfAttention* a = f->attn[layer].get();
     FFN* m = f->ffn[layer].get();
     switch (slot) {
@@ -1574,7 +1680,7 @@ int kfh_set_norm(void* h, int layer, int slot, const void* w, int n, int is_devi
         f->final_norm.w = t;
         return KF_OK;
     }
-    if (layer >= f->config.nLayer) return KF_INVALID_ARGS;
+    if (layer >= (int)f->attn.size()) return KF_INVALID_ARGS;
     SelfAttention* a = f->attn[layer].get();
     switch (slot) {
         case 0: a->norm.w = t; break;
@@ -1595,7 +1701,7 @@ int kfh_forward(void* h, int token, int pos, uint16_t* h_logits) {
     rc = kf_d2h(f->ctx, st, f->d_state, 16);
     if (rc != KF_OK) return rc;
     if (h_logits) {
-        rc = kf_d2h(f->ctx, h_logits, f->head.preLogits->data, (size_t)f->config.vocab * 2);
+        rc = kf_d2h(f->ctx, h_logits, f->LogitsPtr(), (size_t)f->config.vocab * 2);
         if (rc != KF_OK) return rc;
     }
     return f->fuse_level == 0 ? st[2] : st[0];
@@ -1612,7 +1718,7 @@ int kfh_prefill(void* h, const int* tokens, int n, int pos0) { return reinterpre
 int kfh_set_prefill_mode(void* h, int mode, int chunk) {
     Fish* f = reinterpret_cast<Fish*>(h);
     f->prefill_mode = mode;
-    if (chunk > 0 && !f->gBUFF.bX) f->prefill_chunk = chunk;
+    if (chunk > 0 && !f->gBUFF.bX) f->prefill_chunk = chunk; /* (a SeqFish takes it from the next prompt on) */
     return KF_OK;
 }
 int kfh_set_sampler(void* h, float temperature, float top_p, int top_k, uint64_t seed) {
@@ -1630,10 +1736,11 @@ int kfh_get_tokens(void* h, int32_t* out, int n) {
     KF_TRY(f->EngineCheck());
     return kf_d2h(f->ctx, out, f->d_tokens_out, (size_t)n * 4);
 }
-void* kfh_kcache(void* h) { return reinterpret_cast<Fish*>(h)->cache.key->data; }
-void* kfh_vcache(void* h) { return reinterpret_cast<Fish*>(h)->cache.val->data; }
-void* kfh_logits(void* h) { return reinterpret_cast<Fish*>(h)->head.preLogits->data; }
-void* kfh_hidden(void* h) { return reinterpret_cast<Fish*>(h)->x->data; }
+void* kfh_kcache(void* h) { return reinterpret_cast<Fish*>(h)->cache.key ? reinterpret_cast<Fish*>(h)->cache.key->data : nullptr; }
+void* kfh_vcache(void* h) { return reinterpret_cast<Fish*>(h)->cache.val ? reinterpret_cast<Fish*>(h)->cache.val->data : nullptr; }
+void* kfh_logits(void* h) { return reinterpret_cast<Fish*>(h)->LogitsPtr(); }
+void* kfh_hidden(void* h) { return reinterpret_cast<Fish*>(h)->x ? reinterpret_cast<Fish*>(h)->x->data : nullptr; }
+const char* kfh_arch(void* h) { return reinterpret_cast<Fish*>(h)->Arch(); }
 // ---- tensor parallel
 int kfh_tp_init(void* h, int rank, int world, int vocab_row0) { return reinterpret_cast<Fish*>(h)->TPInit(rank, world, vocab_row0); }
 void* kfh_tp_area(void* h) { return reinterpret_cast<Fish*>(h)->tp.area; }
@@ -1737,6 +1844,19 @@ int kfh_xr_chat_each(void* h, const int32_t* prompts, const int32_t* prompt_len,
                      const int32_t* max_new_each) {
     return reinterpret_cast<XcdReplicas*>(h)->Chat(prompts, prompt_len, n_req, stride, max_new, eos, out, out_len, stats, max_new_each);
 }
+// a free slot (< 0: none) / given back; SeqFish models
+int kfh_xr_acquire(void* h) { return reinterpret_cast<XcdReplicas*>(h)->Acquire(); }
+int kfh_xr_release(void* h, int seq) { return reinterpret_cast<XcdReplicas*>(h)->Release(seq); }
+// n_span requests' next tokens (spans [n_span][3] = {slot, first position, tokens}, ids back to back) as one batch; logits of the want [n_want][2] = {span, offset} rows
+int kfh_xr_run(void* h, int n_span, const int32_t* spans3, const int32_t* ids, int n_want, const int32_t* want, float* out) {
+    std::vector<SeqSpan> sp;
+    for (int i = 0; i < n_span; i++) {
+        sp.push_back(SeqSpan{spans3[3 * i], spans3[3 * i + 1], spans3[3 * i + 2], ids});
+        if (spans3[3 * i + 2] < 1) return KF_INVALID_ARGS;
+        ids += spans3[3 * i + 2];
+    }
+    return reinterpret_cast<XcdReplicas*>(h)->Run(sp.data(), n_span, want, n_want, out);
+}
 int kfh_xr_status(void* h, int seq, int32_t* out4) { return reinterpret_cast<XcdReplicas*>(h)->Status(seq, out4); }
 int kfh_xr_set_steps_per_launch(void* h, int n) {
     if (n < 1 || n > 4096) return KF_INVALID_ARGS;
@@ -1755,18 +1875,25 @@ int kfh_xr_get_state(void* h, int seq, int32_t* out2) {
 }
 void* kfh_xr_logits(void* h, int seq) {
     XcdReplicas* r = reinterpret_cast<XcdReplicas*>(h);
+    if (r->slots) {
+        void* p = nullptr;
+        return r->hFish->Seq()->Logits16(*r->slots, seq, &p) == KF_OK ? p : nullptr;
+    }
     return ToX(r->logits) + (size_t)seq * r->hFish->config.vocab;
 }
 void* kfh_xr_hidden(void* h, int seq) {
     XcdReplicas* r = reinterpret_cast<XcdReplicas*>(h);
+    if (!r->x) return nullptr;
     return ToX(r->x) + (size_t)seq * r->hFish->config.nEmbed;
 }
 void* kfh_xr_kcache(void* h, int seq) {
     XcdReplicas* r = reinterpret_cast<XcdReplicas*>(h);
+    if (!r->key) return nullptr;
     return ToX(r->key) + (size_t)seq * r->kv_seq_elems();
 }
 void* kfh_xr_vcache(void* h, int seq) {
     XcdReplicas* r = reinterpret_cast<XcdReplicas*>(h);
+    if (!r->val) return nullptr;
     return ToX(r->val) + (size_t)seq * r->kv_seq_elems();
 }
 void* kfh_xtp_create(void** fishes, int world, int* rc_out) {

@@ -26,6 +26,9 @@ using floatX = kf_bf16;
 enum class typNUMBER : uint8_t { F32 = 0, F64, F16, BF16, F8E5M2, F8E4M3, U8, I8, U16, I16, U32, I32, U64, I64, Q4, Q3, Q2, T_SIGN, T_SEQ, BOOL1, T_BINARY };
 
 struct Fish;
+struct SeqFish;   // kf_seq.hpp: decoders described layer by layer, on the row-batch operators
+struct SeqSlots;
+struct SeqSpan;
 
 #define KF_TRY(expr)                 \
     do {                             \
@@ -70,6 +73,16 @@ struct KVCache {
     int n_layer = 0, max_seq_len = 0, kv_dim = 0;
     int Init(kf_ctx* c, int n_layer, int max_seq, int kv_dim);
     void* Get(CTYPE type, int layer, int pos) const;  // Cache.cpp:42-57
+    // Per-layer rings: layer l of slot s keeps the last `rows` positions (what the layer's mask can still see), position p in row p % rows, a row = dim elements; all
+    // slots of a layer together, a slot rows * dim elements after the one before
+    struct Ring {
+        int rows = 0, dim = 0;
+        size_t begin = 0;  // elements in front of the layer
+    };
+    std::vector<Ring> rings;
+    int n_slot = 0, elem = 2;
+    int InitRings(kf_ctx* c, const std::vector<Ring>& layers, int n_slots, int type);
+    void* Ring0(CTYPE type, int layer) const;  // slot 0 of the layer
 };
 
 struct GeNeuron {
@@ -257,25 +270,29 @@ struct Fish {
     std::vector<int> graph_bound;
     hGTensor x;                   // residual stream
 
-    ~Fish();
+    virtual ~Fish();
+    virtual const char* Arch() const { return "Qwen3"; }
+    virtual SeqFish* Seq() { return nullptr; }
+    virtual void* LogitsPtr() { return head.preLogits ? head.preLogits->data : nullptr; }  // the last step's logits, bf16 [vocab]
     // the attention kernels are instantiated for query-group sizes 1, 2, 4, 8 and head_dim 64 / 128 (every Qwen3 size except the 14B's group of 5)
     static bool ShapeServed(const MODEL_CARD& card, std::string& why);
     int Build(const MODEL_CARD& card, int device, void* stream);
     int pos_bound() const;  // launch-geometry bound for the current bucket
     // one token through every neuron (Fish::ForwardOnRLS, gLLM.cpp:722-787)
-    int ForwardOnRLS(int token, int pos);
-    int EnqueueStep(int bound);  // the launch sequence of one step, positions/tokens from d_state
+    virtual int ForwardOnRLS(int token, int pos);
+    virtual int Warm(int) { return KF_OK; }  // called before a step is captured: whatever must not happen inside the capture
+    virtual int EnqueueStep(int bound);  // the launch sequence of one step, positions/tokens from d_state
     kf_graph* GraphFor(int pos);
     int SetState(int token, int pos);
     // token-serial prefill then greedy decode (Fish::Chat, GoPT.cpp:1139-1159); ids of the new tokens to out
     int Generate(const int* prompt, int n_prompt, int n_new, int* out, bool use_graph);
     // replay n decode steps starting at `pos` with whatever d_forced holds (bench / long runs); no host sync
-    bool OneLaunchStep(); /* the decode step is one kernel launch: launched directly, no graph */
+    virtual bool OneLaunchStep(); /* the decode step is one kernel launch: launched directly, no graph */
     int RunSteps(int pos, int n, bool use_graph);
     // n prompt tokens at positions pos0.. through every layer as token batches (MFMA tile kernels), then the head on the last one:
     // afterwards the KV cache holds rows pos0..pos0+n-1, d_state = {greedy next token, pos0+n}, d_tokens_out[pos0+n-1] = that token.
     // The reference prefills token by token (Fish::Chat, GoPT.cpp:1139-1146); same arithmetic per token, fp32 sums in MFMA order.
-    int Prefill(const int* tokens, int n, int pos0);
+    virtual int Prefill(const int* tokens, int n, int pos0);
     int PrefillReady(int min_rows = 0);  // the token-batch buffers ([rows >= min_rows]), scratch and resident copies: allocated by the first prefill, grown by a larger batch
     // rows per token batch (clamped to n_ctx).  Measured, Qwen3-0.6B 4-bit, prompt filling the context: 2047 tokens 20.9 / 15.5 / 9.8 ms at 512 / 1024 / 2048 rows,
     // 8191 tokens 92.3 / 53.9 / 42.7 / 36.6 ms at 1024 / 2048 / 4096 / 8192 (scratch/prefill_chunk.py): the tile kernels want many rows per launch.
@@ -298,6 +315,15 @@ struct XcdReplicas {
     int32_t* d_forced = nullptr;      // [n_seq][n_ctx], -1 = free running
     int32_t* d_tokens_out = nullptr;  // [n_seq][n_ctx]
     std::string why;        // why the model is not served, "" when it is
+    // a SeqFish has no engine: its slots (rings, logits, work areas) live here, a step is the row-batch launches over all of them; the decode states are the same arrays
+    std::unique_ptr<SeqSlots> slots;
+    int StepAll(int n, bool pick);                 // n steps of every sequence that is not parked
+    int Draw(int seq);                             // the next id of a sequence from its logits (samp_params, its own rng)
+    int Acquire();                                 // a free slot for a new request, < 0: none
+    int Release(int seq);
+    // the next tokens of several requests in one batch; want: (span, offset) pairs, their logits fp32 [n_want][vocab] to the host.  Spans of one token behind position 0 run
+    // as a decode step over the slots, anything else as a prompt batch
+    int Run(const SeqSpan* spans, int n_span, const int32_t* want, int n_want, float* out);
     int steps_per_launch = 32;
     long long steps_run = 0;
     size_t engine_ws_bytes = 0;

@@ -12,6 +12,7 @@
 #include <cstring>
 
 #include "kf_host.hpp"
+#include "kf_seq.hpp"
 
 namespace koifish {
 
@@ -945,6 +946,11 @@ Fish* LoadHF(const std::string& dir, int device, void* stream, typNUMBER layer_t
     JSON cfg;
     std::string jerr;
     if (!JSON::Parse(text.data(), text.size(), cfg, jerr) || cfg.kind != JSON::OBJ) return bail(KF_INVALID_ARGS, "config.json: " + jerr);
+    if (const JSON* arch = cfg.get("architecture")) { /* designs described layer by layer have a registry of their own (kf_tizusun.cpp) */
+        if (layer_nf || head_nf) return bail(KF_UNSUPPORTED_DATATYPE, arch->str + ": storage BF16 or F32");
+        if (layer_type != head_type) return bail(KF_UNSUPPORTED_DATATYPE, arch->str + ": one storage for layers and head");
+        return BuildSeqModel(cfg, dir, device, stream, (int)layer_type, max_seq, rc_out, err);
+    }
     MODEL_CARD card;  // CLI_params.cpp:2177-2300
     card.nEmbed = (int)cfg.number_or("hidden_size", 0);
     card.nLayer = (int)cfg.number_or("num_hidden_layers", 0);
@@ -1067,6 +1073,10 @@ bool is_quant_type(typNUMBER t) { return t == typNUMBER::Q4 || t == typNUMBER::Q
 // (CLI_params.cpp:368-432, cases/qwen3/qwen3_596M_q4.json) and two keys of ours under "parameter" (rope_theta, rms_norm_eps) that the
 // reference takes from the Hugging Face card instead.
 int SaveKun(Fish* f, const std::string& path, std::string& err) {
+    if (f->Seq()) {
+        err = std::string(f->Arch()) + ": the .kun container holds Qwen3 models";
+        return KF_UNSUPPORTED_DATATYPE;
+    }
     const MODEL_CARD& c = f->config;
     std::vector<KunSlot> params = kun_params(f);
     KunWriter w;
@@ -1304,6 +1314,39 @@ void* kfh_load_hf(const char* dir, int device, void* stream, int layer_type, int
                      lnf, hnf);
     if (!f) g_st_err = err;
     return f;
+}
+// a layer-by-layer model from config.json's text, its tensors still to be set (kfh_seq_set_tensor)
+void* kfh_seq_create(const char* config_text, int device, void* stream, int type, int max_seq, int* rc) {
+    JSON cfg;
+    g_st_err.clear();
+    if (!JSON::Parse(config_text, strlen(config_text), cfg, g_st_err) || cfg.kind != JSON::OBJ) {
+        if (rc) *rc = KF_INVALID_ARGS;
+        return nullptr;
+    }
+    return static_cast<Fish*>(BuildSeqModel(cfg, "", device, stream, type, max_seq, rc, g_st_err));
+}
+int kfh_seq_set_tensor(void* h, const char* name, int rows, int cols, const void* bf16, int is_device) {
+    SeqFish* f = reinterpret_cast<Fish*>(h)->Seq();
+    return f ? f->SetTensor(name, rows, cols, bf16, is_device != 0) : KF_INVALID_ARGS;
+}
+// tensor i of the design: its name (into `name`) and shape; returns the number of tensors
+int kfh_seq_tensor(void* h, int i, char* name, int cap, int32_t* shape2) {
+    SeqFish* f = reinterpret_cast<Fish*>(h)->Seq();
+    if (!f) return KF_INVALID_ARGS;
+    if (i >= 0 && i < (int)f->targets.size()) {
+        auto it = f->targets.begin();
+        std::advance(it, i);
+        snprintf(name, cap, "%s", it->first.c_str());
+        shape2[0] = it->second.rows, shape2[1] = it->second.cols;
+    }
+    return (int)f->targets.size();
+}
+// the residual stream after every layer of the next prompt pass, to host memory [layers][rows][width]; NULL: off
+int kfh_seq_tap(void* h, float* out) {
+    SeqFish* f = reinterpret_cast<Fish*>(h)->Seq();
+    if (!f) return KF_INVALID_ARGS;
+    f->tap = out;
+    return KF_OK;
 }
 // ---- `.kun` (the reference's own checkpoint container)
 // Fish -> file; 0 or a negative code with kfh_last_error() set

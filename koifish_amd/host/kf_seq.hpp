@@ -1,0 +1,157 @@
+// kf_seq.hpp -- decoders described layer by layer (every layer its own mixer and feed-forward sizes), on the row-batch operators of include/kf_rb.h.
+//
+// A SeqFish is a Fish: the flat kfh_* surface (generate, prefill, run_steps, sampler, forced ids, graphs) and the slot scheduler (XcdReplicas: prompts in a queue, one slot
+// per live request) drive it as they drive the Qwen3 decoder.  What differs is below the step: a 32-bit residual stream, bf16 or fp32 storage, state rings sized by what
+// a layer can see, and steps over any set of slots at once.
+#pragma once
+#include <map>
+#include <string>
+#include <vector>
+
+#include "../../include/kf_rb.h"
+#include "kf_host.hpp"
+#include "kf_safetensors.hpp"
+
+namespace koifish {
+
+struct ROT_CARD {
+    int dims = 0;
+    double base = 10000, factor = 1, low = 1, high = 4, original = 1;
+    bool operator==(const ROT_CARD& o) const { return dims == o.dims && base == o.base && factor == o.factor && low == o.low && high == o.high && original == o.original; }
+};
+struct MIXER_CARD {
+    int heads = 0, kv_heads = 0, dim = 0, chunk = 0;  // chunk 0: plain causal
+    float scale = 1;
+    bool gated = false, qk_norm = false;
+    ROT_CARD rot;
+};
+struct FF_CARD {
+    enum KIND { NONE = 0, DENSE, MOE } kind = NONE;
+    int ff = 0, act = KF_RB_SILU, experts = 0, top = 0;
+};
+struct LAYER_CARD {
+    MIXER_CARD mix;
+    FF_CARD ff;
+};
+struct SEQ_CARD {
+    std::string arch;
+    int width = 0, vocab = 0, n_ctx = 0, type = KF_BF16;
+    float eps = 1e-6f, alpha = 1;
+    std::vector<LAYER_CARD> layers;
+};
+
+// activations of a row batch; one set for the decode steps (captured graphs hold its addresses), one for prompts
+struct RowWork {
+    int rows = 0, n_seq = 0, head_rows = 0;
+    hGTensor x, z, h, raw, knew, ao, act, y, rlogits, scratch;         // residual and its sum (fp32), bf16 / fp32 rows, expert outputs, router logits, key-range partials
+    hGTensor meta, seqs, tok, ids, weight, list, tile_expert, want, hl;  // int32 tables; hl: the rows the head reads
+    hGTensor logits;                                                     // fp32 [head_rows][padded vocab]
+};
+
+// the state of n slots: K / V rings, decode states, logits, the step graphs
+struct SeqSlots {
+    int n = 0;
+    KVCache kv;
+    int32_t *d_state = nullptr, *d_forced = nullptr, *d_tokens_out = nullptr;  // [n][4], [n][n_ctx], [n][n_ctx]: the owner's
+    RowWork dec;
+    hGTensor pick_ws, logits16;         // [1][vocab] bf16: what kf_sample reads
+    std::vector<int> pos;               // upper bound of every slot's position
+    std::vector<char> parked, taken;
+    std::map<int, kf_graph*> graphs;    // step graphs: 2 * bucket + (1: with the greedy pick)
+    ~SeqSlots();
+};
+
+struct SeqSpan {  // the next n tokens of the sequence in a slot
+    int slot = 0, pos0 = 0, n = 0;
+    const int32_t* tokens = nullptr;
+};
+
+struct SeqFish;
+struct RowProduct : GeNeuron {  // padded weight [m][k] (x experts)
+    hGTensor w;
+    int m = 0, k = 0, experts = 0;
+    int Forw(const void* x, int64_t ldx, int n, void* y, int64_t ldy, int epilogue, int act = 0, const float* res = nullptr, float alpha = 0, int mode = KF_RB_ALL,
+             const kf_rb_experts* ex = nullptr);
+};
+struct RowNorm : GeNeuron {
+    hGTensor w;
+    int dim = 0, ld = 0;
+    int Forw(const float* z, int n, float* x_out, void* h_out, const float* res = nullptr, float alpha = 0, int top = 0, const int32_t* rows = nullptr);
+};
+// chunked gated attention whose values are the projected keys: q | k | gate in one product, then kf_rb_attention_*
+struct ChunkAttention : GeNeuron {
+    MIXER_CARD c;
+    RowProduct qkg, proj;
+    RowNorm norm;
+    hGTensor qn, kn;
+    const float* rope = nullptr;
+    int ldraw = 0, ldout = 0;
+    int Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos);  // n_seq 0: one row per slot
+};
+struct RowFFN : GeNeuron {  // dense gated feed-forward, or routed experts
+    FF_CARD c;
+    RowProduct gateup, down, router;
+    hGTensor router_b;
+    RowNorm norm;
+    int ldact = 0;
+    int Forw(RowWork& w, int n);
+};
+
+struct SeqFish : Fish {
+    SEQ_CARD card;
+    SeqSlots self;  // the single-sequence surface: slot 0
+    RowWork pre;
+    RowProduct seq_head;
+    RowNorm seq_norm;
+    hGTensor table;
+    std::vector<std::unique_ptr<ChunkAttention>> mixers;
+    std::vector<std::unique_ptr<RowFFN>> ffs;
+    std::vector<std::pair<ROT_CARD, float*>> ropes;
+    struct Target {  // where a named tensor of the checkpoint goes
+        hGTensor to;
+        size_t offset = 0;  // elements
+        int rows = 0, cols = 0, ld = 0, half = -1;
+        bool set = false;
+    };
+    std::map<std::string, Target> targets;
+    hGTensor stage;
+    float* tap = nullptr;  // host [layers][rows][width]: the residual stream after every layer of the next prompt pass (diagnosis)
+
+    ~SeqFish() override;
+    const char* Arch() const override { return card.arch.c_str(); }
+    SeqFish* Seq() override { return this; }
+    int BuildSeq(const SEQ_CARD& c, int device, void* stream);
+    int SetTensor(const std::string& name, int rows, int cols, const void* bf16, bool is_device);
+    int Load(K_SafeTensors& st, std::string& err);
+    std::string Missing() const;  // "" when every tensor has been set
+    int Width(int n) const { return (n + KF_RB_PAD - 1) / KF_RB_PAD * KF_RB_PAD; }
+    size_t Elem() const { return card.type == KF_F32 ? 4 : 2; }
+
+    int InitSlots(SeqSlots& s, int n);
+    int Ensure(RowWork& w, int rows, int n_seq, int head_rows, bool decode);
+    int Layers(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos);
+    int HeadRows(RowWork& w, const int32_t* h_rows, int n);  // rows of w.x (host list, NULL: 0 .. n - 1) -> w.logits
+    // n_span spans in one batch (cut into passes of at most prefill_chunk rows); want: (span, offset) pairs whose logits go to out [n_want][vocab] (host);
+    // last: the last row of every span is picked, drawn from or left to the caller's sampler (state, ids out, slot logits)
+    int Spans(SeqSlots& s, const SeqSpan* spans, int n_span, const int32_t* want, int n_want, float* out, bool last);
+    int EnqueueSlots(SeqSlots& s, int bound, bool pick);
+    int StepSlots(SeqSlots& s, int steps, bool pick, bool use_graph);
+    int Draw(SeqSlots& s, int slot, const CHAT_SAMPLER& sp, uint64_t* d_rng);
+    int Logits16(SeqSlots& s, int slot, void** out);  // the slot's logits rounded to bf16
+    void DropGraphs(SeqSlots& s);
+
+    int EnqueueStep(int bound) override;
+    int Warm(int bound) override;
+    int ForwardOnRLS(int token, int pos) override;
+    int Prefill(const int* tokens, int n, int pos0) override;
+    bool OneLaunchStep() override { return false; }
+    void* LogitsPtr() override;
+};
+
+// the registry: config.json's architecture name -> its card
+typedef bool (*seq_card_reader)(const JSON& cfg, SEQ_CARD& card, std::string& err);
+seq_card_reader FindSeqArch(const std::string& architecture);
+bool ReadTizusun(const JSON& cfg, SEQ_CARD& card, std::string& err);
+SeqFish* BuildSeqModel(const JSON& cfg, const std::string& dir, int device, void* stream, int type, int max_seq, int* rc, std::string& err);
+
+}  // namespace koifish

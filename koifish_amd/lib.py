@@ -3,7 +3,7 @@ import ctypes as C
 import os
 
 HERE = os.path.dirname(os.path.abspath(__file__))
-# KF_LIB_DIR (development only: scratch/build_variant.py): a directory holding an A/B build of the two libraries
+# KF_LIB_DIR: a directory holding another build of the two libraries -- the kernels of one family of models only (build.build_part), or an A/B build (scratch/build_variant.py)
 LIB_HIP = os.path.join(os.environ.get("KF_LIB_DIR", HERE), "libkf_hip.so")
 LIB_HOST = os.path.join(os.environ.get("KF_LIB_DIR", HERE), "libkf_host.so")
 
@@ -14,7 +14,7 @@ KF_EPI_RESIDUAL = 1
 QUANT_GROUP, QUANT_ROW_LUT, QUANT_ROW_RTN = 0, 1, 2  # kf_weight.quant
 NF4 = 1000  # not a typNUMBER: "Q4 with the normal-float quant card" (QUANT_MODE::RTNf) for the helpers that take a storage type
 
-# every symbol include/kf_abi.h declares (tests/test_abi_symbols.py checks the header against this list and the .so)
+# every symbol include/kf_abi.h and include/kf_rb.h declare (tests/test_abi_symbols.py checks the header against this list and the .so)
 ABI_SYMBOLS = [
     "kf_init", "kf_destroy", "kf_sync", "kf_last_error", "kf_version", "kf_malloc", "kf_free", "kf_memset", "kf_memset32", "kf_h2d", "kf_d2h", "kf_d2d",
     "kf_graph_begin", "kf_graph_end", "kf_graph_launch", "kf_graph_destroy", "kf_event_create", "kf_event_record", "kf_event_elapsed_ms",
@@ -23,6 +23,8 @@ ABI_SYMBOLS = [
     "kf_norm_gateup_swiglu", "kf_attn_block", "kf_norm_lm_head", "kf_set_state", "kf_embed_state", "kf_embed_batch", "kf_qknorm_rope_batch", "kf_attn_prefill", "kf_sample", "kf_linear_multi", "kf_linear_multi_scratch_bytes", "kf_gateup_swiglu_batch", "kf_adamw", "kf_layernorm", "kf_gelu", "kf_sample_topk", "kf_fused_classifier", "kf_gelu_backward", "kf_swiglu_backward", "kf_rope_backward", "kf_norm_backward", "kf_norm_backward_scratch_bytes", "kf_linear_backward", "kf_linear_backward_scratch_bytes", "kf_embed_backward", "kf_attn_backward", "kf_attn_backward_scratch_bytes", "kf_attn_prefill_batch", "kf_attn_prefill_batch_strided", "kf_embed_pos", "kf_memset2d", "kf_copy_blocks", "kf_argmax_rows_state", "kf_qknorm_rope_train",
     "kf_hot_rows", "kf_linear_masked", "kf_norm_gateup_swiglu_masked", "kf_linear_scratch_bytes", "kf_set_scratch", "kf_engine_workspace_bytes", "kf_engine_create", "kf_engine_step", "kf_engine_check", "kf_engine_destroy", "kf_engine_set_embedding", "kf_engine_set_head", "kf_engine_step_head", "kf_engine_steps_head", "kf_engine_reset", "kf_set_canonical", "kf_get_canonical", "kf_engine_served", "kf_engine_tune", "kf_engine_stats", "kf_qkv_rope_batch", "kf_qkv_rope_seqs", "kf_set_dequant_arena", "kf_dequant_arena_used", "kf_resident_scratch_bytes",
     "kf_xengine_workspace_bytes", "kf_xengine_create", "kf_xengine_served", "kf_xengine_set_embedding", "kf_xengine_set_head", "kf_xengine_steps", "kf_xengine_check", "kf_xengine_reset", "kf_xengine_destroy", "kf_xengine_workspace_bytes_tp", "kf_xengine_create_tp", "kf_xengine_set_head_tp",
+    "kf_rb_linear", "kf_rb_pack", "kf_rb_embed", "kf_rb_embed_state", "kf_rb_norm", "kf_rb_attention_prefill", "kf_rb_attention_decode", "kf_rb_attention_scratch", "kf_rb_rope_table_host",
+    "kf_rb_route", "kf_rb_list_tiles", "kf_rb_pick", "kf_rb_pick_scratch", "kf_rb_to_bf16",
     "kf_tp_recv_bytes", "kf_tp_push_bytes", "kf_tp_commit", "kf_tp_alloc", "kf_tp_ipc_export", "kf_tp_ipc_open", "kf_tp_ipc_close", "kf_linear_f32_push", "kf_tp_reduce_recv", "kf_tp_lm_head", "kf_tp_pick",
 ]
 
@@ -37,7 +39,38 @@ class Weight(C.Structure):
                 ("lGroup", C.c_int32), ("qMin", C.c_int32), ("qMax", C.c_int32), ("qBias", C.c_int32), ("qzeros", C.c_void_p), ("qscales", C.c_void_p), ("quant", C.c_int32), ("reserved_", C.c_int32)]
 
 
+class RbExperts(C.Structure):
+    """struct kf_rb_experts (include/kf_rb.h)"""
+    _fields_ = [("n_expert", C.c_int32), ("top", C.c_int32), ("tile", C.c_int32), ("n_tile", C.c_int32), ("tile_expert", C.c_void_p), ("list", C.c_void_p), ("ids", C.c_void_p),
+                ("weight", C.c_void_p), ("w_stride", C.c_int64)]
+
+
+class RbProduct(C.Structure):
+    """struct kf_rb_product"""
+    _fields_ = [("w", C.c_void_p), ("x", C.c_void_p), ("y", C.c_void_p), ("res", C.c_void_p), ("ldx", C.c_int64), ("ldy", C.c_int64), ("ldr", C.c_int64), ("type", C.c_int32),
+                ("m", C.c_int32), ("k", C.c_int32), ("n", C.c_int32), ("epilogue", C.c_int32), ("act", C.c_int32), ("mode", C.c_int32), ("alpha", C.c_float), ("experts", C.POINTER(RbExperts))]
+
+
+class RbAttention(C.Structure):
+    """struct kf_rb_attention"""
+    _fields_ = [("raw", C.c_void_p), ("out", C.c_void_p), ("k_new", C.c_void_p), ("k_cache", C.c_void_p), ("v_cache", C.c_void_p), ("q_norm", C.c_void_p), ("k_norm", C.c_void_p),
+                ("rope", C.c_void_p), ("scratch", C.c_void_p), ("ldraw", C.c_int64), ("ldout", C.c_int64), ("slot_stride", C.c_int64), ("type", C.c_int32), ("n_head", C.c_int32),
+                ("n_kv", C.c_int32), ("dim", C.c_int32), ("rot_dims", C.c_int32), ("chunk", C.c_int32), ("cache_rows", C.c_int32), ("gated", C.c_int32), ("scale", C.c_float), ("eps", C.c_float)]
+
+
+RB_RELU, RB_SILU, RB_GELU_TANH = range(3)
+RB_STORE, RB_STORE_F32, RB_RESIDUAL, RB_GATED = range(4)
+RB_ALL, RB_UP, RB_DOWN, RB_SUM = range(4)
+
 _libs = None
+
+
+def use(directory):
+    """load the libraries of another build (before anything has loaded them)"""
+    global LIB_HIP, LIB_HOST
+    if _libs is not None and not LIB_HIP.startswith(str(directory)):
+        raise KFError("the libraries are loaded already (%s)" % LIB_HIP)
+    LIB_HIP, LIB_HOST = os.path.join(str(directory), "libkf_hip.so"), os.path.join(str(directory), "libkf_host.so")
 
 
 def load():
@@ -250,6 +283,30 @@ def load():
         for f in ("kfh_xtp_logits", "kfh_xtp_hidden", "kfh_xtp_kcache", "kfh_xtp_vcache"):
             getattr(host, f).restype = C.c_void_p
             getattr(host, f).argtypes = [C.c_void_p]
+        # row batches (include/kf_rb.h) and the models described layer by layer on them
+        hip.kf_rb_linear.argtypes = [C.c_void_p, C.POINTER(RbProduct)]
+        hip.kf_rb_pack.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_void_p, C.c_int64, C.c_int]
+        hip.kf_rb_embed.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_int64, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p]
+        hip.kf_rb_embed_state.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_int64, C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]
+        hip.kf_rb_norm.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_float, C.c_int, C.c_void_p, C.c_float, C.c_int, C.c_int64, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]
+        hip.kf_rb_attention_prefill.argtypes = [C.c_void_p, C.POINTER(RbAttention), C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int]
+        hip.kf_rb_attention_decode.argtypes = [C.c_void_p, C.POINTER(RbAttention), C.c_void_p, C.c_int, C.c_int]
+        hip.kf_rb_attention_scratch.argtypes, hip.kf_rb_attention_scratch.restype = [C.c_int, C.c_int, C.c_int], C.c_size_t
+        hip.kf_rb_rope_table_host.argtypes = [C.c_void_p, C.c_int, C.c_int] + [C.c_double] * 5
+        hip.kf_rb_route.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int64, C.c_void_p, C.c_int, C.c_void_p, C.POINTER(RbExperts)]
+        hip.kf_rb_list_tiles.argtypes = [C.c_int] * 4
+        hip.kf_rb_pick.argtypes = [C.c_void_p, C.c_void_p, C.c_int64, C.c_int, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]
+        hip.kf_rb_pick_scratch.argtypes, hip.kf_rb_pick_scratch.restype = [C.c_int], C.c_size_t
+        hip.kf_rb_to_bf16.argtypes = [C.c_void_p, C.c_void_p, C.c_void_p, C.c_size_t]
+        host.kfh_arch.restype, host.kfh_arch.argtypes = C.c_char_p, [C.c_void_p]
+        host.kfh_seq_create.restype = C.c_void_p
+        host.kfh_seq_create.argtypes = [C.c_char_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.POINTER(C.c_int)]
+        host.kfh_seq_set_tensor.argtypes = [C.c_void_p, C.c_char_p, C.c_int, C.c_int, C.c_void_p, C.c_int]
+        host.kfh_seq_tensor.argtypes = [C.c_void_p, C.c_int, C.c_char_p, C.c_int, C.c_void_p]
+        host.kfh_seq_tap.argtypes = [C.c_void_p, C.c_void_p]
+        host.kfh_xr_acquire.argtypes = [C.c_void_p]
+        host.kfh_xr_release.argtypes = [C.c_void_p, C.c_int]
+        host.kfh_xr_run.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p]
         _libs = (hip, host)
     return _libs
 

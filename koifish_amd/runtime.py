@@ -5,6 +5,8 @@ packed weights are torch.uint8 blobs laid out `data || gama` exactly as the refe
 (GTensor.cpp:456-510).
 """
 import ctypes as C
+import json
+import os
 
 import numpy as np
 import torch
@@ -620,6 +622,81 @@ class Qwen3:
         return wb + norms + kv
 
 
+class Tizusun(Qwen3):
+    """A decoder described layer by layer (koifish::SeqFish, host/kf_seq.hpp): post-norm, chunked gated attention, dense or routed feed-forwards; bf16 or true 32-bit.  The
+    generation surface is the one every model has (generate, prefill, run_steps, set_sampler, ...); XcdReplicas(model, n) serves n requests at once."""
+
+    def __init__(self, config, dtype="bfloat16", max_seq=0, device=0):
+        """config: the dict of a config.json; the tensors are set one by one (set_tensor) before the first step.  See from_dir for a checkpoint."""
+        self._open(device)
+        rc = C.c_int(0)
+        h = self.host.kfh_seq_create(json.dumps(config).encode(), device, C.c_void_p(self._stream.cuda_stream), _storage(dtype), int(max_seq), C.byref(rc))
+        self._made(h, rc, "kfh_seq_create", config, dtype)
+
+    @classmethod
+    def from_dir(cls, path, dtype="bfloat16", max_seq=0, device=0):
+        """a directory with config.json and model.safetensors"""
+        self = cls.__new__(cls)
+        self._open(device)
+        rc = C.c_int(0)
+        st = _storage(dtype)
+        h = self.host.kfh_load_hf(str(path).encode(), device, C.c_void_p(self._stream.cuda_stream), st, st, 0, int(max_seq), C.byref(rc))
+        with open(os.path.join(str(path), "config.json")) as f:
+            self._made(h, rc, "kfh_load_hf(%s)" % path, json.load(f), dtype)
+        return self
+
+    def _open(self, device):
+        self.hip, self.host = L.load()
+        if not torch.cuda.is_available():
+            raise L.KFError("no GPU visible: koifish_amd runs on MI355X only (no CPU fallback)")
+        torch.cuda.set_device(device)
+        self.device, self._stream = torch.device("cuda", device), stream(device)
+
+    def _made(self, h, rc, what, config, dtype):
+        if not h:
+            raise L.KFError("%s failed with %d: %s" % (what, rc.value, self.host.kfh_last_error().decode()))
+        self.h = C.c_void_p(h)
+        self._read_config()
+        self.config, self.dtype = config, dtype
+
+    def tensors(self):
+        """{name: (rows, cols)} of the design; cols 1: a vector"""
+        out, name, shape = {}, C.create_string_buffer(256), (C.c_int32 * 2)()
+        for i in range(self.host.kfh_seq_tensor(self.h, -1, None, 0, None)):
+            self.host.kfh_seq_tensor(self.h, i, name, 256, shape)
+            out[name.value.decode()] = (shape[0], shape[1])
+        return out
+
+    def set_tensor(self, name, w):
+        """w: torch.bfloat16, on the GPU or in host memory, [rows, cols] or [rows]"""
+        w = w.contiguous()
+        assert w.dtype == torch.bfloat16
+        rows, cols = w.shape[0], (w.shape[1] if w.dim() > 1 else 1)
+        L.check(self.host.kfh_seq_set_tensor(self.h, name.encode(), rows, cols, C.c_void_p(w.data_ptr()), int(w.is_cuda)), "kfh_seq_set_tensor(%s)" % name)
+        if w.is_cuda:
+            self.sync()   # the copy reads w on the stream
+
+    def weights_bytes(self):
+        """bytes of the design's tensors in this model's storage"""
+        return sum(r * c for r, c in self.tensors().values()) * (4 if self.dtype == "float32" else 2)
+
+    def tap(self, n_rows):
+        """the residual stream after every layer of the next prompt pass of n_rows tokens: an array [layers, n_rows, width] that the pass fills; tap(0) ends it"""
+        if not n_rows:
+            L.check(self.host.kfh_seq_tap(self.h, None), "kfh_seq_tap")
+            return None
+        self._tap = np.zeros((self.cfg["n_layer"], n_rows, self.cfg["dim"]), dtype=np.float32)
+        L.check(self.host.kfh_seq_tap(self.h, self._tap.ctypes.data_as(C.c_void_p)), "kfh_seq_tap")
+        return self._tap
+
+
+def _storage(dtype):
+    try:
+        return {"bfloat16": L.BF16, "float32": L.F32}[str(dtype)]
+    except KeyError:
+        raise L.KFError("dtype %r (bfloat16 or float32)" % (dtype,))
+
+
 class XcdReplicas:
     """Up to eight independent decoders of ONE model on one GPU, one per XCD (koifish::XcdReplicas over kf_xengine_*): the sequences share the model's weights; each has its
     own KV cache, decode state, forced ids, ids out and logits.  Every sequence's results are bit for bit those of `model.run_steps` for it alone (canonical order)."""
@@ -719,6 +796,28 @@ class XcdReplicas:
                                            out.ctypes.data_as(C.c_void_p), out_len.ctypes.data_as(C.c_void_p), stats.ctypes.data_as(C.c_void_p),
                                            None if each is None else each.ctypes.data_as(C.c_void_p)), "kfh_xr_chat_each")
         return [out[i, :out_len[i]].tolist() for i in range(n)], dict(zip(("launches", "steps", "prefills", "dropped"), (int(v) for v in stats)))
+
+    # ---- models described layer by layer (Tizusun): requests by slot, any mix of prompts and single tokens in one batch
+    def acquire(self):
+        """a slot for a new request"""
+        s = self.host.kfh_xr_acquire(self.h)
+        if s < 0:
+            raise L.KFError("no free slot (%d requests live)" % self.n_seq)
+        return s
+
+    def release(self, seq):
+        """the request in the slot is finished: its state is given back"""
+        L.check(self.host.kfh_xr_release(self.h, int(seq)), "kfh_xr_release")
+
+    def run(self, spans, want=()):
+        """spans: [(slot, first position, tokens)], the next tokens of several requests as one batch; want: [(span, offset)].  Logits of the wanted rows, float32 [len(want), vocab]"""
+        sp = np.array([(s, p, len(t)) for s, p, t in spans], dtype=np.int32).reshape(-1, 3)
+        ids = np.concatenate([np.asarray(t, dtype=np.int32) for _, _, t in spans]).astype(np.int32)
+        w = np.array(want, dtype=np.int32).reshape(-1, 2)
+        out = np.zeros((len(w), self.m.cfg["vocab"]), dtype=np.float32)
+        L.check(self.host.kfh_xr_run(self.h, len(sp), sp.ctypes.data_as(C.c_void_p), ids.ctypes.data_as(C.c_void_p), len(w), w.ctypes.data_as(C.c_void_p), out.ctypes.data_as(C.c_void_p)),
+                "kfh_xr_run")
+        return out
 
     def status(self, seq):
         """{token, pos, parked, status} of the sequence (status 64: the last launch would have left its cache rows and skipped it)"""

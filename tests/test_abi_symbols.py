@@ -11,7 +11,7 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
 def declared_functions():
-    src = open(os.path.join(ROOT, "include", "kf_abi.h")).read()
+    src = "".join(open(os.path.join(ROOT, "include", h)).read() for h in ("kf_abi.h", "kf_rb.h"))
     src = re.sub(r"/\*.*?\*/", "", src, flags=re.S)
     return sorted(set(re.findall(r"\b(kf_[a-z0-9_]+)\s*\(", src)))
 
