@@ -17,7 +17,7 @@ extern "C" {
 #define KF_RB_PAD 64
 #define KF_RB_DECODE_MAX 64 /* rows of a decode batch the streaming products serve; larger batches take the tile kernels */
 
-/* activations: relu(z); z sigmoid(z); 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) */
+/* activations; GELU in its tanh form, as kf_gelu */
 enum kf_rb_act { KF_RB_RELU = 0, KF_RB_SILU = 1, KF_RB_GELU_TANH = 2 };
 
 /* what a product's epilogue does with row dot d[t][m]:
@@ -84,9 +84,9 @@ int kf_rb_norm(kf_ctx* ctx, int type, const float* z, const float* res, float al
 /* a sequence's rows: {first row, rows, position of the first row, slot} */
 
 /* one attention layer over a row batch.  raw [rows][ldraw] holds q (n_head * dim columns), then k (n_kv * dim), then the output gate (n_head * dim, gated != 0).
- * The values ARE the projected keys (before norm and rotation); q and k are RMS-normed per head, then the first rot_dims dimensions of each head rotated (i with
- * i + rot_dims / 2) by the angles of `rope`; score = q . k * scale; position i sees j <= i with floor(i / chunk) == floor(j / chunk) (chunk 0: every j <= i).
- * out [rows][ldout] (columns n_head * dim) = softmax(scores) . v  (* sigmoid(gate)).
+ * There is no v: a row's value is its k column block as the projection left it.  q and k: RMS norm per head, then the leading rot_dims dimensions turned by the table
+ * `rope`, dimension i together with i + rot_dims / 2.  Scores are scale * <q, k>; with chunk > 0 a query sees only its own chunk (positions c chunk .. (c + 1) chunk - 1) up to
+ * itself, with chunk 0 everything up to itself.  out [rows][ldout], columns n_head * dim: softmax-weighted values, times sigmoid(gate) when gated.
  * The state: k (normed, rotated) and v rows of slot s, position j at cache[s * slot_stride + (j % cache_rows) * n_kv * dim]; cache_rows >= min(chunk, positions). */
 typedef struct kf_rb_attention {
     void* raw;
@@ -105,8 +105,8 @@ int kf_rb_attention_prefill(kf_ctx* ctx, const kf_rb_attention* a, const int32_t
 /* one row per slot; max_pos bounds the positions of the active rows (launch geometry) */
 int kf_rb_attention_decode(kf_ctx* ctx, const kf_rb_attention* a, const int32_t* meta, int n_rows, int max_pos);
 size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim);
-/* host: (cos, sin) of pos * f_i, f_i = base^(-2 i / dims), i < dims / 2.  factor != 1: wavelengths above original / low are stretched by factor, those below
- * original / high kept, between the two the blend (1 - s) f / factor + s f with s = (original / wavelength - low) / (high - low). */
+/* host: (cos, sin) of pos * w_i for i < dims / 2, w_i = base^(-2 i / dims) * (t + (1 - t) / factor), t = clamp((original w / 2 pi - low) / (high - low), 0, 1) of the
+ * unscaled w: frequencies that turn more than `high` times over `original` positions stay, those below `low` turns slow down by `factor`, a linear blend between. */
 int kf_rb_rope_table_host(float* h_table, int n_pos, int dims, double base, double factor, double low, double high, double original);
 
 /* router: logits fp32 [n][ld] (+ bias [n_expert] in the batch's storage, may be NULL) -> the `top` largest of every row (ties: the lower expert) and the softmax over them;

@@ -1,5 +1,5 @@
-// kf_rb_attn.hip -- attention of a row batch (kf_rb.h): per-head RMS norm + partial rotation of q and k, values = the projected keys, chunked causal mask, free scale,
-// sigmoid output gate, a ring of cache rows per slot.
+// kf_rb_attn.hip -- attention of a row batch (kf_rb.h): per-head RMS norm and partial rotation of q and k, unrotated k as the value, chunks, free scale, output gate, a ring
+// of cache rows per slot.
 //
 // bf16, dim a multiple of 8 up to 256: MFMA flash form, the register / LDS scheme of kf_attn_prefill.hip (S^T = K Q^T by v_mfma_f32_32x32x16_bf16, a column = one (token,
 // query head) pair per lane pair, P split into a bf16 pair for the P.V product, V^T fragments by ds_read_b64_tr_b16), with

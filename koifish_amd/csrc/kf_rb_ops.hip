@@ -373,13 +373,9 @@ int kf_rb_rope_table_host(float* t, int n_pos, int dims, double base, double fac
     for (int i = 0; i < half; i++) {
         double f = pow(base, -2.0 * i / dims);
         if (factor != 1.0) {
-            const double wavelength = two_pi / f;
-            if (wavelength > original / low) {
-                f /= factor;
-            } else if (!(wavelength < original / high)) {
-                const double s = (original / wavelength - low) / (high - low);
-                f = (1.0 - s) * f / factor + s * f;
-            }
+            const double turns = original * f / two_pi;
+            const double t = turns >= high ? 1.0 : (turns <= low ? 0.0 : (turns - low) / (high - low));
+            f *= t + (1.0 - t) / factor;
         }
         for (int p = 0; p < n_pos; p++) t[((size_t)p * half + i) * 2] = (float)cos(p * f), t[((size_t)p * half + i) * 2 + 1] = (float)sin(p * f);
     }

@@ -1341,11 +1341,11 @@ int kfh_seq_tensor(void* h, int i, char* name, int cap, int32_t* shape2) {
     }
     return (int)f->targets.size();
 }
-// the residual stream after every layer of the next prompt pass, to host memory [layers][rows][width]; NULL: off
-int kfh_seq_tap(void* h, float* out) {
+// the residual stream after every layer of the prompt passes of exactly `rows` rows, to host memory [layers][rows][width]; NULL: off
+int kfh_seq_tap(void* h, float* out, int rows) {
     SeqFish* f = reinterpret_cast<Fish*>(h)->Seq();
     if (!f) return KF_INVALID_ARGS;
-    f->tap = out;
+    f->tap = out, f->tap_rows = rows;
     return KF_OK;
 }
 // ---- `.kun` (the reference's own checkpoint container)

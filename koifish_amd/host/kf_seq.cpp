@@ -341,7 +341,7 @@ int SeqFish::Layers(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, 
     for (size_t l = 0; l < mixers.size(); l++) {
         KF_TRY(mixers[l]->Forw(w, kv, n, n_seq, max_n, max_pos));
         KF_TRY(ffs[l]->Forw(w, n));
-        if (tap && n_seq) {
+        if (tap && n_seq && n == tap_rows) {
             std::vector<float> rows((size_t)n * W);
             KF_TRY(kf_d2h(ctx, rows.data(), w.x->data, rows.size() * 4));
             for (int r = 0; r < n; r++) std::memcpy(tap + ((size_t)l * n + r) * card.width, rows.data() + (size_t)r * W, (size_t)card.width * 4);

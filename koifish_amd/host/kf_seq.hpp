@@ -115,7 +115,8 @@ struct SeqFish : Fish {
     };
     std::map<std::string, Target> targets;
     hGTensor stage;
-    float* tap = nullptr;  // host [layers][rows][width]: the residual stream after every layer of the next prompt pass (diagnosis)
+    float* tap = nullptr;  // host [layers][tap_rows][width]: the residual stream after every layer of a prompt pass of exactly tap_rows rows (diagnosis)
+    int tap_rows = 0;
 
     ~SeqFish() override;
     const char* Arch() const override { return card.arch.c_str(); }

@@ -1,8 +1,7 @@
 // kf_tizusun.cpp -- the registry of layer-by-layer designs and the reader of Tizusun's config.json.
 //
-// Tizusun: a post-norm decoder, x <- norm(alpha x + f(x)) around every sublayer.  Mixer: grouped-query attention inside chunks of `mask.size` positions; the values are the
-// projected keys; q and k RMS-normed per head, the first rot.dims dimensions rotated (wavelength-dependent frequency scaling); a sigmoid gate on the heads' outputs.
-// Feed-forward: none, a dense ReLU-gated one, or SiLU-gated experts of which a softmax over the chosen logits weighs the `top` best.
+// Tizusun: a post-norm decoder (every sublayer f: x' = norm(alpha x + f(x)), 32-bit x).  Mixer: kf_rb_attention with gate, q/k norms and chunks of `mask.size`.
+// Feed-forward: none, one ReLU-gated matrix triple, or routed SiLU-gated triples.
 #include "kf_seq.hpp"
 
 namespace koifish {

@@ -303,7 +303,7 @@ def load():
         host.kfh_seq_create.argtypes = [C.c_char_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.POINTER(C.c_int)]
         host.kfh_seq_set_tensor.argtypes = [C.c_void_p, C.c_char_p, C.c_int, C.c_int, C.c_void_p, C.c_int]
         host.kfh_seq_tensor.argtypes = [C.c_void_p, C.c_int, C.c_char_p, C.c_int, C.c_void_p]
-        host.kfh_seq_tap.argtypes = [C.c_void_p, C.c_void_p]
+        host.kfh_seq_tap.argtypes = [C.c_void_p, C.c_void_p, C.c_int]
         host.kfh_xr_acquire.argtypes = [C.c_void_p]
         host.kfh_xr_release.argtypes = [C.c_void_p, C.c_int]
         host.kfh_xr_run.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p]

@@ -623,7 +623,7 @@ class Qwen3:
 
 
 class Tizusun(Qwen3):
-    """A decoder described layer by layer (koifish::SeqFish, host/kf_seq.hpp): post-norm, chunked gated attention, dense or routed feed-forwards; bf16 or true 32-bit.  The
+    """A decoder described layer by layer (koifish::SeqFish, host/kf_seq.hpp): bf16 or true 32-bit.  The
     generation surface is the one every model has (generate, prefill, run_steps, set_sampler, ...); XcdReplicas(model, n) serves n requests at once."""
 
     def __init__(self, config, dtype="bfloat16", max_seq=0, device=0):
@@ -681,12 +681,12 @@ class Tizusun(Qwen3):
         return sum(r * c for r, c in self.tensors().values()) * (4 if self.dtype == "float32" else 2)
 
     def tap(self, n_rows):
-        """the residual stream after every layer of the next prompt pass of n_rows tokens: an array [layers, n_rows, width] that the pass fills; tap(0) ends it"""
+        """the residual stream after every layer of the prompt passes of exactly n_rows tokens: an array [layers, n_rows, width] that such a pass fills; tap(0) ends it"""
         if not n_rows:
-            L.check(self.host.kfh_seq_tap(self.h, None), "kfh_seq_tap")
+            L.check(self.host.kfh_seq_tap(self.h, None, 0), "kfh_seq_tap")
             return None
         self._tap = np.zeros((self.cfg["n_layer"], n_rows, self.cfg["dim"]), dtype=np.float32)
-        L.check(self.host.kfh_seq_tap(self.h, self._tap.ctypes.data_as(C.c_void_p)), "kfh_seq_tap")
+        L.check(self.host.kfh_seq_tap(self.h, self._tap.ctypes.data_as(C.c_void_p), int(n_rows)), "kfh_seq_tap")
         return self._tap
 
 

@@ -1,10 +1,10 @@
 """Replays a trace of token ids through a model, step by step, and writes the logits asked for.  Nothing is sampled: the model's step, its slots and its kernels are the ones
 that generation uses (runtime.XcdReplicas.run).
 
-Standard input, one JSON object a line:
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
-entries: every request's next tokens, one batch; want: places among them whose logits are written to OUT/<step>.f32 (little-endian fp32 [wanted, vocab], entry order);
-end: requests finished after the step, their slots are given back.  After every step the line `done <step>` is printed.
+Every line of standard input is a step, a JSON object such as
+    {"step": 7, "entries": [{"id": "q1", "tokens": [11], "want": [0]}, {"id": "q2", "tokens": [40], "want": []}], "end": ["q1"]}
+All entries form one batch.  `want` holds offsets into an entry's tokens: the logits of those rows go to OUT/<step>.f32, fp32 little-endian, one row of vocab floats after the
+other in the order the step names them (no file for a step that wants none).  Requests named in `end` leave their slots free.  The answer to a line is `done <step>`.
 """
 import json
 import os

@@ -30,20 +30,18 @@ def softmax(s):
 
 
 def rope_frequencies(base, dims, scaling):
-    """the dims / 2 angular frequencies, long wavelengths stretched by `factor`, short ones kept, a linear blend (in original / wavelength) between"""
+    """the dims / 2 angular frequencies: fast ones kept, slow ones divided by `factor`, a blend between (piecewise in the number of turns over `original` positions)"""
     out = []
     for i in range(dims // 2):
         f = float(base) ** (-2.0 * i / dims)
         if scaling:
-            wavelength = 2.0 * math.pi / f
             factor, low, high, original = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
-            if wavelength < original / high:
-                pass
-            elif wavelength > original / low:
+            turns = original / (2.0 * math.pi / f)
+            if turns < low:
                 f = f / factor
-            else:
-                s = (original / wavelength - low) / (high - low)
-                f = (1.0 - s) * f / factor + s * f
+            elif turns <= high:
+                kept = (turns - low) / (high - low)
+                f = kept * f + (1.0 - kept) * (f / factor)
         out.append(f)
     return np.array(out)
 
@@ -62,13 +60,11 @@ def chunk_mask(T, size):
     return (j <= i) & ((i // size == j // size) if size else True)
 
 
-def attention(h, W, mx, eps):
-    """h [T, width] -> [T, width]; W(name) gives the mixer's tensors"""
-    T, H, G, D = h.shape[0], mx["heads"], mx["kv_heads"], mx["dim"]
-    q = (h @ W("q").T).reshape(T, H, D)
-    k_raw = (h @ W("k").T).reshape(T, G, D)
-    v = k_raw                                                # the values are the projected keys, before norm and rotation
-    q, k = rms_norm(q, W("q.norm"), eps), rms_norm(k_raw, W("k.norm"), eps)
+def attend(q, v, gate, qn, kn, mx, eps):
+    """one sequence's heads: q [T, H, D], v [T, G, D] (the key projection: value as it is, key after norm and rotation), gate [T, H * D] before the sigmoid -> [T, H * D]"""
+    T, H, D = q.shape
+    G = v.shape[1]
+    q, k = rms_norm(q, qn, eps), rms_norm(v, kn, eps)
     freqs = rope_frequencies(mx["rot"]["base"], mx["rot"]["dims"], mx["rot"].get("scaling"))
     pos = np.arange(T, dtype=np.float64)
     q, k = rope(q, pos, freqs), rope(k, pos, freqs)
@@ -78,7 +74,14 @@ def attention(h, W, mx, eps):
         g = n // (H // G)
         s = np.where(seen, (q[:, n] @ k[:, g].T) * mx["scale"], -np.inf)
         out[:, n] = softmax(s) @ v[:, g]
-    return (out.reshape(T, H * D) * sigmoid(h @ W("g").T)) @ W("o").T
+    return out.reshape(T, H * D) * sigmoid(gate)
+
+
+def attention(h, W, mx, eps):
+    """h [T, width] -> [T, width]; W(name) gives the mixer's tensors"""
+    T, H, G, D = h.shape[0], mx["heads"], mx["kv_heads"], mx["dim"]
+    heads = attend((h @ W("q").T).reshape(T, H, D), (h @ W("k").T).reshape(T, G, D), h @ W("g").T, W("q.norm"), W("k.norm"), mx, eps)
+    return heads @ W("o").T
 
 
 def gated_ff(h, gate, up, down, act):
