@@ -79,6 +79,9 @@ def main():
     ap.add_argument("--lean-xcd", type=int, default=0, help="with --lean: also the XCD-confined engines on this many independent sequences of the model being run (xcd_replicas)")
     ap.add_argument("--jump", action="store_true", help="side legs only (never the run behind `value`): no token-serial run-up to the timed window -- the K / V rows of the positions in front of it "
                     "are synthetic N(0, 1) bf16 rows written once (a step's time depends on how many rows it reads, not on their values), the decode state is set to the window's first position")
+    ap.add_argument("--tizusun", default="", help="instead of the run behind `value`: prefill and decode rates of the Tizusun design at these layer sizes (2k, 4k, 2k-moe, comma-separated; "
+                    "random weights), each beside a Qwen3-shaped bf16 decoder of the same sizes; prints one JSON line")
+    ap.add_argument("--tizusun-only", default="", choices=["", "tizusun", "qwen3"], help="with --tizusun: one side alone (profiler runs)")
     ap.add_argument("--lean", action="store_true", help="only the timed decode and step_roofline (what the side legs run in their child processes)")
     ap.add_argument("--leg", default="", choices=["", "config3", "config4cpu"], help="run ONE side leg and print its JSON (child processes of the main run)")
     ap.add_argument("--side-legs", default="config3,config5,config4,qwen3_1p7b,qwen3_1p7b_launches,qwen3_4b", help="side objects beside the line, each measured in a child process after the main measurements "
@@ -93,6 +96,10 @@ def main():
         return
     if args.leg == "config4cpu":
         print(json.dumps(config4_slice_cpu()))
+        return
+
+    if args.tizusun:
+        print(json.dumps(tizusun_rates(args.tizusun.split(","), args.tizusun_only)))
         return
 
     import numpy as np
@@ -810,6 +817,72 @@ def xcd_tp_leg(nt, cfg, ctx, forced, S, K, W, shards, plan, jump=False):
         "summation_order": "canonical, tensor parallel TP = 8 (column shards as fp32 partials summed in rank order: the bits an 8-GPU node computes)",
         "parity": {"first_24_ids_equal_per_launch_rank_step": same, "oracle": "tests/test_gpu_tp.py::test_tp8_ranks_as_the_eight_xcds_of_one_launch_vs_the_oracle (ids, logits, K / V rows bit for bit)"}}
     xt.close()
+    return res
+
+
+def tizusun_rates(names, only=""):
+    """Prefill and decode throughput of Tizusun at a real model's layer sizes beside the framework's Qwen3 decoder with bf16 matrices of the same sizes.  Prompts of 2048 and 8192
+    tokens through the model's own prefill; decode behind a 1024-token prompt: one sequence through run_steps (both), 8 and 32 slots through XcdReplicas.run_steps (Tizusun:
+    Qwen3's slots decode 4-bit models only).  Times are medians over reps, the two models in turn where both run."""
+    import statistics
+    import time
+
+    import numpy as np
+    import torch
+    from koifish_amd import lib as L
+    from koifish_amd import synth
+    from koifish_amd.runtime import XcdReplicas
+
+    def timed(m, fn, reps):
+        fn()
+        m.sync()
+        out = []
+        for _ in range(reps):
+            t0 = time.perf_counter()
+            fn()
+            m.sync()
+            out.append(time.perf_counter() - t0)
+        return statistics.median(out)
+
+    res = {"metric": "Tizusun prefill and decode, tokens/s", "dtype": "bf16", "data": "synthetic", "sizes": {}}
+    for name in names:
+        peer, cfg = synth.tizusun_sizes(name)
+        r = {"layers": peer["n_layer"], "config": {k: peer[k] for k in ("dim", "n_head", "n_kv", "head_dim", "ffn", "vocab")}}
+        ms = {}
+        if only != "qwen3":
+            ms["tizusun"] = synth.tizusun_on_gpu(cfg, max_seq=peer["max_seq"])
+            r["tizusun_weight_bytes"] = ms["tizusun"].weights_bytes()
+        if only != "tizusun":
+            ms["qwen3_bf16"] = synth.build_on_gpu(peer, layer_type=L.BF16, head_type=L.BF16)
+        for n in (2048, 8192):
+            ids = np.random.default_rng(n).integers(0, peer["vocab"], size=n).astype(np.int32)
+            for k, m in ms.items():
+                r["%s_prefill_%d" % (k, n)] = round(n / timed(m, lambda: m.prefill(ids, want_logits=False), 5), 1)
+        ids = np.random.default_rng(5).integers(0, peer["vocab"], size=1024).astype(np.int32)
+        K = 64
+        for k, m in ms.items():
+            m.prefill(ids, want_logits=False)
+
+            def steps():
+                m.set_state(int(ids[0]), 1024)
+                m.run_steps(1024, K)
+            r["%s_decode_1" % k] = round(K / timed(m, steps, 5), 1)
+        if "tizusun" in ms:
+            for B in (8, 32):
+                x = XcdReplicas(ms["tizusun"], B)
+                for s in range(B):
+                    x.prefill(s, ids)
+
+                def slots():
+                    for s in range(B):
+                        x.set_state(s, int(ids[0]), 1024)
+                    x.run_steps(K)
+                r["tizusun_decode_%d" % B] = round(B * K / timed(ms["tizusun"], slots, 3), 1)
+                x.close()
+        res["sizes"][name] = r
+        for m in ms.values():
+            m.close()
+        torch.cuda.empty_cache()
     return res
 
 

@@ -39,6 +39,44 @@ int kf::abi_fail(int code, const char* fmt, ...) {
     return code;
 }
 
+namespace {
+struct UncachedBlock {
+    void* p;
+    size_t bytes;
+    int device;
+    bool used;
+};
+std::mutex g_unc_mu;
+std::vector<UncachedBlock> g_unc;
+}  // namespace
+hipError_t kf::uncached_alloc(void** out, size_t bytes) {
+    int dev = 0;
+    hipError_t e = hipGetDevice(&dev);
+    if (e != hipSuccess) return e;
+    std::lock_guard<std::mutex> lk(g_unc_mu);
+    UncachedBlock* best = nullptr;
+    for (UncachedBlock& b : g_unc)
+        if (!b.used && b.device == dev && b.bytes >= bytes && (!best || b.bytes < best->bytes)) best = &b;
+    if (!best) {
+        void* p = nullptr;
+        e = hipExtMallocWithFlags(&p, bytes, hipDeviceMallocUncached);
+        if (e != hipSuccess) return e;
+        g_unc.push_back(UncachedBlock{p, bytes, dev, false});
+        best = &g_unc.back();
+    }
+    best->used = true, *out = best->p;
+    return hipSuccess;
+}
+bool kf::uncached_free(void* p) {
+    std::lock_guard<std::mutex> lk(g_unc_mu);
+    for (UncachedBlock& b : g_unc)
+        if (b.p == p) {
+            b.used = false;
+            return true;
+        }
+    return false;
+}
+
 extern "C" {
 
 const char* kf_last_error(void) { return g_err; }
@@ -143,6 +181,10 @@ int kf_malloc(kf_ctx* c, size_t bytes, void** out) {
 }
 int kf_free(kf_ctx* c, void* p) {
     CHKCTX(c);
+    if (p && kf::uncached_free(p)) { /* every launch that reads it is over: the next owner may be another stream's */
+        HIPCHK(hipStreamSynchronize(c->stream));
+        return KF_OK;
+    }
     if (p) HIPCHK(hipFree(p));
     return KF_OK;
 }
@@ -471,7 +513,7 @@ int kf_tp_alloc(kf_ctx* c, size_t bytes, void** out) {
     // uncached (fine-grained) device memory: remote writes become visible to this device's polling loads inside a running kernel
     // No fallback to cached (coarse-grained) memory: a peer's stores into it are not guaranteed to reach a running kernel's polls, and every exchange would end in
     // a 2^24-spin timeout with no hint of the cause.
-    hipError_t e = hipExtMallocWithFlags(out, bytes, hipDeviceMallocUncached);
+    hipError_t e = kf::uncached_alloc(out, bytes);
     if (e != hipSuccess) {
         (void)hipGetLastError();
         *out = nullptr;

@@ -1349,7 +1349,7 @@ size_t engine_ws_bytes(const kf_engine_desc* d) {
 static void engine_release(EngineHost* E) {
     if (!E) return;
     if (E->args.dbg) (void)hipFree(E->args.dbg);
-    if (E->xmem) (void)hipFree(E->xmem);
+    if (E->xmem) uncached_free(E->xmem);
     delete E;
 }
 
@@ -1484,7 +1484,7 @@ int engine_build(const kf_engine_desc* d, void* ws, size_t ws_bytes, hipStream_t
     // (scratch/ub_handoff3.hip).  The XCD-local vectors (lqkv, lpart) stay in the caller's cached workspace: they are meant to live in that XCD's L2.
     E->xbytes = (size_t)eng_xoff(E->dim, E->q_dim, E->kv_dim, E->ffn, hd).end * 4;
     E->xmem = nullptr;
-    if (hipExtMallocWithFlags(&E->xmem, E->xbytes, hipDeviceMallocUncached) != hipSuccess) {
+    if (uncached_alloc(&E->xmem, E->xbytes) != hipSuccess) {
         (void)hipGetLastError();
         E->xmem = nullptr; /* the cached workspace serves (slower sweeps, same protocol) */
     }

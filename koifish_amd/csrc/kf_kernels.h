@@ -137,6 +137,11 @@ int qknorm_rope_launch(hipStream_t st, uint16_t* q, uint16_t* k, const uint16_t*
                        const int* d_pos, int n_head, int n_kv, int hd, float eps, int n_tok = 1, long long q_stride = 0, long long k_stride = 0, int seq_len = 0,
                        float* rstd_q = nullptr, float* rstd_k = nullptr);
 
+// Uncached device memory (kf_abi.hip).  A block a kernel has read is never given back to the runtime -- tensors allocated after such a free have held wrong values on this
+// part --: uncached_free puts it aside for the next uncached_alloc that it fits.  hipErrorMemoryAllocation etc. as the runtime reports them.
+hipError_t uncached_alloc(void** out, size_t bytes);
+bool uncached_free(void* p); /* false: not one of these blocks */
+
 // ---- persistent decode engine (kf_engine.hip)
 struct EngineHost;
 // Development knobs (process-wide, default = the product's choice).  Not part of the ABI and never read from the environment: tests and the scripts under

@@ -9,7 +9,7 @@ import numpy as np
 import torch
 
 from . import lib as L
-from .runtime import Qwen3, Context
+from .runtime import Qwen3, Context, Tizusun
 
 CONFIGS = {
     # Qwen3-0.6B: cases/qwen3/qwen3_0.6B.json "transformer" block; tied embeddings
@@ -119,4 +119,34 @@ def build_on_gpu(cfg, seed=1234, layer_type=L.Q4, head_type=L.BF16, device=0, lG
         m.set_norm(li, 2, nrm(cfg["head_dim"]))
         m.set_norm(li, 3, nrm(cfg["head_dim"]))
     ctx.sync()
+    return m
+
+
+# Tizusun at the layer sizes of real models (random weights; a handful of layers: every layer costs the same), each beside a Qwen3-shaped decoder of the same sizes.
+# chunk 4096 positions; `moe`: the expert sizes of a 30B-class sparse model, beside the dense decoder with as many ACTIVE feed-forward rows per token.
+_ROWS = {
+    "2k": dict(dim=2048, n_layer=8, n_head=16, n_kv=8, head_dim=128, ffn=6144, vocab=32768, max_seq=8256, theta=1e6, tied=False),
+    "4k": dict(dim=4096, n_layer=8, n_head=32, n_kv=8, head_dim=128, ffn=12288, vocab=32768, max_seq=8256, theta=1e6, tied=False),
+    "2k-moe": dict(dim=2048, n_layer=8, n_head=32, n_kv=4, head_dim=128, ffn=6144, vocab=32768, max_seq=8256, theta=1e6, tied=False, experts=128, top=8, expert_ffn=768),
+}
+
+
+def tizusun_sizes(name):
+    """(the Qwen3-shaped peer's sizes, the Tizusun config)"""
+    c = _ROWS[name]
+    mix = dict(heads=c["n_head"], kv_heads=c["n_kv"], dim=c["head_dim"], vdim=c["head_dim"], mask=dict(size=4096), scale=c["head_dim"] ** -0.5,
+               rot=dict(base=c["theta"], dims=c["head_dim"], scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192)))
+    mlp = dict(kind="moe", expert=dict(ff=c["expert_ffn"]), router=dict(experts=c["experts"], top=c["top"])) if "experts" in c else dict(kind="dense", ff=c["ffn"])
+    return c, dict(architecture="Tizusun", width=c["dim"], vocab=c["vocab"], norm=dict(eps=1e-6), postln_alpha=1.5, layers=[dict(type="attention", mixer=mix, mlp=mlp)] * c["n_layer"])
+
+
+def tizusun_on_gpu(cfg, dtype="bfloat16", max_seq=0, seed=1234, device=0, w_std=0.02):
+    """random tensors drawn on the GPU"""
+    m = Tizusun(cfg, dtype, max_seq, device)
+    g = torch.Generator(device=m.device)
+    g.manual_seed(seed)
+    for name, (r, c) in m.tensors().items():
+        w = torch.randn((r, c) if c > 1 else (r,), generator=g, device=m.device)
+        norm = c == 1 and not name.endswith(".b")
+        m.set_tensor(name, (1.0 + 0.01 * w if norm else w_std * w).to(torch.bfloat16))
     return m
