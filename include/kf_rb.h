@@ -42,7 +42,7 @@ typedef struct kf_rb_experts {
 /* how a product meets the experts:
  *   ALL   no experts
  *   UP    pair p reads row p / top of x and writes row p of y; GATED only: y is scaled by the pair's weight before it is stored
- *   DOWN  pair p reads row p of x and writes row p of y (fp32, STORE_F32)
+ *   DOWN  pair p reads row p of x and writes row p of y (STORE)
  *   SUM   row t: RESIDUAL with d = the sum over its pairs of (expert's matrix . row p of x) -- decode batches only */
 enum kf_rb_experts_mode { KF_RB_ALL = 0, KF_RB_UP = 1, KF_RB_DOWN = 2, KF_RB_SUM = 3 };
 
@@ -58,8 +58,16 @@ typedef struct kf_rb_product {
     int32_t epilogue, act, mode;
     float alpha;
     const kf_rb_experts* experts;
+    /* norm_z != NULL (decode batches for which kf_rb_linear_norms() says 1, mode ALL): x is FIRST formed as the RMS norm (norm_w, norm_eps, norm_dim columns) of the fp32 rows
+     * norm_z -- rows ldx = k apart, like x -- inside the launch, and left in x (bf16) and norm_x (fp32): kf_rb_norm and the product in one */
+    const float* norm_z;
+    const void* norm_w;
+    float* norm_x;
+    float norm_eps;
+    int32_t norm_dim;
 } kf_rb_product;
 int kf_rb_linear(kf_ctx* ctx, const kf_rb_product* p);
+int kf_rb_linear_norms(int type, int n, int k);
 
 /* load time: a bf16 matrix src [rows][cols] into a padded one of storage `type` with rows ld apart (columns cols .. ld - 1 are left alone: allocate zeroed).
  * half < 0: row r goes to row r; half 0 / 1: to row 32 (r / 16) + 16 half + r % 16, the gate / up halves of a GATED product's weight */
@@ -74,9 +82,9 @@ int kf_rb_embed_state(kf_ctx* ctx, int type, const void* table, int vocab, int d
 
 /* RMS norm of fp32 rows, z / sqrt(mean(z^2) + eps) * w over `dim` columns: x_out (fp32, may be NULL) and h_out (storage `type`) both ld apart, pad columns zero.
  *   plain:   z = row t of z
- *   experts: z = alpha res[t] + sum over the row's `top` pairs of z[t * top + j]      (res != NULL)
+ *   experts: alpha res[t] + sum over the row's `top` pairs of row t * top + j of z, which is in storage `type` then      (res != NULL)
  *   rows != NULL: output row t comes from row rows[t] */
-int kf_rb_norm(kf_ctx* ctx, int type, const float* z, const float* res, float alpha, int top, const void* w, float eps, int dim, int64_t ld, int n, const int32_t* rows,
+int kf_rb_norm(kf_ctx* ctx, int type, const void* z, const float* res, float alpha, int top, const void* w, float eps, int dim, int64_t ld, int n, const int32_t* rows,
                float* x_out, void* h_out);
 
 /* a row's meta: {position (< 0: inactive), slot, position of the sequence's first row in this batch, position of its last row in this batch} */

@@ -184,11 +184,16 @@ struct RbTile {
             st = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, A), __builtin_bit_cast(bf16x8_t, qf[s]), st, 0, 0, 0);
         }
         float mt = -__builtin_inff();
+        if (every) {
 #pragma unroll
-        for (int i = 0; i < 16; i++) {
-            const int key = k0 + 4 * h + (i & 3) + 8 * (i >> 2);
-            st[i] = every || (key >= lo && key <= hi) ? st[i] * sc2 : -__builtin_inff();
-            mt = fmaxf(mt, st[i]);
+            for (int i = 0; i < 16; i++) st[i] *= sc2, mt = fmaxf(mt, st[i]);
+        } else {
+#pragma unroll
+            for (int i = 0; i < 16; i++) {
+                const int key = k0 + 4 * h + (i & 3) + 8 * (i >> 2);
+                st[i] = key >= lo && key <= hi ? st[i] * sc2 : -__builtin_inff();
+                mt = fmaxf(mt, st[i]);
+            }
         }
         mt = xmax32(mt);
         if (mt > M) {
@@ -226,40 +231,26 @@ struct RbTile {
     }
 };
 
-// where key `key` of a sequence lies: the batch's own rows from pos0 on, the ring before
-struct RbKeys {
-    const uint16_t *k_new, *v_new; /* the sequence's first batch row, this kv-head */
-    const uint16_t *k_ring, *v_ring;
-    long long ldk, ldv;            /* batch row strides; a ring row is ldk apart too */
-    int pos0, ring;
-    __device__ __forceinline__ void at(int key, const uint16_t*& k, const uint16_t*& v) const {
-        if (key >= pos0) {
-            k = k_new + (size_t)(key - pos0) * ldk, v = v_new + (size_t)(key - pos0) * ldv;
-        } else {
-            const size_t o = (size_t)(key % ring) * ldk;
-            k = k_ring + o, v = v_ring + o;
-        }
-    }
-};
-
-// q, k_new prepared.  grid (column blocks of the longest sequence, n_kv, sequences); 128 columns per workgroup, 32 per wave, two LDS tiles
-template <int HD>
-__global__ void __launch_bounds__(256, HD <= 128 ? 2 : 1) rb_attn_prefill_kernel(const kf_rb_attention a, const int32_t* __restrict__ seqs) {
+// q, k_new prepared.  grid (column blocks of the longest sequence, n_kv, sequences), 128 columns per workgroup, 32 per wave.  KH = 2: waves 0 - 3 walk the even key tiles,
+// waves 4 - 7 the odd ones, the two partial softmaxes of a column meet in LDS at the end (launches of about one workgroup per CU last as long as their longest walk).
+// Key `key` lies in the batch from the sequence's first position on, in the slot's ring before it.
+template <int HD, int KH>
+__global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_kernel(const kf_rb_attention a, const int32_t* __restrict__ seqs) {
     using Tile = RbTile<HD>;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
-    constexpr int KS = Tile::KS, VS = Tile::VS, CH = HD / 8, CPT = (32 * CH + 255) / 256;
-    uint16_t* ks = reinterpret_cast<uint16_t*>(smem_raw); /* 2 x [32][KS] */
-    uint16_t* vs = ks + 2 * 32 * KS;                      /* 2 x [32][VS] */
+    constexpr int KS = Tile::KS, VS = Tile::VS, CH = HD / 8, CPT = (32 * CH + 255) / 256, NREG = Tile::NDB * 16;
+    const int tid = threadIdx.x & 255, lane = tid & 63, wid = tid >> 6, kh = KH == 2 ? (int)threadIdx.x >> 8 : 0, r = lane & 31, h = lane >> 5, kvd = a.n_kv * a.dim;
+    uint16_t* ks = reinterpret_cast<uint16_t*>(smem_raw) + (size_t)kh * 2 * 32 * (KS + VS); /* 2 x [32][KS] */
+    uint16_t* vs = ks + 2 * 32 * KS;                                                         /* 2 x [32][VS] */
     const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3];
-    const int GQ = a.n_head / a.n_kv, ncol = n * GQ, g = blockIdx.y, bx = (int)gridDim.x - 1 - (int)blockIdx.x;
+    // consecutive workgroups go to consecutive XCDs: the workgroups of a kv-head stay on the same ones, its keys and values in their L2
+    const int wg = (int)blockIdx.x + (int)gridDim.x * (int)blockIdx.y, g = wg % a.n_kv, bx = (int)gridDim.x - 1 - wg / a.n_kv;
+    const int GQ = a.n_head / a.n_kv, ncol = n * GQ;
     if (bx * 128 >= ncol) return; /* workgroup-uniform */
-    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5, kvd = a.n_kv * a.dim;
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw;
-    RbKeys kv;
-    kv.k_new = reinterpret_cast<const uint16_t*>(a.k_new) + (size_t)row0 * kvd + (size_t)g * a.dim, kv.v_new = raw + (size_t)(a.n_head + g) * a.dim;
-    kv.k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
-    kv.v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
-    kv.ldk = kvd, kv.ldv = a.ldraw, kv.pos0 = pos0, kv.ring = a.cache_rows;
+    const uint16_t *k_new = reinterpret_cast<const uint16_t*>(a.k_new) + (size_t)row0 * kvd + (size_t)g * a.dim, *v_new = raw + (size_t)(a.n_head + g) * a.dim;
+    const uint16_t* k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
+    const uint16_t* v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
     // this lane pair's column; columns past the end repeat the last one and are not stored
     int c = bx * 128 + wid * 32 + r;
     const bool col_ok = c < ncol;
@@ -280,16 +271,24 @@ __global__ void __launch_bounds__(256, HD <= 128 ? 2 : 1) rb_attn_prefill_kernel
         }
     }
     u32x4 kr[CPT], vr[CPT];
+    const uint32_t ldk = (uint32_t)kvd, ldv = (uint32_t)a.ldraw, ring = (uint32_t)a.cache_rows; /* offsets inside a batch or a ring fit 32 bits (checked by the launcher) */
     auto tload = [&](int k0) {
+        const int where = k0 >= pos0 ? 0 : (k0 + 31 < pos0 && k0 + 31 <= khi ? 1 : 2); /* all new, all old, a mixture (workgroup-uniform) */
 #pragma unroll
         for (int i = 0; i < CPT; i++) {
             const int ch = tid + 256 * i, key = ch / CH, d = (ch - key * CH) * 8;
             kr[i] = vr[i] = u32x4{0, 0, 0, 0};
-            if (key < 32 && d < a.dim) {
+            if ((32 * CH % 256 == 0 || key < 32) && d < a.dim) {
                 const int kk = k0 + key < khi ? k0 + key : khi; /* past the last key: masked, never read past it */
-                const uint16_t *kp, *vp;
-                kv.at(kk, kp, vp);
-                kr[i] = *reinterpret_cast<const u32x4*>(kp + d), vr[i] = *reinterpret_cast<const u32x4*>(vp + d);
+                const uint16_t *kb = k_new, *vb = v_new;
+                uint32_t ok, ov;
+                if (where == 0 || (where == 2 && kk >= pos0)) {
+                    ok = (uint32_t)(kk - pos0) * ldk, ov = (uint32_t)(kk - pos0) * ldv;
+                } else {
+                    kb = k_ring, vb = v_ring;
+                    ok = ov = ((uint32_t)kk % ring) * ldk;
+                }
+                kr[i] = *reinterpret_cast<const u32x4*>(kb + (ok + d)), vr[i] = *reinterpret_cast<const u32x4*>(vb + (ov + d));
             }
         }
     };
@@ -297,7 +296,7 @@ __global__ void __launch_bounds__(256, HD <= 128 ? 2 : 1) rb_attn_prefill_kernel
 #pragma unroll
         for (int i = 0; i < CPT; i++) {
             const int ch = tid + 256 * i, key = ch / CH, d = (ch - key * CH) * 8;
-            if (key < 32) {
+            if (32 * CH % 256 == 0 || key < 32) {
                 *reinterpret_cast<u32x4*>(ks + (b * 32 + key) * KS + d) = kr[i];
                 *reinterpret_cast<u32x4*>(vs + (b * 32 + key) * VS + d) = vr[i];
             }
@@ -306,17 +305,37 @@ __global__ void __launch_bounds__(256, HD <= 128 ? 2 : 1) rb_attn_prefill_kernel
     Tile T;
     T.init();
     const float sc2 = a.scale * RB_LOG2E;
-    tload(klo);
+    const int ntile = (khi - klo) / 32 + 1, nstep = (ntile + KH - 1) / KH; /* both key halves make the same steps and barriers; the odd half's last may be empty */
+    tload(klo + 32 * (kh < ntile ? kh : ntile - 1));
     tstore(0);
     __syncthreads();
-    int b = 0;
-    for (int k0 = klo; k0 <= khi; k0 += 32, b ^= 1) {
-        const bool more = k0 + 32 <= khi;
-        if (more) tload(k0 + 32);
-        if (k0 + 31 >= wlo && k0 <= w1) /* wave-uniform */
+    for (int j = 0; j < nstep; j++) {
+        const int t = kh + KH * j, k0 = klo + 32 * t, b = j & 1;
+        const bool more = t + KH < ntile;
+        if (more) tload(k0 + 32 * KH);
+        if (t < ntile && k0 + 31 >= wlo && k0 <= w1) /* wave-uniform */
             T.step(ks + b * 32 * KS, vs + b * 32 * VS, qf, sc2, k0, lo, pos, k0 >= wlo1 && k0 + 31 <= w0, lane);
         if (more) tstore(b ^ 1);
         __syncthreads();
+    }
+    if constexpr (KH == 2) { /* the odd half hands its part over, the even half merges */
+        float* ex = reinterpret_cast<float*>(smem_raw); /* [NREG + 2][256] */
+        if (kh == 1) {
+#pragma unroll
+            for (int db = 0; db < Tile::NDB; db++)
+#pragma unroll
+                for (int i = 0; i < 16; i++) ex[(db * 16 + i) * 256 + tid] = T.o[db][i];
+            ex[NREG * 256 + tid] = T.M, ex[(NREG + 1) * 256 + tid] = T.l;
+        }
+        __syncthreads();
+        if (kh == 1) return;
+        const float M1 = ex[NREG * 256 + tid], Mm = fmaxf(T.M, M1); /* one of the halves has seen a key of the column */
+        const float f0 = rb_exp2(T.M - Mm), f1 = rb_exp2(M1 - Mm);
+        T.l = T.l * f0 + ex[(NREG + 1) * 256 + tid] * f1;
+#pragma unroll
+        for (int db = 0; db < Tile::NDB; db++)
+#pragma unroll
+            for (int i = 0; i < 16; i++) T.o[db][i] = T.o[db][i] * f0 + ex[(db * 16 + i) * 256 + tid] * f1;
     }
     const float l = xsum32(T.l);
     if (!col_ok) return;
@@ -339,8 +358,8 @@ __global__ void __launch_bounds__(256, HD <= 128 ? 2 : 1) rb_attn_prefill_kernel
         }
 }
 
-// decode: grid (n_kv * column blocks of 32 query heads, key ranges of `span` keys, rows).  raw is not prepared: q and k are normed and rotated here, the workgroup whose
-// range holds the row's position puts the new key and value into the ring.
+// decode: grid (n_kv * column blocks of 32 query heads, key ranges of `span` keys, rows).  raw is not prepared: q and the new key are normed and rotated here while the first
+// tiles are on their way; the workgroup whose range holds the row's position patches the new key and value into its tile and puts them into the ring.
 template <int HD>
 __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta, int span, int n_range) {
     using Tile = RbTile<HD>;
@@ -352,12 +371,29 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     if (k_lo > pos) return;
     const int GQ = a.n_head / a.n_kv, ncb = (GQ + 31) / 32, g = blockIdx.x / ncb, cb = blockIdx.x % ncb, col0 = cb * 32, ncol = GQ - col0 < 32 ? GQ - col0 : 32;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5, kvd = a.n_kv * a.dim;
-    uint16_t* s_q = reinterpret_cast<uint16_t*>(smem_raw);                  /* [32][KS] */
-    float* s_buf = reinterpret_cast<float*>(smem_raw + 32 * KS * 2);        /* [4][HD] */
-    uint16_t* s_kv = reinterpret_cast<uint16_t*>(smem_raw + 32 * KS * 2 + 16 * HD); /* [4 waves][32][KS] + [32][VS] */
+    uint16_t* s_q = reinterpret_cast<uint16_t*>(smem_raw);                              /* [32][KS] */
+    uint16_t* s_new = s_q + 32 * KS;                                                    /* the new key, the new value: [2][HD] */
+    float* s_buf = reinterpret_cast<float*>(smem_raw + 32 * KS * 2 + 4 * HD);           /* [4][HD] */
+    uint16_t* s_kv = reinterpret_cast<uint16_t*>(smem_raw + 32 * KS * 2 + 4 * HD + 16 * HD); /* [4 waves] [32][KS] + [32][VS] */
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)rr * a.ldraw;
     const size_t base = (size_t)slot * a.slot_stride + (size_t)g * a.dim;
     uint16_t *kc = reinterpret_cast<uint16_t*>(a.k_cache) + base, *vc = reinterpret_cast<uint16_t*>(a.v_cache) + base;
+    constexpr int CPT = CH / 2; /* chunks per lane of a 32-row tile */
+    u32x4 kr[CPT], vr[CPT];
+    auto tload = [&](int k0) { /* (the row's own position still holds an older key: patched below) */
+#pragma unroll
+        for (int i = 0; i < CPT; i++) {
+            const int ch = lane + 64 * i, key = ch / CH, d = (ch - key * CH) * 8;
+            kr[i] = vr[i] = u32x4{0, 0, 0, 0};
+            if (d < a.dim) {
+                const int kk = k0 + key < k_hi ? k0 + key : k_hi;
+                const uint32_t at = ((uint32_t)kk % (uint32_t)a.cache_rows) * (uint32_t)kvd + d;
+                kr[i] = *reinterpret_cast<const u32x4*>(kc + at), vr[i] = *reinterpret_cast<const u32x4*>(vc + at);
+            }
+        }
+    };
+    int k0 = k_lo + wid * 32;
+    if (k0 <= k_hi) tload(k0);
     for (int i = tid; i < 32 * KS / 8; i += 256) reinterpret_cast<u32x4*>(s_q)[i] = u32x4{0, 0, 0, 0};
     __syncthreads();
     for (int u = wid; u <= ncol; u += 4) {
@@ -365,12 +401,17 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
             rb_prep_head(raw + (size_t)(g * GQ + col0 + u) * a.dim, s_q + u * KS, reinterpret_cast<const uint16_t*>(a.q_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
         } else if (k_hi == pos) {
             const uint16_t* k = raw + (size_t)(a.n_head + g) * a.dim;
+            rb_prep_head(k, s_new, reinterpret_cast<const uint16_t*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
             const size_t at = (size_t)(pos % a.cache_rows) * kvd;
-            for (int i = lane; i < a.dim; i += 64) vc[at + i] = k[i];
-            rb_prep_head(k, kc + at, reinterpret_cast<const uint16_t*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
+            for (int i = lane; i < HD; i += 64) {
+                const bool in = i < a.dim;
+                const uint16_t v = in ? k[i] : (uint16_t)0;
+                s_new[HD + i] = v;
+                if (!in) s_new[i] = 0;
+                if (in && cb == 0) kc[at + i] = s_new[i], vc[at + i] = v;
+            }
         }
     }
-    __threadfence_block();
     __syncthreads();
     u32x4 qf[Tile::NS];
 #pragma unroll
@@ -379,35 +420,26 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     Tile T;
     T.init();
     const float sc2 = a.scale * RB_LOG2E;
-    constexpr int CPT = CH / 2; /* chunks per lane of a 32-row tile */
-    for (int k0 = k_lo + wid * 32; k0 <= k_hi; k0 += 128) {
-        u32x4 kr[CPT], vr[CPT];
+    for (; k0 <= k_hi; k0 += 128) {
+        __builtin_amdgcn_wave_barrier(); /* the tile is this wave's own: its LDS accesses are in order, only the compiler has to be told */
 #pragma unroll
         for (int i = 0; i < CPT; i++) {
             const int ch = lane + 64 * i, key = ch / CH, d = (ch - key * CH) * 8;
-            kr[i] = vr[i] = u32x4{0, 0, 0, 0};
-            if (d < a.dim) {
-                const int kk = k0 + key < k_hi ? k0 + key : k_hi;
-                const size_t at = (size_t)(kk % a.cache_rows) * kvd + d;
-                kr[i] = *reinterpret_cast<const u32x4*>(kc + at), vr[i] = *reinterpret_cast<const u32x4*>(vc + at);
-            }
+            const bool own = k_hi == pos && k0 + key >= pos; /* (and the rows behind it: masked, but finite) */
+            *reinterpret_cast<u32x4*>(ks + key * KS + d) = own ? *reinterpret_cast<const u32x4*>(s_new + d) : kr[i];
+            *reinterpret_cast<u32x4*>(vs + key * VS + d) = own ? *reinterpret_cast<const u32x4*>(s_new + HD + d) : vr[i];
         }
-        __builtin_amdgcn_wave_barrier();
-#pragma unroll
-        for (int i = 0; i < CPT; i++) {
-            const int ch = lane + 64 * i, key = ch / CH, d = (ch - key * CH) * 8;
-            *reinterpret_cast<u32x4*>(ks + key * KS + d) = kr[i];
-            *reinterpret_cast<u32x4*>(vs + key * VS + d) = vr[i];
-        }
-        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront"); /* the tile is this wave's own: its LDS accesses are in order, only the compiler has to be told */
+        if (k0 + 128 <= k_hi) tload(k0 + 128);
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
         __builtin_amdgcn_wave_barrier();
         __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
         T.step(ks, vs, qf, sc2, k0, k_lo, k_hi, k0 + 31 <= k_hi, lane);
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+        __builtin_amdgcn_wave_barrier();
     }
     // the four waves' partial softmaxes: registers lane-major per wave, every wave finishes a quarter of them
     __syncthreads();
     float* ex = reinterpret_cast<float*>(s_kv); /* [4][NREG + 2][64] */
-    static_assert((NREG + 2) * 64 * 4 <= WAVE_EL * 2 + 4096, "merge area");
 #pragma unroll
     for (int db = 0; db < Tile::NDB; db++)
 #pragma unroll
@@ -481,19 +513,28 @@ static int big_lds(K kernel, size_t smem, int& done) {
     done = 1;
     return KF_OK;
 }
+template <int HD, int KH>
+static int prefill_kh(hipStream_t st, const kf_rb_attention& a, const int32_t* seqs, dim3 grid) {
+    constexpr size_t tiles = KH * 2 * 2 * 32 * (size_t)(RbTile<HD>::KS + RbTile<HD>::VS), merge = KH == 2 ? 256 * 4 * (size_t)(RbTile<HD>::NDB * 16 + 2) : 0;
+    constexpr size_t smem = tiles > merge ? tiles : merge;
+    static_assert(smem <= 160 * 1024, "LDS");
+    static int done = 0;
+    if (big_lds(rb_attn_prefill_kernel<HD, KH>, smem, done)) return KF_HIP_CHECK;
+    hipLaunchKernelGGL((rb_attn_prefill_kernel<HD, KH>), grid, dim3(256 * KH), smem, st, a, seqs);
+    return KF_OK;
+}
 template <int HD>
 static int prefill_go(hipStream_t st, const kf_rb_attention& a, const int32_t* seqs, int n_seq, int max_n) {
-    constexpr size_t smem = 2 * 2 * 32 * (size_t)(RbTile<HD>::KS + RbTile<HD>::VS);
-    static int done = 0;
-    if (big_lds(rb_attn_prefill_kernel<HD>, smem, done)) return KF_HIP_CHECK;
-    const int GQ = a.n_head / a.n_kv;
-    hipLaunchKernelGGL(rb_attn_prefill_kernel<HD>, dim3((unsigned)(((long long)max_n * GQ + 127) / 128), a.n_kv, n_seq), dim3(256), smem, st, a, seqs);
-    return KF_OK;
+    const dim3 grid((unsigned)(((long long)max_n * (a.n_head / a.n_kv) + 127) / 128), a.n_kv, n_seq);
+    if constexpr (HD <= 128) {
+        if ((long)grid.x * grid.y * grid.z <= 512 && max_n >= 256) return prefill_kh<HD, 2>(st, a, seqs, grid);
+    }
+    return prefill_kh<HD, 1>(st, a, seqs, grid);
 }
 template <int HD>
 static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n_rows, int span, int n_range) {
     constexpr size_t tiles = 4 * 2 * 32 * (size_t)(RbTile<HD>::KS + RbTile<HD>::VS), merge = 4 * (size_t)(RbTile<HD>::NDB * 16 + 2) * 256;
-    constexpr size_t smem = 32 * RbTile<HD>::KS * 2 + 16 * HD + (tiles > merge ? tiles : merge);
+    constexpr size_t smem = 32 * RbTile<HD>::KS * 2 + 20 * HD + (tiles > merge ? tiles : merge);
     static_assert(smem <= 160 * 1024, "LDS");
     static int done = 0;
     if (big_lds(rb_attn_decode_kernel<HD>, smem, done)) return KF_HIP_CHECK;
@@ -502,8 +543,8 @@ static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* me
     if (n_range > 1) hipLaunchKernelGGL(rb_attn_combine_kernel, dim3(a.n_head, n_rows), dim3(64), 0, st, a, meta, span, n_range);
     return KF_OK;
 }
-static bool mfma_served(const kf_rb_attention& a) {
-    return a.type == KF_BF16 && a.dim % 8 == 0 && a.dim <= 256 && a.ldraw % 8 == 0 && a.ldout % 4 == 0 && a.slot_stride % 8 == 0;
+static bool mfma_served(const kf_rb_attention& a, int n_rows) {
+    return a.type == KF_BF16 && (int64_t)n_rows * a.ldraw < ((int64_t)1 << 30) && (int64_t)a.cache_rows * a.n_kv * a.dim < ((int64_t)1 << 30) && a.dim % 8 == 0 && a.dim <= 256 && a.ldraw % 8 == 0 && a.ldout % 4 == 0 && a.slot_stride % 8 == 0;
 }
 #define RB_BY_DIM(call)                       \
     (a.dim <= 32    ? call(32)                \
@@ -558,7 +599,7 @@ int kf_rb_attention_prefill(kf_ctx* c, const kf_rb_attention* ap, const int32_t*
     int r = KF_OK;
     if (a.type == KF_BF16) {
         prep_go<uint16_t>(st, a, meta, n_rows, false);
-        if (mfma_served(a)) {
+        if (mfma_served(a, n_rows)) {
 #define RB_CALL(HD) prefill_go<HD>(st, a, seqs, n_seq, max_n)
             r = RB_BY_DIM(RB_CALL);
 #undef RB_CALL
@@ -582,7 +623,7 @@ int kf_rb_attention_decode(kf_ctx* c, const kf_rb_attention* ap, const int32_t* 
     const kf_rb_attention& a = *ap;
     hipStream_t st = c->stream;
     int r = KF_OK;
-    if (mfma_served(a)) {
+    if (mfma_served(a, n_rows)) {
         int keys = max_pos + 1, span, n_range;
         if (a.chunk > 0 && keys > a.chunk) keys = a.chunk;
         decode_ranges(n_rows, a.n_kv * ((a.n_head / a.n_kv + 31) / 32), keys, span, n_range);

@@ -12,6 +12,7 @@ using RbBig = G3Cfg<256, 256, 8>;
 using RbSmall = G3Cfg<128, 128, 4>;
 using RbMid = G3Cfg<64, 128, 4>;
 using RbTiny = G3Cfg<64, 64, 4>;
+using RbPairs = G3Cfg<128, 64, 4>; /* experts of about a hundred pairs: half the padding of 128-pair tiles, each weight tile read about once */
 
 template <class C, bool EXPERTS>
 __global__ void __launch_bounds__(C::NTH, C::WGS_PER_CU * C::NW / 4) rb_gemm_kernel(const RbProduct q) {
@@ -101,7 +102,7 @@ int rb_gemm_launch(hipStream_t st, const RbProduct& q) {
     auto tiles = [&](int bm, int bn) { return (long)((p.m + bm - 1) / bm) * ((p.n + bn - 1) / bn); };
     if (p.mode != KF_RB_ALL) {
         if (q.e.tile == 128) return rb_go<RbSmall, true>(st, q, (long)((p.m + 127) / 128) * q.e.n_tile);
-        if (q.e.tile == 64) return rb_go<RbTiny, true>(st, q, (long)((p.m + 63) / 64) * q.e.n_tile);
+        if (q.e.tile == 64) return rb_go<RbPairs, true>(st, q, (long)((p.m + 127) / 128) * q.e.n_tile);
         return 1;
     }
     // the measured thresholds of gemm3_launch: big tiles from 160 of them, then smaller ones that fill the chip

@@ -1,10 +1,11 @@
 // kf_rb_linear.hip -- row-batch products y[t][m] = W[m] . x[t] for few rows (decode batches) and in 32-bit, and the ABI entry that picks the form.
 //
-// Decode batches stream the weights: a workgroup owns 16 weight rows (GATED: 16 gate and the 16 up rows that follow them), its waves take the 32-deep k-steps round robin --
-// a wave instruction reads 16 rows x 64 contiguous bytes -- and multiply them against up to 64 token columns by v_mfma_f32_16x16x32_bf16 (A = weight rows, B = token rows,
-// straight from global memory: the activations of a decode batch are a few KB and stay in L2).  The waves' partial tiles meet in LDS, one thread per output finishes it.
-// With experts a workgroup's columns are the pairs of one expert (UP), or it walks every chosen expert with the columns that did not choose it held at zero (SUM): an
-// expert's rows are read once per workgroup whoever chose them.
+// Decode batches stream the weights: a workgroup owns 16 weight rows (GATED: 16 gate and the 16 up rows that follow them), its waves take runs of 32-deep k-steps -- 256
+// contiguous bytes of each of the 16 rows per run -- and multiply them against up to 64 token columns by v_mfma_f32_16x16x32_bf16 (A = weight rows, B = token rows, straight
+// from global memory: the activations of a decode batch are a few KB and stay in L2).  The next run's weights are in flight while a run is multiplied; the first run's
+// while the RMS norm in front of the product (NORM: few rows of the 32-bit residual sum, kept in LDS as bf16) is formed.  The waves' partial tiles meet in LDS, one thread
+// per output finishes it.  With experts a workgroup's columns are the pairs of one expert (UP, DOWN), or it walks all chosen experts' k-steps as one list dealt to its waves,
+// columns that did not choose an expert held at zero (SUM): an expert's rows are read once per workgroup whoever chose them.
 #include "kf_ctx.h"
 #include "kf_rb_common.h"
 
@@ -16,91 +17,50 @@ __device__ __forceinline__ f32x4 rb_mfma16(u32x4 a, u32x4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
-// k-steps wid, wid + NW, ... of the MG 16-row blocks at w (row stride k) against NT column blocks; xp[nt] = this lane's token row + 8 (lane >> 4), NULL: a zero column
-template <int NT, int MG, int NW>
-__device__ __forceinline__ void rb_stream_k(const uint16_t* __restrict__ w, int k, const uint16_t* const (&xp)[NT], f32x4 (&acc)[MG][NT], int wid, int lane) {
-    const int r16 = lane & 15, q4 = lane >> 4, nstep = k / 32;
-    const uint16_t* wr = w + (size_t)r16 * k + 8 * q4;
-    constexpr int U = NT >= 4 ? 2 : 4; /* steps in flight */
-    for (int s0 = wid; s0 < nstep; s0 += NW * U) {
-        u32x4 a[U][MG], b[U][NT];
-#pragma unroll
-        for (int u = 0; u < U; u++) {
-            const int s = s0 + u * NW;
-            const bool on = s < nstep; /* wave-uniform */
-#pragma unroll
-            for (int g = 0; g < MG; g++) {
-                a[u][g] = u32x4{0, 0, 0, 0};
-                if (on) a[u][g] = ld_nt(reinterpret_cast<const u32x4*>(wr + (size_t)g * 16 * k + 32 * s));
-            }
-#pragma unroll
-            for (int t = 0; t < NT; t++) {
-                b[u][t] = u32x4{0, 0, 0, 0};
-                if (on && xp[t]) b[u][t] = *reinterpret_cast<const u32x4*>(xp[t] + 32 * s);
-            }
-        }
-#pragma unroll
-        for (int u = 0; u < U; u++)
-#pragma unroll
-            for (int g = 0; g < MG; g++)
-#pragma unroll
-                for (int t = 0; t < NT; t++) acc[g][t] = rb_mfma16(a[u][g], b[u][t], acc[g][t]);
-    }
-}
+constexpr int RB_NORM_ROWS = 8, RB_NORM_LDS = 64 * 1024;
 
-template <int NT, bool GATED, int NW>
-__global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
-    const kf_rb_product& p = q.p;
-    constexpr int MG = GATED ? 2 : 1, COLS = 16 * NT;
-    __shared__ float red[NW][MG][COLS][17]; /* [wave][block][column][row], padded */
-    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, q4 = lane >> 4;
-    const int m0 = blockIdx.x * (16 * MG);
-    const uint16_t* W = reinterpret_cast<const uint16_t*>(p.w);
-    const uint16_t* X = reinterpret_cast<const uint16_t*>(p.x);
-    f32x4 acc[MG][NT];
+// the run of U k-steps from step s of the MG 16-row blocks at wr (this lane's row and k octet; row stride k)
+template <int MG, int U>
+__device__ __forceinline__ void rb_load_w(u32x4 (&a)[U][MG], const uint16_t* __restrict__ wr, int k, int s, int s_end) {
 #pragma unroll
-    for (int g = 0; g < MG; g++)
+    for (int u = 0; u < U; u++)
 #pragma unroll
-        for (int t = 0; t < NT; t++) acc[g][t] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const uint16_t* xp[NT];
-    const int32_t* list = nullptr;
-    if (p.mode == KF_RB_SUM) {
-        int last = -1;
-        for (int i = 0; i < q.e.n_tile; i++) {
-            const int ex = q.e.tile_expert[i];
-            if (ex < 0) break;
-            if (ex == last) continue; /* an expert with more pairs than a tile holds: its tiles follow each other */
-            last = ex;
-#pragma unroll
-            for (int t = 0; t < NT; t++) {
-                const int row = t * 16 + r16;
-                xp[t] = nullptr;
-                if (row < p.n)
-                    for (int j = 0; j < q.e.top; j++)
-                        if (q.e.ids[row * q.e.top + j] == ex) xp[t] = X + (size_t)(row * q.e.top + j) * p.ldx + 8 * q4;
-            }
-            rb_stream_k<NT, MG, NW>(W + (size_t)ex * q.e.w_stride + (size_t)m0 * p.k, p.k, xp, acc, wid, lane);
+        for (int g = 0; g < MG; g++) {
+            a[u][g] = u32x4{0, 0, 0, 0};
+            if (s + u < s_end) a[u][g] = ld_nt(reinterpret_cast<const u32x4*>(wr + (size_t)g * 16 * k + 32 * (s + u))); /* wave-uniform */
         }
-    } else {
-        if (p.mode != KF_RB_ALL) {
-            const int ex = q.e.tile_expert[blockIdx.y];
-            if (ex < 0) return;
-            W += (size_t)ex * q.e.w_stride;
-            list = q.e.list + (size_t)blockIdx.y * q.e.tile;
-        }
+}
+// token fragments of the same steps; xp[t]: this lane's token row + its k octet (NULLABLE: NULL is a zero column), steps past s_end read step s_end - 1 against zero weights
+template <int NT, int U, bool NULLABLE>
+__device__ __forceinline__ void rb_load_x(u32x4 (&b)[U][NT], const uint16_t* const (&xp)[NT], int s, int s_end) {
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+        const int st = s + u < s_end ? s + u : s_end - 1;
 #pragma unroll
         for (int t = 0; t < NT; t++) {
-            const int col = t * 16 + r16;
-            xp[t] = nullptr;
-            if (list) {
-                const int pair = list[col];
-                if (pair >= 0) xp[t] = X + (size_t)(p.mode == KF_RB_UP ? pair / q.e.top : pair) * p.ldx + 8 * q4;
-            } else if (col < p.n) {
-                xp[t] = X + (size_t)col * p.ldx + 8 * q4;
+            if (NULLABLE) {
+                b[u][t] = u32x4{0, 0, 0, 0};
+                if (xp[t]) b[u][t] = *reinterpret_cast<const u32x4*>(xp[t] + 32 * st);
+            } else {
+                b[u][t] = *reinterpret_cast<const u32x4*>(xp[t] + 32 * st);
             }
         }
-        rb_stream_k<NT, MG, NW>(W + (size_t)m0 * p.k, p.k, xp, acc, wid, lane);
     }
+}
+template <int NT, int MG, int U>
+__device__ __forceinline__ void rb_multiply(const u32x4 (&a)[U][MG], const u32x4 (&b)[U][NT], f32x4 (&acc)[MG][NT]) {
+#pragma unroll
+    for (int u = 0; u < U; u++)
+#pragma unroll
+        for (int g = 0; g < MG; g++)
+#pragma unroll
+            for (int t = 0; t < NT; t++) acc[g][t] = rb_mfma16(a[u][g], b[u][t], acc[g][t]);
+}
+// the waves' partial tiles -> outputs; list: the columns are pairs
+template <int NT, int MG, int NW>
+__device__ __forceinline__ void rb_stream_finish(const RbProduct& q, const f32x4 (&acc)[MG][NT], float (&red)[NW][MG][16 * NT][17], const int32_t* list, int m0, int tid) {
+    const kf_rb_product& p = q.p;
+    const int lane = tid & 63, wid = tid >> 6, r16 = lane & 15, q4 = lane >> 4;
 #pragma unroll
     for (int g = 0; g < MG; g++)
 #pragma unroll
@@ -108,7 +68,8 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
 #pragma unroll
             for (int j = 0; j < 4; j++) red[wid][g][t * 16 + r16][4 * q4 + j] = acc[g][t][j];
     __syncthreads();
-    for (int i = tid; i < COLS * 16; i += 64 * NW) {
+    const int cols = list ? 16 * NT : p.n;
+    for (int i = tid; i < cols * 16; i += 64 * NW) {
         const int row = i & 15, col = i >> 4;
         int yr = col;
         float scale = 1.f;
@@ -116,13 +77,11 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
             yr = list[col];
             if (yr < 0) continue;
             if (p.mode == KF_RB_UP) scale = q.e.weight[yr];
-        } else if (col >= p.n) {
-            continue;
         }
         float d = 0.f;
 #pragma unroll
         for (int w = 0; w < NW; w++) d += red[w][0][col][row];
-        if constexpr (GATED) {
+        if constexpr (MG == 2) {
             float u = 0.f;
 #pragma unroll
             for (int w = 0; w < NW; w++) u += red[w][MG - 1][col][row];
@@ -136,18 +95,181 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
         }
     }
 }
+
+template <int NT, bool GATED, int NW, bool NORM>
+__global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
+    const kf_rb_product& p = q.p;
+    constexpr int MG = GATED ? 2 : 1, U = NT >= 4 ? 2 : 4;
+    __shared__ float red[NW][MG][16 * NT][17]; /* [wave][block][column][row], padded */
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, q4 = lane >> 4;
+    const int m0 = blockIdx.x * (16 * MG), nstep = p.k / 32;
+    const uint16_t* W = reinterpret_cast<const uint16_t*>(p.w);
+    const uint16_t* X = reinterpret_cast<const uint16_t*>(p.x);
+    const int32_t* list = nullptr;
+    if (p.mode != KF_RB_ALL) {
+        const int ex = q.e.tile_expert[blockIdx.y];
+        if (ex < 0) return;
+        W += (size_t)ex * q.e.w_stride;
+        list = q.e.list + (size_t)blockIdx.y * q.e.tile;
+    }
+    const uint16_t* wr = W + (size_t)(m0 + r16) * p.k + 8 * q4;
+    u32x4 a[U][MG], b[U][NT];
+    int s = wid * U;
+    rb_load_w<MG, U>(a, wr, p.k, s, nstep);
+    const uint16_t* xp[NT];
+    if constexpr (NORM) {
+        static_assert(NT == 1, "a few rows");
+        uint16_t* sx = reinterpret_cast<uint16_t*>(smem_raw); /* [n][k + 8] */
+        float* part = &red[0][0][0][0];                       /* [NW][RB_NORM_ROWS] sums of squares: 8 NW floats of the (unused so far) partial tiles */
+        for (int t = 0; t < p.n; t++) {
+            float ss = 0.f;
+            for (int c = 4 * tid; c < p.k; c += 256 * NW) {
+                const f32x4 v = rb_ld4(p.norm_z + (size_t)t * p.ldx + c);
+#pragma unroll
+                for (int j = 0; j < 4; j++)
+                    if (c + j < p.norm_dim) ss = fmaf(v[j], v[j], ss);
+            }
+            ss = wave_sum(ss);
+            if (lane == 0) part[wid * RB_NORM_ROWS + t] = ss;
+        }
+        __syncthreads();
+        for (int t = 0; t < p.n; t++) {
+            float ss = 0.f;
+#pragma unroll
+            for (int w = 0; w < NW; w++) ss += part[w * RB_NORM_ROWS + t];
+            const float rs = 1.0f / sqrtf(ss / (float)p.norm_dim + p.norm_eps);
+            for (int c = 4 * tid; c < p.k; c += 256 * NW) {
+                const f32x4 v = rb_ld4(p.norm_z + (size_t)t * p.ldx + c), g = rb_ld4(reinterpret_cast<const uint16_t*>(p.norm_w) + c);
+                f32x4 o;
+#pragma unroll
+                for (int j = 0; j < 4; j++) o[j] = c + j < p.norm_dim ? v[j] * rs * g[j] : 0.f;
+                rb_st4(sx + t * (p.k + 8) + c, o);
+                if (blockIdx.x == 0) { /* the normed rows themselves, once */
+                    rb_st4(p.norm_x + (size_t)t * p.ldx + c, o);
+                    rb_st4(reinterpret_cast<uint16_t*>(const_cast<void*>(p.x)) + (size_t)t * p.ldx + c, o);
+                }
+            }
+        }
+        __syncthreads();
+        xp[0] = sx + (r16 < p.n ? r16 : p.n - 1) * (p.k + 8) + 8 * q4;
+    } else {
+#pragma unroll
+        for (int t = 0; t < NT; t++) { /* columns past the end repeat a row: their outputs are not stored */
+            const int col = t * 16 + r16;
+            int row = col < p.n ? col : p.n - 1;
+            if (list) {
+                const int pair = list[col];
+                row = pair < 0 ? 0 : (p.mode == KF_RB_UP ? pair / q.e.top : pair);
+            }
+            xp[t] = X + (size_t)row * p.ldx + 8 * q4;
+        }
+    }
+    f32x4 acc[MG][NT];
+#pragma unroll
+    for (int g = 0; g < MG; g++)
+#pragma unroll
+        for (int t = 0; t < NT; t++) acc[g][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (; s < nstep; s += NW * U) {
+        u32x4 an[U][MG];
+        rb_load_x<NT, U, false>(b, xp, s, nstep);
+        rb_load_w<MG, U>(an, wr, p.k, s + NW * U, nstep);
+        rb_multiply<NT, MG, U>(a, b, acc);
+#pragma unroll
+        for (int u = 0; u < U; u++)
+#pragma unroll
+            for (int g = 0; g < MG; g++) a[u][g] = an[u][g];
+    }
+    if constexpr (NORM) __syncthreads(); /* `part` shares the partial tiles' memory: every wave is past it */
+    rb_stream_finish<NT, MG, NW>(q, acc, red, list, m0, tid);
+}
+
+// RESIDUAL with the rows' experts summed: (chosen expert, k-step) pairs as one list, cut evenly over the waves
+constexpr int RB_SUM_IDS = 1024;
+template <int NT, int NW>
+__global__ void __launch_bounds__(64 * NW) rb_stream_sum_kernel(const RbProduct q) {
+    const kf_rb_product& p = q.p;
+    constexpr int U = NT >= 4 ? 2 : 4;
+    __shared__ float red[NW][1][16 * NT][17];
+    __shared__ int32_t s_ex[RB_SUM_IDS], s_ids[RB_SUM_IDS];
+    __shared__ int s_n;
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, q4 = lane >> 4;
+    const int m0 = blockIdx.x * 16, nstep = p.k / 32, pairs = p.n * q.e.top;
+    const uint16_t* X = reinterpret_cast<const uint16_t*>(p.x);
+    for (int i = tid; i < pairs; i += 64 * NW) s_ids[i] = q.e.ids[i];
+    if (wid == 0) { /* the chosen experts, each once: a tile per expert (a tile holds as many pairs as the batch has rows) */
+        int cnt = 0;
+        for (int i0 = 0; i0 < q.e.n_tile; i0 += 64) {
+            const int ex = i0 + lane < q.e.n_tile ? q.e.tile_expert[i0 + lane] : -1;
+            const unsigned long long on = __ballot(ex >= 0);
+            if (ex >= 0) s_ex[cnt + __popcll(on & ((1ull << lane) - 1))] = ex;
+            cnt += __popcll(on);
+        }
+        if (lane == 0) s_n = cnt;
+    }
+    __syncthreads();
+    const int total = s_n * nstep, span = (total + NW - 1) / NW;
+    int at = wid * span;
+    const int end = at + span < total ? at + span : total;
+    f32x4 acc[1][NT];
+#pragma unroll
+    for (int t = 0; t < NT; t++) acc[0][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    while (at < end) { /* an expert's part of this wave's range (wave-uniform) */
+        const int i = at / nstep, s0 = at - i * nstep, s1 = s0 + (end - at) < nstep ? s0 + (end - at) : nstep;
+        const int ex = s_ex[i];
+        const uint16_t* wr = reinterpret_cast<const uint16_t*>(p.w) + (size_t)ex * q.e.w_stride + (size_t)(m0 + r16) * p.k + 8 * q4;
+        u32x4 a[U][1], b[U][NT];
+        rb_load_w<1, U>(a, wr, p.k, s0, s1);
+        const uint16_t* xp[NT];
+#pragma unroll
+        for (int t = 0; t < NT; t++) {
+            const int row = t * 16 + r16;
+            xp[t] = nullptr;
+            if (row < p.n)
+                for (int j = 0; j < q.e.top; j++)
+                    if (s_ids[row * q.e.top + j] == ex) xp[t] = X + (size_t)(row * q.e.top + j) * p.ldx + 8 * q4;
+        }
+        for (int s = s0; s < s1; s += U) {
+            u32x4 an[U][1];
+            rb_load_x<NT, U, true>(b, xp, s, s1);
+            rb_load_w<1, U>(an, wr, p.k, s + U, s1);
+            rb_multiply<NT, 1, U>(a, b, acc);
+#pragma unroll
+            for (int u = 0; u < U; u++) a[u][0] = an[u][0];
+        }
+        at += s1 - s0;
+    }
+    rb_stream_finish<NT, 1, NW>(q, acc, red, nullptr, m0, tid);
+}
 template <int NT, int NW>
 static void stream_go(hipStream_t st, const RbProduct& q, dim3 grid) {
-    if (q.p.epilogue == KF_RB_GATED) hipLaunchKernelGGL((rb_stream_kernel<NT, true, NW>), grid, dim3(64 * NW), 0, st, q);
-    else hipLaunchKernelGGL((rb_stream_kernel<NT, false, NW>), grid, dim3(64 * NW), 0, st, q);
+    if (q.p.mode == KF_RB_SUM) hipLaunchKernelGGL((rb_stream_sum_kernel<NT, NW>), grid, dim3(64 * NW), 0, st, q);
+    else if (q.p.epilogue == KF_RB_GATED) hipLaunchKernelGGL((rb_stream_kernel<NT, true, NW, false>), grid, dim3(64 * NW), 0, st, q);
+    else hipLaunchKernelGGL((rb_stream_kernel<NT, false, NW, false>), grid, dim3(64 * NW), 0, st, q);
+}
+static size_t norm_lds(int n, int k) { return (size_t)n * (k + 8) * 2; }
+template <int NW>
+static int norm_stream_go(hipStream_t st, const RbProduct& q, dim3 grid) {
+    const size_t smem = norm_lds(q.p.n, q.p.k);
+    static int done = 0;
+    if (!done) {
+        for (const void* f : {(const void*)rb_stream_kernel<1, true, NW, true>, (const void*)rb_stream_kernel<1, false, NW, true>})
+            if (hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, RB_NORM_LDS) != hipSuccess) return KF_HIP_CHECK;
+        done = 1;
+    }
+    if (q.p.epilogue == KF_RB_GATED) hipLaunchKernelGGL((rb_stream_kernel<1, true, NW, true>), grid, dim3(64 * NW), smem, st, q);
+    else hipLaunchKernelGGL((rb_stream_kernel<1, false, NW, true>), grid, dim3(64 * NW), smem, st, q);
+    return KF_OK;
 }
 int rb_stream_launch(hipStream_t st, const RbProduct& q) {
     const kf_rb_product& p = q.p;
     const bool tiles = p.mode == KF_RB_UP || p.mode == KF_RB_DOWN;
     const int cols = tiles ? q.e.tile : p.n, nt = (cols + 15) / 16;
     if (nt > 4 || (tiles && q.e.tile % 16)) return 1;
+    if (p.mode == KF_RB_SUM && ((long)p.n * q.e.top > RB_SUM_IDS || q.e.tile < p.n)) return 1;
     dim3 grid(p.m / (p.epilogue == KF_RB_GATED ? 32 : 16), tiles ? q.e.n_tile : 1);
     const bool wide = (long)grid.x * grid.y < 768 && p.k >= 512; /* few workgroups: more waves each, more loads in flight per CU */
+    if (p.norm_z) return wide ? norm_stream_go<8>(st, q, grid) : norm_stream_go<4>(st, q, grid);
     switch (nt) {
         case 1: wide ? stream_go<1, 8>(st, q, grid) : stream_go<1, 4>(st, q, grid); break;
         case 2: wide ? stream_go<2, 8>(st, q, grid) : stream_go<2, 4>(st, q, grid); break;
@@ -248,6 +370,7 @@ int rb_f32_launch(hipStream_t st, const RbProduct& q) {
 }  // namespace kf
 
 using namespace kf;
+extern "C" int kf_rb_linear_norms(int type, int n, int k) { return type == KF_BF16 && n >= 1 && n <= RB_NORM_ROWS && norm_lds(n, k) + 20 * 1024 <= RB_NORM_LDS; }
 extern "C" int kf_rb_linear(kf_ctx* c, const kf_rb_product* p) {
     CHKCTX(c);
     if (!p || !p->w || !p->x || !p->y) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: null pointer");
@@ -257,6 +380,9 @@ extern "C" int kf_rb_linear(kf_ctx* c, const kf_rb_product* p) {
     if (!al16(p->w) || !al16(p->x) || !al16(p->y)) return abi_fail(KF_BLAS_UNALIGN, "kf_rb_linear: unaligned pointer");
     if (p->epilogue < KF_RB_STORE || p->epilogue > KF_RB_GATED || p->mode < KF_RB_ALL || p->mode > KF_RB_SUM) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: epilogue or mode");
     if (p->epilogue == KF_RB_RESIDUAL && (!p->res || !al16(p->res) || p->ldr < p->m || p->ldr % 4)) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: residual");
+    if (p->norm_z && (!kf_rb_linear_norms(p->type, p->n, p->k) || p->mode != KF_RB_ALL || !p->norm_w || !p->norm_x || p->norm_dim < 1 || p->norm_dim > p->k || p->ldx != p->k || !al16(p->norm_z) ||
+                      !al16(p->norm_w) || !al16(p->norm_x)))
+        return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: norm in front of the product");
     RbProduct q;
     q.p = *p;
     q.e = kf_rb_experts{};
@@ -264,7 +390,7 @@ extern "C" int kf_rb_linear(kf_ctx* c, const kf_rb_product* p) {
         const kf_rb_experts* e = p->experts;
         if (!e || e->n_expert < 1 || e->top < 1 || e->tile < 1 || e->n_tile < 1 || !e->tile_expert || !e->list || !e->ids || !e->weight) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: experts");
         if (e->w_stride < (int64_t)p->m * p->k || e->w_stride % 8) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: expert stride");
-        if ((p->mode == KF_RB_UP) != (p->epilogue == KF_RB_GATED) || (p->mode == KF_RB_DOWN && p->epilogue != KF_RB_STORE_F32) || (p->mode == KF_RB_SUM && p->epilogue != KF_RB_RESIDUAL))
+        if ((p->mode == KF_RB_UP) != (p->epilogue == KF_RB_GATED) || (p->mode == KF_RB_DOWN && p->epilogue != KF_RB_STORE) || (p->mode == KF_RB_SUM && p->epilogue != KF_RB_RESIDUAL))
             return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: this mode has another epilogue");
         q.e = *e;
     }

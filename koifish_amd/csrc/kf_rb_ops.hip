@@ -46,7 +46,8 @@ __global__ void rb_embed_state_kernel(const T* table, int vocab, int dim, long l
 }
 
 struct RbNorm {
-    const float *z, *res;
+    const void* z;
+    const float* res;
     const int32_t* rows;
     const void* w;
     float* x_out;
@@ -69,11 +70,11 @@ __global__ void __launch_bounds__(256) rb_norm_kernel(const RbNorm a) {
             if (a.res) {
                 const f32x4 r = rb_ld4(a.res + (size_t)src * a.ld + c);
                 f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
-                for (int j = 0; j < a.top; j++) s += rb_ld4(a.z + ((size_t)src * a.top + j) * a.ld + c);
+                for (int j = 0; j < a.top; j++) s += rb_ld4(reinterpret_cast<const T*>(a.z) + ((size_t)src * a.top + j) * a.ld + c);
 #pragma unroll
                 for (int j = 0; j < 4; j++) v[i][j] = fmaf(a.alpha, r[j], s[j]);
             } else {
-                v[i] = rb_ld4(a.z + (size_t)src * a.ld + c);
+                v[i] = rb_ld4(reinterpret_cast<const float*>(a.z) + (size_t)src * a.ld + c);
             }
 #pragma unroll
             for (int j = 0; j < 4; j++) { /* pad columns do not count, whatever they hold */
@@ -123,16 +124,28 @@ static int norm_go(hipStream_t st, const RbNorm& a, int n) {
 
 // ---- router: one wave per row; expert e sits in lane e % 64, register e / 64
 constexpr int RB_MAX_EXPERTS = 1024;
-template <class T>
-__global__ void __launch_bounds__(256) rb_topk_kernel(const float* __restrict__ logits, long long ld, const T* __restrict__ bias, int n, const int32_t* __restrict__ meta, int n_expert,
-                                                      int top, int32_t* __restrict__ ids, float* __restrict__ weight) {
-    const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (t >= n) return;
+struct RbRoute {
+    const float* logits;
+    const void* bias;
+    const int32_t* meta;
+    int32_t *ids, *tile_expert, *list;
+    float* weight;
+    long long ld;
+    int n, n_expert, top, tile, n_tile;
+};
+template <class T, int NV> /* NV registers of 64 experts */
+__device__ __forceinline__ void rb_topk_row(const RbRoute& a, int t, int lane) {
+    const float* logits = a.logits;
+    const T* bias = reinterpret_cast<const T*>(a.bias);
+    const int32_t* meta = a.meta;
+    int32_t* ids = a.ids;
+    float* weight = a.weight;
+    const long long ld = a.ld;
+    const int n_expert = a.n_expert, top = a.top;
     if (meta && meta[KF_RB_META * t] < 0) {
         for (int j = lane; j < top; j += 64) ids[(size_t)t * top + j] = -1, weight[(size_t)t * top + j] = 0.f;
         return;
     }
-    constexpr int NV = RB_MAX_EXPERTS / 64;
     float v[NV];
 #pragma unroll
     for (int i = 0; i < NV; i++) {
@@ -162,15 +175,21 @@ __global__ void __launch_bounds__(256) rb_topk_kernel(const float* __restrict__ 
         for (int i = 0; i < NV; i++)
             if (lane + 64 * i == cand) v[i] = -__builtin_inff();
     }
-    if (lane == 0) { /* the lane that wrote them reads them back */
-        const float inv = 1.0f / sum;
+    const float inv = 1.0f / sum;
+    if (lane == 0) /* the lane that wrote them reads them back */
         for (int j = 0; j < top; j++) weight[(size_t)t * top + j] *= inv;
-    }
+}
+template <class T, int NV>
+__global__ void __launch_bounds__(256) rb_topk_kernel(const RbRoute a) {
+    const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t < a.n) rb_topk_row<T, NV>(a, t, threadIdx.x & 63);
 }
 // ---- pairs grouped by expert, one workgroup: count, tile-aligned offsets, fill
-__global__ void __launch_bounds__(1024) rb_list_kernel(const int32_t* __restrict__ ids, int n_pair, int n_expert, int tile, int n_tile, int32_t* __restrict__ tile_expert,
-                                                       int32_t* __restrict__ list) {
+__device__ __forceinline__ void rb_list(const RbRoute& a) {
     __shared__ int cnt[RB_MAX_EXPERTS], off[RB_MAX_EXPERTS];
+    const int32_t* ids = a.ids;
+    int32_t *tile_expert = a.tile_expert, *list = a.list;
+    const int n_pair = a.n * a.top, n_expert = a.n_expert, tile = a.tile, n_tile = a.n_tile;
     const int tid = threadIdx.x, nt = blockDim.x;
     for (int e = tid; e < n_expert; e += nt) cnt[e] = 0;
     for (int i = tid; i < n_tile; i += nt) tile_expert[i] = -1;
@@ -208,6 +227,31 @@ __global__ void __launch_bounds__(1024) rb_list_kernel(const int32_t* __restrict
         const int p = off[e] * tile + atomicAdd(&cnt[e], 1);
         if (p < n_tile * tile) list[p] = i;
     }
+}
+__global__ void __launch_bounds__(1024) rb_list_kernel(const RbRoute a) { rb_list(a); }
+/* a decode batch: both in one workgroup */
+template <class T, int NV>
+__global__ void __launch_bounds__(1024) rb_route_kernel(const RbRoute a) {
+    for (int t = threadIdx.x >> 6; t < a.n; t += (int)blockDim.x >> 6) rb_topk_row<T, NV>(a, t, threadIdx.x & 63);
+    __threadfence_block();
+    __syncthreads();
+    rb_list(a);
+}
+template <class T, int NV>
+static void route_nv(hipStream_t st, const RbRoute& a) {
+    if (a.n <= KF_RB_DECODE_MAX) {
+        hipLaunchKernelGGL((rb_route_kernel<T, NV>), dim3(1), dim3(a.n <= 4 ? 256 : 1024), 0, st, a);
+        return;
+    }
+    hipLaunchKernelGGL((rb_topk_kernel<T, NV>), dim3((a.n + 3) / 4), dim3(256), 0, st, a);
+    hipLaunchKernelGGL(rb_list_kernel, dim3(1), dim3(1024), 0, st, a);
+}
+template <class T>
+static void route_go(hipStream_t st, const RbRoute& a) {
+    if (a.n_expert <= 64) route_nv<T, 1>(st, a);
+    else if (a.n_expert <= 128) route_nv<T, 2>(st, a);
+    else if (a.n_expert <= 256) route_nv<T, 4>(st, a);
+    else route_nv<T, RB_MAX_EXPERTS / 64>(st, a);
 }
 
 // ---- greedy pick: maxima of PICK_SPAN-wide pieces, then the first maximum over the pieces
@@ -304,7 +348,7 @@ int kf_rb_embed_state(kf_ctx* c, int type, const void* table, int vocab, int dim
                            (float*)h, meta);
     return launched("kf_rb_embed_state");
 }
-int kf_rb_norm(kf_ctx* c, int type, const float* z, const float* res, float alpha, int top, const void* w, float eps, int dim, int64_t ld, int n, const int32_t* rows, float* x_out,
+int kf_rb_norm(kf_ctx* c, int type, const void* z, const float* res, float alpha, int top, const void* w, float eps, int dim, int64_t ld, int n, const int32_t* rows, float* x_out,
                void* h_out) {
     CHKCTX(c);
     if (!type_ok(type)) return abi_fail(KF_UNSUPPORTED_DATATYPE, "kf_rb_norm: storage %d", type);
@@ -327,15 +371,10 @@ int kf_rb_route(kf_ctx* c, int type, const float* logits, int64_t ld, const void
         return abi_fail(KF_INVALID_ARGS, "kf_rb_route: bad arguments");
     if (e->n_expert > RB_MAX_EXPERTS) return abi_fail(KF_UNSUPPORTED_DATATYPE, "kf_rb_route: %d experts (served: up to %d)", e->n_expert, RB_MAX_EXPERTS);
     if (e->n_tile < kf_rb_list_tiles(n, e->top, e->n_expert, e->tile)) return abi_fail(KF_INVALID_ARGS, "kf_rb_route: the list has %d tiles", e->n_tile);
-    int32_t* ids = const_cast<int32_t*>(e->ids);
-    float* wt = const_cast<float*>(e->weight);
-    if (type == KF_BF16)
-        hipLaunchKernelGGL(rb_topk_kernel<uint16_t>, dim3((n + 3) / 4), dim3(256), 0, c->stream, logits, (long long)ld, (const uint16_t*)bias, n, meta, e->n_expert, e->top, ids, wt);
-    else
-        hipLaunchKernelGGL(rb_topk_kernel<float>, dim3((n + 3) / 4), dim3(256), 0, c->stream, logits, (long long)ld, (const float*)bias, n, meta, e->n_expert, e->top, ids, wt);
-    const int pairs = n * e->top;
-    hipLaunchKernelGGL(rb_list_kernel, dim3(1), dim3(pairs > 2048 ? 1024 : 256), 0, c->stream, ids, pairs, e->n_expert, e->tile, e->n_tile, const_cast<int32_t*>(e->tile_expert),
-                       const_cast<int32_t*>(e->list));
+    RbRoute a{logits, bias, meta, const_cast<int32_t*>(e->ids), const_cast<int32_t*>(e->tile_expert), const_cast<int32_t*>(e->list), const_cast<float*>(e->weight), (long long)ld, n,
+              e->n_expert, e->top, e->tile, e->n_tile};
+    if (type == KF_BF16) route_go<uint16_t>(c->stream, a);
+    else route_go<float>(c->stream, a);
     return launched("kf_rb_route");
 }
 size_t kf_rb_pick_scratch(int n) { return n < 1 ? 0 : (size_t)n * PICK_PIECES * 8; }

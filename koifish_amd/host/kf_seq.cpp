@@ -30,13 +30,23 @@ int RowProduct::Forw(const void* x, int64_t ldx, int n, void* y, int64_t ldy, in
     if (ex) e = *ex, e.w_stride = (int64_t)m * k, p.experts = &e;
     return kf_rb_linear(hFish->ctx, &p);
 }
-int RowNorm::Forw(const float* z, int n, float* x_out, void* h_out, const float* res, float alpha, int top, const int32_t* rows) {
+int RowProduct::ForwNormed(RowWork& w, int n, void* y, int64_t ldy, int epilogue, int act) {
+    if (!w.pending) return Forw(P(w.h), k, n, y, ldy, epilogue, act);
+    const SEQ_CARD& c = hFish->Seq()->card;
+    kf_rb_product p;
+    std::memset(&p, 0, sizeof(p));
+    p.w = this->w->data, p.x = P(w.h), p.y = y, p.ldx = k, p.ldy = ldy, p.type = c.type, p.m = m, p.k = k, p.n = n, p.epilogue = epilogue, p.act = act;
+    p.norm_z = F(w.z), p.norm_w = P(w.pending->w), p.norm_x = F(w.x), p.norm_eps = c.eps, p.norm_dim = c.width;
+    w.pending = nullptr;
+    return kf_rb_linear(hFish->ctx, &p);
+}
+int RowNorm::Forw(const void* z, int n, float* x_out, void* h_out, const float* res, float alpha, int top, const int32_t* rows) {
     const SEQ_CARD& c = hFish->Seq()->card;
     return kf_rb_norm(hFish->ctx, c.type, z, res, alpha, top, w->data, c.eps, dim, ld, n, rows, x_out, h_out);
 }
-int ChunkAttention::Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos) {
+int ChunkAttention::Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos, bool defer) {
     const SEQ_CARD& card = hFish->Seq()->card;
-    KF_TRY(qkg.Forw(P(w.h), qkg.k, n, P(w.raw), ldraw, KF_RB_STORE));
+    KF_TRY(qkg.ForwNormed(w, n, P(w.raw), ldraw, KF_RB_STORE));
     const KVCache::Ring& ring = kv.rings[layid - 1];
     kf_rb_attention a;
     std::memset(&a, 0, sizeof(a));
@@ -48,34 +58,46 @@ int ChunkAttention::Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int ma
     if (n_seq) KF_TRY(kf_rb_attention_prefill(hFish->ctx, &a, I(w.meta), n, I(w.seqs), n_seq, max_n));
     else KF_TRY(kf_rb_attention_decode(hFish->ctx, &a, I(w.meta), n, max_pos));
     KF_TRY(proj.Forw(P(w.ao), ldout, n, F(w.z), proj.m, KF_RB_RESIDUAL, 0, F(w.x), card.alpha));
+    if (defer) {
+        w.pending = &norm;
+        return KF_OK;
+    }
     return norm.Forw(F(w.z), n, F(w.x), P(w.h));
 }
-int RowFFN::Forw(RowWork& w, int n) {
+int RowFFN::Forw(RowWork& w, int n, bool defer) {
     const SEQ_CARD& card = hFish->Seq()->card;
     if (c.kind == FF_CARD::NONE) return KF_OK;
     const int64_t ld = gateup.k;
     if (c.kind == FF_CARD::DENSE) {
-        KF_TRY(gateup.Forw(P(w.h), ld, n, P(w.act), ldact, KF_RB_GATED, c.act));
+        KF_TRY(gateup.ForwNormed(w, n, P(w.act), ldact, KF_RB_GATED, c.act));
         KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha));
+        if (defer) {
+            w.pending = &norm;
+            return KF_OK;
+        }
         return norm.Forw(F(w.z), n, F(w.x), P(w.h));
     }
     const bool few = card.type == KF_BF16 && n <= KF_RB_DECODE_MAX;
     kf_rb_experts e;
     std::memset(&e, 0, sizeof(e));
     e.n_expert = c.experts, e.top = c.top;
-    // few rows: an expert never has more pairs than the batch has rows, one tile each; many: 128-pair tiles where the experts have about that many
-    e.tile = few ? up(n, 16) : (card.type == KF_BF16 && (long long)n * c.top >= 96LL * c.experts ? 128 : 64);
+    // few rows: an expert never has more pairs than the batch has rows, one tile each; many: 128-pair tiles where the experts fill several
+    e.tile = few ? up(n, 16) : (card.type == KF_BF16 && (long long)n * c.top >= 256LL * c.experts ? 128 : 64);
     e.n_tile = kf_rb_list_tiles(n, c.top, c.experts, e.tile);
     e.tile_expert = I(w.tile_expert), e.list = I(w.list), e.ids = I(w.ids), e.weight = F(w.weight);
-    KF_TRY(router.Forw(P(w.h), ld, n, F(w.rlogits), router.m, KF_RB_STORE_F32));
+    KF_TRY(router.ForwNormed(w, n, F(w.rlogits), router.m, KF_RB_STORE_F32));
     KF_TRY(kf_rb_route(hFish->ctx, card.type, F(w.rlogits), router.m, P(router_b), n, I(w.meta), &e));
     KF_TRY(gateup.Forw(P(w.h), ld, n, P(w.act), ldact, KF_RB_GATED, c.act, nullptr, 0, KF_RB_UP, &e));
     if (few) {
         KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_SUM, &e));
+        if (defer) {
+            w.pending = &norm;
+            return KF_OK;
+        }
         return norm.Forw(F(w.z), n, F(w.x), P(w.h));
     }
-    KF_TRY(down.Forw(P(w.act), ldact, n, F(w.y), ld, KF_RB_STORE_F32, 0, nullptr, 0, KF_RB_DOWN, &e));
-    return norm.Forw(F(w.y), n, F(w.x), P(w.h), F(w.x), card.alpha, c.top);
+    KF_TRY(down.Forw(P(w.act), ldact, n, P(w.y), ld, KF_RB_STORE, 0, nullptr, 0, KF_RB_DOWN, &e));
+    return norm.Forw(P(w.y), n, F(w.x), P(w.h), F(w.x), card.alpha, c.top);
 }
 
 // ------------------------------------------------------------------------------------------------ build
@@ -322,7 +344,7 @@ int SeqFish::Ensure(RowWork& w, int rows, int n_seq, int head_rows, bool decode)
             }
         }
         get(w.x, "x", KF_F32, (size_t)rows * W), get(w.z, "z", KF_F32, (size_t)rows * W), get(w.h, "h", T, (size_t)rows * W);
-        get(w.raw, "raw", T, raw), get(w.ao, "ao", T, ao), get(w.knew, "knew", T, kn), get(w.act, "act", T, act), get(w.y, "y", KF_F32, y), get(w.rlogits, "rlogits", KF_F32, rl);
+        get(w.raw, "raw", T, raw), get(w.ao, "ao", T, ao), get(w.knew, "knew", T, kn), get(w.act, "act", T, act), get(w.y, "y", T, y), get(w.rlogits, "rlogits", KF_F32, rl);
         get(w.meta, "meta", KF_F32, (size_t)rows * KF_RB_META), get(w.tok, "tok", KF_F32, rows), get(w.ids, "ids", KF_F32, pairs), get(w.weight, "weight", KF_F32, pairs);
         get(w.list, "list", KF_F32, list), get(w.tile_expert, "tile_expert", KF_F32, tiles), get(w.scratch, "scratch", KF_F32, scratch);
         w.rows = rows;
@@ -338,14 +360,20 @@ int SeqFish::Ensure(RowWork& w, int rows, int n_seq, int head_rows, bool decode)
 // ------------------------------------------------------------------------------------------------ steps
 int SeqFish::Layers(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos) {
     const int W = Width(card.width);
+    const bool defer = n_seq == 0 && kf_rb_linear_norms(card.type, n, W); /* few rows: every norm inside the product behind it */
+    w.pending = nullptr;
     for (size_t l = 0; l < mixers.size(); l++) {
-        KF_TRY(mixers[l]->Forw(w, kv, n, n_seq, max_n, max_pos));
-        KF_TRY(ffs[l]->Forw(w, n));
+        KF_TRY(mixers[l]->Forw(w, kv, n, n_seq, max_n, max_pos, defer));
+        KF_TRY(ffs[l]->Forw(w, n, defer));
         if (tap && n_seq && n == tap_rows) {
             std::vector<float> rows((size_t)n * W);
             KF_TRY(kf_d2h(ctx, rows.data(), w.x->data, rows.size() * 4));
             for (int r = 0; r < n; r++) std::memcpy(tap + ((size_t)l * n + r) * card.width, rows.data() + (size_t)r * W, (size_t)card.width * 4);
         }
+    }
+    if (RowNorm* last = w.pending) {
+        w.pending = nullptr;
+        return last->Forw(F(w.z), n, F(w.x), P(w.h));
     }
     return KF_OK;
 }

@@ -41,7 +41,9 @@ struct SEQ_CARD {
 };
 
 // activations of a row batch; one set for the decode steps (captured graphs hold its addresses), one for prompts
+struct RowNorm;
 struct RowWork {
+    RowNorm* pending = nullptr;  // decode: z holds a residual sum whose norm the next product forms itself
     int rows = 0, n_seq = 0, head_rows = 0;
     hGTensor x, z, h, raw, knew, ao, act, y, rlogits, scratch;         // residual and its sum (fp32), bf16 / fp32 rows, expert outputs, router logits, key-range partials
     hGTensor meta, seqs, tok, ids, weight, list, tile_expert, want, hl;  // int32 tables; hl: the rows the head reads
@@ -72,11 +74,12 @@ struct RowProduct : GeNeuron {  // padded weight [m][k] (x experts)
     int m = 0, k = 0, experts = 0;
     int Forw(const void* x, int64_t ldx, int n, void* y, int64_t ldy, int epilogue, int act = 0, const float* res = nullptr, float alpha = 0, int mode = KF_RB_ALL,
              const kf_rb_experts* ex = nullptr);
+    int ForwNormed(RowWork& w, int n, void* y, int64_t ldy, int epilogue, int act = 0);  // of w.h, the pending norm first
 };
 struct RowNorm : GeNeuron {
     hGTensor w;
     int dim = 0, ld = 0;
-    int Forw(const float* z, int n, float* x_out, void* h_out, const float* res = nullptr, float alpha = 0, int top = 0, const int32_t* rows = nullptr);
+    int Forw(const void* z, int n, float* x_out, void* h_out, const float* res = nullptr, float alpha = 0, int top = 0, const int32_t* rows = nullptr);
 };
 // chunked gated attention whose values are the projected keys: q | k | gate in one product, then kf_rb_attention_*
 struct ChunkAttention : GeNeuron {
@@ -86,7 +89,7 @@ struct ChunkAttention : GeNeuron {
     hGTensor qn, kn;
     const float* rope = nullptr;
     int ldraw = 0, ldout = 0;
-    int Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos);  // n_seq 0: one row per slot
+    int Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos, bool defer);  // n_seq 0: one row per slot; defer: leave the norm pending
 };
 struct RowFFN : GeNeuron {  // dense gated feed-forward, or routed experts
     FF_CARD c;
@@ -94,7 +97,7 @@ struct RowFFN : GeNeuron {  // dense gated feed-forward, or routed experts
     hGTensor router_b;
     RowNorm norm;
     int ldact = 0;
-    int Forw(RowWork& w, int n);
+    int Forw(RowWork& w, int n, bool defer);
 };
 
 struct SeqFish : Fish {

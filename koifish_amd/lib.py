@@ -23,7 +23,7 @@ ABI_SYMBOLS = [
     "kf_norm_gateup_swiglu", "kf_attn_block", "kf_norm_lm_head", "kf_set_state", "kf_embed_state", "kf_embed_batch", "kf_qknorm_rope_batch", "kf_attn_prefill", "kf_sample", "kf_linear_multi", "kf_linear_multi_scratch_bytes", "kf_gateup_swiglu_batch", "kf_adamw", "kf_layernorm", "kf_gelu", "kf_sample_topk", "kf_fused_classifier", "kf_gelu_backward", "kf_swiglu_backward", "kf_rope_backward", "kf_norm_backward", "kf_norm_backward_scratch_bytes", "kf_linear_backward", "kf_linear_backward_scratch_bytes", "kf_embed_backward", "kf_attn_backward", "kf_attn_backward_scratch_bytes", "kf_attn_prefill_batch", "kf_attn_prefill_batch_strided", "kf_embed_pos", "kf_memset2d", "kf_copy_blocks", "kf_argmax_rows_state", "kf_qknorm_rope_train",
     "kf_hot_rows", "kf_linear_masked", "kf_norm_gateup_swiglu_masked", "kf_linear_scratch_bytes", "kf_set_scratch", "kf_engine_workspace_bytes", "kf_engine_create", "kf_engine_step", "kf_engine_check", "kf_engine_destroy", "kf_engine_set_embedding", "kf_engine_set_head", "kf_engine_step_head", "kf_engine_steps_head", "kf_engine_reset", "kf_set_canonical", "kf_get_canonical", "kf_engine_served", "kf_engine_tune", "kf_engine_stats", "kf_qkv_rope_batch", "kf_qkv_rope_seqs", "kf_set_dequant_arena", "kf_dequant_arena_used", "kf_resident_scratch_bytes",
     "kf_xengine_workspace_bytes", "kf_xengine_create", "kf_xengine_served", "kf_xengine_set_embedding", "kf_xengine_set_head", "kf_xengine_steps", "kf_xengine_check", "kf_xengine_reset", "kf_xengine_destroy", "kf_xengine_workspace_bytes_tp", "kf_xengine_create_tp", "kf_xengine_set_head_tp",
-    "kf_rb_linear", "kf_rb_pack", "kf_rb_embed", "kf_rb_embed_state", "kf_rb_norm", "kf_rb_attention_prefill", "kf_rb_attention_decode", "kf_rb_attention_scratch", "kf_rb_rope_table_host",
+    "kf_rb_linear", "kf_rb_linear_norms", "kf_rb_pack", "kf_rb_embed", "kf_rb_embed_state", "kf_rb_norm", "kf_rb_attention_prefill", "kf_rb_attention_decode", "kf_rb_attention_scratch", "kf_rb_rope_table_host",
     "kf_rb_route", "kf_rb_list_tiles", "kf_rb_pick", "kf_rb_pick_scratch", "kf_rb_to_bf16",
     "kf_tp_recv_bytes", "kf_tp_push_bytes", "kf_tp_commit", "kf_tp_alloc", "kf_tp_ipc_export", "kf_tp_ipc_open", "kf_tp_ipc_close", "kf_linear_f32_push", "kf_tp_reduce_recv", "kf_tp_lm_head", "kf_tp_pick",
 ]
@@ -48,7 +48,8 @@ class RbExperts(C.Structure):
 class RbProduct(C.Structure):
     """struct kf_rb_product"""
     _fields_ = [("w", C.c_void_p), ("x", C.c_void_p), ("y", C.c_void_p), ("res", C.c_void_p), ("ldx", C.c_int64), ("ldy", C.c_int64), ("ldr", C.c_int64), ("type", C.c_int32),
-                ("m", C.c_int32), ("k", C.c_int32), ("n", C.c_int32), ("epilogue", C.c_int32), ("act", C.c_int32), ("mode", C.c_int32), ("alpha", C.c_float), ("experts", C.POINTER(RbExperts))]
+                ("m", C.c_int32), ("k", C.c_int32), ("n", C.c_int32), ("epilogue", C.c_int32), ("act", C.c_int32), ("mode", C.c_int32), ("alpha", C.c_float), ("experts", C.POINTER(RbExperts)),
+                ("norm_z", C.c_void_p), ("norm_w", C.c_void_p), ("norm_x", C.c_void_p), ("norm_eps", C.c_float), ("norm_dim", C.c_int32)]
 
 
 class RbAttention(C.Structure):

@@ -61,14 +61,15 @@ def test_norm(ctx, kind, dim, n):
     g = torch.Generator().manual_seed(dim)
     w = pad(dev(torch.rand(1, dim, generator=g) + 0.5, dt), 1, ld)
     res, z = pad(dev(torch.randn(n, dim, generator=g)), n, ld), pad(dev(torch.randn(n * top, dim, generator=g)), n * top, ld)
+    zt = z.to(dt)
     x, h = torch.full((n, ld), 7.0, device="cuda"), torch.full((n, ld), 7.0, dtype=dt, device="cuda")
     L.check(ctx.hip.kf_rb_norm(ctx.h, typ, z.data_ptr(), None, 0.0, 0, w.data_ptr(), 1e-5, dim, ld, n, None, x.data_ptr(), h.data_ptr()))
     ref = P.rms_norm(f64(z)[:n, :dim], f64(w)[0, :dim], 1e-5)
     assert np.abs(f64(x)[:, :dim] - ref).max() < 1e-5 and not f64(x)[:, dim:].any() and np.abs(f64(h)[:, :dim] - ref).max() < tol * 8
     # the sum over a row's experts on the scaled residual, in place
     r0 = f64(res)[:, :dim]
-    L.check(ctx.hip.kf_rb_norm(ctx.h, typ, z.data_ptr(), res.data_ptr(), 1.7, top, w.data_ptr(), 1e-5, dim, ld, n, None, res.data_ptr(), h.data_ptr()))
-    ref = P.rms_norm(1.7 * r0 + f64(z)[:, :dim].reshape(n, top, dim).sum(1), f64(w)[0, :dim], 1e-5)
+    L.check(ctx.hip.kf_rb_norm(ctx.h, typ, zt.data_ptr(), res.data_ptr(), 1.7, top, w.data_ptr(), 1e-5, dim, ld, n, None, res.data_ptr(), h.data_ptr()))
+    ref = P.rms_norm(1.7 * r0 + f64(zt)[:, :dim].reshape(n, top, dim).sum(1), f64(w)[0, :dim], 1e-5)
     assert np.abs(f64(res)[:, :dim] - ref).max() < 1e-5
     # rows picked from a list
     rows = torch.tensor([n - 1, 0], dtype=torch.int32, device="cuda")
@@ -99,6 +100,27 @@ def test_product_epilogues(ctx, kind, n, m, k):
         p = L.RbProduct(w.data_ptr(), x.data_ptr(), y.data_ptr(), None, k + 8, m // 2, 0, typ, m, k, n, L.RB_GATED, act, L.RB_ALL, 0.0, None)
         L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
         assert np.abs(f64(y) - fn(gate) * upw).max() < tol * 8
+
+
+@pytest.mark.parametrize("n,m,k,dim", [(1, 64, 64, 50), (3, 192, 320, 300), (8, 448, 1024, 1024), (2, 256, 4096, 4090)])
+def test_norm_in_front_of_a_product(ctx, n, m, k, dim):
+    assert ctx.hip.kf_rb_linear_norms(L.BF16, n, k) and not ctx.hip.kf_rb_linear_norms(L.F32, n, k) and not ctx.hip.kf_rb_linear_norms(L.BF16, 9, k)
+    w, z = (torch.randn(m, k, device="cuda") / k ** 0.5).bfloat16(), torch.randn(n, k, device="cuda")
+    z[:, dim:] = 99.0                         # pad columns do not count
+    g = (torch.rand(k, device="cuda") + 0.5).bfloat16()
+    il = f64(w).reshape(m // 32, 2, 16, k)
+    ref = P.rms_norm(f64(z)[:, :dim], f64(g)[:dim], 1e-5)
+    for epi in (L.RB_STORE, L.RB_STORE_F32, L.RB_GATED):
+        x, h = torch.full((n, k), 7.0, device="cuda"), torch.full((n, k), 7.0, dtype=torch.bfloat16, device="cuda")
+        y = torch.zeros(n, m, dtype=torch.float32 if epi == L.RB_STORE_F32 else torch.bfloat16, device="cuda")
+        p = L.RbProduct(w.data_ptr(), h.data_ptr(), y.data_ptr(), None, k, m, 0, L.BF16, m, k, n, epi, L.RB_SILU, L.RB_ALL, 0.0, None, z.data_ptr(), g.data_ptr(), x.data_ptr(), 1e-5, dim)
+        L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
+        assert np.abs(f64(x)[:, :dim] - ref).max() < 1e-5 and not f64(x)[:, dim:].any() and torch.equal(h, x.bfloat16())
+        full = f64(h) @ f64(w).T
+        if epi == L.RB_GATED:
+            full = P.silu(f64(h) @ il[:, 0].reshape(-1, k).T) * (f64(h) @ il[:, 1].reshape(-1, k).T)
+        got = f64(y).reshape(-1)[:n * m].reshape(n, m)[:, :full.shape[1]]
+        assert np.abs(got - full).max() < (2e-5 if epi == L.RB_STORE_F32 else 0.04)
 
 
 def test_product_many_tiles(ctx):
@@ -175,10 +197,10 @@ def test_experts(ctx, kind, n, E, top, tile):
         y[q] = f64(dn)[ids[q]] @ f64(act)[q]
     assert np.abs(f64(act) - A).max() < tol * 8
     e.w_stride = C_ * ff
-    yd = torch.zeros(n * top, C_, device="cuda")
-    p = L.RbProduct(dn.data_ptr(), act.data_ptr(), yd.data_ptr(), None, ff, C_, 0, typ, C_, ff, n, L.RB_STORE_F32, 0, L.RB_DOWN, 0.0, C.pointer(e))
+    yd = torch.zeros(n * top, C_, dtype=dt, device="cuda")
+    p = L.RbProduct(dn.data_ptr(), act.data_ptr(), yd.data_ptr(), None, ff, C_, 0, typ, C_, ff, n, L.RB_STORE, 0, L.RB_DOWN, 0.0, C.pointer(e))
     L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
-    assert np.abs(f64(yd) - y).max() < 2e-5
+    assert np.abs(f64(yd) - y).max() < tol * 4
     z = torch.zeros(n, C_, device="cuda")
     p = L.RbProduct(dn.data_ptr(), act.data_ptr(), z.data_ptr(), res.data_ptr(), ff, C_, C_, typ, C_, ff, n, L.RB_RESIDUAL, 0, L.RB_SUM, 1.25, C.pointer(e))
     rc = ctx.hip.kf_rb_linear(ctx.h, C.byref(p))

@@ -129,7 +129,7 @@ def test_slots_give_the_same_whatever_else_runs(served):
     da = np.concatenate([x.run([(0, 40 + i, t[40 + i:41 + i])], [(0, 0)]) for i in range(10)])
     b = x.run([(1, 0, other[:63]), (2, 0, t[:40])], [(1, i) for i in range(40)])
     db = np.concatenate([x.run([(1, 63 + i % 7, [5]), (2, 40 + i, t[40 + i:41 + i])], [(1, 0)]) for i in range(7)])
-    tol = 1e-5 if m.dtype == "float32" else 0.03
+    tol = 1e-5 if m.dtype == "float32" else TOL["bfloat16"]   # (40 rows and 103 take different kernels: another set of bf16 roundings)
     assert rel(b, a).max() < tol and rel(db, da[:7]).max() < tol
     x.close()
 
