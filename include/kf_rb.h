@@ -95,7 +95,8 @@ int kf_rb_norm(kf_ctx* ctx, int type, const void* z, const float* res, float alp
  * There is no v: a row's value is its k column block as the projection left it.  q and k: RMS norm per head, then the leading rot_dims dimensions turned by the table
  * `rope`, dimension i together with i + rot_dims / 2.  Scores are scale * <q, k>; with chunk > 0 a query sees only its own chunk (positions c chunk .. (c + 1) chunk - 1) up to
  * itself, with chunk 0 everything up to itself.  out [rows][ldout], columns n_head * dim: softmax-weighted values, times sigmoid(gate) when gated.
- * The state: k (normed, rotated) and v rows of slot s, position j at cache[s * slot_stride + (j % cache_rows) * n_kv * dim]; cache_rows >= min(chunk, positions). */
+ * The state: kv-head g's key (normed, rotated) and value of position j in slot s lie at cache[s * slot_stride + (g * cache_rows + j % cache_rows) * dim]; cache_rows >=
+ * min(chunk, positions).  scratch holds arrival counters: zero it once after allocation. */
 typedef struct kf_rb_attention {
     void* raw;
     void* out;

@@ -22,6 +22,9 @@ typedef float f32x16_t __attribute__((ext_vector_type(16)));
 
 constexpr float RB_LOG2E = 1.44269502162933349609375f;
 __device__ __forceinline__ float rb_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ void rb_st_sc1(float* p, float v) { __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
+__device__ __forceinline__ float rb_ld_sc1(const float* p) { return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
+constexpr int RB_CNT_STRIDE = 16; /* words between arrival counters: one cache line each */
 __device__ __forceinline__ int rb_first_key(int pos, int chunk) { return chunk > 0 ? pos - pos % chunk : 0; }
 
 // one head (dim elements at src) normed and rotated by one wave into dst; buf: dim floats of LDS of this wave
@@ -70,7 +73,7 @@ __global__ void __launch_bounds__(256) rb_prep_kernel(const kf_rb_attention a, c
     const T* k = raw + (size_t)u * a.dim;
     T* dst;
     if constexpr (STORE) {
-        const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * kvd + (size_t)g * a.dim;
+        const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + ((size_t)g * a.cache_rows + pos % a.cache_rows) * a.dim;
         dst = reinterpret_cast<T*>(a.k_cache) + at;
         T* v = reinterpret_cast<T*>(a.v_cache) + at;
         for (int i = lane; i < a.dim; i += 64) v[i] = k[i];
@@ -79,17 +82,62 @@ __global__ void __launch_bounds__(256) rb_prep_kernel(const kf_rb_attention a, c
     }
     rb_prep_head(k, dst, reinterpret_cast<const T*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, buf, lane);
 }
+// the prompt form, bf16, L lanes per head: lane j < rot / 8 holds the rotation pairs 4 j .. 4 j + 3 (a quad of each half), the next lanes a quad of the dimensions behind
+template <int L>
+__global__ void __launch_bounds__(256) rb_prep_vec_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta) {
+    const int r = blockIdx.x, u = blockIdx.y * (256 / L) + (int)threadIdx.x / L, j = threadIdx.x % L;
+    const int pos = meta[KF_RB_META * r];
+    const bool head_on = pos >= 0 && u < a.n_head + a.n_kv;
+    uint16_t* src = reinterpret_cast<uint16_t*>(a.raw) + (size_t)r * a.ldraw + (size_t)(head_on ? u : 0) * a.dim;
+    const bool key = u >= a.n_head;
+    uint16_t* dst = key ? reinterpret_cast<uint16_t*>(a.k_new) + ((size_t)r * a.n_kv + (u - a.n_head)) * a.dim : src;
+    const uint16_t* w = reinterpret_cast<const uint16_t*>(key ? a.k_norm : a.q_norm);
+    const int half = a.rot_dims / 2, np = a.rot_dims / 8, i0 = j < np ? 4 * j : a.rot_dims + 4 * (j - np);
+    const bool on = head_on && i0 < a.dim, pair = on && j < np;
+    f32x4 x = f32x4{0.f, 0.f, 0.f, 0.f}, y = x;
+    if (on) x = rb_ld4(src + i0);
+    if (pair) y = rb_ld4(src + i0 + half);
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; e++) ss = fmaf(x[e], x[e], fmaf(y[e], y[e], ss));
+#pragma unroll
+    for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
+    if (!on) return;
+    const float rs = 1.0f / sqrtf(ss / (float)a.dim + a.eps);
+    const f32x4 wx = rb_ld4(w + i0);
+#pragma unroll
+    for (int e = 0; e < 4; e++) x[e] *= rs * wx[e];
+    if (pair) {
+        const f32x4 wy = rb_ld4(w + i0 + half);
+        const f32x4* cs = reinterpret_cast<const f32x4*>(a.rope + ((size_t)pos * half + i0) * 2);
+        const f32x4 c01 = cs[0], c23 = cs[1];
+        const float co[4] = {c01.x, c01.z, c23.x, c23.z}, si[4] = {c01.y, c01.w, c23.y, c23.w};
+        f32x4 p, q;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const float yy = y[e] * rs * wy[e];
+            p[e] = x[e] * co[e] - yy * si[e], q[e] = yy * co[e] + x[e] * si[e];
+        }
+        rb_st4(dst + i0, p), rb_st4(dst + i0 + half, q);
+    } else {
+        rb_st4(dst + i0, x);
+    }
+}
 // ---- the batch's last cache_rows keys / values of every sequence into its slot's ring
 template <class T>
 __global__ void __launch_bounds__(256) rb_store_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta) {
     const int r = blockIdx.x, pos = meta[KF_RB_META * r], last = meta[KF_RB_META * r + 3];
     if (pos < 0 || pos <= last - a.cache_rows) return;
     const int kvd = a.n_kv * a.dim;
-    const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * kvd;
+    const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * a.dim, head = (size_t)a.cache_rows * a.dim;
     const T* k = reinterpret_cast<const T*>(a.k_new) + (size_t)r * kvd;
     const T* v = reinterpret_cast<const T*>(a.raw) + (size_t)r * a.ldraw + (size_t)a.n_head * a.dim;
     T *kc = reinterpret_cast<T*>(a.k_cache) + at, *vc = reinterpret_cast<T*>(a.v_cache) + at;
-    for (int i = threadIdx.x; i < kvd; i += blockDim.x) kc[i] = k[i], vc[i] = v[i];
+    for (int i = threadIdx.x; i < kvd; i += blockDim.x) {
+        const int g = i / a.dim;
+        const size_t o = g * head + (i - g * a.dim);
+        kc[o] = k[i], vc[o] = v[i];
+    }
 }
 
 // ---- the plain form: one wave per (row, head); scores of 64 keys at a time, one key per lane, then the values with one dimension per lane.
@@ -122,7 +170,7 @@ __global__ void __launch_bounds__(64) rb_attn_plain_kernel(const kf_rb_attention
                 k = reinterpret_cast<const T*>(a.k_new) + row * kvd + (size_t)g * a.dim;
                 v = raw + row * a.ldraw + (size_t)(a.n_head + g) * a.dim;
             } else {
-                const size_t at = (size_t)slot * a.slot_stride + (size_t)(key % a.cache_rows) * kvd + (size_t)g * a.dim;
+                const size_t at = (size_t)slot * a.slot_stride + ((size_t)g * a.cache_rows + key % a.cache_rows) * a.dim;
                 k = reinterpret_cast<const T*>(a.k_cache) + at, v = reinterpret_cast<const T*>(a.v_cache) + at;
             }
             float d = 0.f;
@@ -249,8 +297,8 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
     if (bx * 128 >= ncol) return; /* workgroup-uniform */
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw;
     const uint16_t *k_new = reinterpret_cast<const uint16_t*>(a.k_new) + (size_t)row0 * kvd + (size_t)g * a.dim, *v_new = raw + (size_t)(a.n_head + g) * a.dim;
-    const uint16_t* k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
-    const uint16_t* v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.dim;
+    const uint16_t* k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.cache_rows * a.dim;
+    const uint16_t* v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.cache_rows * a.dim;
     // this lane pair's column; columns past the end repeat the last one and are not stored
     int c = bx * 128 + wid * 32 + r;
     const bool col_ok = c < ncol;
@@ -286,7 +334,7 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
                     ok = (uint32_t)(kk - pos0) * ldk, ov = (uint32_t)(kk - pos0) * ldv;
                 } else {
                     kb = k_ring, vb = v_ring;
-                    ok = ov = ((uint32_t)kk % ring) * ldk;
+                    ok = ov = ((uint32_t)kk % ring) * (uint32_t)a.dim;
                 }
                 kr[i] = *reinterpret_cast<const u32x4*>(kb + (ok + d)), vr[i] = *reinterpret_cast<const u32x4*>(vb + (ov + d));
             }
@@ -370,13 +418,13 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     const int first = rb_first_key(pos, a.chunk), k_lo = first + (int)blockIdx.y * span, k_hi = k_lo + span - 1 < pos ? k_lo + span - 1 : pos;
     if (k_lo > pos) return;
     const int GQ = a.n_head / a.n_kv, ncb = (GQ + 31) / 32, g = blockIdx.x / ncb, cb = blockIdx.x % ncb, col0 = cb * 32, ncol = GQ - col0 < 32 ? GQ - col0 : 32;
-    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5, kvd = a.n_kv * a.dim;
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5;
     uint16_t* s_q = reinterpret_cast<uint16_t*>(smem_raw);                              /* [32][KS] */
     uint16_t* s_new = s_q + 32 * KS;                                                    /* the new key, the new value: [2][HD] */
     float* s_buf = reinterpret_cast<float*>(smem_raw + 32 * KS * 2 + 4 * HD);           /* [4][HD] */
     uint16_t* s_kv = reinterpret_cast<uint16_t*>(smem_raw + 32 * KS * 2 + 4 * HD + 16 * HD); /* [4 waves] [32][KS] + [32][VS] */
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)rr * a.ldraw;
-    const size_t base = (size_t)slot * a.slot_stride + (size_t)g * a.dim;
+    const size_t base = (size_t)slot * a.slot_stride + (size_t)g * a.cache_rows * a.dim;
     uint16_t *kc = reinterpret_cast<uint16_t*>(a.k_cache) + base, *vc = reinterpret_cast<uint16_t*>(a.v_cache) + base;
     constexpr int CPT = CH / 2; /* chunks per lane of a 32-row tile */
     u32x4 kr[CPT], vr[CPT];
@@ -387,7 +435,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
             kr[i] = vr[i] = u32x4{0, 0, 0, 0};
             if (d < a.dim) {
                 const int kk = k0 + key < k_hi ? k0 + key : k_hi;
-                const uint32_t at = ((uint32_t)kk % (uint32_t)a.cache_rows) * (uint32_t)kvd + d;
+                const uint32_t at = ((uint32_t)kk % (uint32_t)a.cache_rows) * (uint32_t)a.dim + d;
                 kr[i] = *reinterpret_cast<const u32x4*>(kc + at), vr[i] = *reinterpret_cast<const u32x4*>(vc + at);
             }
         }
@@ -402,7 +450,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
         } else if (k_hi == pos) {
             const uint16_t* k = raw + (size_t)(a.n_head + g) * a.dim;
             rb_prep_head(k, s_new, reinterpret_cast<const uint16_t*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
-            const size_t at = (size_t)(pos % a.cache_rows) * kvd;
+            const size_t at = (size_t)(pos % a.cache_rows) * a.dim;
             for (int i = lane; i < HD; i += 64) {
                 const bool in = i < a.dim;
                 const uint16_t v = in ? k[i] : (uint16_t)0;
@@ -455,13 +503,14 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
         f[w] = rb_exp2(ex[((size_t)w * (NREG + 2) + NREG) * 64 + lane] - M);
         L += f[w] * ex[((size_t)w * (NREG + 2) + NREG + 1) * 64 + lane];
     }
-    if (r >= ncol) return;
-    const int head = g * GQ + col0 + r;
+    const int n_used = (pos - first) / span + 1; /* key ranges this row has */
+    const int head = g * GQ + col0 + (r < ncol ? r : 0);
     const uint16_t* gate = raw + (size_t)(a.n_head + a.n_kv + head) * a.dim;
     uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)rr * a.ldout + (size_t)head * a.dim;
-    float* part = reinterpret_cast<float*>(a.scratch) + (((size_t)rr * a.n_head + head) * n_range + blockIdx.y) * (a.dim + 2);
+    float* parts = reinterpret_cast<float*>(a.scratch) + RB_CNT_STRIDE * (size_t)gridDim.z * a.n_head; /* behind the arrival counters: [row][head][range][dim + 2] */
+    float* part = parts + (((size_t)rr * a.n_head + head) * n_range + blockIdx.y) * (a.dim + 2);
     const float inv = 1.0f / L;
-    for (int q = wid; q < Tile::NDB * 4; q += 4) { /* a quad of registers = four consecutive d */
+    for (int q = wid; q < Tile::NDB * 4 && r < ncol; q += 4) { /* a quad of registers = four consecutive d */
         const int d = 8 * q + 4 * h;
         if (d >= a.dim) continue;
         f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -469,9 +518,9 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
         for (int w = 0; w < 4; w++)
 #pragma unroll
             for (int j = 0; j < 4; j++) v[j] = fmaf(f[w], ex[((size_t)w * (NREG + 2) + 4 * q + j) * 64 + lane], v[j]);
-        if (n_range > 1) {
+        if (n_used > 1) {
 #pragma unroll
-            for (int j = 0; j < 4; j++) part[2 + d + j] = v[j];
+            for (int j = 0; j < 4; j++) rb_st_sc1(part + 2 + d + j, v[j]);
         } else {
             const f32x4 gv = a.gated ? rb_ld4(gate + d) : f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -479,25 +528,50 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
             rb_st4(out + d, v);
         }
     }
-    if (n_range > 1 && wid == 0 && h == 0) part[0] = M, part[1] = L;
-}
-__global__ void __launch_bounds__(64) rb_attn_combine_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta, int span, int n_range) {
-    const int rr = blockIdx.y, head = blockIdx.x, lane = threadIdx.x, pos = meta[KF_RB_META * rr];
-    if (pos < 0) return;
-    const int used = (pos - rb_first_key(pos, a.chunk)) / span + 1;
-    const float* part = reinterpret_cast<const float*>(a.scratch) + ((size_t)rr * a.n_head + head) * n_range * (a.dim + 2);
-    float M = -__builtin_inff(), L = 0.f;
-    for (int s = 0; s < used; s++) M = fmaxf(M, part[(size_t)s * (a.dim + 2)]);
-    for (int s = 0; s < used; s++) L += rb_exp2(part[(size_t)s * (a.dim + 2)] - M) * part[(size_t)s * (a.dim + 2) + 1];
-    const uint16_t* gate = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)rr * a.ldraw + (size_t)(a.n_head + a.n_kv + head) * a.dim;
-    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)rr * a.ldout + (size_t)head * a.dim;
-    for (int d = lane; d < a.dim; d += 64) {
-        float v = 0.f;
-        for (int s = 0; s < used; s++) v = fmaf(rb_exp2(part[(size_t)s * (a.dim + 2)] - M), part[(size_t)s * (a.dim + 2) + 2 + d], v);
-        out[d] = f2bf(v / L * (a.gated ? rb_sigmoid(bf2f(gate[d])) : 1.f));
+    if (n_used == 1) return;
+    // the ranges' parts leave with write-through stores; every wave has their acknowledgements before one lane counts the workgroup in; the last one in merges and puts the
+    // counter back to zero (kf_attn.hip's scheme)
+    if (wid == 0 && h == 0 && r < ncol) rb_st_sc1(part, M), rb_st_sc1(part + 1, L);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    int* s_last = reinterpret_cast<int*>(s_buf);
+    int* counter = reinterpret_cast<int*>(a.scratch) + RB_CNT_STRIDE * ((size_t)rr * a.n_head + blockIdx.x);
+    if (tid == 0) *s_last = __hip_atomic_fetch_add(counter, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == n_used - 1;
+    __syncthreads();
+    if (!*s_last) return;
+    if (tid == 0) __hip_atomic_store(counter, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    for (int c = wid; c < ncol; c += 4) {
+        const int hd = g * GQ + col0 + c;
+        const float* p = parts + ((size_t)rr * a.n_head + hd) * n_range * (a.dim + 2);
+        const bool mine = lane < n_used;
+        const float ms = mine ? rb_ld_sc1(p + (size_t)lane * (a.dim + 2)) : -__builtin_inff(), ls = mine ? rb_ld_sc1(p + (size_t)lane * (a.dim + 2) + 1) : 0.f;
+        const float fs = rb_exp2(ms - wave_max(ms)), tot = 1.0f / wave_sum(fs * ls);
+        constexpr int DPL = (HD + 63) / 64;
+        float v[DPL];
+#pragma unroll
+        for (int e = 0; e < DPL; e++) v[e] = 0.f;
+        for (int s0 = 0; s0 < n_used; s0 += 8) {
+            float w[DPL][8];
+#pragma unroll
+            for (int e = 0; e < DPL; e++)
+#pragma unroll
+                for (int s = 0; s < 8; s++) w[e][s] = s0 + s < n_used && lane + 64 * e < a.dim ? rb_ld_sc1(p + (size_t)(s0 + s) * (a.dim + 2) + 2 + lane + 64 * e) : 0.f;
+#pragma unroll
+            for (int s = 0; s < 8; s++) {
+                const float f1 = __shfl(fs, (s0 + s) & 63, 64); /* past n_used: exp2(-inf) = 0 */
+#pragma unroll
+                for (int e = 0; e < DPL; e++) v[e] = fmaf(f1, w[e][s], v[e]);
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < DPL; e++) {
+            const int d = lane + 64 * e;
+            if (d < a.dim)
+                reinterpret_cast<uint16_t*>(a.out)[(size_t)rr * a.ldout + (size_t)hd * a.dim + d] =
+                    f2bf(v[e] * tot * (a.gated ? rb_sigmoid(bf2f(raw[(size_t)(a.n_head + a.n_kv + hd) * a.dim + d])) : 1.f));
+        }
     }
 }
-
 constexpr int RB_MAX_RANGES = 32;
 static void decode_ranges(int n_rows, int n_kv, int keys, int& span, int& n_range) {
     n_range = (keys + 255) / 256; /* a range is at least two tiles per wave */
@@ -540,7 +614,6 @@ static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* me
     if (big_lds(rb_attn_decode_kernel<HD>, smem, done)) return KF_HIP_CHECK;
     const int ncb = (a.n_head / a.n_kv + 31) / 32;
     hipLaunchKernelGGL(rb_attn_decode_kernel<HD>, dim3(a.n_kv * ncb, n_range, n_rows), dim3(256), smem, st, a, meta, span, n_range);
-    if (n_range > 1) hipLaunchKernelGGL(rb_attn_combine_kernel, dim3(a.n_head, n_rows), dim3(64), 0, st, a, meta, span, n_range);
     return KF_OK;
 }
 static bool mfma_served(const kf_rb_attention& a, int n_rows) {
@@ -554,10 +627,22 @@ static bool mfma_served(const kf_rb_attention& a, int n_rows) {
      : a.dim <= 192 ? call(192)               \
                     : call(256))
 
+/* vector form of the prep of a prompt batch: a head's lanes fit 16 or 32, quads of both halves */
+static int prep_vec_lanes(const kf_rb_attention& a) {
+    if (a.type != KF_BF16 || a.dim % 4 || a.rot_dims % 8 || a.ldraw % 4 || !a.q_norm || !a.k_norm) return 0;
+    const int need = a.rot_dims / 8 + (a.dim - a.rot_dims) / 4;
+    return need <= 16 ? 16 : (need <= 32 ? 32 : 0);
+}
 template <class T>
 static void prep_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n, bool store) {
     const dim3 grid(n, (a.n_head + a.n_kv + 3) / 4);
     const size_t smem = 4 * (size_t)a.dim * sizeof(float);
+    if (const int L = store ? 0 : prep_vec_lanes(a)) {
+        const dim3 vgrid(n, (a.n_head + a.n_kv + 256 / L - 1) / (256 / L));
+        if (L == 16) hipLaunchKernelGGL(rb_prep_vec_kernel<16>, vgrid, dim3(256), 0, st, a, meta);
+        else hipLaunchKernelGGL(rb_prep_vec_kernel<32>, vgrid, dim3(256), 0, st, a, meta);
+        return;
+    }
     if (store) hipLaunchKernelGGL((rb_prep_kernel<T, true>), grid, dim3(256), smem, st, a, meta);
     else hipLaunchKernelGGL((rb_prep_kernel<T, false>), grid, dim3(256), smem, st, a, meta);
 }
@@ -587,7 +672,7 @@ static int check_attention(const kf_rb_attention* a, const int32_t* meta, int n,
 }
 extern "C" {
 
-size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim) { return n_rows < 1 || n_head < 1 || dim < 1 ? 0 : (size_t)n_rows * n_head * RB_MAX_RANGES * (dim + 2) * sizeof(float); }
+size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim) { return n_rows < 1 || n_head < 1 || dim < 1 ? 0 : (size_t)n_rows * n_head * (RB_CNT_STRIDE + (size_t)RB_MAX_RANGES * (dim + 2)) * sizeof(float); }
 
 int kf_rb_attention_prefill(kf_ctx* c, const kf_rb_attention* ap, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n) {
     CHKCTX(c);

@@ -122,13 +122,28 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
         static_assert(NT == 1, "a few rows");
         uint16_t* sx = reinterpret_cast<uint16_t*>(smem_raw); /* [n][k + 8] */
         float* part = &red[0][0][0][0];                       /* [NW][RB_NORM_ROWS] sums of squares: 8 NW floats of the (unused so far) partial tiles */
+        constexpr int NQ = 4; /* quads of z a thread keeps (one row of up to 1024 NW columns); more are read again */
+        const int per = (p.k + 256 * NW - 1) / (256 * NW), nq = per * p.n;
+        f32x4 zq[NQ], gq[NQ];
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            const int c = 4 * tid + (i % per) * 256 * NW;
+            zq[i] = gq[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (i < nq && c < p.k) zq[i] = rb_ld4(p.norm_z + (size_t)(i / per) * p.ldx + c), gq[i] = rb_ld4(reinterpret_cast<const uint16_t*>(p.norm_w) + c);
+        }
         for (int t = 0; t < p.n; t++) {
             float ss = 0.f;
-            for (int c = 4 * tid; c < p.k; c += 256 * NW) {
-                const f32x4 v = rb_ld4(p.norm_z + (size_t)t * p.ldx + c);
+            auto add = [&](int c, const f32x4& v) {
 #pragma unroll
                 for (int j = 0; j < 4; j++)
                     if (c + j < p.norm_dim) ss = fmaf(v[j], v[j], ss);
+            };
+            if (nq <= NQ) {
+#pragma unroll
+                for (int i = 0; i < NQ; i++)
+                    if (i / per == t) add(4 * tid + (i % per) * 256 * NW, zq[i]);
+            } else {
+                for (int c = 4 * tid; c < p.k; c += 256 * NW) add(c, rb_ld4(p.norm_z + (size_t)t * p.ldx + c));
             }
             ss = wave_sum(ss);
             if (lane == 0) part[wid * RB_NORM_ROWS + t] = ss;
@@ -139,8 +154,7 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
 #pragma unroll
             for (int w = 0; w < NW; w++) ss += part[w * RB_NORM_ROWS + t];
             const float rs = 1.0f / sqrtf(ss / (float)p.norm_dim + p.norm_eps);
-            for (int c = 4 * tid; c < p.k; c += 256 * NW) {
-                const f32x4 v = rb_ld4(p.norm_z + (size_t)t * p.ldx + c), g = rb_ld4(reinterpret_cast<const uint16_t*>(p.norm_w) + c);
+            auto put = [&](int c, const f32x4& v, const f32x4& g) {
                 f32x4 o;
 #pragma unroll
                 for (int j = 0; j < 4; j++) o[j] = c + j < p.norm_dim ? v[j] * rs * g[j] : 0.f;
@@ -149,6 +163,13 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
                     rb_st4(p.norm_x + (size_t)t * p.ldx + c, o);
                     rb_st4(reinterpret_cast<uint16_t*>(const_cast<void*>(p.x)) + (size_t)t * p.ldx + c, o);
                 }
+            };
+            if (nq <= NQ) {
+#pragma unroll
+                for (int i = 0; i < NQ; i++)
+                    if (i / per == t && 4 * tid + (i % per) * 256 * NW < p.k) put(4 * tid + (i % per) * 256 * NW, zq[i], gq[i]);
+            } else {
+                for (int c = 4 * tid; c < p.k; c += 256 * NW) put(c, rb_ld4(p.norm_z + (size_t)t * p.ldx + c), rb_ld4(reinterpret_cast<const uint16_t*>(p.norm_w) + c));
             }
         }
         __syncthreads();

@@ -73,7 +73,8 @@ struct KVCache {
     int n_layer = 0, max_seq_len = 0, kv_dim = 0;
     int Init(kf_ctx* c, int n_layer, int max_seq, int kv_dim);
     void* Get(CTYPE type, int layer, int pos) const;  // Cache.cpp:42-57
-    // Per-layer rings: layer l of slot s keeps the last `rows` positions (what the layer's mask can still see), position p in row p % rows, a row = dim elements; all
+    // Per-layer rings: layer l of slot s keeps the last `rows` positions (what the layer's mask can still see), position p in row p % rows, dim elements per position (the kv-heads' rows
+    // one head after the other); all
     // slots of a layer together, a slot rows * dim elements after the one before
     struct Ring {
         int rows = 0, dim = 0;
