@@ -4,6 +4,9 @@
  * every mechanism (activation, chunk size, rotation, gate, scale, experts ...) as a parameter and exist in two storages: KF_BF16 (bf16 operands, 32-bit accumulation)
  * and KF_F32 (true 32-bit throughout).  Conventions of kf_abi.h apply: device pointers, a stream of one ctx, 0 or a negative code, no allocation.
  *
+ * Weights of a product in bf16 are stored as MFMA operands: tiles of 16 rows x 32 columns, 1 KB each, in row-of-tiles order; inside a tile the 16-byte piece of row r, columns
+ * 8 q .. 8 q + 7 (q < 4) is number 16 q + r -- a wave reads a tile as one contiguous kilobyte, whichever lane it hands a piece to.  fp32 weights stay row-major.
+ *
  * Padding: the widths a product runs over are padded with zeros to multiples of KF_RB_PAD in weights and activations alike, weight rows too: tile kernels need no tails.
  */
 #ifndef KF_RB_H
@@ -15,6 +18,7 @@ extern "C" {
 #endif
 
 #define KF_RB_PAD 64
+#define KF_RB_NORM_ROWS 4
 #define KF_RB_DECODE_MAX 64 /* rows of a decode batch the streaming products serve; larger batches take the tile kernels */
 
 /* activations; GELU in its tanh form, as kf_gelu */
@@ -47,7 +51,7 @@ typedef struct kf_rb_experts {
 enum kf_rb_experts_mode { KF_RB_ALL = 0, KF_RB_UP = 1, KF_RB_DOWN = 2, KF_RB_SUM = 3 };
 
 typedef struct kf_rb_product {
-    const void* w;   /* [m][k] row-major (x n_expert) */
+    const void* w;   /* [m][k] (x n_expert), bf16: in tiles */
     const void* x;   /* rows ldx apart */
     void* y;         /* rows ldy apart */
     const float* res;
@@ -58,9 +62,13 @@ typedef struct kf_rb_product {
     int32_t epilogue, act, mode;
     float alpha;
     const kf_rb_experts* experts;
-    /* norm_z != NULL (decode batches for which kf_rb_linear_norms() says 1, mode ALL): x is FIRST formed as the RMS norm (norm_w, norm_eps, norm_dim columns) of the fp32 rows
-     * norm_z -- rows ldx = k apart, like x -- inside the launch, and left in x (bf16) and norm_x (fp32): kf_rb_norm and the product in one */
+    /* The norm between two products of a decode batch inside the second (where kf_rb_linear_norms() says 1):
+     *   ssq != NULL (RESIDUAL): the sums of squares of y's columns 16 i .. 16 i + 15 go to ssq[i][KF_RB_NORM_ROWS] (row t in column t)
+     *   norm_z != NULL (mode ALL): x is FIRST formed as the RMS norm (norm_w, norm_eps, norm_dim columns; pad columns of norm_z and norm_w zero) of the fp32 rows norm_z --
+     *     rows ldx = k apart, like x, their sums of squares in norm_ssq -- and left in x (bf16) and norm_x (fp32): kf_rb_norm and the product in one */
+    float* ssq;
     const float* norm_z;
+    const float* norm_ssq;
     const void* norm_w;
     float* norm_x;
     float norm_eps;
@@ -69,9 +77,10 @@ typedef struct kf_rb_product {
 int kf_rb_linear(kf_ctx* ctx, const kf_rb_product* p);
 int kf_rb_linear_norms(int type, int n, int k);
 
-/* load time: a bf16 matrix src [rows][cols] into a padded one of storage `type` with rows ld apart (columns cols .. ld - 1 are left alone: allocate zeroed).
- * half < 0: row r goes to row r; half 0 / 1: to row 32 (r / 16) + 16 half + r % 16, the gate / up halves of a GATED product's weight */
-int kf_rb_pack(kf_ctx* ctx, int type, const kf_bf16* src, int rows, int cols, void* dst, int64_t ld, int half);
+/* load time: a bf16 matrix src [rows][cols] into rows row0 .. of a padded one (ld columns; columns cols .. ld - 1 are left alone: allocate zeroed) of storage `type`.
+ * half < 0: row r goes to row row0 + r; half 0 / 1: to row 32 (r / 16) + 16 half + r % 16, the gate / up halves of a GATED product's weight.  tiled (bf16): a product's
+ * weight; otherwise row-major (embedding tables, norm weights) */
+int kf_rb_pack(kf_ctx* ctx, int type, const kf_bf16* src, int rows, int cols, void* dst, int64_t ld, int row0, int half, int tiled);
 
 /* tokens -> rows of the table: x fp32 [n][ldx] and h (storage `type`) [n][ldx]; columns dim .. ldx - 1 are written as zeros.  table rows are ldx apart too. */
 int kf_rb_embed(kf_ctx* ctx, int type, const void* table, int vocab, int dim, int64_t ldx, const int32_t* tokens, int n, float* x, void* h);

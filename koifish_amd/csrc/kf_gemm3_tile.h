@@ -81,11 +81,16 @@ __device__ __forceinline__ bf16x8 g3_frag_km(const unsigned char* tile, int rowb
 // 1000 on the forward shapes at 246 VGPRs, and the k-major forms spill; four waves of 128 x 128 outputs each (256 accumulator AGPRs, a third less LDS traffic per MFMA,
 // the vendor library's shape): the compiler fills all 512 registers and still spills inside the loop, 228 TFLOP/s -- that form needs a hand-scheduled loop.
 // `rows` (G3Rows: plain; G3Gather: row r of the token tile is row map[r] of x) says where the tile's token rows lie.
+// TILED: w is stored in MFMA tiles (kf_rb.h: 16 rows x 32 columns, piece (r, q) at number 16 q + r) instead of rows: a load
+// instruction moves one tile, contiguous in memory and in LDS, and a fragment read is lane-linear -- no swizzle on this operand.
 struct G3Rows {
-    static constexpr bool GATHER = false;
+    static constexpr bool GATHER = false, TILED = false;
 };
-struct G3Gather {
-    static constexpr bool GATHER = true;
+struct G3Tiled {
+    static constexpr bool GATHER = false, TILED = true;
+};
+struct G3GatherTiled {
+    static constexpr bool GATHER = true, TILED = true;
     const int32_t* map; /* [BN] rows of x, every entry valid */
 };
 template <bool AKM, bool BKM, int BK, class C, class ROWS = G3Rows>
@@ -100,7 +105,15 @@ __device__ __forceinline__ void g3_mainloop(const GemmArgs& a, int m0, int t0, i
     // Per-lane source pointers are set up once; a step adds a uniform offset (a 64-bit multiply per load and step was a tenth of the loop's issue slots).
     const uint16_t *pa[C::NIA], *pb[C::NIB];
 #pragma unroll
-    for (int i = 0; i < C::NIA; i++) pa[i] = AKM ? g3_src_km<BK, C::BM, C::NIA>(W, a.ldr, m0, a.M, i, wid, lane) : g3_src<BK, C::NIA>(W, a.K, m0, a.M, i, wid, lane);
+    for (int i = 0; i < C::NIA; i++) {
+        if constexpr (ROWS::TILED) {
+            static_assert(!AKM && BK == 64, "two tiles per row block and step");
+            const int j = wid * C::NIA + i, last = (a.M - 1) >> 4, rb = (m0 >> 4) + (j >> 1); /* tile (row block j / 2, k-half j % 2) */
+            pa[i] = W + ((size_t)(rb < last ? rb : last) * (a.K / 32) + (j & 1)) * 512 + lane * 8;
+            continue;
+        }
+        pa[i] = AKM ? g3_src_km<BK, C::BM, C::NIA>(W, a.ldr, m0, a.M, i, wid, lane) : g3_src<BK, C::NIA>(W, a.K, m0, a.M, i, wid, lane);
+    }
 #pragma unroll
     for (int i = 0; i < C::NIB; i++) {
         if constexpr (ROWS::GATHER) {
@@ -111,7 +124,7 @@ __device__ __forceinline__ void g3_mainloop(const GemmArgs& a, int m0, int t0, i
             pb[i] = BKM ? g3_src_km<BK, C::BN, C::NIB>(a.x, a.ldx, t0, a.n, i, wid, lane) : g3_src<BK, C::NIB>(a.x, a.ldx, t0, a.n, i, wid, lane);
         }
     }
-    const long long stepA = AKM ? (long long)BK * a.ldr : BK, stepB = BKM ? (long long)BK * a.ldx : BK;
+    const long long stepA = ROWS::TILED ? 1024 : (AKM ? (long long)BK * a.ldr : BK), stepB = BKM ? (long long)BK * a.ldx : BK;
     auto stage = [&](int kt, int b) {
         const long long oa = stepA * kt, ob = stepB * kt;
 #pragma unroll
@@ -146,7 +159,8 @@ __device__ __forceinline__ void g3_mainloop(const GemmArgs& a, int m0, int t0, i
             }
 #pragma unroll
             for (int mt = 0; mt < C::MT; mt++) {
-                if constexpr (AKM) af[mt] = g3_frag_km<C::BM>(bufA(cur), wm * C::MT + mt, kk * 32 + 8 * q4, r16);
+                if constexpr (ROWS::TILED) af[mt] = *reinterpret_cast<const bf16x8*>(bufA(cur) + ((wm * C::MT + mt) * 2 + kk) * 1024 + lane * 16);
+                else if constexpr (AKM) af[mt] = g3_frag_km<C::BM>(bufA(cur), wm * C::MT + mt, kk * 32 + 8 * q4, r16);
                 else af[mt] = g3_frag<BK>(bufA(cur), wm * (16 * C::MT) + mt * 16 + r16, kk * 4 + q4);
             }
 #pragma unroll

@@ -419,10 +419,11 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     if (k_lo > pos) return;
     const int GQ = a.n_head / a.n_kv, ncb = (GQ + 31) / 32, g = blockIdx.x / ncb, cb = blockIdx.x % ncb, col0 = cb * 32, ncol = GQ - col0 < 32 ? GQ - col0 : 32;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5;
-    uint16_t* s_q = reinterpret_cast<uint16_t*>(smem_raw);                              /* [32][KS] */
-    uint16_t* s_new = s_q + 32 * KS;                                                    /* the new key, the new value: [2][HD] */
-    float* s_buf = reinterpret_cast<float*>(smem_raw + 32 * KS * 2 + 4 * HD);           /* [4][HD] */
-    uint16_t* s_kv = reinterpret_cast<uint16_t*>(smem_raw + 32 * KS * 2 + 4 * HD + 16 * HD); /* [4 waves] [32][KS] + [32][VS] */
+    uint16_t* s_new = reinterpret_cast<uint16_t*>(smem_raw);             /* the new key, the new value: [2][HD] */
+    uint16_t* s_kv = s_new + 2 * HD;                                     /* [4 waves] [32][KS] + [32][VS]; before the walk: */
+    uint16_t* s_q = s_kv;                                                /* [32][KS] */
+    float* s_buf = reinterpret_cast<float*>(s_q + 32 * KS);              /* [4][HD] */
+    __shared__ int s_last;
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)rr * a.ldraw;
     const size_t base = (size_t)slot * a.slot_stride + (size_t)g * a.cache_rows * a.dim;
     uint16_t *kc = reinterpret_cast<uint16_t*>(a.k_cache) + base, *vc = reinterpret_cast<uint16_t*>(a.v_cache) + base;
@@ -464,6 +465,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     u32x4 qf[Tile::NS];
 #pragma unroll
     for (int s = 0; s < Tile::NS; s++) qf[s] = *reinterpret_cast<const u32x4*>(s_q + r * KS + 16 * s + 8 * h);
+    __syncthreads(); /* the queries are in registers: their place is a tile's from here on */
     uint16_t *ks = s_kv + (size_t)wid * WAVE_EL, *vs = ks + 32 * KS;
     Tile T;
     T.init();
@@ -534,11 +536,10 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     if (wid == 0 && h == 0 && r < ncol) rb_st_sc1(part, M), rb_st_sc1(part + 1, L);
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
-    int* s_last = reinterpret_cast<int*>(s_buf);
     int* counter = reinterpret_cast<int*>(a.scratch) + RB_CNT_STRIDE * ((size_t)rr * a.n_head + blockIdx.x);
-    if (tid == 0) *s_last = __hip_atomic_fetch_add(counter, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == n_used - 1;
+    if (tid == 0) s_last = __hip_atomic_fetch_add(counter, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == n_used - 1;
     __syncthreads();
-    if (!*s_last) return;
+    if (!s_last) return;
     if (tid == 0) __hip_atomic_store(counter, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     for (int c = wid; c < ncol; c += 4) {
         const int hd = g * GQ + col0 + c;
@@ -608,7 +609,8 @@ static int prefill_go(hipStream_t st, const kf_rb_attention& a, const int32_t* s
 template <int HD>
 static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n_rows, int span, int n_range) {
     constexpr size_t tiles = 4 * 2 * 32 * (size_t)(RbTile<HD>::KS + RbTile<HD>::VS), merge = 4 * (size_t)(RbTile<HD>::NDB * 16 + 2) * 256;
-    constexpr size_t smem = 32 * RbTile<HD>::KS * 2 + 20 * HD + (tiles > merge ? tiles : merge);
+    constexpr size_t smem = 4 * HD + (tiles > merge ? tiles : merge);
+    static_assert(32 * RbTile<HD>::KS * 2 + 16 * HD <= tiles, "queries in the tiles' place");
     static_assert(smem <= 160 * 1024, "LDS");
     static int done = 0;
     if (big_lds(rb_attn_decode_kernel<HD>, smem, done)) return KF_HIP_CHECK;

@@ -38,9 +38,9 @@ __global__ void __launch_bounds__(C::NTH, C::WGS_PER_CU * C::NW / 4) rb_gemm_ker
             s_dst[i] = pair, s_src[i] = pair < 0 ? 0 : (p.mode == KF_RB_UP ? pair / q.e.top : pair);
         }
         __syncthreads();
-        g3_mainloop<false, false, G3_BK, C, G3Gather>(a, m0, 0, 0, p.k / G3_BK, acc, smem_raw, wid, lane, G3Gather{s_src});
+        g3_mainloop<false, false, G3_BK, C, G3GatherTiled>(a, m0, 0, 0, p.k / G3_BK, acc, smem_raw, wid, lane, G3GatherTiled{s_src});
     } else {
-        g3_mainloop<false, false, G3_BK, C>(a, m0, t0, 0, p.k / G3_BK, acc, smem_raw, wid, lane);
+        g3_mainloop<false, false, G3_BK, C, G3Tiled>(a, m0, t0, 0, p.k / G3_BK, acc, smem_raw, wid, lane);
     }
     const int wm = wid / C::WN, wn = wid % C::WN, r16 = lane & 15, q4 = lane >> 4;
 #pragma unroll

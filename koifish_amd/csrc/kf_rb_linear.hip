@@ -1,10 +1,10 @@
 // kf_rb_linear.hip -- row-batch products y[t][m] = W[m] . x[t] for few rows (decode batches) and in 32-bit, and the ABI entry that picks the form.
 //
-// Decode batches stream the weights: a workgroup owns 16 weight rows (GATED: 16 gate and the 16 up rows that follow them), its waves take runs of 32-deep k-steps -- 256
-// contiguous bytes of each of the 16 rows per run -- and multiply them against up to 64 token columns by v_mfma_f32_16x16x32_bf16 (A = weight rows, B = token rows, straight
-// from global memory: the activations of a decode batch are a few KB and stay in L2).  The next run's weights are in flight while a run is multiplied; the first run's
-// while the RMS norm in front of the product (NORM: few rows of the 32-bit residual sum, kept in LDS as bf16) is formed.  The waves' partial tiles meet in LDS, one thread
-// per output finishes it.  With experts a workgroup's columns are the pairs of one expert (UP, DOWN), or it walks all chosen experts' k-steps as one list dealt to its waves,
+// Decode batches stream the weights: a workgroup owns 16 weight rows (GATED: 16 gate and the 16 up rows that follow them), its waves take runs of 32-deep k-steps -- a
+// step's 16 x 32 weights are one stored tile, a contiguous kilobyte -- and multiply them against up to 64 token columns by v_mfma_f32_16x16x32_bf16 (A = weight rows, B = token rows, straight
+// from global memory: the activations of a decode batch are a few KB and stay in L2), the next run's weights in flight.  The waves' partial tiles meet in LDS, one thread
+// per output finishes it.  The RMS norm in front of a product (NORM: few rows of the 32-bit residual sum) costs no pass: the product that formed the sum left its squares
+// per 16 columns, every wave adds them up for itself and norms its token fragments as it reads them.  With experts a workgroup's columns are the pairs of one expert (UP, DOWN), or it walks all chosen experts' k-steps as one list dealt to its waves,
 // columns that did not choose an expert held at zero (SUM): an expert's rows are read once per workgroup whoever chose them.
 #include "kf_ctx.h"
 #include "kf_rb_common.h"
@@ -17,9 +17,7 @@ __device__ __forceinline__ f32x4 rb_mfma16(u32x4 a, u32x4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
-constexpr int RB_NORM_ROWS = 8, RB_NORM_LDS = 64 * 1024;
-
-// the run of U k-steps from step s of the MG 16-row blocks at wr (this lane's row and k octet; row stride k)
+// the run of U k-steps from step s of the MG 16-row blocks at wr (this lane's piece of the first block's first tile; a tile per step)
 template <int MG, int U>
 __device__ __forceinline__ void rb_load_w(u32x4 (&a)[U][MG], const uint16_t* __restrict__ wr, int k, int s, int s_end) {
 #pragma unroll
@@ -27,7 +25,7 @@ __device__ __forceinline__ void rb_load_w(u32x4 (&a)[U][MG], const uint16_t* __r
 #pragma unroll
         for (int g = 0; g < MG; g++) {
             a[u][g] = u32x4{0, 0, 0, 0};
-            if (s + u < s_end) a[u][g] = ld_nt(reinterpret_cast<const u32x4*>(wr + (size_t)g * 16 * k + 32 * (s + u))); /* wave-uniform */
+            if (s + u < s_end) a[u][g] = ld_nt(reinterpret_cast<const u32x4*>(wr + (size_t)g * 16 * k + 512 * (s + u))); /* wave-uniform */
         }
 }
 // token fragments of the same steps; xp[t]: this lane's token row + its k octet (NULLABLE: NULL is a zero column), steps past s_end read step s_end - 1 against zero weights
@@ -91,7 +89,16 @@ __device__ __forceinline__ void rb_stream_finish(const RbProduct& q, const f32x4
         } else if (p.epilogue == KF_RB_STORE_F32) {
             reinterpret_cast<float*>(p.y)[(size_t)yr * p.ldy + m0 + row] = d;
         } else {
-            reinterpret_cast<float*>(p.y)[(size_t)yr * p.ldy + m0 + row] = fmaf(p.alpha, p.res[(size_t)yr * p.ldr + m0 + row], d);
+            const float z = fmaf(p.alpha, p.res[(size_t)yr * p.ldr + m0 + row], d);
+            reinterpret_cast<float*>(p.y)[(size_t)yr * p.ldy + m0 + row] = z;
+            if (NT == 1 && p.ssq) { /* 16 lanes = the 16 columns of one row */
+                float ss = z * z;
+                ss += dpp_f<0xB1>(ss);
+                ss += dpp_f<0x4E>(ss);
+                ss += dpp_f<0x141>(ss);
+                ss += dpp_f<0x140>(ss);
+                if (row == 0) p.ssq[(size_t)(m0 / 16) * KF_RB_NORM_ROWS + yr] = ss;
+            }
         }
     }
 }
@@ -101,7 +108,6 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
     const kf_rb_product& p = q.p;
     constexpr int MG = GATED ? 2 : 1, U = NT >= 4 ? 2 : 4;
     __shared__ float red[NW][MG][16 * NT][17]; /* [wave][block][column][row], padded */
-    extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, q4 = lane >> 4;
     const int m0 = blockIdx.x * (16 * MG), nstep = p.k / 32;
     const uint16_t* W = reinterpret_cast<const uint16_t*>(p.w);
@@ -113,67 +119,25 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
         W += (size_t)ex * q.e.w_stride;
         list = q.e.list + (size_t)blockIdx.y * q.e.tile;
     }
-    const uint16_t* wr = W + (size_t)(m0 + r16) * p.k + 8 * q4;
+    const uint16_t* wr = W + (size_t)m0 * p.k + 8 * lane;
     u32x4 a[U][MG], b[U][NT];
     int s = wid * U;
     rb_load_w<MG, U>(a, wr, p.k, s, nstep);
     const uint16_t* xp[NT];
+    const float* zp = nullptr;   /* NORM: this lane's row of the residual sum, and 1 / its root mean square */
+    const uint16_t* gp = nullptr;
+    float rs = 0.f;
     if constexpr (NORM) {
         static_assert(NT == 1, "a few rows");
-        uint16_t* sx = reinterpret_cast<uint16_t*>(smem_raw); /* [n][k + 8] */
-        float* part = &red[0][0][0][0];                       /* [NW][RB_NORM_ROWS] sums of squares: 8 NW floats of the (unused so far) partial tiles */
-        constexpr int NQ = 4; /* quads of z a thread keeps (one row of up to 1024 NW columns); more are read again */
-        const int per = (p.k + 256 * NW - 1) / (256 * NW), nq = per * p.n;
-        f32x4 zq[NQ], gq[NQ];
-#pragma unroll
-        for (int i = 0; i < NQ; i++) {
-            const int c = 4 * tid + (i % per) * 256 * NW;
-            zq[i] = gq[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-            if (i < nq && c < p.k) zq[i] = rb_ld4(p.norm_z + (size_t)(i / per) * p.ldx + c), gq[i] = rb_ld4(reinterpret_cast<const uint16_t*>(p.norm_w) + c);
-        }
-        for (int t = 0; t < p.n; t++) {
+        const int row = r16 < p.n ? r16 : p.n - 1, parts = p.k / 16;
+        zp = p.norm_z + (size_t)row * p.ldx + 8 * q4, gp = reinterpret_cast<const uint16_t*>(p.norm_w) + 8 * q4;
+        for (int t = 0; t < p.n; t++) { /* the sums of squares the product in front left per 16 columns: no barrier, every wave for itself */
             float ss = 0.f;
-            auto add = [&](int c, const f32x4& v) {
-#pragma unroll
-                for (int j = 0; j < 4; j++)
-                    if (c + j < p.norm_dim) ss = fmaf(v[j], v[j], ss);
-            };
-            if (nq <= NQ) {
-#pragma unroll
-                for (int i = 0; i < NQ; i++)
-                    if (i / per == t) add(4 * tid + (i % per) * 256 * NW, zq[i]);
-            } else {
-                for (int c = 4 * tid; c < p.k; c += 256 * NW) add(c, rb_ld4(p.norm_z + (size_t)t * p.ldx + c));
-            }
+            for (int i = lane; i < parts; i += 64) ss += p.norm_ssq[(size_t)i * KF_RB_NORM_ROWS + t];
             ss = wave_sum(ss);
-            if (lane == 0) part[wid * RB_NORM_ROWS + t] = ss;
+            if (row == t) rs = 1.0f / sqrtf(ss / (float)p.norm_dim + p.norm_eps);
         }
-        __syncthreads();
-        for (int t = 0; t < p.n; t++) {
-            float ss = 0.f;
-#pragma unroll
-            for (int w = 0; w < NW; w++) ss += part[w * RB_NORM_ROWS + t];
-            const float rs = 1.0f / sqrtf(ss / (float)p.norm_dim + p.norm_eps);
-            auto put = [&](int c, const f32x4& v, const f32x4& g) {
-                f32x4 o;
-#pragma unroll
-                for (int j = 0; j < 4; j++) o[j] = c + j < p.norm_dim ? v[j] * rs * g[j] : 0.f;
-                rb_st4(sx + t * (p.k + 8) + c, o);
-                if (blockIdx.x == 0) { /* the normed rows themselves, once */
-                    rb_st4(p.norm_x + (size_t)t * p.ldx + c, o);
-                    rb_st4(reinterpret_cast<uint16_t*>(const_cast<void*>(p.x)) + (size_t)t * p.ldx + c, o);
-                }
-            };
-            if (nq <= NQ) {
-#pragma unroll
-                for (int i = 0; i < NQ; i++)
-                    if (i / per == t && 4 * tid + (i % per) * 256 * NW < p.k) put(4 * tid + (i % per) * 256 * NW, zq[i], gq[i]);
-            } else {
-                for (int c = 4 * tid; c < p.k; c += 256 * NW) put(c, rb_ld4(p.norm_z + (size_t)t * p.ldx + c), rb_ld4(reinterpret_cast<const uint16_t*>(p.norm_w) + c));
-            }
-        }
-        __syncthreads();
-        xp[0] = sx + (r16 < p.n ? r16 : p.n - 1) * (p.k + 8) + 8 * q4;
+        xp[0] = nullptr;
     } else {
 #pragma unroll
         for (int t = 0; t < NT; t++) { /* columns past the end repeat a row: their outputs are not stored */
@@ -193,15 +157,36 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
         for (int t = 0; t < NT; t++) acc[g][t] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (; s < nstep; s += NW * U) {
         u32x4 an[U][MG];
-        rb_load_x<NT, U, false>(b, xp, s, nstep);
-        rb_load_w<MG, U>(an, wr, p.k, s + NW * U, nstep);
+        if constexpr (NORM) {
+            f32x4 z0[U], z1[U];
+            u32x4 g[U];
+#pragma unroll
+            for (int u = 0; u < U; u++) {
+                const int k0 = 32 * (s + u < nstep ? s + u : nstep - 1);
+                z0[u] = rb_ld4(zp + k0), z1[u] = rb_ld4(zp + k0 + 4), g[u] = *reinterpret_cast<const u32x4*>(gp + k0);
+            }
+            rb_load_w<MG, U>(an, wr, p.k, s + NW * U, nstep);
+#pragma unroll
+            for (int u = 0; u < U; u++) {
+                const f32x4 o0 = f32x4{z0[u].x * rs * bf_lo(g[u].x), z0[u].y * rs * bf_hi(g[u].x), z0[u].z * rs * bf_lo(g[u].y), z0[u].w * rs * bf_hi(g[u].y)};
+                const f32x4 o1 = f32x4{z1[u].x * rs * bf_lo(g[u].z), z1[u].y * rs * bf_hi(g[u].z), z1[u].z * rs * bf_lo(g[u].w), z1[u].w * rs * bf_hi(g[u].w)};
+                b[u][0] = u32x4{pack_bf16x2(o0.x, o0.y), pack_bf16x2(o0.z, o0.w), pack_bf16x2(o1.x, o1.y), pack_bf16x2(o1.z, o1.w)};
+                if (blockIdx.x == 0 && r16 < p.n && s + u < nstep) { /* the normed rows themselves, once */
+                    const size_t at = (size_t)r16 * p.ldx + 32 * (s + u) + 8 * q4;
+                    rb_st4(p.norm_x + at, o0), rb_st4(p.norm_x + at + 4, o1);
+                    *reinterpret_cast<u32x4*>(reinterpret_cast<uint16_t*>(const_cast<void*>(p.x)) + at) = b[u][0];
+                }
+            }
+        } else {
+            rb_load_x<NT, U, false>(b, xp, s, nstep);
+            rb_load_w<MG, U>(an, wr, p.k, s + NW * U, nstep);
+        }
         rb_multiply<NT, MG, U>(a, b, acc);
 #pragma unroll
         for (int u = 0; u < U; u++)
 #pragma unroll
             for (int g = 0; g < MG; g++) a[u][g] = an[u][g];
     }
-    if constexpr (NORM) __syncthreads(); /* `part` shares the partial tiles' memory: every wave is past it */
     rb_stream_finish<NT, MG, NW>(q, acc, red, list, m0, tid);
 }
 
@@ -238,7 +223,7 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_sum_kernel(const RbProduct 
     while (at < end) { /* an expert's part of this wave's range (wave-uniform) */
         const int i = at / nstep, s0 = at - i * nstep, s1 = s0 + (end - at) < nstep ? s0 + (end - at) : nstep;
         const int ex = s_ex[i];
-        const uint16_t* wr = reinterpret_cast<const uint16_t*>(p.w) + (size_t)ex * q.e.w_stride + (size_t)(m0 + r16) * p.k + 8 * q4;
+        const uint16_t* wr = reinterpret_cast<const uint16_t*>(p.w) + (size_t)ex * q.e.w_stride + (size_t)m0 * p.k + 8 * lane;
         u32x4 a[U][1], b[U][NT];
         rb_load_w<1, U>(a, wr, p.k, s0, s1);
         const uint16_t* xp[NT];
@@ -268,19 +253,10 @@ static void stream_go(hipStream_t st, const RbProduct& q, dim3 grid) {
     else if (q.p.epilogue == KF_RB_GATED) hipLaunchKernelGGL((rb_stream_kernel<NT, true, NW, false>), grid, dim3(64 * NW), 0, st, q);
     else hipLaunchKernelGGL((rb_stream_kernel<NT, false, NW, false>), grid, dim3(64 * NW), 0, st, q);
 }
-static size_t norm_lds(int n, int k) { return (size_t)n * (k + 8) * 2; }
 template <int NW>
-static int norm_stream_go(hipStream_t st, const RbProduct& q, dim3 grid) {
-    const size_t smem = norm_lds(q.p.n, q.p.k);
-    static int done = 0;
-    if (!done) {
-        for (const void* f : {(const void*)rb_stream_kernel<1, true, NW, true>, (const void*)rb_stream_kernel<1, false, NW, true>})
-            if (hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, RB_NORM_LDS) != hipSuccess) return KF_HIP_CHECK;
-        done = 1;
-    }
-    if (q.p.epilogue == KF_RB_GATED) hipLaunchKernelGGL((rb_stream_kernel<1, true, NW, true>), grid, dim3(64 * NW), smem, st, q);
-    else hipLaunchKernelGGL((rb_stream_kernel<1, false, NW, true>), grid, dim3(64 * NW), smem, st, q);
-    return KF_OK;
+static void norm_stream_go(hipStream_t st, const RbProduct& q, dim3 grid) {
+    if (q.p.epilogue == KF_RB_GATED) hipLaunchKernelGGL((rb_stream_kernel<1, true, 4, true>), grid, dim3(256), 0, st, q);
+    else hipLaunchKernelGGL((rb_stream_kernel<1, false, NW, true>), grid, dim3(64 * NW), 0, st, q);
 }
 int rb_stream_launch(hipStream_t st, const RbProduct& q) {
     const kf_rb_product& p = q.p;
@@ -290,7 +266,10 @@ int rb_stream_launch(hipStream_t st, const RbProduct& q) {
     if (p.mode == KF_RB_SUM && ((long)p.n * q.e.top > RB_SUM_IDS || q.e.tile < p.n)) return 1;
     dim3 grid(p.m / (p.epilogue == KF_RB_GATED ? 32 : 16), tiles ? q.e.n_tile : 1);
     const bool wide = (long)grid.x * grid.y < 768 && p.k >= 512; /* few workgroups: more waves each, more loads in flight per CU */
-    if (p.norm_z) return wide ? norm_stream_go<8>(st, q, grid) : norm_stream_go<4>(st, q, grid);
+    if (p.norm_z) {
+        wide ? norm_stream_go<8>(st, q, grid) : norm_stream_go<4>(st, q, grid);
+        return KF_OK;
+    }
     switch (nt) {
         case 1: wide ? stream_go<1, 8>(st, q, grid) : stream_go<1, 4>(st, q, grid); break;
         case 2: wide ? stream_go<2, 8>(st, q, grid) : stream_go<2, 4>(st, q, grid); break;
@@ -391,7 +370,7 @@ int rb_f32_launch(hipStream_t st, const RbProduct& q) {
 }  // namespace kf
 
 using namespace kf;
-extern "C" int kf_rb_linear_norms(int type, int n, int k) { return type == KF_BF16 && n >= 1 && n <= RB_NORM_ROWS && norm_lds(n, k) + 20 * 1024 <= RB_NORM_LDS; }
+extern "C" int kf_rb_linear_norms(int type, int n, int k) { return type == KF_BF16 && n >= 1 && n <= KF_RB_NORM_ROWS && k % KF_RB_PAD == 0; }
 extern "C" int kf_rb_linear(kf_ctx* c, const kf_rb_product* p) {
     CHKCTX(c);
     if (!p || !p->w || !p->x || !p->y) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: null pointer");
@@ -401,7 +380,8 @@ extern "C" int kf_rb_linear(kf_ctx* c, const kf_rb_product* p) {
     if (!al16(p->w) || !al16(p->x) || !al16(p->y)) return abi_fail(KF_BLAS_UNALIGN, "kf_rb_linear: unaligned pointer");
     if (p->epilogue < KF_RB_STORE || p->epilogue > KF_RB_GATED || p->mode < KF_RB_ALL || p->mode > KF_RB_SUM) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: epilogue or mode");
     if (p->epilogue == KF_RB_RESIDUAL && (!p->res || !al16(p->res) || p->ldr < p->m || p->ldr % 4)) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: residual");
-    if (p->norm_z && (!kf_rb_linear_norms(p->type, p->n, p->k) || p->mode != KF_RB_ALL || !p->norm_w || !p->norm_x || p->norm_dim < 1 || p->norm_dim > p->k || p->ldx != p->k || !al16(p->norm_z) ||
+    if (p->ssq && (!kf_rb_linear_norms(p->type, p->n, p->m) || p->epilogue != KF_RB_RESIDUAL)) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: sums of squares");
+    if (p->norm_z && (!kf_rb_linear_norms(p->type, p->n, p->k) || p->mode != KF_RB_ALL || p->epilogue == KF_RB_RESIDUAL || !p->norm_w || !p->norm_x || !p->norm_ssq || p->norm_dim < 1 || p->norm_dim > p->k || p->ldx != p->k || !al16(p->norm_z) ||
                       !al16(p->norm_w) || !al16(p->norm_x)))
         return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: norm in front of the product");
     RbProduct q;

@@ -153,31 +153,34 @@ __device__ __forceinline__ void rb_topk_row(const RbRoute& a, int t, int lane) {
         v[i] = -__builtin_inff();
         if (e < n_expert) v[i] = logits[(size_t)t * ld + e] + (bias ? rb_ld(bias + e) : 0.f);
     }
-    float best0 = 0.f, sum = 0.f;
+    float best0 = 0.f, sum = 0.f, my_p = 0.f;
+    int my_id = -1; /* choice j sits in lane j % 64 */
+    auto flush = [&](int j0, int j1, float scale) {
+        if (lane < j1 - j0) ids[(size_t)t * top + j0 + lane] = my_id, weight[(size_t)t * top + j0 + lane] = my_p * scale;
+    };
     for (int j = 0; j < top; j++) {
         float m = v[0];
-        int idx = lane;
 #pragma unroll
-        for (int i = 1; i < NV; i++)
-            if (v[i] > m) m = v[i], idx = lane + 64 * i;
+        for (int i = 1; i < NV; i++) m = fmaxf(m, v[i]);
         const float wm = wave_max(m);
-        int cand = m == wm ? idx : 0x7fffffff; /* ties: the lower expert */
+        int cand = -1; /* ties: the lower expert.  NaN logits: none */
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const int other = __shfl_xor(cand, o, 64);
-            cand = other < cand ? other : cand;
+        for (int i = NV - 1; i >= 0; i--) {
+            const unsigned long long on = __ballot(v[i] == wm && lane + 64 * i < n_expert);
+            if (on) cand = 64 * i + __ffsll((long long)on) - 1;
         }
         if (j == 0) best0 = wm;
         const float p = expf(wm - best0);
         sum += p;
-        if (lane == 0) ids[(size_t)t * top + j] = cand < n_expert ? cand : -1 /* NaN logits */, weight[(size_t)t * top + j] = p;
+        if (lane == (j & 63)) my_p = p, my_id = cand;
 #pragma unroll
         for (int i = 0; i < NV; i++)
             if (lane + 64 * i == cand) v[i] = -__builtin_inff();
+        if ((j & 63) == 63 && j + 1 < top) flush(j - 63, j + 1, 1.f);
     }
     const float inv = 1.0f / sum;
-    if (lane == 0) /* the lane that wrote them reads them back */
-        for (int j = 0; j < top; j++) weight[(size_t)t * top + j] *= inv;
+    flush((top - 1) & ~63, top, inv);
+    for (int j = lane; j < ((top - 1) & ~63); j += 64) weight[(size_t)t * top + j] *= inv; /* (more than 64 choices: a lane reads back what it wrote) */
 }
 template <class T, int NV>
 __global__ void __launch_bounds__(256) rb_topk_kernel(const RbRoute a) {
@@ -308,10 +311,13 @@ __global__ void __launch_bounds__(256) rb_to_bf16_kernel(const float* __restrict
 }
 
 template <class T>
-__global__ void __launch_bounds__(256) rb_pack_kernel(const uint16_t* __restrict__ src, int cols, T* __restrict__ dst, long long ld, int half) {
+__global__ void __launch_bounds__(256) rb_pack_kernel(const uint16_t* __restrict__ src, int cols, T* __restrict__ dst, long long ld, int row0, int half, int tiled) {
     const int r = blockIdx.x;
-    const size_t d = half < 0 ? (size_t)r : (size_t)(32 * (r / 16) + 16 * half + r % 16);
-    for (int i = threadIdx.x; i < cols; i += 256) rb_st(dst + d * ld + i, bf2f(src[(size_t)r * cols + i]));
+    const size_t d = half < 0 ? (size_t)row0 + r : (size_t)(32 * (r / 16) + 16 * half + r % 16);
+    for (int i = threadIdx.x; i < cols; i += 256) {
+        const size_t at = tiled ? ((d / 16) * (ld / 32) + i / 32) * 512 + (d % 16 + 16 * ((i % 32) / 8)) * 8 + i % 8 : d * ld + i;
+        rb_st(dst + at, bf2f(src[(size_t)r * cols + i]));
+    }
 }
 
 }  // namespace kf
@@ -390,12 +396,12 @@ int kf_rb_pick(kf_ctx* c, const float* logits, int64_t ld, int vocab, int n, con
     hipLaunchKernelGGL(rb_pick_finish_kernel, dim3(n), dim3(64), 0, c->stream, pv, pi, pieces, vocab, meta, d_state, d_tokens_out, tokens_stride);
     return launched("kf_rb_pick");
 }
-int kf_rb_pack(kf_ctx* c, int type, const kf_bf16* src, int rows, int cols, void* dst, int64_t ld, int half) {
+int kf_rb_pack(kf_ctx* c, int type, const kf_bf16* src, int rows, int cols, void* dst, int64_t ld, int row0, int half, int tiled) {
     CHKCTX(c);
     if (!type_ok(type)) return abi_fail(KF_UNSUPPORTED_DATATYPE, "kf_rb_pack: storage %d", type);
-    if (!src || !dst || rows < 1 || cols < 1 || ld < cols || half > 1) return abi_fail(KF_INVALID_ARGS, "kf_rb_pack: bad arguments");
-    if (type == KF_BF16) hipLaunchKernelGGL(rb_pack_kernel<uint16_t>, dim3(rows), dim3(256), 0, c->stream, src, cols, (uint16_t*)dst, (long long)ld, half);
-    else hipLaunchKernelGGL(rb_pack_kernel<float>, dim3(rows), dim3(256), 0, c->stream, src, cols, (float*)dst, (long long)ld, half);
+    if (!src || !dst || rows < 1 || cols < 1 || ld < cols || row0 < 0 || half > 1 || (tiled && (type != KF_BF16 || ld % KF_RB_PAD))) return abi_fail(KF_INVALID_ARGS, "kf_rb_pack: bad arguments");
+    if (type == KF_BF16) hipLaunchKernelGGL(rb_pack_kernel<uint16_t>, dim3(rows), dim3(256), 0, c->stream, src, cols, (uint16_t*)dst, (long long)ld, row0, half, tiled);
+    else hipLaunchKernelGGL(rb_pack_kernel<float>, dim3(rows), dim3(256), 0, c->stream, src, cols, (float*)dst, (long long)ld, row0, half, 0);
     return launched("kf_rb_pack");
 }
 int kf_rb_to_bf16(kf_ctx* c, const float* src, kf_bf16* dst, size_t n) {

@@ -21,11 +21,11 @@ static hGTensor Mem(kf_ctx* c, const char* name, int type, size_t n) {
 }
 
 // ------------------------------------------------------------------------------------------------ neurons
-int RowProduct::Forw(const void* x, int64_t ldx, int n, void* y, int64_t ldy, int epilogue, int act, const float* res, float alpha, int mode, const kf_rb_experts* ex) {
+int RowProduct::Forw(const void* x, int64_t ldx, int n, void* y, int64_t ldy, int epilogue, int act, const float* res, float alpha, int mode, const kf_rb_experts* ex, float* ssq) {
     kf_rb_product p;
     std::memset(&p, 0, sizeof(p));
     p.w = w->data, p.x = x, p.y = y, p.res = res, p.ldx = ldx, p.ldy = ldy, p.ldr = ldy;
-    p.type = hFish->Seq()->card.type, p.m = m, p.k = k, p.n = n, p.epilogue = epilogue, p.act = act, p.mode = mode, p.alpha = alpha;
+    p.type = hFish->Seq()->card.type, p.m = m, p.k = k, p.n = n, p.epilogue = epilogue, p.act = act, p.mode = mode, p.alpha = alpha, p.ssq = ssq;
     kf_rb_experts e;
     if (ex) e = *ex, e.w_stride = (int64_t)m * k, p.experts = &e;
     return kf_rb_linear(hFish->ctx, &p);
@@ -36,7 +36,7 @@ int RowProduct::ForwNormed(RowWork& w, int n, void* y, int64_t ldy, int epilogue
     kf_rb_product p;
     std::memset(&p, 0, sizeof(p));
     p.w = this->w->data, p.x = P(w.h), p.y = y, p.ldx = k, p.ldy = ldy, p.type = c.type, p.m = m, p.k = k, p.n = n, p.epilogue = epilogue, p.act = act;
-    p.norm_z = F(w.z), p.norm_w = P(w.pending->w), p.norm_x = F(w.x), p.norm_eps = c.eps, p.norm_dim = c.width;
+    p.norm_z = F(w.z), p.norm_ssq = F(w.ssq), p.norm_w = P(w.pending->w), p.norm_x = F(w.x), p.norm_eps = c.eps, p.norm_dim = c.width;
     w.pending = nullptr;
     return kf_rb_linear(hFish->ctx, &p);
 }
@@ -57,7 +57,7 @@ int ChunkAttention::Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int ma
     a.scale = c.scale, a.eps = card.eps;
     if (n_seq) KF_TRY(kf_rb_attention_prefill(hFish->ctx, &a, I(w.meta), n, I(w.seqs), n_seq, max_n));
     else KF_TRY(kf_rb_attention_decode(hFish->ctx, &a, I(w.meta), n, max_pos));
-    KF_TRY(proj.Forw(P(w.ao), ldout, n, F(w.z), proj.m, KF_RB_RESIDUAL, 0, F(w.x), card.alpha));
+    KF_TRY(proj.Forw(P(w.ao), ldout, n, F(w.z), proj.m, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_ALL, nullptr, defer ? F(w.ssq) : nullptr));
     if (defer) {
         w.pending = &norm;
         return KF_OK;
@@ -70,7 +70,7 @@ int RowFFN::Forw(RowWork& w, int n, bool defer) {
     const int64_t ld = gateup.k;
     if (c.kind == FF_CARD::DENSE) {
         KF_TRY(gateup.ForwNormed(w, n, P(w.act), ldact, KF_RB_GATED, c.act));
-        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha));
+        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_ALL, nullptr, defer ? F(w.ssq) : nullptr));
         if (defer) {
             w.pending = &norm;
             return KF_OK;
@@ -89,7 +89,7 @@ int RowFFN::Forw(RowWork& w, int n, bool defer) {
     KF_TRY(kf_rb_route(hFish->ctx, card.type, F(w.rlogits), router.m, P(router_b), n, I(w.meta), &e));
     KF_TRY(gateup.Forw(P(w.h), ld, n, P(w.act), ldact, KF_RB_GATED, c.act, nullptr, 0, KF_RB_UP, &e));
     if (few) {
-        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_SUM, &e));
+        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_SUM, &e, defer ? F(w.ssq) : nullptr));
         if (defer) {
             w.pending = &norm;
             return KF_OK;
@@ -141,12 +141,12 @@ int SeqFish::BuildSeq(const SEQ_CARD& c, int device, void* stream) {
     };
     auto norm = [&](RowNorm& n, const std::string& name) {
         n.hFish = this, n.name = name, n.dim = c.width, n.ld = W, n.w = mem(name, W);
-        targets[name] = Target{n.w, 0, c.width, 1, 1, -1, false};
+        targets[name] = Target{n.w, 0, 0, c.width, 1, 1, -1, false, false};
     };
     table = mem("embed", (size_t)V * W);
-    targets["embed"] = Target{table, 0, c.vocab, c.width, W, -1, false};
+    targets["embed"] = Target{table, 0, 0, c.vocab, c.width, W, -1, false, false};
     product(seq_head, "head", V, W);
-    targets["head"] = Target{seq_head.w, 0, c.vocab, c.width, W, -1, false};
+    targets["head"] = Target{seq_head.w, 0, 0, c.vocab, c.width, W, -1, true, false};
     norm(seq_norm, "final.norm");
     for (size_t l = 0; l < c.layers.size(); l++) {
         const LAYER_CARD& L = c.layers[l];
@@ -157,14 +157,14 @@ int SeqFish::BuildSeq(const SEQ_CARD& c, int device, void* stream) {
         a->ldraw = Width(rows), a->ldout = Width(qd);
         product(a->qkg, p + "mix.qkg", a->ldraw, W);
         product(a->proj, p + "mix.o", W, a->ldout);
-        targets[p + "mix.q"] = Target{a->qkg.w, 0, qd, c.width, W, -1, false};
-        targets[p + "mix.k"] = Target{a->qkg.w, (size_t)qd * W, kd, c.width, W, -1, false};
-        if (L.mix.gated) targets[p + "mix.g"] = Target{a->qkg.w, (size_t)(qd + kd) * W, qd, c.width, W, -1, false};
-        targets[p + "mix.o"] = Target{a->proj.w, 0, c.width, qd, a->ldout, -1, false};
+        targets[p + "mix.q"] = Target{a->qkg.w, 0, 0, qd, c.width, W, -1, true, false};
+        targets[p + "mix.k"] = Target{a->qkg.w, 0, qd, kd, c.width, W, -1, true, false};
+        if (L.mix.gated) targets[p + "mix.g"] = Target{a->qkg.w, 0, qd + kd, qd, c.width, W, -1, true, false};
+        targets[p + "mix.o"] = Target{a->proj.w, 0, 0, c.width, qd, a->ldout, -1, true, false};
         if (L.mix.qk_norm) {
             a->qn = mem(p + "mix.q.norm", Width(L.mix.dim)), a->kn = mem(p + "mix.k.norm", Width(L.mix.dim));
-            targets[p + "mix.q.norm"] = Target{a->qn, 0, L.mix.dim, 1, 1, -1, false};
-            targets[p + "mix.k.norm"] = Target{a->kn, 0, L.mix.dim, 1, 1, -1, false};
+            targets[p + "mix.q.norm"] = Target{a->qn, 0, 0, L.mix.dim, 1, 1, -1, false, false};
+            targets[p + "mix.k.norm"] = Target{a->kn, 0, 0, L.mix.dim, 1, 1, -1, false, false};
         }
         norm(a->norm, p + "norm1");
         for (auto& r : ropes)
@@ -190,15 +190,15 @@ int SeqFish::BuildSeq(const SEQ_CARD& c, int device, void* stream) {
             for (int e = 0; e < std::max(E, 1); e++) {
                 const std::string q = p + "mlp." + (E ? "e" + std::to_string(e) + "." : "");
                 const size_t gu = (size_t)e * 2 * ff * W, dn = (size_t)e * W * ff;
-                targets[q + "gate"] = Target{f->gateup.w, gu, L.ff.ff, c.width, W, 0, false};
-                targets[q + "up"] = Target{f->gateup.w, gu, L.ff.ff, c.width, W, 1, false};
-                targets[q + "down"] = Target{f->down.w, dn, c.width, L.ff.ff, ff, -1, false};
+                targets[q + "gate"] = Target{f->gateup.w, gu, 0, L.ff.ff, c.width, W, 0, true, false};
+                targets[q + "up"] = Target{f->gateup.w, gu, 0, L.ff.ff, c.width, W, 1, true, false};
+                targets[q + "down"] = Target{f->down.w, dn, 0, c.width, L.ff.ff, ff, -1, true, false};
             }
             if (E) {
                 product(f->router, p + "mlp.router", Width(E), W);
                 f->router_b = mem(p + "mlp.router.b", Width(E));
-                targets[p + "mlp.router"] = Target{f->router.w, 0, E, c.width, W, -1, false};
-                targets[p + "mlp.router.b"] = Target{f->router_b, 0, E, 1, 1, -1, false};
+                targets[p + "mlp.router"] = Target{f->router.w, 0, 0, E, c.width, W, -1, true, false};
+                targets[p + "mlp.router.b"] = Target{f->router_b, 0, 0, E, 1, 1, -1, false, false};
             }
             norm(f->norm, p + "norm2");
         }
@@ -230,8 +230,8 @@ int SeqFish::SetTensor(const std::string& name, int rows, int cols, const void* 
         src = stage->data;
     }
     uint8_t* dst = reinterpret_cast<uint8_t*>(t.to->data) + t.offset * Elem();
-    const bool vec = cols == 1;  // a norm weight or a bias: one row of `rows` values
-    KF_TRY(kf_rb_pack(ctx, card.type, reinterpret_cast<const kf_bf16*>(src), vec ? 1 : rows, vec ? rows : cols, dst, vec ? rows : t.ld, vec ? -1 : t.half));
+    const bool vec = !t.product && cols == 1;  // a norm weight or a bias: one row of `rows` values
+    KF_TRY(kf_rb_pack(ctx, card.type, reinterpret_cast<const kf_bf16*>(src), vec ? 1 : rows, vec ? rows : cols, dst, vec ? rows : t.ld, t.row0, vec ? -1 : t.half, t.product && card.type == KF_BF16));
     t.set = true;
     return KF_OK;
 }
@@ -347,6 +347,7 @@ int SeqFish::Ensure(RowWork& w, int rows, int n_seq, int head_rows, bool decode)
         get(w.raw, "raw", T, raw), get(w.ao, "ao", T, ao), get(w.knew, "knew", T, kn), get(w.act, "act", T, act), get(w.y, "y", T, y), get(w.rlogits, "rlogits", KF_F32, rl);
         get(w.meta, "meta", KF_F32, (size_t)rows * KF_RB_META), get(w.tok, "tok", KF_F32, rows), get(w.ids, "ids", KF_F32, pairs), get(w.weight, "weight", KF_F32, pairs);
         get(w.list, "list", KF_F32, list), get(w.tile_expert, "tile_expert", KF_F32, tiles), get(w.scratch, "scratch", KF_F32, scratch);
+        if (decode) get(w.ssq, "ssq", KF_F32, (size_t)(W / 16) * KF_RB_NORM_ROWS);
         w.rows = rows;
     }
     if (n_seq > w.n_seq) get(w.seqs, "seqs", KF_F32, (size_t)n_seq * 4), w.n_seq = n_seq;

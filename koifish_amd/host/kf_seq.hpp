@@ -45,6 +45,7 @@ struct RowNorm;
 struct RowWork {
     RowNorm* pending = nullptr;  // decode: z holds a residual sum whose norm the next product forms itself
     int rows = 0, n_seq = 0, head_rows = 0;
+    hGTensor ssq;                                                      // decode: z's sums of squares
     hGTensor x, z, h, raw, knew, ao, act, y, rlogits, scratch;         // residual and its sum (fp32), bf16 / fp32 rows, expert outputs, router logits, key-range partials
     hGTensor meta, seqs, tok, ids, weight, list, tile_expert, want, hl;  // int32 tables; hl: the rows the head reads
     hGTensor logits;                                                     // fp32 [head_rows][padded vocab]
@@ -73,7 +74,7 @@ struct RowProduct : GeNeuron {  // padded weight [m][k] (x experts)
     hGTensor w;
     int m = 0, k = 0, experts = 0;
     int Forw(const void* x, int64_t ldx, int n, void* y, int64_t ldy, int epilogue, int act = 0, const float* res = nullptr, float alpha = 0, int mode = KF_RB_ALL,
-             const kf_rb_experts* ex = nullptr);
+             const kf_rb_experts* ex = nullptr, float* ssq = nullptr);
     int ForwNormed(RowWork& w, int n, void* y, int64_t ldy, int epilogue, int act = 0);  // of w.h, the pending norm first
 };
 struct RowNorm : GeNeuron {
@@ -112,9 +113,9 @@ struct SeqFish : Fish {
     std::vector<std::pair<ROT_CARD, float*>> ropes;
     struct Target {  // where a named tensor of the checkpoint goes
         hGTensor to;
-        size_t offset = 0;  // elements
-        int rows = 0, cols = 0, ld = 0, half = -1;
-        bool set = false;
+        size_t offset = 0;  // elements in front of the matrix
+        int row0 = 0, rows = 0, cols = 0, ld = 0, half = -1;
+        bool product = false, set = false;
     };
     std::map<std::string, Target> targets;
     hGTensor stage;

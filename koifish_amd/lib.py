@@ -49,7 +49,7 @@ class RbProduct(C.Structure):
     """struct kf_rb_product"""
     _fields_ = [("w", C.c_void_p), ("x", C.c_void_p), ("y", C.c_void_p), ("res", C.c_void_p), ("ldx", C.c_int64), ("ldy", C.c_int64), ("ldr", C.c_int64), ("type", C.c_int32),
                 ("m", C.c_int32), ("k", C.c_int32), ("n", C.c_int32), ("epilogue", C.c_int32), ("act", C.c_int32), ("mode", C.c_int32), ("alpha", C.c_float), ("experts", C.POINTER(RbExperts)),
-                ("norm_z", C.c_void_p), ("norm_w", C.c_void_p), ("norm_x", C.c_void_p), ("norm_eps", C.c_float), ("norm_dim", C.c_int32)]
+                ("ssq", C.c_void_p), ("norm_z", C.c_void_p), ("norm_ssq", C.c_void_p), ("norm_w", C.c_void_p), ("norm_x", C.c_void_p), ("norm_eps", C.c_float), ("norm_dim", C.c_int32)]
 
 
 class RbAttention(C.Structure):
@@ -286,7 +286,7 @@ def load():
             getattr(host, f).argtypes = [C.c_void_p]
         # row batches (include/kf_rb.h) and the models described layer by layer on them
         hip.kf_rb_linear.argtypes = [C.c_void_p, C.POINTER(RbProduct)]
-        hip.kf_rb_pack.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_void_p, C.c_int64, C.c_int]
+        hip.kf_rb_pack.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_void_p, C.c_int64, C.c_int, C.c_int, C.c_int]
         hip.kf_rb_embed.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_int64, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p]
         hip.kf_rb_embed_state.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int, C.c_int64, C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]
         hip.kf_rb_norm.argtypes = [C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_float, C.c_int, C.c_void_p, C.c_float, C.c_int, C.c_int64, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]

@@ -34,6 +34,14 @@ def ptr(t):
     return None if t is None else t.data_ptr()
 
 
+def stored(w):
+    """a product's weight [..., m, k] as the library stores it: bf16 in 16 x 32 tiles, piece (row r, octet q) at number 16 q + r; fp32 as it is"""
+    if w.dtype != torch.bfloat16:
+        return w
+    m, k = w.shape[-2:]
+    return w.reshape(-1, m // 16, 16, k // 32, 4, 8).permute(0, 1, 3, 4, 2, 5).contiguous().reshape(w.shape)
+
+
 @pytest.fixture(params=list(TYPES))
 def kind(request):
     return TYPES[request.param]
@@ -85,9 +93,9 @@ def test_product_epilogues(ctx, kind, n, m, k):
     typ, dt, tol = kind
     g = torch.Generator().manual_seed(n * m + k)
     w, x, res = dev(torch.randn(m, k, generator=g) / k ** 0.5, dt), dev(torch.randn(n, k + 8, generator=g), dt), dev(torch.randn(n, m, generator=g))
-    ref = f64(x)[:, :k] @ f64(w).T
+    ref, ws = f64(x)[:, :k] @ f64(w).T, stored(w)
     for epi, y in ((L.RB_STORE, torch.zeros(n, m, dtype=dt, device="cuda")), (L.RB_STORE_F32, torch.zeros(n, m, device="cuda")), (L.RB_RESIDUAL, torch.zeros(n, m, device="cuda"))):
-        p = L.RbProduct(w.data_ptr(), x.data_ptr(), y.data_ptr(), res.data_ptr(), k + 8, m, m, typ, m, k, n, epi, 0, L.RB_ALL, -0.75, None)
+        p = L.RbProduct(ws.data_ptr(), x.data_ptr(), y.data_ptr(), res.data_ptr(), k + 8, m, m, typ, m, k, n, epi, 0, L.RB_ALL, -0.75, None)
         L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
         want = ref + (-0.75 * f64(res) if epi == L.RB_RESIDUAL else 0)
         assert np.abs(f64(y) - want).max() < (tol * 4 if epi == L.RB_STORE else 2e-5)
@@ -97,23 +105,30 @@ def test_product_epilogues(ctx, kind, n, m, k):
     gelu = lambda z: 0.5 * z * (1 + np.tanh(np.sqrt(2 / np.pi) * (z + 0.044715 * z ** 3)))
     for act, fn in ((L.RB_RELU, P.relu), (L.RB_SILU, P.silu), (L.RB_GELU_TANH, gelu)):
         y = torch.zeros(n, m // 2, dtype=dt, device="cuda")
-        p = L.RbProduct(w.data_ptr(), x.data_ptr(), y.data_ptr(), None, k + 8, m // 2, 0, typ, m, k, n, L.RB_GATED, act, L.RB_ALL, 0.0, None)
+        p = L.RbProduct(ws.data_ptr(), x.data_ptr(), y.data_ptr(), None, k + 8, m // 2, 0, typ, m, k, n, L.RB_GATED, act, L.RB_ALL, 0.0, None)
         L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
         assert np.abs(f64(y) - fn(gate) * upw).max() < tol * 8
 
 
-@pytest.mark.parametrize("n,m,k,dim", [(1, 64, 64, 50), (3, 192, 320, 300), (8, 448, 1024, 1024), (2, 256, 4096, 4090)])
+@pytest.mark.parametrize("n,m,k,dim", [(1, 64, 64, 50), (3, 192, 320, 300), (4, 448, 1024, 1024), (2, 256, 4096, 4090)])
 def test_norm_in_front_of_a_product(ctx, n, m, k, dim):
-    assert ctx.hip.kf_rb_linear_norms(L.BF16, n, k) and not ctx.hip.kf_rb_linear_norms(L.F32, n, k) and not ctx.hip.kf_rb_linear_norms(L.BF16, 9, k)
+    assert ctx.hip.kf_rb_linear_norms(L.BF16, n, k) and not ctx.hip.kf_rb_linear_norms(L.F32, n, k) and not ctx.hip.kf_rb_linear_norms(L.BF16, 5, k)
     w, z = (torch.randn(m, k, device="cuda") / k ** 0.5).bfloat16(), torch.randn(n, k, device="cuda")
-    z[:, dim:] = 99.0                         # pad columns do not count
+    z[:, dim:] = 0.0
     g = (torch.rand(k, device="cuda") + 0.5).bfloat16()
-    il = f64(w).reshape(m // 32, 2, 16, k)
+    g[dim:] = 0.0
+    # the sums of squares come from the product in front: z = 0.5 res + W0 x0 with its epilogue's partial sums
+    w0, x0, res = torch.zeros(k, 64, dtype=torch.bfloat16, device="cuda"), torch.zeros(n, 64, dtype=torch.bfloat16, device="cuda"), 2.0 * z
+    ssq = torch.full((k // 16, 4), 7.0, device="cuda")
+    p = L.RbProduct(w0.data_ptr(), x0.data_ptr(), z.data_ptr(), res.data_ptr(), 64, k, k, L.BF16, k, 64, n, L.RB_RESIDUAL, 0, L.RB_ALL, 0.5, None, ssq.data_ptr())
+    L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
+    assert np.abs(f64(ssq)[:, :n] - (f64(z) ** 2).reshape(n, k // 16, 16).sum(2).T).max() < 1e-4 and (ssq[:, n:] == 7.0).all()
+    il, ws = f64(w).reshape(m // 32, 2, 16, k), stored(w)
     ref = P.rms_norm(f64(z)[:, :dim], f64(g)[:dim], 1e-5)
     for epi in (L.RB_STORE, L.RB_STORE_F32, L.RB_GATED):
         x, h = torch.full((n, k), 7.0, device="cuda"), torch.full((n, k), 7.0, dtype=torch.bfloat16, device="cuda")
         y = torch.zeros(n, m, dtype=torch.float32 if epi == L.RB_STORE_F32 else torch.bfloat16, device="cuda")
-        p = L.RbProduct(w.data_ptr(), h.data_ptr(), y.data_ptr(), None, k, m, 0, L.BF16, m, k, n, epi, L.RB_SILU, L.RB_ALL, 0.0, None, z.data_ptr(), g.data_ptr(), x.data_ptr(), 1e-5, dim)
+        p = L.RbProduct(ws.data_ptr(), h.data_ptr(), y.data_ptr(), None, k, m, 0, L.BF16, m, k, n, epi, L.RB_SILU, L.RB_ALL, 0.0, None, None, z.data_ptr(), ssq.data_ptr(), g.data_ptr(), x.data_ptr(), 1e-5, dim)
         L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
         assert np.abs(f64(x)[:, :dim] - ref).max() < 1e-5 and not f64(x)[:, dim:].any() and torch.equal(h, x.bfloat16())
         full = f64(h) @ f64(w).T
@@ -127,8 +142,8 @@ def test_product_many_tiles(ctx):
     """the larger tiles of the bf16 product (256 x 256, 128 x 128, 64 x 128)"""
     for m, n, k in ((2560, 4096, 128), (2048, 2048, 64), (1024, 1500, 192)):
         w, x = (torch.randn(m, k, device="cuda") / k ** 0.5).bfloat16(), torch.randn(n, k, device="cuda").bfloat16()
-        y = torch.zeros(n, m, device="cuda")
-        p = L.RbProduct(w.data_ptr(), x.data_ptr(), y.data_ptr(), None, k, m, m, L.BF16, m, k, n, L.RB_STORE_F32, 0, L.RB_ALL, 0.0, None)
+        y, ws = torch.zeros(n, m, device="cuda"), stored(w)
+        p = L.RbProduct(ws.data_ptr(), x.data_ptr(), y.data_ptr(), None, k, m, m, L.BF16, m, k, n, L.RB_STORE_F32, 0, L.RB_ALL, 0.0, None)
         L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
         assert (y - x.float() @ w.float().T).abs().max().item() < 1e-4
 
@@ -141,7 +156,7 @@ def test_product_refuses_what_it_cannot_do(ctx):
         assert ctx.hip.kf_rb_linear(ctx.h, C.byref(p)) < 0, bad
 
 
-@pytest.mark.parametrize("n,E,top,tile", [(1, 4, 2, 16), (5, 7, 7, 16), (40, 3, 1, 48), (200, 70, 4, 64), (700, 130, 8, 128)])
+@pytest.mark.parametrize("n,E,top,tile", [(1, 4, 2, 16), (5, 7, 7, 16), (3, 200, 150, 16), (40, 3, 1, 48), (200, 70, 4, 64), (700, 130, 8, 128)])
 def test_route(ctx, kind, n, E, top, tile):
     typ, dt, _ = kind
     g = torch.Generator().manual_seed(n + E)
@@ -182,11 +197,12 @@ def test_experts(ctx, kind, n, E, top, tile):
         tile = 64
     C_, ff, g = 128, 64, torch.Generator().manual_seed(n)
     gu, dn = dev(torch.randn(E, 2 * ff, C_, generator=g) / C_ ** 0.5, dt), dev(torch.randn(E, C_, ff, generator=g) / ff ** 0.5, dt)
+    gus, dns = stored(gu), stored(dn)
     x, res = dev(torch.randn(n, C_, generator=g), dt), dev(torch.randn(n, C_, generator=g))
     logits = pad(dev(torch.randn(n, E, generator=g)), n, up(E))
     e, b = route(ctx, logits, None, n, E, top, tile, typ, w_stride=2 * ff * C_)
     act = torch.zeros(n * top, ff, dtype=dt, device="cuda")
-    p = L.RbProduct(gu.data_ptr(), x.data_ptr(), act.data_ptr(), None, C_, ff, 0, typ, 2 * ff, C_, n, L.RB_GATED, L.RB_SILU, L.RB_UP, 0.0, C.pointer(e))
+    p = L.RbProduct(gus.data_ptr(), x.data_ptr(), act.data_ptr(), None, C_, ff, 0, typ, 2 * ff, C_, n, L.RB_GATED, L.RB_SILU, L.RB_UP, 0.0, C.pointer(e))
     L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
     ids, wt = b["ids"].cpu().numpy(), b["weight"].double().cpu().numpy()
     il = f64(gu).reshape(E, ff // 16, 2, 16, C_)
@@ -198,11 +214,11 @@ def test_experts(ctx, kind, n, E, top, tile):
     assert np.abs(f64(act) - A).max() < tol * 8
     e.w_stride = C_ * ff
     yd = torch.zeros(n * top, C_, dtype=dt, device="cuda")
-    p = L.RbProduct(dn.data_ptr(), act.data_ptr(), yd.data_ptr(), None, ff, C_, 0, typ, C_, ff, n, L.RB_STORE, 0, L.RB_DOWN, 0.0, C.pointer(e))
+    p = L.RbProduct(dns.data_ptr(), act.data_ptr(), yd.data_ptr(), None, ff, C_, 0, typ, C_, ff, n, L.RB_STORE, 0, L.RB_DOWN, 0.0, C.pointer(e))
     L.check(ctx.hip.kf_rb_linear(ctx.h, C.byref(p)))
     assert np.abs(f64(yd) - y).max() < tol * 4
     z = torch.zeros(n, C_, device="cuda")
-    p = L.RbProduct(dn.data_ptr(), act.data_ptr(), z.data_ptr(), res.data_ptr(), ff, C_, C_, typ, C_, ff, n, L.RB_RESIDUAL, 0, L.RB_SUM, 1.25, C.pointer(e))
+    p = L.RbProduct(dns.data_ptr(), act.data_ptr(), z.data_ptr(), res.data_ptr(), ff, C_, C_, typ, C_, ff, n, L.RB_RESIDUAL, 0, L.RB_SUM, 1.25, C.pointer(e))
     rc = ctx.hip.kf_rb_linear(ctx.h, C.byref(p))
     if typ == L.F32 or n > 64:
         assert rc == -1000
@@ -395,7 +411,7 @@ def test_embed_and_pack(ctx, kind):
     V, dim, ld = 11, 75, 128
     src = torch.randn(V, dim).bfloat16().cuda()
     tab = torch.zeros(64, ld, dtype=dt, device="cuda")
-    L.check(ctx.hip.kf_rb_pack(ctx.h, typ, src.data_ptr(), V, dim, tab.data_ptr(), ld, -1))
+    L.check(ctx.hip.kf_rb_pack(ctx.h, typ, src.data_ptr(), V, dim, tab.data_ptr(), ld, 0, -1, 0))
     assert torch.equal(tab[:V, :dim].float(), src.float()) and not tab[:, dim:].any() and not tab[V:].any()
     tok = torch.tensor([3, 10, 0], dtype=torch.int32, device="cuda")
     x, h = torch.full((3, ld), 9.0, device="cuda"), torch.full((3, ld), 9.0, dtype=dt, device="cuda")
@@ -403,9 +419,14 @@ def test_embed_and_pack(ctx, kind):
     assert torch.equal(x[:, :dim], src[tok.long()].float()) and not x[:, dim:].any() and torch.equal(h.float(), x)
     gu = torch.zeros(96, 64, dtype=dt, device="cuda")
     w = torch.randn(40, 50).bfloat16().cuda()
-    L.check(ctx.hip.kf_rb_pack(ctx.h, typ, w.data_ptr(), 40, 50, gu.data_ptr(), 64, 1))
+    L.check(ctx.hip.kf_rb_pack(ctx.h, typ, w.data_ptr(), 40, 50, gu.data_ptr(), 64, 0, 1, 0))
     for r in range(40):
         assert torch.equal(gu[32 * (r // 16) + 16 + r % 16, :50].float(), w[r].float())
+    if typ == L.BF16:      # a product's weight, from a row no tile starts at
+        pw, row = torch.zeros(64, 64, dtype=dt, device="cuda"), torch.zeros(64, 64, dtype=dt, device="cuda")
+        row[21:61, :50] = w
+        L.check(ctx.hip.kf_rb_pack(ctx.h, typ, w.data_ptr(), 40, 50, pw.data_ptr(), 64, 21, -1, 1))
+        assert torch.equal(pw, stored(row))
     # states: forced ids, a parked slot, a position outside
     state = torch.tensor([[1, 2, 0, 0], [4, 0, 1, 0], [5, 8, 0, 0], [6, 7, 0, 0]], dtype=torch.int32, device="cuda")
     forced = torch.full((4, 8), -1, dtype=torch.int32, device="cuda")
