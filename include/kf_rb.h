@@ -104,8 +104,8 @@ int kf_rb_norm(kf_ctx* ctx, int type, const void* z, const float* res, float alp
  * There is no v: a row's value is its k column block as the projection left it.  q and k: RMS norm per head, then the leading rot_dims dimensions turned by the table
  * `rope`, dimension i together with i + rot_dims / 2.  Scores are scale * <q, k>; with chunk > 0 a query sees only its own chunk (positions c chunk .. (c + 1) chunk - 1) up to
  * itself, with chunk 0 everything up to itself.  out [rows][ldout], columns n_head * dim: softmax-weighted values, times sigmoid(gate) when gated.
- * The state: kv-head g's key (normed, rotated) and value of position j in slot s lie at cache[s * slot_stride + (g * cache_rows + j % cache_rows) * dim]; cache_rows >=
- * min(chunk, positions).  scratch holds arrival counters: zero it once after allocation. */
+ * The state: kv-head g's key (normed, rotated) and value of position j in slot s lie at cache[s * slot_stride + g * head_stride + (j % cache_rows) * dim];
+ * cache_rows >= min(chunk, positions).  scratch holds arrival counters: zero it once after allocation. */
 typedef struct kf_rb_attention {
     void* raw;
     void* out;
@@ -114,7 +114,7 @@ typedef struct kf_rb_attention {
     const void *q_norm, *k_norm; /* [dim], NULL: no norm */
     const float* rope;      /* [max_pos][rot_dims / 2][2] (cos, sin) */
     void* scratch;          /* decode form, kf_rb_attention_scratch() bytes */
-    int64_t ldraw, ldout, slot_stride;
+    int64_t ldraw, ldout, slot_stride, head_stride;
     int32_t type, n_head, n_kv, dim, rot_dims, chunk, cache_rows, gated;
     float scale, eps;
 } kf_rb_attention;

@@ -73,7 +73,7 @@ __global__ void __launch_bounds__(256) rb_prep_kernel(const kf_rb_attention a, c
     const T* k = raw + (size_t)u * a.dim;
     T* dst;
     if constexpr (STORE) {
-        const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + ((size_t)g * a.cache_rows + pos % a.cache_rows) * a.dim;
+        const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)g * a.head_stride + (size_t)(pos % a.cache_rows) * a.dim;
         dst = reinterpret_cast<T*>(a.k_cache) + at;
         T* v = reinterpret_cast<T*>(a.v_cache) + at;
         for (int i = lane; i < a.dim; i += 64) v[i] = k[i];
@@ -129,7 +129,7 @@ __global__ void __launch_bounds__(256) rb_store_kernel(const kf_rb_attention a, 
     const int r = blockIdx.x, pos = meta[KF_RB_META * r], last = meta[KF_RB_META * r + 3];
     if (pos < 0 || pos <= last - a.cache_rows) return;
     const int kvd = a.n_kv * a.dim;
-    const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * a.dim, head = (size_t)a.cache_rows * a.dim;
+    const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * a.dim, head = a.head_stride;
     const T* k = reinterpret_cast<const T*>(a.k_new) + (size_t)r * kvd;
     const T* v = reinterpret_cast<const T*>(a.raw) + (size_t)r * a.ldraw + (size_t)a.n_head * a.dim;
     T *kc = reinterpret_cast<T*>(a.k_cache) + at, *vc = reinterpret_cast<T*>(a.v_cache) + at;
@@ -170,7 +170,7 @@ __global__ void __launch_bounds__(64) rb_attn_plain_kernel(const kf_rb_attention
                 k = reinterpret_cast<const T*>(a.k_new) + row * kvd + (size_t)g * a.dim;
                 v = raw + row * a.ldraw + (size_t)(a.n_head + g) * a.dim;
             } else {
-                const size_t at = (size_t)slot * a.slot_stride + ((size_t)g * a.cache_rows + key % a.cache_rows) * a.dim;
+                const size_t at = (size_t)slot * a.slot_stride + (size_t)g * a.head_stride + (size_t)(key % a.cache_rows) * a.dim;
                 k = reinterpret_cast<const T*>(a.k_cache) + at, v = reinterpret_cast<const T*>(a.v_cache) + at;
             }
             float d = 0.f;
@@ -297,8 +297,8 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
     if (bx * 128 >= ncol) return; /* workgroup-uniform */
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw;
     const uint16_t *k_new = reinterpret_cast<const uint16_t*>(a.k_new) + (size_t)row0 * kvd + (size_t)g * a.dim, *v_new = raw + (size_t)(a.n_head + g) * a.dim;
-    const uint16_t* k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.cache_rows * a.dim;
-    const uint16_t* v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.cache_rows * a.dim;
+    const uint16_t* k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.head_stride;
+    const uint16_t* v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.head_stride;
     // this lane pair's column; columns past the end repeat the last one and are not stored
     int c = bx * 128 + wid * 32 + r;
     const bool col_ok = c < ncol;
@@ -425,7 +425,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     float* s_buf = reinterpret_cast<float*>(s_q + 32 * KS);              /* [4][HD] */
     __shared__ int s_last;
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)rr * a.ldraw;
-    const size_t base = (size_t)slot * a.slot_stride + (size_t)g * a.cache_rows * a.dim;
+    const size_t base = (size_t)slot * a.slot_stride + (size_t)g * a.head_stride;
     uint16_t *kc = reinterpret_cast<uint16_t*>(a.k_cache) + base, *vc = reinterpret_cast<uint16_t*>(a.v_cache) + base;
     constexpr int CPT = CH / 2; /* chunks per lane of a 32-row tile */
     u32x4 kr[CPT], vr[CPT];
@@ -576,7 +576,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
 constexpr int RB_MAX_RANGES = 32;
 static void decode_ranges(int n_rows, int n_kv, int keys, int& span, int& n_range) {
     n_range = (keys + 255) / 256; /* a range is at least two tiles per wave */
-    const int want = (1024 + n_rows * n_kv - 1) / (n_rows * n_kv);
+    const int want = (512 + n_rows * n_kv - 1) / (n_rows * n_kv); /* two workgroups per CU: one round */
     n_range = std::max(1, std::min(n_range, std::min(want, RB_MAX_RANGES)));
     span = ((keys + n_range - 1) / n_range + 127) / 128 * 128;
     n_range = (keys + span - 1) / span;
@@ -619,7 +619,7 @@ static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* me
     return KF_OK;
 }
 static bool mfma_served(const kf_rb_attention& a, int n_rows) {
-    return a.type == KF_BF16 && (int64_t)n_rows * a.ldraw < ((int64_t)1 << 30) && (int64_t)a.cache_rows * a.n_kv * a.dim < ((int64_t)1 << 30) && a.dim % 8 == 0 && a.dim <= 256 && a.ldraw % 8 == 0 && a.ldout % 4 == 0 && a.slot_stride % 8 == 0;
+    return a.type == KF_BF16 && (int64_t)n_rows * a.ldraw < ((int64_t)1 << 30) && (int64_t)a.cache_rows * a.n_kv * a.dim < ((int64_t)1 << 30) && a.dim % 8 == 0 && a.dim <= 256 && a.ldraw % 8 == 0 && a.ldout % 4 == 0 && a.slot_stride % 8 == 0 && a.head_stride % 8 == 0;
 }
 #define RB_BY_DIM(call)                       \
     (a.dim <= 32    ? call(32)                \
@@ -668,7 +668,7 @@ static int check_attention(const kf_rb_attention* a, const int32_t* meta, int n,
         return abi_fail(KF_INVALID_ARGS, "%s: %d / %d heads of %d, %d rotated, chunk %d, %d cache rows", who, a->n_head, a->n_kv, a->dim, a->rot_dims, a->chunk, a->cache_rows);
     if (a->dim > 512) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: head size %d (served: up to 512)", who, a->dim);
     const int64_t cols = (int64_t)(a->gated ? 2 : 1) * a->n_head * a->dim + (int64_t)a->n_kv * a->dim;
-    if (a->ldraw < cols || a->ldout < (int64_t)a->n_head * a->dim || a->slot_stride < (int64_t)a->cache_rows * a->n_kv * a->dim) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
+    if (a->ldraw < cols || a->ldout < (int64_t)a->n_head * a->dim || a->head_stride < (int64_t)a->cache_rows * a->dim || a->slot_stride < a->head_stride * a->n_kv) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
     if (!al16(a->raw) || !al16(a->out) || !al16(a->k_cache) || !al16(a->v_cache)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
     return KF_OK;
 }

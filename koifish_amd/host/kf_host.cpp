@@ -65,7 +65,7 @@ int KVCache::InitRings(kf_ctx* c, const std::vector<Ring>& layers, int n_slots, 
     size_t n = 0;
     for (Ring& r : rings) {
         r.begin = n;
-        n += ((size_t)r.rows * r.dim * n_slots + 127) & ~(size_t)127;
+        n += (r.slot_stride() * n_slots + 127) & ~(size_t)127;
     }
     for (hGTensor* t : {&key, &val}) {
         *t = std::make_shared<GTensor>();

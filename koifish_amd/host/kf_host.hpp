@@ -73,11 +73,13 @@ struct KVCache {
     int n_layer = 0, max_seq_len = 0, kv_dim = 0;
     int Init(kf_ctx* c, int n_layer, int max_seq, int kv_dim);
     void* Get(CTYPE type, int layer, int pos) const;  // Cache.cpp:42-57
-    // Per-layer rings: layer l of slot s keeps the last `rows` positions (what the layer's mask can still see), position p in row p % rows, dim elements per position (the kv-heads' rows
-    // one head after the other); all
-    // slots of a layer together, a slot rows * dim elements after the one before
+    // Per-layer rings: layer l of slot s keeps the last `rows` positions (what the layer's mask can still see), position p in row p % rows of every kv-head; all
+    // slots of a layer together.  A kv-head's rows are followed by a gap of a page and a quarter kilobyte: streams that walk different heads or slots in step otherwise meet
+    // in the same memory channels (their distance would be a power of two)
     struct Ring {
-        int rows = 0, dim = 0;
+        int rows = 0, heads = 0, dim = 0;  // dim: of one head
+        size_t head_stride() const { return (((size_t)rows * dim + 7) & ~(size_t)7) + 2176; }
+        size_t slot_stride() const { return heads * head_stride(); }
         size_t begin = 0;  // elements in front of the layer
     };
     std::vector<Ring> rings;

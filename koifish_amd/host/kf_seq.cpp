@@ -52,7 +52,7 @@ int ChunkAttention::Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int ma
     std::memset(&a, 0, sizeof(a));
     a.raw = P(w.raw), a.out = P(w.ao), a.k_new = P(w.knew), a.k_cache = kv.Ring0(KVCache::KV_KEY, layid - 1), a.v_cache = kv.Ring0(KVCache::KV_VAL, layid - 1);
     a.q_norm = c.qk_norm ? P(qn) : nullptr, a.k_norm = c.qk_norm ? P(kn) : nullptr, a.rope = rope, a.scratch = P(w.scratch);
-    a.ldraw = ldraw, a.ldout = ldout, a.slot_stride = (int64_t)ring.rows * ring.dim;
+    a.ldraw = ldraw, a.ldout = ldout, a.slot_stride = (int64_t)ring.slot_stride(), a.head_stride = (int64_t)ring.head_stride();
     a.type = card.type, a.n_head = c.heads, a.n_kv = c.kv_heads, a.dim = c.dim, a.rot_dims = c.rot.dims, a.chunk = c.chunk, a.cache_rows = ring.rows, a.gated = c.gated;
     a.scale = c.scale, a.eps = card.eps;
     if (n_seq) KF_TRY(kf_rb_attention_prefill(hFish->ctx, &a, I(w.meta), n, I(w.seqs), n_seq, max_n));
@@ -307,8 +307,7 @@ SeqFish* BuildSeqModel(const JSON& cfg, const std::string& dir, int device, void
 int SeqFish::InitSlots(SeqSlots& s, int n) {
     s.n = n;
     std::vector<KVCache::Ring> rings;
-    for (const LAYER_CARD& L : card.layers) rings.push_back(KVCache::Ring{L.mix.chunk > 0 ? std::min(L.mix.chunk, card.n_ctx) : card.n_ctx, up(L.mix.kv_heads * L.mix.dim, 8), 0});
-    for (size_t l = 0; l < rings.size(); l++) rings[l].dim = card.layers[l].mix.kv_heads * card.layers[l].mix.dim;
+    for (const LAYER_CARD& L : card.layers) rings.push_back(KVCache::Ring{L.mix.chunk > 0 ? std::min(L.mix.chunk, card.n_ctx) : card.n_ctx, L.mix.kv_heads, L.mix.dim, 0});
     KF_TRY(s.kv.InitRings(ctx, rings, n, card.type));
     s.pos.assign(n, 0), s.parked.assign(n, 0), s.taken.assign(n, 0);
     s.pick_ws = Mem(ctx, "pick", KF_F32, kf_rb_pick_scratch(n) / 4), s.logits16 = Mem(ctx, "logits16", KF_BF16, card.vocab);

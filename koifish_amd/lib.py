@@ -55,7 +55,7 @@ class RbProduct(C.Structure):
 class RbAttention(C.Structure):
     """struct kf_rb_attention"""
     _fields_ = [("raw", C.c_void_p), ("out", C.c_void_p), ("k_new", C.c_void_p), ("k_cache", C.c_void_p), ("v_cache", C.c_void_p), ("q_norm", C.c_void_p), ("k_norm", C.c_void_p),
-                ("rope", C.c_void_p), ("scratch", C.c_void_p), ("ldraw", C.c_int64), ("ldout", C.c_int64), ("slot_stride", C.c_int64), ("type", C.c_int32), ("n_head", C.c_int32),
+                ("rope", C.c_void_p), ("scratch", C.c_void_p), ("ldraw", C.c_int64), ("ldout", C.c_int64), ("slot_stride", C.c_int64), ("head_stride", C.c_int64), ("type", C.c_int32), ("n_head", C.c_int32),
                 ("n_kv", C.c_int32), ("dim", C.c_int32), ("rot_dims", C.c_int32), ("chunk", C.c_int32), ("cache_rows", C.c_int32), ("gated", C.c_int32), ("scale", C.c_float), ("eps", C.c_float)]
 
 

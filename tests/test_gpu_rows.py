@@ -242,7 +242,7 @@ class Attn:
         self.qn, self.kn = (dev(torch.rand(up(D), generator=g) + 0.5, self.dt) for _ in range(2))
         chunk = mx["mask"]["size"] if mx["mask"] else 0
         rows = min(chunk, n_ctx) if chunk else n_ctx
-        self.kc, self.vc = (torch.zeros(n_slots * rows * G * D + 64, dtype=self.dt, device="cuda") for _ in range(2))
+        self.kc, self.vc = (torch.zeros(n_slots * (rows * D + 24) * G + 64, dtype=self.dt, device="cuda") for _ in range(2))
         self.tab = np.zeros((n_ctx, max(mx["rot"]["dims"], 2) // 2, 2), dtype=np.float32)
         if mx["rot"]["dims"]:
             s = mx["rot"]["scaling"]
@@ -252,7 +252,7 @@ class Attn:
         self.n_slots, self.cols = n_slots, 2 * H * D + G * D
         self.a = L.RbAttention(type=self.typ, n_head=H, n_kv=G, dim=D, rot_dims=mx["rot"]["dims"], chunk=chunk, cache_rows=rows, gated=1, scale=mx["scale"], eps=1e-5, k_cache=self.kc.data_ptr(),
                                v_cache=self.vc.data_ptr(), q_norm=self.qn.data_ptr(), k_norm=self.kn.data_ptr(), rope=self.tab.data_ptr(), ldraw=self.ldraw, ldout=self.ldout,
-                               slot_stride=rows * G * D)
+                               slot_stride=(rows * D + 24) * G, head_stride=rows * D + 24)
         self.hist = {}
         self.rng = np.random.default_rng(seed)
 
@@ -379,7 +379,7 @@ def test_attention_refuses(ctx):
     m = torch.zeros(4, dtype=torch.int32, device="cuda")
     for f in ("raw", "out", "k_new", "scratch"):
         setattr(a.a, f, t.data_ptr())
-    for f, v in (("n_kv", 3), ("rot_dims", 66), ("rot_dims", 3), ("ldraw", 64), ("slot_stride", 8), ("cache_rows", 0), ("dim", 1024), ("type", L.Q4), ("raw", None)):
+    for f, v in (("n_kv", 3), ("rot_dims", 66), ("rot_dims", 3), ("ldraw", 64), ("slot_stride", 8), ("head_stride", 8), ("cache_rows", 0), ("dim", 1024), ("type", L.Q4), ("raw", None)):
         old = getattr(a.a, f)
         setattr(a.a, f, v)
         assert ctx.hip.kf_rb_attention_prefill(ctx.h, C.byref(a.a), m.data_ptr(), 1, m.data_ptr(), 1, 1) < 0, f
