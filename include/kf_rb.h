@@ -19,6 +19,7 @@ extern "C" {
 
 #define KF_RB_PAD 64
 #define KF_RB_NORM_ROWS 4
+#define KF_RB_SUM_PAIRS 1024 /* (row, choice) pairs of a batch the SUM mode takes */
 #define KF_RB_DECODE_MAX 64 /* rows of a decode batch the streaming products serve; larger batches take the tile kernels */
 
 /* activations; GELU in its tanh form, as kf_gelu */

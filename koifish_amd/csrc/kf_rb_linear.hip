@@ -191,13 +191,12 @@ __global__ void __launch_bounds__(64 * NW) rb_stream_kernel(const RbProduct q) {
 }
 
 // RESIDUAL with the rows' experts summed: (chosen expert, k-step) pairs as one list, cut evenly over the waves
-constexpr int RB_SUM_IDS = 1024;
 template <int NT, int NW>
 __global__ void __launch_bounds__(64 * NW) rb_stream_sum_kernel(const RbProduct q) {
     const kf_rb_product& p = q.p;
     constexpr int U = NT >= 4 ? 2 : 4;
     __shared__ float red[NW][1][16 * NT][17];
-    __shared__ int32_t s_ex[RB_SUM_IDS], s_ids[RB_SUM_IDS];
+    __shared__ int32_t s_ex[KF_RB_SUM_PAIRS], s_ids[KF_RB_SUM_PAIRS];
     __shared__ int s_n;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, q4 = lane >> 4;
     const int m0 = blockIdx.x * 16, nstep = p.k / 32, pairs = p.n * q.e.top;
@@ -263,7 +262,7 @@ int rb_stream_launch(hipStream_t st, const RbProduct& q) {
     const bool tiles = p.mode == KF_RB_UP || p.mode == KF_RB_DOWN;
     const int cols = tiles ? q.e.tile : p.n, nt = (cols + 15) / 16;
     if (nt > 4 || (tiles && q.e.tile % 16)) return 1;
-    if (p.mode == KF_RB_SUM && ((long)p.n * q.e.top > RB_SUM_IDS || q.e.tile < p.n)) return 1;
+    if (p.mode == KF_RB_SUM && ((long)p.n * q.e.top > KF_RB_SUM_PAIRS || q.e.tile < p.n)) return 1;
     dim3 grid(p.m / (p.epilogue == KF_RB_GATED ? 32 : 16), tiles ? q.e.n_tile : 1);
     const bool wide = (long)grid.x * grid.y < 768 && p.k >= 512; /* few workgroups: more waves each, more loads in flight per CU */
     if (p.norm_z) {

@@ -77,7 +77,7 @@ int RowFFN::Forw(RowWork& w, int n, bool defer) {
         }
         return norm.Forw(F(w.z), n, F(w.x), P(w.h));
     }
-    const bool few = card.type == KF_BF16 && n <= KF_RB_DECODE_MAX;
+    const bool few = Sums(card.type, n);
     kf_rb_experts e;
     std::memset(&e, 0, sizeof(e));
     e.n_expert = c.experts, e.top = c.top;
@@ -336,7 +336,7 @@ int SeqFish::Ensure(RowWork& w, int rows, int n_seq, int head_rows, bool decode)
             act = std::max<size_t>(act, (size_t)rows * (moe ? f->c.top : 1) * f->ldact);
             if (!moe) continue;
             rl = std::max<size_t>(rl, (size_t)rows * f->router.m), pairs = std::max<size_t>(pairs, (size_t)rows * f->c.top);
-            if (T == KF_F32 || rows > KF_RB_DECODE_MAX) y = std::max<size_t>(y, (size_t)rows * f->c.top * W);
+            if (!f->Sums(T, rows)) y = std::max<size_t>(y, (size_t)rows * f->c.top * W);
             for (int tile : {16, 32, 48, 64, 128}) { /* whichever tile a batch of at most `rows` rows picks */
                 const size_t n = kf_rb_list_tiles(rows, f->c.top, f->c.experts, tile);
                 tiles = std::max(tiles, n), list = std::max(list, n * tile);

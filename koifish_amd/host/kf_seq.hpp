@@ -99,6 +99,7 @@ struct RowFFN : GeNeuron {  // dense gated feed-forward, or routed experts
     RowNorm norm;
     int ldact = 0;
     int Forw(RowWork& w, int n, bool defer);
+    bool Sums(int type, int n) const { return type == KF_BF16 && n <= KF_RB_DECODE_MAX && n * c.top <= KF_RB_SUM_PAIRS; }  // the experts' outputs summed inside one product
 };
 
 struct SeqFish : Fish {

@@ -253,6 +253,23 @@ def test_every_replay_of_a_captured_step_equals_the_eager_one():
     m.close()
 
 
+@pytest.mark.parametrize("n", [9, 60, 70])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_many_slots_decode_together(n, dtype):
+    """decode batches past the sizes the streaming products, their norms and the in-product expert sums take; a third of the slots parked"""
+    cfg = dict(architecture="Tizusun", width=64, vocab=60, postln_alpha=1.2, norm={"eps": 1e-6}, layers=[M.layer(M.mixer(2, 1, 32, 12, 8), M.moe(16, 24, 20)), M.layer(M.mixer(2, 2, 32, 9, 32), M.dense(48))])
+    m, w = make(cfg, dtype, 40)
+    s = Seqs(m, w, cfg, n)
+    for i in range(n):
+        s.open("s%d" % i, M.tokens(cfg, 14, i))
+    s.feed({"s%d" % i: 5 + i % 4 for i in range(n)})
+    for _ in range(5):
+        s.feed({"s%d" % i: 1 for i in range(n)})
+    s.feed({"s%d" % i: 1 for i in range(n) if i % 3 and len(s.tok["s%d" % i][1])})
+    s.x.close()
+    m.close()
+
+
 def test_sampler_draws_through_the_framework():
     from koifish_amd.runtime import XcdReplicas
     cfg = M.CONFIGS["mixed"]
