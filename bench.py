@@ -238,7 +238,7 @@ def main():
         }
         # `value` was timed in the library's default summation order: the CANONICAL one (kf_abi.h kf_set_canonical; round 4), every logit, greedy id and KV row bit-exact against
         # the CPU oracle (cpu_baseline.parity_timed_order).  Beside it, never `value`: the same positions in the v_dot2c / fp32 order (kf_set_canonical(ctx, 0)).
-        out["config"]["summation_order"] = "canonical (the library default): two v_pk_fma_f32 chains per lane + tree, exact power-of-two softmax with fp64 sums -- bit-exact against the CPU oracle"
+        out["config"]["summation_order"] = "canonical (the library default): two fused multiply-add chains per lane + tree, exact power-of-two softmax with fp64 sums -- bit-exact against the CPU oracle"
         ids_timed_run = m.tokens_out(S).copy()   # the greedy ids of the timed (canonical) run at every position: what sequence 0 of the xcd_replicas leg must reproduce
         try:
             ids0 = m.tokens_out(S)

@@ -46,7 +46,7 @@ int RowNorm::Forw(const void* z, int n, float* x_out, void* h_out, const float* 
 }
 int ChunkAttention::Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos, bool defer) {
     const SEQ_CARD& card = hFish->Seq()->card;
-    KF_TRY(qkg.ForwNormed(w, n, P(w.raw), ldraw, KF_RB_STORE));
+    KF_TRY(qkg.Forw(P(w.h), qkg.k, n, P(w.raw), ldraw, KF_RB_STORE));
     const KVCache::Ring& ring = kv.rings[layid - 1];
     kf_rb_attention a;
     std::memset(&a, 0, sizeof(a));
@@ -64,17 +64,13 @@ int ChunkAttention::Forw(RowWork& w, const KVCache& kv, int n, int n_seq, int ma
     }
     return norm.Forw(F(w.z), n, F(w.x), P(w.h));
 }
-int RowFFN::Forw(RowWork& w, int n, bool defer) {
+int RowFFN::Forw(RowWork& w, int n) {
     const SEQ_CARD& card = hFish->Seq()->card;
     if (c.kind == FF_CARD::NONE) return KF_OK;
     const int64_t ld = gateup.k;
     if (c.kind == FF_CARD::DENSE) {
         KF_TRY(gateup.ForwNormed(w, n, P(w.act), ldact, KF_RB_GATED, c.act));
-        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_ALL, nullptr, defer ? F(w.ssq) : nullptr));
-        if (defer) {
-            w.pending = &norm;
-            return KF_OK;
-        }
+        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha));
         return norm.Forw(F(w.z), n, F(w.x), P(w.h));
     }
     const bool few = Sums(card.type, n);
@@ -85,15 +81,11 @@ int RowFFN::Forw(RowWork& w, int n, bool defer) {
     e.tile = few ? up(n, 16) : (card.type == KF_BF16 && (long long)n * c.top >= 256LL * c.experts ? 128 : 64);
     e.n_tile = kf_rb_list_tiles(n, c.top, c.experts, e.tile);
     e.tile_expert = I(w.tile_expert), e.list = I(w.list), e.ids = I(w.ids), e.weight = F(w.weight);
-    KF_TRY(router.ForwNormed(w, n, F(w.rlogits), router.m, KF_RB_STORE_F32));
+    KF_TRY(router.Forw(P(w.h), ld, n, F(w.rlogits), router.m, KF_RB_STORE_F32));
     KF_TRY(kf_rb_route(hFish->ctx, card.type, F(w.rlogits), router.m, P(router_b), n, I(w.meta), &e));
     KF_TRY(gateup.Forw(P(w.h), ld, n, P(w.act), ldact, KF_RB_GATED, c.act, nullptr, 0, KF_RB_UP, &e));
     if (few) {
-        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_SUM, &e, defer ? F(w.ssq) : nullptr));
-        if (defer) {
-            w.pending = &norm;
-            return KF_OK;
-        }
+        KF_TRY(down.Forw(P(w.act), ldact, n, F(w.z), ld, KF_RB_RESIDUAL, 0, F(w.x), card.alpha, KF_RB_SUM, &e));
         return norm.Forw(F(w.z), n, F(w.x), P(w.h));
     }
     KF_TRY(down.Forw(P(w.act), ldact, n, P(w.y), ld, KF_RB_STORE, 0, nullptr, 0, KF_RB_DOWN, &e));
@@ -360,20 +352,17 @@ int SeqFish::Ensure(RowWork& w, int rows, int n_seq, int head_rows, bool decode)
 // ------------------------------------------------------------------------------------------------ steps
 int SeqFish::Layers(RowWork& w, const KVCache& kv, int n, int n_seq, int max_n, int max_pos) {
     const int W = Width(card.width);
-    const bool defer = n_seq == 0 && kf_rb_linear_norms(card.type, n, W); /* few rows: every norm inside the product behind it */
+    // few rows: the norm in front of a dense gate | up inside that product (in front of the q | k | gate product and of a router the separate launch measured the same or faster)
+    const bool fuse = n_seq == 0 && kf_rb_linear_norms(card.type, n, W);
     w.pending = nullptr;
     for (size_t l = 0; l < mixers.size(); l++) {
-        KF_TRY(mixers[l]->Forw(w, kv, n, n_seq, max_n, max_pos, defer));
-        KF_TRY(ffs[l]->Forw(w, n, defer));
+        KF_TRY(mixers[l]->Forw(w, kv, n, n_seq, max_n, max_pos, fuse && ffs[l]->c.kind == FF_CARD::DENSE));
+        KF_TRY(ffs[l]->Forw(w, n));
         if (tap && n_seq && n == tap_rows) {
             std::vector<float> rows((size_t)n * W);
             KF_TRY(kf_d2h(ctx, rows.data(), w.x->data, rows.size() * 4));
             for (int r = 0; r < n; r++) std::memcpy(tap + ((size_t)l * n + r) * card.width, rows.data() + (size_t)r * W, (size_t)card.width * 4);
         }
-    }
-    if (RowNorm* last = w.pending) {
-        w.pending = nullptr;
-        return last->Forw(F(w.z), n, F(w.x), P(w.h));
     }
     return KF_OK;
 }

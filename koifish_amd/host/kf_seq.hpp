@@ -98,7 +98,7 @@ struct RowFFN : GeNeuron {  // dense gated feed-forward, or routed experts
     hGTensor router_b;
     RowNorm norm;
     int ldact = 0;
-    int Forw(RowWork& w, int n, bool defer);
+    int Forw(RowWork& w, int n);
     bool Sums(int type, int n) const { return type == KF_BF16 && n <= KF_RB_DECODE_MAX && n * c.top <= KF_RB_SUM_PAIRS; }  // the experts' outputs summed inside one product
 };
 
