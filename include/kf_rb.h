@@ -26,7 +26,7 @@ extern "C" {
 enum kf_rb_act { KF_RB_RELU = 0, KF_RB_SILU = 1, KF_RB_GELU_TANH = 2 };
 
 /* what a product's epilogue does with row dot d[t][m]:
- *   STORE      y[t][m] = d             (y in the batch's storage)
+ *   STORE      y[t][m] = d             (y in the batch's storage; columns act_lo <= m < act_hi: act(d))
  *   STORE_F32  y[t][m] = d             (fp32)
  *   RESIDUAL   y[t][m] = alpha res[t][m] + d   (fp32)
  *   GATED      y[t][f] = act(d[t][gate f]) * d[t][up f]; the weight holds gate and up interleaved in blocks of 16 rows (16 gate, 16 up, ...), m counts both */
@@ -74,6 +74,7 @@ typedef struct kf_rb_product {
     float* norm_x;
     float norm_eps;
     int32_t norm_dim;
+    int32_t act_lo, act_hi; /* STORE: the columns that pass through act; equal: none */
 } kf_rb_product;
 int kf_rb_linear(kf_ctx* ctx, const kf_rb_product* p);
 int kf_rb_linear_norms(int type, int n, int k);
@@ -97,6 +98,30 @@ int kf_rb_embed_state(kf_ctx* ctx, int type, const void* table, int vocab, int d
 int kf_rb_norm(kf_ctx* ctx, int type, const void* z, const float* res, float alpha, int top, const void* w, float eps, int dim, int64_t ld, int n, const int32_t* rows,
                float* x_out, void* h_out);
 
+/* the norm of a sublayer's OUTPUT, added to the residual, and the norm of an input that takes a position vector first: rows z (fp32, ld apart)
+ *   z += the sinusoid of the row's position (pos_hi != NULL; kf_rb_sinusoid_tables_host, position in meta)
+ *   n  = the norm of z over `dim` columns, times w:  RMS  z / sqrt(mean(z^2) + eps),  LAYER  (z - mean) / sqrt(mean((z - mean)^2) + eps)
+ *   x_out (fp32, may be NULL) and h_out (storage `type`, may be NULL): add + n (add NULL: n), pad columns zero
+ * rows != NULL: output row t comes from row rows[t] of z.  In place on z or add is fine without `rows`. */
+enum kf_rb_norm_kind { KF_RB_RMS = 0, KF_RB_LAYER = 1 };
+typedef struct kf_rb_norming {
+    const float* z;
+    const float* add;
+    const int32_t* rows;
+    const void* w; /* [dim], padded to ld, in storage `type` */
+    float* x_out;
+    void* h_out;
+    const float *pos_hi, *pos_lo;
+    const int32_t* meta;
+    int64_t ld;
+    int32_t type, kind, dim, n;
+    float eps;
+} kf_rb_norming;
+int kf_rb_norm_rows(kf_ctx* ctx, const kf_rb_norming* a);
+/* host: (sin, cos) of p * base^(-2 i / width) for column pair i, as two factors of the angle: hi [(n_pos + 63) / 64][ld / 2][2] at p = 64 j, lo [64][ld / 2][2]; column 2 i of
+ * a position vector is the sine, 2 i + 1 the cosine */
+int kf_rb_sinusoid_tables_host(float* hi, float* lo, int n_pos, int width, int64_t ld, double base);
+
 /* a row's meta: {position (< 0: inactive), slot, position of the sequence's first row in this batch, position of its last row in this batch} */
 #define KF_RB_META 4
 /* a sequence's rows: {first row, rows, position of the first row, slot} */
@@ -105,6 +130,12 @@ int kf_rb_norm(kf_ctx* ctx, int type, const void* z, const float* res, float alp
  * There is no v: a row's value is its k column block as the projection left it.  q and k: RMS norm per head, then the leading rot_dims dimensions turned by the table
  * `rope`, dimension i together with i + rot_dims / 2.  Scores are scale * <q, k>; with chunk > 0 a query sees only its own chunk (positions c chunk .. (c + 1) chunk - 1) up to
  * itself, with chunk 0 everything up to itself.  out [rows][ldout], columns n_head * dim: softmax-weighted values, times sigmoid(gate) when gated.
+ * Variants (zero: the form above):
+ *   v_col   values are raw columns v_col .. v_col + n_kv * vdim - 1, `vdim` per head; the output gate then starts at column gate_col
+ *   unit    q and k are divided by their root mean square, no weight (q_norm = k_norm = NULL)
+ *   window  position i sees j with 0 <= i - j < window (chunk 0)
+ *   sink    one more score of 0 in the softmax's denominator, without a value
+ *   scaled  the output is multiplied by out_scale
  * The state: kv-head g's key (normed, rotated) and value of position j in slot s lie at cache[s * slot_stride + g * head_stride + (j % cache_rows) * dim];
  * cache_rows >= min(chunk, positions).  scratch holds arrival counters: zero it once after allocation. */
 typedef struct kf_rb_attention {
@@ -113,11 +144,13 @@ typedef struct kf_rb_attention {
     void* k_new;            /* [rows][n_kv * dim] scratch: the batch's normed, rotated keys (prefill form) */
     void *k_cache, *v_cache;
     const void *q_norm, *k_norm; /* [dim], NULL: no norm */
-    const float* rope;      /* [max_pos][rot_dims / 2][2] (cos, sin) */
+    const float* rope;      /* [max_pos][rot_dims / 2][2] (cos, sin); rot_dims 0: not read */
     void* scratch;          /* decode form, kf_rb_attention_scratch() bytes */
     int64_t ldraw, ldout, slot_stride, head_stride;
     int32_t type, n_head, n_kv, dim, rot_dims, chunk, cache_rows, gated;
     float scale, eps;
+    int32_t v_col, vdim, gate_col, unit, window, sink, scaled;
+    float out_scale;
 } kf_rb_attention;
 /* rows of n_seq sequences, longest max_n rows: seqs [n_seq][4], meta [n_rows][4] on the device */
 int kf_rb_attention_prefill(kf_ctx* ctx, const kf_rb_attention* a, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n);
@@ -127,6 +160,52 @@ size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim);
 /* host: (cos, sin) of pos * w_i for i < dims / 2, w_i = base^(-2 i / dims) * (t + (1 - t) / factor), t = clamp((original w / 2 pi - low) / (high - low), 0, 1) of the
  * unscaled w: frequencies that turn more than `high` times over `original` positions stay, those below `low` turns slow down by `factor`, a linear blend between. */
 int kf_rb_rope_table_host(float* h_table, int n_pos, int dims, double base, double factor, double low, double high, double original);
+
+/* ---- recurrent layers: a 32-bit state matrix S [dim][vdim] per head and slot, carried from row to row
+ * state: head h of slot s at state[((s * 2 + side) * n_head + h) * dim * vs], rows of vs = vdim rounded up to 4 floats.  The state AFTER position p lies on side p & 1: a step reads
+ * side (p - 1) & 1 and writes the other one, so a step that is run twice on the same position gives the same.  Position 0 starts from zero whatever the slot holds.
+ *
+ * The gated delta rule with one decay per head and key channel.  raw [rows][ldraw] holds, as projected: q (n_kv * dim) from column 0, k (n_kv * dim), v (n_head * vdim), and from columns
+ * col_b: n_head logits of the step sizes, col_a: rank_a, col_g: rank_g inputs of the low-rank factors.  q, k, v: causal convolution over time per channel (conv [channels][taps], last
+ * tap the row itself, nothing before position 0), SiLU; q and k per head divided by sqrt(sum of squares + unit_eps), q times q_scale.  Head h uses q / k head h / (n_head / n_kv).
+ *   beta = sigmoid(b),  decay g = exp(-exp(a_log[h]) softplus(a + dt_bias)) with a = w_a2 . (rank_a columns), [n_head][dim]
+ *   S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+ *   out = o / sqrt(mean over vdim (o^2) + eps) * norm_w * sigmoid(w_g2 . (rank_g columns)), [n_head][vdim]
+ * hist: the convolution's last inputs, raw columns 0 .. channels - 1 of position p at hist[s * hist_slot + (p % taps) * channels].
+ * w_a2 / w_g2 are products' weights of ld_a / ld_g columns; the prompt form takes their products from the caller: a_z fp32 [rows][ld_az], g_z (storage) [rows][ld_gz]. */
+typedef struct kf_rb_delta {
+    const void* raw;
+    void* out;
+    const void *conv, *w_a2, *w_g2, *a_log, *dt_bias, *norm_w;
+    const float* a_z;
+    const void* g_z;
+    float* state;
+    void* hist;
+    float* scratch; /* prompt form: kf_rb_delta_scratch() bytes */
+    int64_t ldraw, ldout, ld_az, ld_gz, hist_slot;
+    int32_t type, n_head, n_kv, dim, vdim, taps, col_b, col_a, col_g, rank_a, rank_g, ld_a, ld_g;
+    float q_scale, unit_eps, eps;
+} kf_rb_delta;
+int kf_rb_delta_prefill(kf_ctx* ctx, const kf_rb_delta* a, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n);
+int kf_rb_delta_decode(kf_ctx* ctx, const kf_rb_delta* a, const int32_t* meta, int n_rows);
+size_t kf_rb_delta_scratch(int type, int n_rows, int n_seq, int n_head, int n_kv, int dim, int vdim);
+
+/* A sum with one constant decay per head: S <- decay[h] S + k v^T, o = S^T q.  raw holds q (n_head * dim) from column col_q, k behind it, v (n_head * vdim) behind that -- activated
+ * already -- and from col_g n_head * vdim gate logits.  All heads together: out = out_scale * o / sqrt(mean(o^2) + eps) * norm_w * sigmoid(gate). */
+typedef struct kf_rb_decay {
+    const void* raw;
+    void* out;
+    const void* norm_w;   /* [n_head * vdim] */
+    const float* decay;   /* [n_head] on the device */
+    float* state;
+    float* scratch;       /* kf_rb_decay_scratch() bytes, zeroed once after allocation (arrival counters) */
+    int64_t ldraw, ldout;
+    int32_t type, n_head, dim, vdim, col_q, col_g;
+    float out_scale, eps;
+} kf_rb_decay;
+int kf_rb_decay_prefill(kf_ctx* ctx, const kf_rb_decay* a, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n);
+int kf_rb_decay_decode(kf_ctx* ctx, const kf_rb_decay* a, const int32_t* meta, int n_rows);
+size_t kf_rb_decay_scratch(int type, int n_rows, int n_seq, int n_head, int dim, int vdim);
 
 /* router: logits fp32 [n][ld] (+ bias [n_expert] in the batch's storage, may be NULL) -> the `top` largest of every row (ties: the lower expert) and the softmax over them;
  * rows whose meta position is < 0 (meta != NULL) choose nothing.  Then the pairs grouped by expert into the list.  experts: the arrays it points to are written. */

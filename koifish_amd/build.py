@@ -13,7 +13,7 @@ import sys
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 HOST = os.path.join(HERE, "host")
-HIP_SOURCES = ["kf_gemv.hip", "kf_gemv_canon.hip", "kf_gemm.hip", "kf_gemm2.hip", "kf_gemm3.hip", "kf_attn.hip", "kf_engine.hip", "kf_xengine.hip", "kf_xengine_q1.hip", "kf_attn_prefill.hip", "kf_ops.hip", "kf_lut.hip", "kf_loss.hip", "kf_norm_bwd.hip", "kf_linear_bwd.hip", "kf_embed_bwd.hip", "kf_attn_bwd_mfma.hip", "kf_awq.hip", "kf_tp.hip", "kf_rb_ops.hip", "kf_rb_linear.hip", "kf_rb_gemm.hip", "kf_rb_attn.hip", "kf_abi.hip"]
+HIP_SOURCES = ["kf_gemv.hip", "kf_gemv_canon.hip", "kf_gemm.hip", "kf_gemm2.hip", "kf_gemm3.hip", "kf_attn.hip", "kf_engine.hip", "kf_xengine.hip", "kf_xengine_q1.hip", "kf_attn_prefill.hip", "kf_ops.hip", "kf_lut.hip", "kf_loss.hip", "kf_norm_bwd.hip", "kf_linear_bwd.hip", "kf_embed_bwd.hip", "kf_attn_bwd_mfma.hip", "kf_awq.hip", "kf_tp.hip", "kf_rb_ops.hip", "kf_rb_linear.hip", "kf_rb_gemm.hip", "kf_rb_attn.hip", "kf_rb_recur.hip", "kf_abi.hip"]
 LIB_HIP = os.path.join(HERE, "libkf_hip.so")
 LIB_HOST = os.path.join(HERE, "libkf_host.so")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
@@ -79,7 +79,7 @@ def build_hip(force=False, verbose=False):
     return LIB_HIP
 
 
-HOST_SOURCES = ["kf_host.cpp", "kf_safetensors.cpp", "kf_train.cpp", "kf_seq.cpp", "kf_tizusun.cpp"]
+HOST_SOURCES = ["kf_host.cpp", "kf_safetensors.cpp", "kf_train.cpp", "kf_seq.cpp", "kf_tizusun.cpp", "kf_bolopel.cpp"]
 
 
 def _host_cmd(out, libdir, opt):
@@ -103,7 +103,7 @@ def build_host(force=False, verbose=False):
 
 
 # What one family of models launches.  A fresh checkout that only serves such a model (bin/trace_run) compiles these files and no others: seconds instead of minutes.
-PARTS = {"rows": ["kf_rb_ops.hip", "kf_rb_linear.hip", "kf_rb_gemm.hip", "kf_rb_attn.hip", "kf_ops.hip", "kf_abi.hip"]}
+PARTS = {"rows": ["kf_rb_ops.hip", "kf_rb_linear.hip", "kf_rb_gemm.hip", "kf_rb_attn.hip", "kf_rb_recur.hip", "kf_ops.hip", "kf_abi.hip"]}
 
 
 def build_part(part, verbose=False):

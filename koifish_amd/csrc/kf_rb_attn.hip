@@ -25,12 +25,16 @@ __device__ __forceinline__ float rb_exp2(float x) { return __builtin_amdgcn_exp2
 __device__ __forceinline__ void rb_st_sc1(float* p, float v) { __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
 __device__ __forceinline__ float rb_ld_sc1(const float* p) { return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
 constexpr int RB_CNT_STRIDE = 16; /* words between arrival counters: one cache line each */
-__device__ __forceinline__ int rb_first_key(int pos, int chunk) { return chunk > 0 ? pos - pos % chunk : 0; }
+__device__ __forceinline__ int rb_first_key(int pos, const kf_rb_attention& a) {
+    if (a.window > 0) return pos >= a.window ? pos - a.window + 1 : 0;
+    return a.chunk > 0 ? pos - pos % a.chunk : 0;
+}
+// the launchers fill in what the caller left zero (whole_form): vdim, v_col, gate_col and out_scale hold real values in the kernels
 
 // one head (dim elements at src) normed and rotated by one wave into dst; buf: dim floats of LDS of this wave
 template <class T>
-__device__ __forceinline__ void rb_prep_head(const T* __restrict__ src, T* dst, const T* __restrict__ w, const float* __restrict__ rope, int rot, int dim, int pos, float eps, float* buf,
-                                             int lane) {
+__device__ __forceinline__ void rb_prep_head(const T* __restrict__ src, T* dst, const T* __restrict__ w, bool unit, const float* __restrict__ rope, int rot, int dim, int pos, float eps,
+                                             float* buf, int lane) {
     float ss = 0.f;
     for (int i = lane; i < dim; i += 64) {
         const float v = rb_ld(src + i);
@@ -38,7 +42,7 @@ __device__ __forceinline__ void rb_prep_head(const T* __restrict__ src, T* dst, 
         ss = fmaf(v, v, ss);
     }
     ss = wave_sum(ss);
-    const float rs = w ? 1.0f / sqrtf(ss / (float)dim + eps) : 1.0f;
+    const float rs = w || unit ? 1.0f / sqrtf(ss / (float)dim + eps) : 1.0f;
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
@@ -66,21 +70,22 @@ __global__ void __launch_bounds__(256) rb_prep_kernel(const kf_rb_attention a, c
     float* buf = s_buf + wid * a.dim;
     if (u < a.n_head) {
         T* q = raw + (size_t)u * a.dim;
-        rb_prep_head(q, q, reinterpret_cast<const T*>(a.q_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, buf, lane);
+        rb_prep_head(q, q, reinterpret_cast<const T*>(a.q_norm), a.unit, a.rope, a.rot_dims, a.dim, pos, a.eps, buf, lane);
         return;
     }
     const int g = u - a.n_head, kvd = a.n_kv * a.dim;
     const T* k = raw + (size_t)u * a.dim;
     T* dst;
     if constexpr (STORE) {
-        const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)g * a.head_stride + (size_t)(pos % a.cache_rows) * a.dim;
-        dst = reinterpret_cast<T*>(a.k_cache) + at;
-        T* v = reinterpret_cast<T*>(a.v_cache) + at;
-        for (int i = lane; i < a.dim; i += 64) v[i] = k[i];
+        const size_t head = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)g * a.head_stride, row = pos % a.cache_rows;
+        dst = reinterpret_cast<T*>(a.k_cache) + head + row * a.dim;
+        const T* vn = raw + a.v_col + (size_t)g * a.vdim;
+        T* v = reinterpret_cast<T*>(a.v_cache) + head + row * a.vdim;
+        for (int i = lane; i < a.vdim; i += 64) v[i] = vn[i];
     } else {
         dst = reinterpret_cast<T*>(a.k_new) + (size_t)r * kvd + (size_t)g * a.dim;
     }
-    rb_prep_head(k, dst, reinterpret_cast<const T*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, buf, lane);
+    rb_prep_head(k, dst, reinterpret_cast<const T*>(a.k_norm), a.unit, a.rope, a.rot_dims, a.dim, pos, a.eps, buf, lane);
 }
 // the prompt form, bf16, L lanes per head: lane j < rot / 8 holds the rotation pairs 4 j .. 4 j + 3 (a quad of each half), the next lanes a quad of the dimensions behind
 template <int L>
@@ -104,11 +109,11 @@ __global__ void __launch_bounds__(256) rb_prep_vec_kernel(const kf_rb_attention 
     for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
     if (!on) return;
     const float rs = 1.0f / sqrtf(ss / (float)a.dim + a.eps);
-    const f32x4 wx = rb_ld4(w + i0);
+    const f32x4 one = f32x4{1.f, 1.f, 1.f, 1.f}, wx = w ? rb_ld4(w + i0) : one;
 #pragma unroll
     for (int e = 0; e < 4; e++) x[e] *= rs * wx[e];
     if (pair) {
-        const f32x4 wy = rb_ld4(w + i0 + half);
+        const f32x4 wy = w ? rb_ld4(w + i0 + half) : one;
         const f32x4* cs = reinterpret_cast<const f32x4*>(a.rope + ((size_t)pos * half + i0) * 2);
         const f32x4 c01 = cs[0], c23 = cs[1];
         const float co[4] = {c01.x, c01.z, c23.x, c23.z}, si[4] = {c01.y, c01.w, c23.y, c23.w};
@@ -128,15 +133,18 @@ template <class T>
 __global__ void __launch_bounds__(256) rb_store_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta) {
     const int r = blockIdx.x, pos = meta[KF_RB_META * r], last = meta[KF_RB_META * r + 3];
     if (pos < 0 || pos <= last - a.cache_rows) return;
-    const int kvd = a.n_kv * a.dim;
-    const size_t at = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride + (size_t)(pos % a.cache_rows) * a.dim, head = a.head_stride;
+    const int kvd = a.n_kv * a.dim, vvd = a.n_kv * a.vdim;
+    const size_t slot = (size_t)meta[KF_RB_META * r + 1] * a.slot_stride, row = pos % a.cache_rows, head = a.head_stride;
     const T* k = reinterpret_cast<const T*>(a.k_new) + (size_t)r * kvd;
-    const T* v = reinterpret_cast<const T*>(a.raw) + (size_t)r * a.ldraw + (size_t)a.n_head * a.dim;
-    T *kc = reinterpret_cast<T*>(a.k_cache) + at, *vc = reinterpret_cast<T*>(a.v_cache) + at;
+    const T* v = reinterpret_cast<const T*>(a.raw) + (size_t)r * a.ldraw + a.v_col;
+    T *kc = reinterpret_cast<T*>(a.k_cache) + slot + row * a.dim, *vc = reinterpret_cast<T*>(a.v_cache) + slot + row * a.vdim;
     for (int i = threadIdx.x; i < kvd; i += blockDim.x) {
         const int g = i / a.dim;
-        const size_t o = g * head + (i - g * a.dim);
-        kc[o] = k[i], vc[o] = v[i];
+        kc[g * head + (i - g * a.dim)] = k[i];
+    }
+    for (int i = threadIdx.x; i < vvd; i += blockDim.x) {
+        const int g = i / a.vdim;
+        vc[g * head + (i - g * a.vdim)] = v[i];
     }
 }
 
@@ -154,12 +162,12 @@ __global__ void __launch_bounds__(64) rb_attn_plain_kernel(const kf_rb_attention
     const T* raw = reinterpret_cast<const T*>(a.raw);
     for (int i = lane; i < a.dim; i += 64) s_q[i] = rb_ld(raw + (size_t)r * a.ldraw + (size_t)n * a.dim + i);
     __syncthreads();
-    constexpr int ND = 8; /* dims per lane: dim <= 512 */
+    constexpr int ND = 8; /* dims per lane: vdim <= 512 */
     float o[ND];
 #pragma unroll
     for (int j = 0; j < ND; j++) o[j] = 0.f;
     float M = -__builtin_inff(), l = 0.f;
-    for (int k0 = rb_first_key(pos, a.chunk); k0 <= pos; k0 += 64) {
+    for (int k0 = rb_first_key(pos, a); k0 <= pos; k0 += 64) {
         const int key = k0 + lane;
         float s = -__builtin_inff();
         const T* v = nullptr;
@@ -168,10 +176,10 @@ __global__ void __launch_bounds__(64) rb_attn_plain_kernel(const kf_rb_attention
             if (key >= pos0) {
                 const size_t row = (size_t)r - (pos - key);
                 k = reinterpret_cast<const T*>(a.k_new) + row * kvd + (size_t)g * a.dim;
-                v = raw + row * a.ldraw + (size_t)(a.n_head + g) * a.dim;
+                v = raw + row * a.ldraw + a.v_col + (size_t)g * a.vdim;
             } else {
-                const size_t at = (size_t)slot * a.slot_stride + (size_t)g * a.head_stride + (size_t)(key % a.cache_rows) * a.dim;
-                k = reinterpret_cast<const T*>(a.k_cache) + at, v = reinterpret_cast<const T*>(a.v_cache) + at;
+                const size_t head = (size_t)slot * a.slot_stride + (size_t)g * a.head_stride, row = key % a.cache_rows;
+                k = reinterpret_cast<const T*>(a.k_cache) + head + row * a.dim, v = reinterpret_cast<const T*>(a.v_cache) + head + row * a.vdim;
             }
             float d = 0.f;
             for (int i = 0; i < a.dim; i++) d = fmaf(s_q[i], rb_ld(k + i), d);
@@ -193,17 +201,29 @@ __global__ void __launch_bounds__(64) rb_attn_plain_kernel(const kf_rb_attention
 #pragma unroll
             for (int j = 0; j < ND; j++) {
                 const int d = lane + 64 * j;
-                if (d < a.dim) o[j] = fmaf(pi, rb_ld(vi + d), o[j]);
+                if (d < a.vdim) o[j] = fmaf(pi, rb_ld(vi + d), o[j]);
             }
         }
     }
-    const T* gate = raw + (size_t)r * a.ldraw + (size_t)(a.n_head + a.n_kv + n) * a.dim;
-    T* out = reinterpret_cast<T*>(a.out) + (size_t)r * a.ldout + (size_t)n * a.dim;
+    float f = a.out_scale;
+    if (a.sink) {
+        const float Ms = fmaxf(M, 0.f), fs = expf(M - Ms);
+        l = l * fs + expf(-Ms), f *= fs;
+    }
+    const T* gate = raw + (size_t)r * a.ldraw + a.gate_col + (size_t)n * a.vdim;
+    T* out = reinterpret_cast<T*>(a.out) + (size_t)r * a.ldout + (size_t)n * a.vdim;
 #pragma unroll
     for (int j = 0; j < ND; j++) {
         const int d = lane + 64 * j;
-        if (d < a.dim) rb_st(out + d, o[j] / l * (a.gated ? rb_sigmoid(rb_ld(gate + d)) : 1.f));
+        if (d < a.vdim) rb_st(out + d, o[j] * f / l * (a.gated ? rb_sigmoid(rb_ld(gate + d)) : 1.f));
     }
+}
+
+// what a column's sum of values is multiplied by, from its maximum M (in powers of two) and its sum l: 1 / l, or with the sink's score of 0 in the denominator
+__device__ __forceinline__ float rb_softmax_factor(float M, float l, int sink) {
+    if (!sink) return 1.0f / l;
+    const float Ms = fmaxf(M, 0.f), f = rb_exp2(M - Ms);
+    return f / (l * f + rb_exp2(-Ms));
 }
 
 // ---- MFMA form: one 32-key tile against a wave's 32 columns
@@ -296,19 +316,19 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
     const int GQ = a.n_head / a.n_kv, ncol = n * GQ;
     if (bx * 128 >= ncol) return; /* workgroup-uniform */
     const uint16_t* raw = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw;
-    const uint16_t *k_new = reinterpret_cast<const uint16_t*>(a.k_new) + (size_t)row0 * kvd + (size_t)g * a.dim, *v_new = raw + (size_t)(a.n_head + g) * a.dim;
+    const uint16_t *k_new = reinterpret_cast<const uint16_t*>(a.k_new) + (size_t)row0 * kvd + (size_t)g * a.dim, *v_new = raw + a.v_col + (size_t)g * a.vdim;
     const uint16_t* k_ring = reinterpret_cast<const uint16_t*>(a.k_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.head_stride;
     const uint16_t* v_ring = reinterpret_cast<const uint16_t*>(a.v_cache) + (size_t)slot * a.slot_stride + (size_t)g * a.head_stride;
     // this lane pair's column; columns past the end repeat the last one and are not stored
     int c = bx * 128 + wid * 32 + r;
     const bool col_ok = c < ncol;
     c = col_ok ? c : ncol - 1;
-    const int tok = c / GQ, head = g * GQ + (c - tok * GQ), pos = pos0 + tok, lo = rb_first_key(pos, a.chunk);
+    const int tok = c / GQ, head = g * GQ + (c - tok * GQ), pos = pos0 + tok, lo = rb_first_key(pos, a);
     // the wave's and the workgroup's key ranges
     auto tok_of = [&](int cc) { return (cc < ncol ? cc : ncol - 1) / GQ; };
     const int w0 = pos0 + tok_of(bx * 128 + wid * 32), w1 = pos0 + tok_of(bx * 128 + wid * 32 + 31);
-    const int wlo = rb_first_key(w0, a.chunk), wlo1 = rb_first_key(w1, a.chunk);
-    const int klo = rb_first_key(pos0 + tok_of(bx * 128), a.chunk), khi = pos0 + tok_of(bx * 128 + 127);
+    const int wlo = rb_first_key(w0, a), wlo1 = rb_first_key(w1, a);
+    const int klo = rb_first_key(pos0 + tok_of(bx * 128), a), khi = pos0 + tok_of(bx * 128 + 127);
     u32x4 qf[Tile::NS];
     {
         const uint16_t* q = raw + (size_t)tok * a.ldraw + (size_t)head * a.dim;
@@ -326,7 +346,7 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
         for (int i = 0; i < CPT; i++) {
             const int ch = tid + 256 * i, key = ch / CH, d = (ch - key * CH) * 8;
             kr[i] = vr[i] = u32x4{0, 0, 0, 0};
-            if ((32 * CH % 256 == 0 || key < 32) && d < a.dim) {
+            if (32 * CH % 256 == 0 || key < 32) {
                 const int kk = k0 + key < khi ? k0 + key : khi; /* past the last key: masked, never read past it */
                 const uint16_t *kb = k_new, *vb = v_new;
                 uint32_t ok, ov;
@@ -334,9 +354,11 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
                     ok = (uint32_t)(kk - pos0) * ldk, ov = (uint32_t)(kk - pos0) * ldv;
                 } else {
                     kb = k_ring, vb = v_ring;
-                    ok = ov = ((uint32_t)kk % ring) * (uint32_t)a.dim;
+                    const uint32_t row = (uint32_t)kk % ring;
+                    ok = row * (uint32_t)a.dim, ov = row * (uint32_t)a.vdim;
                 }
-                kr[i] = *reinterpret_cast<const u32x4*>(kb + (ok + d)), vr[i] = *reinterpret_cast<const u32x4*>(vb + (ov + d));
+                if (d < a.dim) kr[i] = *reinterpret_cast<const u32x4*>(kb + (ok + d));
+                if (d < a.vdim) vr[i] = *reinterpret_cast<const u32x4*>(vb + (ov + d));
             }
         }
     };
@@ -387,15 +409,15 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
     }
     const float l = xsum32(T.l);
     if (!col_ok) return;
-    const float inv = 1.0f / l;
-    const uint16_t* gate = raw + (size_t)tok * a.ldraw + (size_t)(a.n_head + a.n_kv + head) * a.dim;
-    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)(row0 + tok) * a.ldout + (size_t)head * a.dim;
+    const float inv = a.out_scale * rb_softmax_factor(T.M, l, a.sink);
+    const uint16_t* gate = raw + (size_t)tok * a.ldraw + a.gate_col + (size_t)head * a.vdim;
+    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)(row0 + tok) * a.ldout + (size_t)head * a.vdim;
 #pragma unroll
     for (int db = 0; db < Tile::NDB; db++)
 #pragma unroll
         for (int q = 0; q < 4; q++) {
             const int d = 32 * db + 8 * q + 4 * h;
-            if (d >= a.dim) continue;
+            if (d >= a.vdim) continue;
             f32x4 v = f32x4{T.o[db][4 * q] * inv, T.o[db][4 * q + 1] * inv, T.o[db][4 * q + 2] * inv, T.o[db][4 * q + 3] * inv};
             if (a.gated) {
                 const f32x4 gv = rb_ld4(gate + d);
@@ -415,7 +437,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     constexpr int KS = Tile::KS, VS = Tile::VS, CH = HD / 8, WAVE_EL = 32 * (KS + VS), NREG = Tile::NDB * 16;
     const int rr = blockIdx.z, pos = meta[KF_RB_META * rr], slot = meta[KF_RB_META * rr + 1];
     if (pos < 0) return; /* workgroup-uniform, like the next */
-    const int first = rb_first_key(pos, a.chunk), k_lo = first + (int)blockIdx.y * span, k_hi = k_lo + span - 1 < pos ? k_lo + span - 1 : pos;
+    const int first = rb_first_key(pos, a), k_lo = first + (int)blockIdx.y * span, k_hi = k_lo + span - 1 < pos ? k_lo + span - 1 : pos;
     if (k_lo > pos) return;
     const int GQ = a.n_head / a.n_kv, ncb = (GQ + 31) / 32, g = blockIdx.x / ncb, cb = blockIdx.x % ncb, col0 = cb * 32, ncol = GQ - col0 < 32 ? GQ - col0 : 32;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5;
@@ -434,11 +456,10 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
         for (int i = 0; i < CPT; i++) {
             const int ch = lane + 64 * i, key = ch / CH, d = (ch - key * CH) * 8;
             kr[i] = vr[i] = u32x4{0, 0, 0, 0};
-            if (d < a.dim) {
-                const int kk = k0 + key < k_hi ? k0 + key : k_hi;
-                const uint32_t at = ((uint32_t)kk % (uint32_t)a.cache_rows) * (uint32_t)a.dim + d;
-                kr[i] = *reinterpret_cast<const u32x4*>(kc + at), vr[i] = *reinterpret_cast<const u32x4*>(vc + at);
-            }
+            const int kk = k0 + key < k_hi ? k0 + key : k_hi;
+            const uint32_t row = (uint32_t)kk % (uint32_t)a.cache_rows;
+            if (d < a.dim) kr[i] = *reinterpret_cast<const u32x4*>(kc + (row * (uint32_t)a.dim + d));
+            if (d < a.vdim) vr[i] = *reinterpret_cast<const u32x4*>(vc + (row * (uint32_t)a.vdim + d));
         }
     };
     int k0 = k_lo + wid * 32;
@@ -447,17 +468,18 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     __syncthreads();
     for (int u = wid; u <= ncol; u += 4) {
         if (u < ncol) {
-            rb_prep_head(raw + (size_t)(g * GQ + col0 + u) * a.dim, s_q + u * KS, reinterpret_cast<const uint16_t*>(a.q_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
+            rb_prep_head(raw + (size_t)(g * GQ + col0 + u) * a.dim, s_q + u * KS, reinterpret_cast<const uint16_t*>(a.q_norm), a.unit, a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
         } else if (k_hi == pos) {
             const uint16_t* k = raw + (size_t)(a.n_head + g) * a.dim;
-            rb_prep_head(k, s_new, reinterpret_cast<const uint16_t*>(a.k_norm), a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
-            const size_t at = (size_t)(pos % a.cache_rows) * a.dim;
+            rb_prep_head(k, s_new, reinterpret_cast<const uint16_t*>(a.k_norm), a.unit, a.rope, a.rot_dims, a.dim, pos, a.eps, s_buf + wid * HD, lane);
+            const uint16_t* vn = raw + a.v_col + (size_t)g * a.vdim;
+            const size_t row = pos % a.cache_rows;
             for (int i = lane; i < HD; i += 64) {
-                const bool in = i < a.dim;
-                const uint16_t v = in ? k[i] : (uint16_t)0;
+                const uint16_t v = i < a.vdim ? vn[i] : (uint16_t)0;
                 s_new[HD + i] = v;
-                if (!in) s_new[i] = 0;
-                if (in && cb == 0) kc[at + i] = s_new[i], vc[at + i] = v;
+                if (i >= a.dim) s_new[i] = 0;
+                if (i < a.dim && cb == 0) kc[row * a.dim + i] = s_new[i];
+                if (i < a.vdim && cb == 0) vc[row * a.vdim + i] = v;
             }
         }
     }
@@ -507,14 +529,14 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     }
     const int n_used = (pos - first) / span + 1; /* key ranges this row has */
     const int head = g * GQ + col0 + (r < ncol ? r : 0);
-    const uint16_t* gate = raw + (size_t)(a.n_head + a.n_kv + head) * a.dim;
-    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)rr * a.ldout + (size_t)head * a.dim;
-    float* parts = reinterpret_cast<float*>(a.scratch) + RB_CNT_STRIDE * (size_t)gridDim.z * a.n_head; /* behind the arrival counters: [row][head][range][dim + 2] */
-    float* part = parts + (((size_t)rr * a.n_head + head) * n_range + blockIdx.y) * (a.dim + 2);
-    const float inv = 1.0f / L;
+    const uint16_t* gate = raw + a.gate_col + (size_t)head * a.vdim;
+    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)rr * a.ldout + (size_t)head * a.vdim;
+    float* parts = reinterpret_cast<float*>(a.scratch) + RB_CNT_STRIDE * (size_t)gridDim.z * a.n_head; /* behind the arrival counters: [row][head][range][vdim + 2] */
+    float* part = parts + (((size_t)rr * a.n_head + head) * n_range + blockIdx.y) * (a.vdim + 2);
+    const float inv = a.out_scale * rb_softmax_factor(M, L, a.sink);
     for (int q = wid; q < Tile::NDB * 4 && r < ncol; q += 4) { /* a quad of registers = four consecutive d */
         const int d = 8 * q + 4 * h;
-        if (d >= a.dim) continue;
+        if (d >= a.vdim) continue;
         f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int w = 0; w < 4; w++)
@@ -543,10 +565,10 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     if (tid == 0) __hip_atomic_store(counter, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     for (int c = wid; c < ncol; c += 4) {
         const int hd = g * GQ + col0 + c;
-        const float* p = parts + ((size_t)rr * a.n_head + hd) * n_range * (a.dim + 2);
+        const float* p = parts + ((size_t)rr * a.n_head + hd) * n_range * (a.vdim + 2);
         const bool mine = lane < n_used;
-        const float ms = mine ? rb_ld_sc1(p + (size_t)lane * (a.dim + 2)) : -__builtin_inff(), ls = mine ? rb_ld_sc1(p + (size_t)lane * (a.dim + 2) + 1) : 0.f;
-        const float fs = rb_exp2(ms - wave_max(ms)), tot = 1.0f / wave_sum(fs * ls);
+        const float ms = mine ? rb_ld_sc1(p + (size_t)lane * (a.vdim + 2)) : -__builtin_inff(), ls = mine ? rb_ld_sc1(p + (size_t)lane * (a.vdim + 2) + 1) : 0.f;
+        const float mw = wave_max(ms), mx = a.sink ? fmaxf(mw, 0.f) : mw, fs = rb_exp2(ms - mx), tot = a.out_scale / (wave_sum(fs * ls) + (a.sink ? rb_exp2(-mx) : 0.f));
         constexpr int DPL = (HD + 63) / 64;
         float v[DPL];
 #pragma unroll
@@ -556,7 +578,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
 #pragma unroll
             for (int e = 0; e < DPL; e++)
 #pragma unroll
-                for (int s = 0; s < 8; s++) w[e][s] = s0 + s < n_used && lane + 64 * e < a.dim ? rb_ld_sc1(p + (size_t)(s0 + s) * (a.dim + 2) + 2 + lane + 64 * e) : 0.f;
+                for (int s = 0; s < 8; s++) w[e][s] = s0 + s < n_used && lane + 64 * e < a.vdim ? rb_ld_sc1(p + (size_t)(s0 + s) * (a.vdim + 2) + 2 + lane + 64 * e) : 0.f;
 #pragma unroll
             for (int s = 0; s < 8; s++) {
                 const float f1 = __shfl(fs, (s0 + s) & 63, 64); /* past n_used: exp2(-inf) = 0 */
@@ -567,9 +589,9 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
 #pragma unroll
         for (int e = 0; e < DPL; e++) {
             const int d = lane + 64 * e;
-            if (d < a.dim)
-                reinterpret_cast<uint16_t*>(a.out)[(size_t)rr * a.ldout + (size_t)hd * a.dim + d] =
-                    f2bf(v[e] * tot * (a.gated ? rb_sigmoid(bf2f(raw[(size_t)(a.n_head + a.n_kv + hd) * a.dim + d])) : 1.f));
+            if (d < a.vdim)
+                reinterpret_cast<uint16_t*>(a.out)[(size_t)rr * a.ldout + (size_t)hd * a.vdim + d] =
+                    f2bf(v[e] * tot * (a.gated ? rb_sigmoid(bf2f(raw[a.gate_col + (size_t)hd * a.vdim + d])) : 1.f));
         }
     }
 }
@@ -619,19 +641,19 @@ static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* me
     return KF_OK;
 }
 static bool mfma_served(const kf_rb_attention& a, int n_rows) {
-    return a.type == KF_BF16 && (int64_t)n_rows * a.ldraw < ((int64_t)1 << 30) && (int64_t)a.cache_rows * a.n_kv * a.dim < ((int64_t)1 << 30) && a.dim % 8 == 0 && a.dim <= 256 && a.ldraw % 8 == 0 && a.ldout % 4 == 0 && a.slot_stride % 8 == 0 && a.head_stride % 8 == 0;
+    return a.type == KF_BF16 && (int64_t)n_rows * a.ldraw < ((int64_t)1 << 30) && (int64_t)a.cache_rows * a.n_kv * std::max(a.dim, a.vdim) < ((int64_t)1 << 30) && a.dim % 8 == 0 && a.dim <= 256 && a.vdim % 8 == 0 && a.vdim <= 256 && a.v_col % 8 == 0 && a.gate_col % 4 == 0 && a.ldraw % 8 == 0 && a.ldout % 4 == 0 && a.slot_stride % 8 == 0 && a.head_stride % 8 == 0;
 }
-#define RB_BY_DIM(call)                       \
-    (a.dim <= 32    ? call(32)                \
-     : a.dim <= 64  ? call(64)                \
-     : a.dim <= 96  ? call(96)                \
-     : a.dim <= 128 ? call(128)               \
-     : a.dim <= 192 ? call(192)               \
-                    : call(256))
+#define RB_BY_DIM(call)                                 \
+    (std::max(a.dim, a.vdim) <= 32    ? call(32)        \
+     : std::max(a.dim, a.vdim) <= 64  ? call(64)        \
+     : std::max(a.dim, a.vdim) <= 96  ? call(96)        \
+     : std::max(a.dim, a.vdim) <= 128 ? call(128)       \
+     : std::max(a.dim, a.vdim) <= 192 ? call(192)       \
+                                      : call(256))
 
 /* vector form of the prep of a prompt batch: a head's lanes fit 16 or 32, quads of both halves */
 static int prep_vec_lanes(const kf_rb_attention& a) {
-    if (a.type != KF_BF16 || a.dim % 4 || a.rot_dims % 8 || a.ldraw % 4 || !a.q_norm || !a.k_norm) return 0;
+    if (a.type != KF_BF16 || a.dim % 4 || a.rot_dims % 8 || a.ldraw % 4 || (!a.unit && (!a.q_norm || !a.k_norm))) return 0;
     const int need = a.rot_dims / 8 + (a.dim - a.rot_dims) / 4;
     return need <= 16 ? 16 : (need <= 32 ? 32 : 0);
 }
@@ -661,14 +683,23 @@ static void store_go(hipStream_t st, const kf_rb_attention& a, const int32_t* me
 }  // namespace kf
 
 using namespace kf;
+static kf_rb_attention whole_form(const kf_rb_attention& in) {
+    kf_rb_attention a = in;
+    if (!a.vdim) a.vdim = a.dim;
+    if (!a.v_col) a.v_col = a.n_head * a.dim;                       /* the keys as they were projected */
+    if (!a.gate_col) a.gate_col = (a.n_head + a.n_kv) * a.dim;
+    if (!a.scaled) a.out_scale = 1.f;
+    return a;
+}
 static int check_attention(const kf_rb_attention* a, const int32_t* meta, int n, const char* who) {
-    if (!a || !meta || n < 1 || !a->raw || !a->out || !a->k_cache || !a->v_cache || !a->rope) return abi_fail(KF_INVALID_ARGS, "%s: null pointer", who);
+    if (!a || !meta || n < 1 || !a->raw || !a->out || !a->k_cache || !a->v_cache || (a->rot_dims && !a->rope)) return abi_fail(KF_INVALID_ARGS, "%s: null pointer", who);
     if (a->type != KF_BF16 && a->type != KF_F32) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: storage %d", who, a->type);
     if (a->n_head < 1 || a->n_kv < 1 || a->n_head % a->n_kv || a->dim < 1 || a->rot_dims < 0 || a->rot_dims > a->dim || (a->rot_dims & 1) || a->chunk < 0 || a->cache_rows < 1)
         return abi_fail(KF_INVALID_ARGS, "%s: %d / %d heads of %d, %d rotated, chunk %d, %d cache rows", who, a->n_head, a->n_kv, a->dim, a->rot_dims, a->chunk, a->cache_rows);
-    if (a->dim > 512) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: head size %d (served: up to 512)", who, a->dim);
-    const int64_t cols = (int64_t)(a->gated ? 2 : 1) * a->n_head * a->dim + (int64_t)a->n_kv * a->dim;
-    if (a->ldraw < cols || a->ldout < (int64_t)a->n_head * a->dim || a->head_stride < (int64_t)a->cache_rows * a->dim || a->slot_stride < a->head_stride * a->n_kv) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
+    if (a->dim > 512 || a->vdim > 512) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: head sizes %d / %d (served: up to 512)", who, a->dim, a->vdim);
+    if (a->vdim < 1 || a->window < 0 || (a->window && a->chunk) || (a->unit && (a->q_norm || a->k_norm)) || a->v_col < a->n_head * a->dim) return abi_fail(KF_INVALID_ARGS, "%s: values or mask", who);
+    const int64_t cols = std::max((int64_t)a->v_col + (int64_t)a->n_kv * a->vdim, a->gated ? (int64_t)a->gate_col + (int64_t)a->n_head * a->vdim : 0);
+    if (a->ldraw < cols || a->ldout < (int64_t)a->n_head * a->vdim || a->head_stride < (int64_t)a->cache_rows * std::max(a->dim, a->vdim) || a->slot_stride < a->head_stride * a->n_kv) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
     if (!al16(a->raw) || !al16(a->out) || !al16(a->k_cache) || !al16(a->v_cache)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
     return KF_OK;
 }
@@ -678,10 +709,11 @@ size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim) { return n_rows 
 
 int kf_rb_attention_prefill(kf_ctx* c, const kf_rb_attention* ap, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n) {
     CHKCTX(c);
-    const int rc = check_attention(ap, meta, n_rows, "kf_rb_attention_prefill");
+    if (!ap) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_prefill: null pointer");
+    const kf_rb_attention a = whole_form(*ap);
+    const int rc = check_attention(&a, meta, n_rows, "kf_rb_attention_prefill");
     if (rc) return rc;
-    if (!seqs || n_seq < 1 || max_n < 1 || max_n > n_rows || !ap->k_new || !al16(ap->k_new)) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_prefill: bad arguments");
-    const kf_rb_attention& a = *ap;
+    if (!seqs || n_seq < 1 || max_n < 1 || max_n > n_rows || !a.k_new || !al16(a.k_new)) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_prefill: bad arguments");
     hipStream_t st = c->stream;
     int r = KF_OK;
     if (a.type == KF_BF16) {
@@ -704,15 +736,17 @@ int kf_rb_attention_prefill(kf_ctx* c, const kf_rb_attention* ap, const int32_t*
 }
 int kf_rb_attention_decode(kf_ctx* c, const kf_rb_attention* ap, const int32_t* meta, int n_rows, int max_pos) {
     CHKCTX(c);
-    const int rc = check_attention(ap, meta, n_rows, "kf_rb_attention_decode");
+    if (!ap) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: null pointer");
+    const kf_rb_attention a = whole_form(*ap);
+    const int rc = check_attention(&a, meta, n_rows, "kf_rb_attention_decode");
     if (rc) return rc;
     if (max_pos < 0) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: max_pos %d", max_pos);
-    const kf_rb_attention& a = *ap;
     hipStream_t st = c->stream;
     int r = KF_OK;
     if (mfma_served(a, n_rows)) {
         int keys = max_pos + 1, span, n_range;
-        if (a.chunk > 0 && keys > a.chunk) keys = a.chunk;
+        const int seen = a.window > 0 ? a.window : a.chunk;
+        if (seen > 0 && keys > seen) keys = seen;
         decode_ranges(n_rows, a.n_kv * ((a.n_head / a.n_kv + 31) / 32), keys, span, n_range);
         if (n_range > 1 && !a.scratch) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: null scratch");
 #define RB_CALL(HD) decode_go<HD>(st, a, meta, n_rows, span, n_range)

@@ -19,6 +19,7 @@ __device__ __forceinline__ void rb_st4(uint16_t* p, f32x4 v) { *reinterpret_cast
 __device__ __forceinline__ void rb_st4(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
 
 __device__ __forceinline__ float rb_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float rb_softplus(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ float rb_activate(int act, float z) {
     if (act == KF_RB_RELU) return fmaxf(z, 0.0f);
     if (act == KF_RB_SILU) return z * rb_sigmoid(z);

@@ -73,6 +73,11 @@ __global__ void __launch_bounds__(C::NTH, C::WGS_PER_CU * C::NW / 4) rb_gemm_ker
                 if (m >= p.m) continue;
                 f32x4 d = acc[mt][nt];
                 if (p.epilogue == KF_RB_STORE) {
+                    if (m + 3 >= p.act_lo && m < p.act_hi) {
+#pragma unroll
+                        for (int j = 0; j < 4; j++)
+                            if (m + j >= p.act_lo && m + j < p.act_hi) d[j] = rb_activate(p.act, d[j]);
+                    }
                     rb_st4(reinterpret_cast<uint16_t*>(p.y) + (size_t)row * p.ldy + m, d);
                 } else {
                     if (p.epilogue == KF_RB_RESIDUAL) {

@@ -85,7 +85,8 @@ __device__ __forceinline__ void rb_stream_finish(const RbProduct& q, const f32x4
             for (int w = 0; w < NW; w++) u += red[w][MG - 1][col][row];
             reinterpret_cast<uint16_t*>(p.y)[(size_t)yr * p.ldy + (m0 >> 1) + row] = f2bf(scale * (rb_activate(p.act, d) * u));
         } else if (p.epilogue == KF_RB_STORE) {
-            reinterpret_cast<uint16_t*>(p.y)[(size_t)yr * p.ldy + m0 + row] = f2bf(d);
+            const int m = m0 + row;
+            reinterpret_cast<uint16_t*>(p.y)[(size_t)yr * p.ldy + m] = f2bf(m >= p.act_lo && m < p.act_hi ? rb_activate(p.act, d) : d);
         } else if (p.epilogue == KF_RB_STORE_F32) {
             reinterpret_cast<float*>(p.y)[(size_t)yr * p.ldy + m0 + row] = d;
         } else {
@@ -354,6 +355,10 @@ __global__ void __launch_bounds__(256) rb_f32_kernel(const RbProduct q) {
             const f32x4 r = *reinterpret_cast<const f32x4*>(p.res + (size_t)yr * p.ldr + m0 + tm);
 #pragma unroll
             for (int i = 0; i < 4; i++) d[i] = fmaf(p.alpha, r[i], d[i]);
+        } else if (p.epilogue == KF_RB_STORE && m0 + tm + 3 >= p.act_lo && m0 + tm < p.act_hi) {
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                if (m0 + tm + i >= p.act_lo && m0 + tm + i < p.act_hi) d[i] = rb_activate(p.act, d[i]);
         }
         *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(p.y) + (size_t)yr * p.ldy + m0 + tm) = d;
     }
@@ -379,6 +384,7 @@ extern "C" int kf_rb_linear(kf_ctx* c, const kf_rb_product* p) {
     if (!al16(p->w) || !al16(p->x) || !al16(p->y)) return abi_fail(KF_BLAS_UNALIGN, "kf_rb_linear: unaligned pointer");
     if (p->epilogue < KF_RB_STORE || p->epilogue > KF_RB_GATED || p->mode < KF_RB_ALL || p->mode > KF_RB_SUM) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: epilogue or mode");
     if (p->epilogue == KF_RB_RESIDUAL && (!p->res || !al16(p->res) || p->ldr < p->m || p->ldr % 4)) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: residual");
+    if (p->act_lo < p->act_hi && (p->epilogue != KF_RB_STORE || p->mode != KF_RB_ALL || p->act_lo < 0 || p->act_hi > p->m)) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: activated columns");
     if (p->ssq && (!kf_rb_linear_norms(p->type, p->n, p->m) || p->epilogue != KF_RB_RESIDUAL)) return abi_fail(KF_INVALID_ARGS, "kf_rb_linear: sums of squares");
     if (p->norm_z && (!kf_rb_linear_norms(p->type, p->n, p->k) || p->mode != KF_RB_ALL || p->epilogue == KF_RB_RESIDUAL || !p->norm_w || !p->norm_x || !p->norm_ssq || p->norm_dim < 1 || p->norm_dim > p->k || p->ldx != p->k || !al16(p->norm_z) ||
                       !al16(p->norm_w) || !al16(p->norm_x)))

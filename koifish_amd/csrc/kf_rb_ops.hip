@@ -122,6 +122,88 @@ static int norm_go(hipStream_t st, const RbNorm& a, int n) {
     return KF_OK;
 }
 
+// the sum over a workgroup of up to 256 threads; red: 4 floats of LDS that no earlier sum still uses
+__device__ __forceinline__ float group_sum(float v, float* red, int nt) {
+    v = wave_sum(v);
+    if (nt > 64) {
+        if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+        __syncthreads();
+        v = 0.f;
+        for (int w = 0; w < nt / 64; w++) v += red[w];
+    }
+    return v;
+}
+// kf_rb_norm_rows: VPT float4 columns per thread in registers, as above; the LAYER kind takes the mean off first (two sums, no difference of large numbers)
+template <class T, int VPT>
+__global__ void __launch_bounds__(256) rb_norm_rows_kernel(const kf_rb_norming a) {
+    __shared__ float red[2][4];
+    const int t = blockIdx.x, src = a.rows ? a.rows[t] : t, nt = blockDim.x;
+    f32x4 v[VPT];
+    float s = 0.f;
+    const float *hi = nullptr, *lo = nullptr;
+    if (a.pos_hi) {
+        const int p = a.meta[KF_RB_META * src], pos = p > 0 ? p : 0; /* (an inactive row: whatever) */
+        hi = a.pos_hi + (size_t)(pos >> 6) * a.ld, lo = a.pos_lo + (size_t)(pos & 63) * a.ld;
+    }
+#pragma unroll
+    for (int i = 0; i < VPT; i++) {
+        const int c = 4 * ((int)threadIdx.x + i * nt);
+        v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (c < a.ld) {
+            v[i] = rb_ld4(a.z + (size_t)src * a.ld + c);
+            if (hi) { /* two (sin, cos) pairs of each factor */
+                const f32x4 p = rb_ld4(hi + c), q = rb_ld4(lo + c);
+                v[i].x += p.x * q.y + p.y * q.x, v[i].y += p.y * q.y - p.x * q.x;
+                v[i].z += p.z * q.w + p.w * q.z, v[i].w += p.w * q.w - p.z * q.z;
+            }
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                if (c + j >= a.dim) v[i][j] = 0.f;
+                s += v[i][j];
+            }
+        }
+    }
+    float mean = 0.f, ss = 0.f;
+    if (a.kind == KF_RB_LAYER) mean = group_sum(s, red[0], nt) / (float)a.dim;
+#pragma unroll
+    for (int i = 0; i < VPT; i++) {
+        const int c = 4 * ((int)threadIdx.x + i * nt);
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            v[i][j] = c + j < a.dim ? v[i][j] - mean : 0.f;
+            ss = fmaf(v[i][j], v[i][j], ss);
+        }
+    }
+    const float rs = 1.0f / sqrtf(group_sum(ss, red[1], nt) / (float)a.dim + a.eps);
+#pragma unroll
+    for (int i = 0; i < VPT; i++) {
+        const int c = 4 * ((int)threadIdx.x + i * nt);
+        if (c < a.ld) {
+            const f32x4 g = rb_ld4(reinterpret_cast<const T*>(a.w) + c);
+            f32x4 o = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (a.add) o = rb_ld4(a.add + (size_t)src * a.ld + c);
+#pragma unroll
+            for (int j = 0; j < 4; j++) o[j] = c + j < a.dim ? o[j] + v[i][j] * rs * g[j] : 0.f;
+            if (a.x_out) rb_st4(a.x_out + (size_t)t * a.ld + c, o);
+            if (a.h_out) rb_st4(reinterpret_cast<T*>(a.h_out) + (size_t)t * a.ld + c, o);
+        }
+    }
+}
+template <class T>
+static int norm_rows_go(hipStream_t st, const kf_rb_norming& a) {
+    const int quads = (int)(a.ld / 4);
+    int nt = (quads + 63) / 64 * 64;
+    nt = nt > 256 ? 256 : nt;
+    const int vpt = (quads + nt - 1) / nt;
+    if (vpt <= 1) hipLaunchKernelGGL((rb_norm_rows_kernel<T, 1>), dim3(a.n), dim3(nt), 0, st, a);
+    else if (vpt <= 2) hipLaunchKernelGGL((rb_norm_rows_kernel<T, 2>), dim3(a.n), dim3(nt), 0, st, a);
+    else if (vpt <= 4) hipLaunchKernelGGL((rb_norm_rows_kernel<T, 4>), dim3(a.n), dim3(nt), 0, st, a);
+    else if (vpt <= 8) hipLaunchKernelGGL((rb_norm_rows_kernel<T, 8>), dim3(a.n), dim3(nt), 0, st, a);
+    else if (vpt <= 16) hipLaunchKernelGGL((rb_norm_rows_kernel<T, 16>), dim3(a.n), dim3(nt), 0, st, a);
+    else return 1;
+    return KF_OK;
+}
+
 // ---- router: one wave per row; expert e sits in lane e % 64, register e / 64
 constexpr int RB_MAX_EXPERTS = 1024;
 struct RbRoute {
@@ -364,6 +446,26 @@ int kf_rb_norm(kf_ctx* c, int type, const void* z, const float* res, float alpha
     const int rc = type == KF_BF16 ? norm_go<uint16_t>(c->stream, a, n) : norm_go<float>(c->stream, a, n);
     if (rc) return abi_fail(KF_UNSUPPORTED_DATATYPE, "kf_rb_norm: rows of %d columns (served: up to 16384)", dim);
     return launched("kf_rb_norm");
+}
+int kf_rb_norm_rows(kf_ctx* c, const kf_rb_norming* a) {
+    CHKCTX(c);
+    if (!a || !a->z || !a->w || (!a->x_out && !a->h_out) || a->dim < 1 || a->ld < a->dim || a->ld % KF_RB_PAD || a->n < 1 || a->kind < KF_RB_RMS || a->kind > KF_RB_LAYER)
+        return abi_fail(KF_INVALID_ARGS, "kf_rb_norm_rows: bad arguments");
+    if (!type_ok(a->type)) return abi_fail(KF_UNSUPPORTED_DATATYPE, "kf_rb_norm_rows: storage %d", a->type);
+    if (a->pos_hi && (!a->pos_lo || !a->meta || !al16(a->pos_hi) || !al16(a->pos_lo))) return abi_fail(KF_INVALID_ARGS, "kf_rb_norm_rows: positions");
+    if (!al16(a->z) || (a->add && !al16(a->add)) || !al16(a->w) || (a->x_out && !al16(a->x_out)) || (a->h_out && !al16(a->h_out))) return abi_fail(KF_BLAS_UNALIGN, "kf_rb_norm_rows: unaligned pointer");
+    const int rc = a->type == KF_BF16 ? norm_rows_go<uint16_t>(c->stream, *a) : norm_rows_go<float>(c->stream, *a);
+    if (rc) return abi_fail(KF_UNSUPPORTED_DATATYPE, "kf_rb_norm_rows: rows of %d columns (served: up to 16384)", a->dim);
+    return launched("kf_rb_norm_rows");
+}
+int kf_rb_sinusoid_tables_host(float* hi, float* lo, int n_pos, int width, int64_t ld, double base) {
+    if (!hi || !lo || n_pos < 1 || width < 1 || ld < width || (ld & 1) || !(base > 0)) return abi_fail(KF_INVALID_ARGS, "kf_rb_sinusoid_tables_host: bad arguments");
+    for (int64_t i = 0; i < ld / 2; i++) {
+        const double f = 2 * i < width ? pow(base, -2.0 * (double)i / width) : 0.0;
+        for (int j = 0; j < (n_pos + 63) / 64; j++) hi[j * ld + 2 * i] = (float)sin(64.0 * j * f), hi[j * ld + 2 * i + 1] = (float)cos(64.0 * j * f);
+        for (int j = 0; j < 64; j++) lo[j * ld + 2 * i] = (float)sin(j * f), lo[j * ld + 2 * i + 1] = (float)cos(j * f);
+    }
+    return KF_OK;
 }
 int kf_rb_list_tiles(int n, int top, int n_expert, int tile) {
     if (n < 1 || top < 1 || n_expert < 1 || tile < 1) return 0;

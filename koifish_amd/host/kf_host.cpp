@@ -67,6 +67,7 @@ int KVCache::InitRings(kf_ctx* c, const std::vector<Ring>& layers, int n_slots, 
         r.begin = n;
         n += (r.slot_stride() * n_slots + 127) & ~(size_t)127;
     }
+    n = std::max<size_t>(n, 128); /* (a model without a ring) */
     for (hGTensor* t : {&key, &val}) {
         *t = std::make_shared<GTensor>();
         (*t)->type = type == KF_F32 ? typNUMBER::F32 : typNUMBER::BF16, (*t)->szData = n * elem;
@@ -78,6 +79,26 @@ int KVCache::InitRings(kf_ctx* c, const std::vector<Ring>& layers, int n_slots, 
 void* KVCache::Ring0(CTYPE type, int layer) const {
     return reinterpret_cast<uint8_t*>((type == KV_KEY ? key : val)->data) + rings[layer].begin * elem;
 }
+
+int KVCache::InitRecurrent(kf_ctx* c, const std::vector<Recurrent>& layers, int n_slots, int type) {
+    recurrent = layers, n_slot = n_slots, elem = type == KF_F32 ? 4 : 2;
+    size_t n = 0, m = 0;
+    for (Recurrent& r : recurrent) {
+        r.begin = n, r.hist_begin = m;
+        n += (r.slot_stride() * n_slots + 63) & ~(size_t)63, m += (r.hist_slot() * n_slots + 63) & ~(size_t)63;
+    }
+    auto make = [&](hGTensor& t, typNUMBER tp, size_t bytes) {
+        t = std::make_shared<GTensor>();
+        t->type = tp, t->szData = bytes;
+        KF_TRY(t->Alloc(c, bytes));
+        return kf_memset(c, t->data, 0, bytes);
+    };
+    if (n) KF_TRY(make(state, typNUMBER::F32, n * 4));
+    if (m) KF_TRY(make(hist, type == KF_F32 ? typNUMBER::F32 : typNUMBER::BF16, m * elem));
+    return KF_OK;
+}
+float* KVCache::State0(int layer) const { return reinterpret_cast<float*>(state->data) + recurrent[layer].begin; }
+void* KVCache::Hist0(int layer) const { return reinterpret_cast<uint8_t*>(hist->data) + recurrent[layer].hist_begin * elem; }
 
 // ------------------------------------------------------------------------------------------------ neurons
 hGTensor LayerNormal::cuFlow(hGTensor inp, int) {

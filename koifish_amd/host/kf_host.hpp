@@ -86,6 +86,19 @@ struct KVCache {
     int n_slot = 0, elem = 2;
     int InitRings(kf_ctx* c, const std::vector<Ring>& layers, int n_slots, int type);
     void* Ring0(CTYPE type, int layer) const;  // slot 0 of the layer
+    // Per-layer recurrent state: slot s holds two sides of 32-bit matrices [heads][dim][vdim rounded up to 4] (the state after position p on side p & 1, kf_rb.h) and the last
+    // `taps` inputs of a short convolution over `channels` (position p in row p % taps).  Nothing is cleared for a new sequence: position 0 starts from zero.
+    struct Recurrent {
+        int heads = 0, dim = 0, vdim = 0, taps = 0, channels = 0;
+        size_t slot_stride() const { return (size_t)2 * heads * dim * ((vdim + 3) / 4 * 4); }
+        size_t hist_slot() const { return ((size_t)taps * channels + 7) & ~(size_t)7; }
+        size_t begin = 0, hist_begin = 0;  // elements in front of the layer
+    };
+    std::vector<Recurrent> recurrent;
+    hGTensor state, hist;
+    int InitRecurrent(kf_ctx* c, const std::vector<Recurrent>& layers, int n_slots, int type);
+    float* State0(int layer) const;  // slot 0 of the layer
+    void* Hist0(int layer) const;
 };
 
 struct GeNeuron {

@@ -6,8 +6,7 @@
 
 namespace koifish {
 
-namespace {
-bool need(const JSON* o, const char* key, double lo, double& out, std::string& err, const std::string& where) {
+bool CardNumber(const JSON* o, const char* key, double lo, double& out, std::string& err, const std::string& where) {
     const JSON* v = o ? o->get(key) : nullptr;
     if (!v || v->kind != JSON::NUM || !(v->num >= lo)) {
         err = "config.json: " + where + "." + key + " is missing or out of range";
@@ -16,9 +15,9 @@ bool need(const JSON* o, const char* key, double lo, double& out, std::string& e
     out = v->num;
     return true;
 }
-bool need(const JSON* o, const char* key, int lo, int& out, std::string& err, const std::string& where) {
+bool CardNumber(const JSON* o, const char* key, int lo, int& out, std::string& err, const std::string& where) {
     double v;
-    if (!need(o, key, (double)lo, v, err, where)) return false;
+    if (!CardNumber(o, key, (double)lo, v, err, where)) return false;
     if (v != (double)(int)v) {
         err = "config.json: " + where + "." + key + " is not an integer";
         return false;
@@ -26,9 +25,9 @@ bool need(const JSON* o, const char* key, int lo, int& out, std::string& err, co
     out = (int)v;
     return true;
 }
-}  // namespace
 
-bool ReadTizusun(const JSON& cfg, SEQ_CARD& card, std::string& err) {
+bool ReadTizusun(const JSON& cfg, const seq_shapes&, SEQ_CARD& card, std::string& err) {
+    const auto need = [](auto&&... a) { return CardNumber(a...); };
     double eps, alpha;
     if (!need(&cfg, "width", 1, card.width, err, "") || !need(&cfg, "vocab", 1, card.vocab, err, "") || !need(cfg.get("norm"), "eps", 0.0, eps, err, "norm")) return false;
     if (!need(&cfg, "postln_alpha", -1e30, alpha, err, "")) return false;
@@ -95,7 +94,7 @@ bool ReadTizusun(const JSON& cfg, SEQ_CARD& card, std::string& err) {
 static const struct {
     const char* name;
     seq_card_reader read;
-} kSeqArchs[] = {{"Tizusun", ReadTizusun}};
+} kSeqArchs[] = {{"Tizusun", ReadTizusun}, {"Bolopel", ReadBolopel}};
 seq_card_reader FindSeqArch(const std::string& architecture) {
     for (const auto& e : kSeqArchs)
         if (architecture == e.name) return e.read;

@@ -24,7 +24,8 @@ ABI_SYMBOLS = [
     "kf_hot_rows", "kf_linear_masked", "kf_norm_gateup_swiglu_masked", "kf_linear_scratch_bytes", "kf_set_scratch", "kf_engine_workspace_bytes", "kf_engine_create", "kf_engine_step", "kf_engine_check", "kf_engine_destroy", "kf_engine_set_embedding", "kf_engine_set_head", "kf_engine_step_head", "kf_engine_steps_head", "kf_engine_reset", "kf_set_canonical", "kf_get_canonical", "kf_engine_served", "kf_engine_tune", "kf_engine_stats", "kf_qkv_rope_batch", "kf_qkv_rope_seqs", "kf_set_dequant_arena", "kf_dequant_arena_used", "kf_resident_scratch_bytes",
     "kf_xengine_workspace_bytes", "kf_xengine_create", "kf_xengine_served", "kf_xengine_set_embedding", "kf_xengine_set_head", "kf_xengine_steps", "kf_xengine_check", "kf_xengine_reset", "kf_xengine_destroy", "kf_xengine_workspace_bytes_tp", "kf_xengine_create_tp", "kf_xengine_set_head_tp",
     "kf_rb_linear", "kf_rb_linear_norms", "kf_rb_pack", "kf_rb_embed", "kf_rb_embed_state", "kf_rb_norm", "kf_rb_attention_prefill", "kf_rb_attention_decode", "kf_rb_attention_scratch", "kf_rb_rope_table_host",
-    "kf_rb_route", "kf_rb_list_tiles", "kf_rb_pick", "kf_rb_pick_scratch", "kf_rb_to_bf16",
+    "kf_rb_route", "kf_rb_list_tiles", "kf_rb_pick", "kf_rb_pick_scratch", "kf_rb_to_bf16", "kf_rb_norm_rows", "kf_rb_sinusoid_tables_host",
+    "kf_rb_delta_prefill", "kf_rb_delta_decode", "kf_rb_delta_scratch", "kf_rb_decay_prefill", "kf_rb_decay_decode", "kf_rb_decay_scratch",
     "kf_tp_recv_bytes", "kf_tp_push_bytes", "kf_tp_commit", "kf_tp_alloc", "kf_tp_ipc_export", "kf_tp_ipc_open", "kf_tp_ipc_close", "kf_linear_f32_push", "kf_tp_reduce_recv", "kf_tp_lm_head", "kf_tp_pick",
 ]
 
@@ -49,16 +50,39 @@ class RbProduct(C.Structure):
     """struct kf_rb_product"""
     _fields_ = [("w", C.c_void_p), ("x", C.c_void_p), ("y", C.c_void_p), ("res", C.c_void_p), ("ldx", C.c_int64), ("ldy", C.c_int64), ("ldr", C.c_int64), ("type", C.c_int32),
                 ("m", C.c_int32), ("k", C.c_int32), ("n", C.c_int32), ("epilogue", C.c_int32), ("act", C.c_int32), ("mode", C.c_int32), ("alpha", C.c_float), ("experts", C.POINTER(RbExperts)),
-                ("ssq", C.c_void_p), ("norm_z", C.c_void_p), ("norm_ssq", C.c_void_p), ("norm_w", C.c_void_p), ("norm_x", C.c_void_p), ("norm_eps", C.c_float), ("norm_dim", C.c_int32)]
+                ("ssq", C.c_void_p), ("norm_z", C.c_void_p), ("norm_ssq", C.c_void_p), ("norm_w", C.c_void_p), ("norm_x", C.c_void_p), ("norm_eps", C.c_float), ("norm_dim", C.c_int32),
+                ("act_lo", C.c_int32), ("act_hi", C.c_int32)]
 
 
 class RbAttention(C.Structure):
     """struct kf_rb_attention"""
     _fields_ = [("raw", C.c_void_p), ("out", C.c_void_p), ("k_new", C.c_void_p), ("k_cache", C.c_void_p), ("v_cache", C.c_void_p), ("q_norm", C.c_void_p), ("k_norm", C.c_void_p),
                 ("rope", C.c_void_p), ("scratch", C.c_void_p), ("ldraw", C.c_int64), ("ldout", C.c_int64), ("slot_stride", C.c_int64), ("head_stride", C.c_int64), ("type", C.c_int32), ("n_head", C.c_int32),
-                ("n_kv", C.c_int32), ("dim", C.c_int32), ("rot_dims", C.c_int32), ("chunk", C.c_int32), ("cache_rows", C.c_int32), ("gated", C.c_int32), ("scale", C.c_float), ("eps", C.c_float)]
+                ("n_kv", C.c_int32), ("dim", C.c_int32), ("rot_dims", C.c_int32), ("chunk", C.c_int32), ("cache_rows", C.c_int32), ("gated", C.c_int32), ("scale", C.c_float), ("eps", C.c_float),
+                ("v_col", C.c_int32), ("vdim", C.c_int32), ("gate_col", C.c_int32), ("unit", C.c_int32), ("window", C.c_int32), ("sink", C.c_int32), ("scaled", C.c_int32), ("out_scale", C.c_float)]
 
 
+class RbNorming(C.Structure):
+    """struct kf_rb_norming"""
+    _fields_ = [("z", C.c_void_p), ("add", C.c_void_p), ("rows", C.c_void_p), ("w", C.c_void_p), ("x_out", C.c_void_p), ("h_out", C.c_void_p), ("pos_hi", C.c_void_p), ("pos_lo", C.c_void_p),
+                ("meta", C.c_void_p), ("ld", C.c_int64), ("type", C.c_int32), ("kind", C.c_int32), ("dim", C.c_int32), ("n", C.c_int32), ("eps", C.c_float)]
+
+
+class RbDelta(C.Structure):
+    """struct kf_rb_delta"""
+    _fields_ = [("raw", C.c_void_p), ("out", C.c_void_p), ("conv", C.c_void_p), ("w_a2", C.c_void_p), ("w_g2", C.c_void_p), ("a_log", C.c_void_p), ("dt_bias", C.c_void_p), ("norm_w", C.c_void_p),
+                ("a_z", C.c_void_p), ("g_z", C.c_void_p), ("state", C.c_void_p), ("hist", C.c_void_p), ("scratch", C.c_void_p), ("ldraw", C.c_int64), ("ldout", C.c_int64), ("ld_az", C.c_int64),
+                ("ld_gz", C.c_int64), ("hist_slot", C.c_int64)] + [(n, C.c_int32) for n in "type n_head n_kv dim vdim taps col_b col_a col_g rank_a rank_g ld_a ld_g".split()] + \
+               [("q_scale", C.c_float), ("unit_eps", C.c_float), ("eps", C.c_float)]
+
+
+class RbDecay(C.Structure):
+    """struct kf_rb_decay"""
+    _fields_ = [("raw", C.c_void_p), ("out", C.c_void_p), ("norm_w", C.c_void_p), ("decay", C.c_void_p), ("state", C.c_void_p), ("scratch", C.c_void_p), ("ldraw", C.c_int64), ("ldout", C.c_int64),
+                ("type", C.c_int32), ("n_head", C.c_int32), ("dim", C.c_int32), ("vdim", C.c_int32), ("col_q", C.c_int32), ("col_g", C.c_int32), ("out_scale", C.c_float), ("eps", C.c_float)]
+
+
+RB_RMS, RB_LAYER = range(2)
 RB_RELU, RB_SILU, RB_GELU_TANH = range(3)
 RB_STORE, RB_STORE_F32, RB_RESIDUAL, RB_GATED = range(4)
 RB_ALL, RB_UP, RB_DOWN, RB_SUM = range(4)
@@ -298,6 +322,14 @@ def load():
         hip.kf_rb_list_tiles.argtypes = [C.c_int] * 4
         hip.kf_rb_pick.argtypes = [C.c_void_p, C.c_void_p, C.c_int64, C.c_int, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p]
         hip.kf_rb_pick_scratch.argtypes, hip.kf_rb_pick_scratch.restype = [C.c_int], C.c_size_t
+        hip.kf_rb_norm_rows.argtypes = [C.c_void_p, C.POINTER(RbNorming)]
+        hip.kf_rb_sinusoid_tables_host.argtypes = [C.c_void_p, C.c_void_p, C.c_int, C.c_int, C.c_int64, C.c_double]
+        hip.kf_rb_delta_prefill.argtypes = [C.c_void_p, C.POINTER(RbDelta), C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int]
+        hip.kf_rb_delta_decode.argtypes = [C.c_void_p, C.POINTER(RbDelta), C.c_void_p, C.c_int]
+        hip.kf_rb_delta_scratch.argtypes, hip.kf_rb_delta_scratch.restype = [C.c_int] * 7, C.c_size_t
+        hip.kf_rb_decay_prefill.argtypes = [C.c_void_p, C.POINTER(RbDecay), C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int]
+        hip.kf_rb_decay_decode.argtypes = [C.c_void_p, C.POINTER(RbDecay), C.c_void_p, C.c_int]
+        hip.kf_rb_decay_scratch.argtypes, hip.kf_rb_decay_scratch.restype = [C.c_int] * 6, C.c_size_t
         hip.kf_rb_to_bf16.argtypes = [C.c_void_p, C.c_void_p, C.c_void_p, C.c_size_t]
         host.kfh_arch.restype, host.kfh_arch.argtypes = C.c_char_p, [C.c_void_p]
         host.kfh_seq_create.restype = C.c_void_p

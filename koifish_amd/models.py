@@ -7,11 +7,15 @@ import os
 
 from . import lib as L
 from .build import PARTS
-from .runtime import Qwen3, Tizusun
+from .runtime import Bolopel, Qwen3, Tizusun
 
 
 def _tizusun(path, dtype, max_seq, device):
     return Tizusun.from_dir(path, dtype=dtype, max_seq=max_seq, device=device)
+
+
+def _bolopel(path, dtype, max_seq, device):
+    return Bolopel.from_dir(path, dtype=dtype, max_seq=max_seq, device=device)
 
 
 def _qwen3(path, dtype, max_seq, device):
@@ -21,7 +25,7 @@ def _qwen3(path, dtype, max_seq, device):
 
 
 # name -> (loader, the part of the device code it needs: build.PARTS, None = all of it)
-ARCHITECTURES = {"Tizusun": (_tizusun, "rows"), "Qwen3ForCausalLM": (_qwen3, None), "qwen3": (_qwen3, None)}
+ARCHITECTURES = {"Tizusun": (_tizusun, "rows"), "Bolopel": (_bolopel, "rows"), "Qwen3ForCausalLM": (_qwen3, None), "qwen3": (_qwen3, None)}
 assert all(p is None or p in PARTS for _, p in ARCHITECTURES.values())
 
 

@@ -622,15 +622,17 @@ class Qwen3:
         return wb + norms + kv
 
 
-class Tizusun(Qwen3):
+class LayeredDecoder(Qwen3):
     """A decoder described layer by layer (koifish::SeqFish, host/kf_seq.hpp): bf16 or true 32-bit.  The
     generation surface is the one every model has (generate, prefill, run_steps, set_sampler, ...); XcdReplicas(model, n) serves n requests at once."""
 
-    def __init__(self, config, dtype="bfloat16", max_seq=0, device=0):
-        """config: the dict of a config.json; the tensors are set one by one (set_tensor) before the first step.  See from_dir for a checkpoint."""
+    def __init__(self, config, dtype="bfloat16", max_seq=0, device=0, shapes=None):
+        """config: the dict of a config.json; the tensors are set one by one (set_tensor) before the first step.  shapes: {tensor name: shape} for the sizes that a design's
+        config.json leaves to its tensors.  See from_dir for a checkpoint."""
         self._open(device)
         rc = C.c_int(0)
-        h = self.host.kfh_seq_create(json.dumps(config).encode(), device, C.c_void_p(self._stream.cuda_stream), _storage(dtype), int(max_seq), C.byref(rc))
+        doc = dict(config, tensor_shapes={k: list(v) for k, v in shapes.items()}) if shapes else config
+        h = self.host.kfh_seq_create(json.dumps(doc).encode(), device, C.c_void_p(self._stream.cuda_stream), _storage(dtype), int(max_seq), C.byref(rc))
         self._made(h, rc, "kfh_seq_create", config, dtype)
 
     @classmethod
@@ -688,6 +690,14 @@ class Tizusun(Qwen3):
         self._tap = np.zeros((self.cfg["n_layer"], n_rows, self.cfg["dim"]), dtype=np.float32)
         L.check(self.host.kfh_seq_tap(self.h, self._tap.ctypes.data_as(C.c_void_p), int(n_rows)), "kfh_seq_tap")
         return self._tap
+
+
+class Tizusun(LayeredDecoder):
+    """chunked gated attention, post-norm residual, dense or routed feed-forwards (host/kf_tizusun.cpp)"""
+
+
+class Bolopel(LayeredDecoder):
+    """gated delta rule layers and windowed attention beside a decayed sum, normed outputs added to the residual (host/kf_bolopel.cpp)"""
 
 
 def _storage(dtype):
@@ -797,7 +807,7 @@ class XcdReplicas:
                                            None if each is None else each.ctypes.data_as(C.c_void_p)), "kfh_xr_chat_each")
         return [out[i, :out_len[i]].tolist() for i in range(n)], dict(zip(("launches", "steps", "prefills", "dropped"), (int(v) for v in stats)))
 
-    # ---- models described layer by layer (Tizusun): requests by slot, any mix of prompts and single tokens in one batch
+    # ---- models described layer by layer (LayeredDecoder): requests by slot, any mix of prompts and single tokens in one batch
     def acquire(self):
         """a slot for a new request"""
         s = self.host.kfh_xr_acquire(self.h)
