@@ -401,7 +401,7 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
         if (kh == 1) return;
         const float M1 = ex[NREG * 256 + tid], Mm = fmaxf(T.M, M1); /* one of the halves has seen a key of the column */
         const float f0 = rb_exp2(T.M - Mm), f1 = rb_exp2(M1 - Mm);
-        T.l = T.l * f0 + ex[(NREG + 1) * 256 + tid] * f1;
+        T.l = T.l * f0 + ex[(NREG + 1) * 256 + tid] * f1, T.M = Mm;
 #pragma unroll
         for (int db = 0; db < Tile::NDB; db++)
 #pragma unroll
