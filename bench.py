@@ -81,6 +81,8 @@ def main():
                     "are synthetic N(0, 1) bf16 rows written once (a step's time depends on how many rows it reads, not on their values), the decode state is set to the window's first position")
     ap.add_argument("--tizusun", default="", help="instead of the run behind `value`: prefill and decode rates of the Tizusun design at these layer sizes (2k, 4k, 2k-moe, comma-separated; "
                     "random weights), each beside a Qwen3-shaped bf16 decoder of the same sizes; prints one JSON line")
+    ap.add_argument("--bolopel", default="", help="the same for the Bolopel design (2k, 4k)")
+    ap.add_argument("--bolopel-only", default="", choices=["", "bolopel", "qwen3"], help="with --bolopel: one side alone (profiler runs)")
     ap.add_argument("--tizusun-only", default="", choices=["", "tizusun", "qwen3"], help="with --tizusun: one side alone (profiler runs)")
     ap.add_argument("--lean", action="store_true", help="only the timed decode and step_roofline (what the side legs run in their child processes)")
     ap.add_argument("--leg", default="", choices=["", "config3", "config4cpu"], help="run ONE side leg and print its JSON (child processes of the main run)")
@@ -99,7 +101,10 @@ def main():
         return
 
     if args.tizusun:
-        print(json.dumps(tizusun_rates(args.tizusun.split(","), args.tizusun_only)))
+        print(json.dumps(layered_rates("tizusun", args.tizusun.split(","), args.tizusun_only)))
+        return
+    if args.bolopel:
+        print(json.dumps(layered_rates("bolopel", args.bolopel.split(","), args.bolopel_only)))
         return
 
     import numpy as np
@@ -820,10 +825,10 @@ def xcd_tp_leg(nt, cfg, ctx, forced, S, K, W, shards, plan, jump=False):
     return res
 
 
-def tizusun_rates(names, only=""):
-    """Prefill and decode throughput of Tizusun at a real model's layer sizes beside the framework's Qwen3 decoder with bf16 matrices of the same sizes.  Prompts of 2048 and 8192
-    tokens through the model's own prefill; decode behind a 1024-token prompt: one sequence through run_steps (both), 8 and 32 slots through XcdReplicas.run_steps (Tizusun:
-    Qwen3's slots decode 4-bit models only).  Times are medians over reps, the two models in turn where both run."""
+def layered_rates(design, names, only=""):
+    """Prefill and decode throughput of a design described layer by layer (tizusun, bolopel) at a real model's layer sizes beside the framework's Qwen3 decoder with bf16 matrices of the same sizes.  Prompts of 2048 and 8192
+    tokens through the model's own prefill; decode behind a 1024-token prompt: one sequence through run_steps (both), 8 and 32 slots through XcdReplicas.run_steps (the
+    design alone: Qwen3's slots decode 4-bit models only).  Times are medians over reps, the two models in turn where both run."""
     import statistics
     import time
 
@@ -831,7 +836,7 @@ def tizusun_rates(names, only=""):
     import torch
     from koifish_amd import lib as L
     from koifish_amd import synth
-    from koifish_amd.runtime import XcdReplicas
+    from koifish_amd.runtime import Bolopel, Tizusun, XcdReplicas
 
     def timed(m, fn, reps):
         fn()
@@ -844,15 +849,15 @@ def tizusun_rates(names, only=""):
             out.append(time.perf_counter() - t0)
         return statistics.median(out)
 
-    res = {"metric": "Tizusun prefill and decode, tokens/s", "dtype": "bf16", "data": "synthetic", "sizes": {}}
+    res = {"metric": "%s prefill and decode, tokens/s" % design.capitalize(), "dtype": "bf16", "data": "synthetic", "sizes": {}}
     for name in names:
-        peer, cfg = synth.tizusun_sizes(name)
+        peer, cfg, shapes = synth.tizusun_sizes(name) + (None,) if design == "tizusun" else synth.bolopel_sizes(name)
         r = {"layers": peer["n_layer"], "config": {k: peer[k] for k in ("dim", "n_head", "n_kv", "head_dim", "ffn", "vocab")}}
         ms = {}
         if only != "qwen3":
-            ms["tizusun"] = synth.tizusun_on_gpu(cfg, max_seq=peer["max_seq"])
-            r["tizusun_weight_bytes"] = ms["tizusun"].weights_bytes()
-        if only != "tizusun":
+            ms[design] = synth.layered_on_gpu(Tizusun if design == "tizusun" else Bolopel, cfg, max_seq=peer["max_seq"], shapes=shapes)
+            r[design + "_weight_bytes"] = ms[design].weights_bytes()
+        if only != design:
             ms["qwen3_bf16"] = synth.build_on_gpu(peer, layer_type=L.BF16, head_type=L.BF16)
         for n in (2048, 8192):
             ids = np.random.default_rng(n).integers(0, peer["vocab"], size=n).astype(np.int32)
@@ -867,9 +872,9 @@ def tizusun_rates(names, only=""):
                 m.set_state(int(ids[0]), 1024)
                 m.run_steps(1024, K)
             r["%s_decode_1" % k] = round(K / timed(m, steps, 5), 1)
-        if "tizusun" in ms:
+        if design in ms:
             for B in (8, 32):
-                x = XcdReplicas(ms["tizusun"], B)
+                x = XcdReplicas(ms[design], B)
                 for s in range(B):
                     x.prefill(s, ids)
 
@@ -877,7 +882,7 @@ def tizusun_rates(names, only=""):
                     for s in range(B):
                         x.set_state(s, int(ids[0]), 1024)
                     x.run_steps(K)
-                r["tizusun_decode_%d" % B] = round(B * K / timed(ms["tizusun"], slots, 3), 1)
+                r["%s_decode_%d" % (design, B)] = round(B * K / timed(ms[design], slots, 3), 1)
                 x.close()
         res["sizes"][name] = r
         for m in ms.values():

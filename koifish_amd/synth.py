@@ -9,7 +9,7 @@ import numpy as np
 import torch
 
 from . import lib as L
-from .runtime import Qwen3, Context, Tizusun
+from .runtime import Qwen3, Context
 
 CONFIGS = {
     # Qwen3-0.6B: cases/qwen3/qwen3_0.6B.json "transformer" block; tied embeddings
@@ -140,13 +140,32 @@ def tizusun_sizes(name):
     return c, dict(architecture="Tizusun", width=c["dim"], vocab=c["vocab"], norm=dict(eps=1e-6), postln_alpha=1.5, layers=[dict(type="attention", mixer=mix, mlp=mlp)] * c["n_layer"])
 
 
-def tizusun_on_gpu(cfg, dtype="bfloat16", max_seq=0, seed=1234, device=0, w_std=0.02):
-    """random tensors drawn on the GPU"""
-    m = Tizusun(cfg, dtype, max_seq, device)
+def bolopel_sizes(name):
+    """(the Qwen3-shaped peer's sizes, the Bolopel config, the shapes its config leaves to the tensors): the two kinds of layers in turn, window 4096"""
+    c = _ROWS[name]
+    H, D = c["n_head"], c["head_dim"]
+    delta = dict(type="channel_delta", mixer=dict(heads=H, kv_heads=H, dim=D, vdim=D, conv=4), mlp=dict(kind="dense", ff=c["ffn"]))
+    both = dict(type="parallel", mixer=dict(left=dict(heads=H, kv_heads=c["n_kv"], dim=D, vdim=D, mask=dict(size=4096), scale=D ** -0.5),
+                                            right=dict(heads=H, dim=D, vdim=D, decay=[1.0 - 2.0 ** (-3 - 7 * h / H) for h in range(H)]), left_scale=1.0, right_scale=1.0), mlp=dict(kind="dense", ff=c["ffn"]))
+    layers = [delta, both] * (c["n_layer"] // 2)
+    shapes = {"l%d.mix.%s" % (i, n): (D, c["dim"]) for i in range(0, len(layers), 2) for n in ("a1", "g1")}
+    return c, dict(architecture="Bolopel", width=c["dim"], vocab=c["vocab"], norm=dict(eps=1e-6), layers=layers), shapes
+
+
+def layered_on_gpu(cls, cfg, dtype="bfloat16", max_seq=0, seed=1234, device=0, w_std=0.02, shapes=None):
+    """a model described layer by layer, random tensors drawn on the GPU"""
+    m = cls(cfg, dtype, max_seq, device, shapes)
     g = torch.Generator(device=m.device)
     g.manual_seed(seed)
     for name, (r, c) in m.tensors().items():
         w = torch.randn((r, c) if c > 1 else (r,), generator=g, device=m.device)
-        norm = c == 1 and not name.endswith(".b")
-        m.set_tensor(name, (1.0 + 0.01 * w if norm else w_std * w).to(torch.bfloat16))
+        if name.endswith("dt_bias"):
+            w = w - 4.0
+        elif name.endswith("conv"):
+            w = 0.5 * w
+        elif c == 1 and not name.endswith((".b", "A_log")):
+            w = 1.0 + 0.01 * w
+        else:
+            w = w_std * w
+        m.set_tensor(name, w.to(torch.bfloat16))
     return m

@@ -39,7 +39,7 @@ def sinusoid(positions, width):
 def short_conv(x, taps):
     """x [T, channels], taps [channels, n]: y_t = sum over j of taps[:, n - 1 - j] x_(t - j), zeros before the start"""
     y, n = np.zeros_like(x), taps.shape[1]
-    for j in range(n):
+    for j in range(min(n, len(x))):
         y[j:] += taps[:, n - 1 - j] * x[:len(x) - j]
     return y
 

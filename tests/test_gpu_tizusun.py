@@ -8,9 +8,11 @@ import numpy as np
 import pytest
 import torch
 
+import layered_helpers
 import plain_tizusun as P
 import tizusun_models as M
 from koifish_amd import lib as L
+from layered_helpers import bf16_view, rel
 
 pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
@@ -28,39 +30,8 @@ def make(cfg, dtype="float32", max_seq=400, seed=0, qk=1.5):
     return m, M.arrays(w)
 
 
-def rel(got, ref):
-    """row-wise rms difference of the centred logits against the rms of the reference"""
-    d = got - ref
-    d = d - d.mean(-1, keepdims=True)
-    return np.sqrt((d ** 2).mean(-1)) / np.sqrt(((ref - ref.mean(-1, keepdims=True)) ** 2).mean())
-
-
-class Seqs:
-    """requests in slots, fed in any cut; every fed row's logits against the plain model over the whole history"""
-
-    def __init__(self, m, w, cfg, n=4):
-        from koifish_amd.runtime import XcdReplicas
-        self.m, self.w, self.cfg, self.x, self.tok, self.slot, self.ref = m, w, cfg, XcdReplicas(m, n), {}, {}, {}
-
-    def open(self, name, tokens):
-        self.slot[name], self.tok[name] = self.x.acquire(), [[], list(tokens)]
-        self.ref[name] = P.forward(self.cfg, self.w, tokens)
-
-    def feed(self, cut):
-        spans, want, rows = [], [], []
-        for k, (name, n) in enumerate(cut.items()):
-            done, left = self.tok[name]
-            spans.append((self.slot[name], len(done), left[:n]))
-            want += [(k, t) for t in range(n)]
-            rows += [self.ref[name][len(done) + t] for t in range(n)]
-            self.tok[name] = [done + left[:n], left[n:]]
-        got = self.x.run(spans, want)
-        e = rel(got, np.array(rows))
-        i = int(e.argmax())
-        assert e[i] < TOL[self.m.dtype], (cut, want[i], e[i])
-
-    def close(self, name):
-        self.x.release(self.slot.pop(name))
+def Seqs(m, w, cfg, n=4):
+    return layered_helpers.Seqs(P, m, w, cfg, TOL, n)
 
 
 @pytest.fixture(scope="module", params=[(c, d) for c in M.CONFIGS for d in ("float32", "bfloat16")], ids=lambda p: p[0] + "-" + p[1])
@@ -188,16 +159,12 @@ def test_greedy_generation_matches_the_plain_model():
     assert m.generate(p, 24, use_graph=True) == want                 # batched prompt
     assert m.num_graphs() >= 1
     nxt, lg = m.prefill(p)
-    assert nxt == want[0] and int(L_bf16(lg).argmax()) >= 0
+    assert nxt == want[0] and int(bf16_view(lg).argmax()) >= 0
     r, lg = m.forward(int(want[0]), 30)
     assert r == want[1]
     ref = P.forward(cfg, w, list(p) + want[:1])[-1]
-    assert rel(L_bf16(lg)[None], ref[None])[0] < 0.01                # kfh_logits is the bf16 view
+    assert rel(bf16_view(lg)[None], ref[None])[0] < 0.01                # kfh_logits is the bf16 view
     m.close()
-
-
-def L_bf16(u):
-    return (u.astype(np.uint32) << 16).view(np.float32)
 
 
 def test_queue_of_prompts_through_the_slots():

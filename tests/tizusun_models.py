@@ -1,10 +1,7 @@
 """Small Tizusun models for the tests: configurations of their own, random bf16 weights, and a writer for checkpoint directories."""
-import json
-import os
-import struct
-
-import numpy as np
 import torch
+
+from layered_helpers import arrays, tokens, write_dir  # noqa: F401
 
 
 def mixer(heads, kv, dim, chunk, rot, base=1000.0, scale=None, scaling=(8.0, 1.0, 4.0, 32)):
@@ -79,26 +76,3 @@ def weights(cfg, seed=0, qk=1.5, settled=False):
             w = w * (2.0 if name.endswith((".k", ".o", ".down")) else 1.0) / s[1] ** 0.5
         out[name] = w.to(torch.bfloat16)
     return out
-
-
-def arrays(w):
-    return {k: v.float().numpy() for k, v in w.items()}
-
-
-def write_dir(path, cfg, w):
-    os.makedirs(path, exist_ok=True)
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    hdr, data, at = {}, [], 0
-    for name, t in w.items():
-        b = t.contiguous().view(torch.int16).numpy().tobytes()
-        hdr[name] = {"dtype": "BF16", "shape": list(t.shape), "data_offsets": [at, at + len(b)]}
-        data.append(b)
-        at += len(b)
-    h = json.dumps(hdr).encode()
-    with open(os.path.join(path, "model.safetensors"), "wb") as f:
-        f.write(struct.pack("<Q", len(h)) + h + b"".join(data))
-
-
-def tokens(cfg, n, seed=3):
-    return np.random.default_rng(seed).integers(0, cfg["vocab"], size=n).astype(np.int32)
