@@ -3,7 +3,7 @@
 // Decode: one workgroup per (head, row) holds the head's whole state matrix in registers -- a thread a few rows of four neighbouring columns -- and does the whole layer between the
 // two products: convolution, SiLU, unit norms, the low-rank decay and gate, the state's step, the norm and the gate of the output.  S^T k and S^T q come from ONE walk over the old
 // state: with k' = g k and q' = g q (row by row) S'^T q = S^T q' + (q . k) u, so the new state is only written, never read again.
-// Prompts: a preparation pass per row and head, the walk over the tokens, the norm and gate per row.
+// Prompts: in chunks (below), or where the sizes are not served that way a preparation pass per row and head and a walk over the tokens; then the norm and gate per row.
 #include <math.h>
 
 #include <algorithm>
@@ -272,11 +272,11 @@ __global__ void __launch_bounds__(NT) rb_decay_step_kernel(const kf_rb_decay a, 
 // ---- prompts
 // where a delta layer's prepared rows lie in its scratch (floats)
 struct RcPrep {
-    float *qk, *v, *g, *beta; /* [rows][2 n_kv dim] q then k, [rows][n_head vdim] (the outputs take its place), [rows][n_head dim], [rows][n_head] */
+    float *v, *qk, *g, *beta; /* [rows][n_head vdim] (the outputs take its place), [rows][2 n_kv dim] q then k, [rows][n_head dim], [rows][n_head] */
 };
 static RcPrep rc_prep_at(float* s, size_t rows, int n_head, int n_kv, int dim, int vdim) {
     RcPrep p;
-    p.qk = s, p.v = p.qk + rows * 2 * n_kv * dim, p.g = p.v + rows * n_head * vdim, p.beta = p.g + rows * n_head * dim;
+    p.v = s, p.qk = p.v + rows * n_head * vdim, p.g = p.qk + rows * 2 * n_kv * dim, p.beta = p.g + rows * n_head * dim;
     return p;
 }
 // one wave per (row, unit): a q head, a k head, a v head, a head's decays and step size
@@ -410,6 +410,604 @@ static int scan_go(hipStream_t st, const RcScan<T>& a, const int32_t* seqs, int 
     return KF_OK;
 }
 
+// ---- the delta rule in chunks of 64 tokens (prompts).  With G the logarithm of the decays' product from the chunk's start through a token, S0 the state in front of the chunk:
+//   A_ij = sum over d of k_i k_j e^(G_i - G_j),  (I + diag(beta) A below the diagonal) [W U] = diag(beta) [k e^G, v],  u = U - W S0
+//   o = (q e^G) S0 + (the same A with q_i, diagonal included) u,   S = e^(G_end) S0 + (k e^(G_end - G))^T u
+// Everything but u is known without the state: one workgroup per (chunk, head) prepares it (rb_delta_chunk_kernel), then a workgroup per (head, 16 value columns) walks the chunks
+// (rb_delta_walk_kernel).  All of it in 32 bits: v_mfma_f32_16x16x4_f32.  Its operands are read four k at a time (lane group g, register i holds k = 4 g + i): the register layout of a
+// result is then the layout of a right operand, and a solved block feeds the next product without leaving its registers.
+// No exponent is ever positive beyond what a float holds: logarithms are summed within blocks of 16 tokens and between blocks; a block row's left factors are taken from its own start
+// (e^(G_i - start) <= 1), its right factors to that start (<= 1 in earlier blocks).  In the diagonal block the right factor is e^(start - G_j) >= 1: where a block's decays multiply to less
+// than 2^-100 its entries are summed pair by pair instead.
+constexpr int RC_C = 64;
+__device__ __forceinline__ f32x4 rc_mfma(f32x4 a, f32x4 b, f32x4 c) { /* 16 x 16 x 16 */
+#pragma unroll
+    for (int i = 0; i < 4; i++) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
+    return c;
+}
+__device__ __forceinline__ float rc_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+constexpr float RC_LOG2E = 1.44269502162933349609375f;
+__device__ __forceinline__ float rc_fast_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + rc_exp2(-RC_LOG2E * z)); }
+// softplus in units of ln 2: log2(1 + e^z); the correction factor keeps the small ones exact to rounding
+__device__ __forceinline__ float rc_softplus2(float z) {
+    const float e = rc_exp2(-RC_LOG2E * fabsf(z)), u = 1.0f + e, d = u - 1.0f;
+    const float l = d == 0.f ? e * RC_LOG2E : __builtin_amdgcn_logf(u) * (e * __builtin_amdgcn_rcpf(d));
+    return fmaxf(z, 0.f) * RC_LOG2E + l;
+}
+// what a chunk leaves for the walk, floats: W [64][DP], q e^G [64][DP], (k e^(G_end - G))^T [DP][64], q-k products [64][64], U [64][Vp], e^(G_end) [DP]
+static __host__ __device__ inline size_t rc_chunk_floats(int DP, int Vp) { return (size_t)RC_C * (3 * DP + RC_C + Vp) + DP; }
+static __host__ __device__ inline int rc_chunk_index(int row0, int seq) { return row0 / RC_C + seq; } /* of a sequence's first chunk: the sequences' chunks never meet */
+
+template <class T>
+__device__ __forceinline__ const T* rc_input_row(const kf_rb_delta& a, const T* raw0, const T* hist, int channels, int row, int pos0) {
+    /* the projected channels of the sequence's row `row` (row < 0: before the batch), NULL: before the sequence */
+    if (row >= 0) return raw0 + (int64_t)row * a.ldraw;
+    const int p = pos0 + row;
+    return p < 0 ? nullptr : hist + (size_t)(p % a.taps) * channels;
+}
+// silu(conv) of channel c at N consecutive rows from `row`; rows at or past n_end give 0
+template <class T, int N>
+__device__ __forceinline__ void rc_conv_run(const kf_rb_delta& a, const T* raw0, const T* hist, int channels, int c, int row, int n_end, int pos0, float (&y)[N]) {
+    const T* w = reinterpret_cast<const T*>(a.conv) + (size_t)c * a.taps;
+#pragma unroll
+    for (int t = 0; t < N; t++) y[t] = 0.f;
+    if (a.taps == 4) {
+        float wt[4], x[N + 3];
+#pragma unroll
+        for (int j = 0; j < 4; j++) wt[j] = rb_ld(w + j);
+#pragma unroll
+        for (int t = 0; t < N + 3; t++) {
+            const T* p = row + t - 3 < n_end ? rc_input_row(a, raw0, hist, channels, row + t - 3, pos0) : nullptr;
+            x[t] = p ? rb_ld(p + c) : 0.f;
+        }
+#pragma unroll
+        for (int t = 0; t < N; t++)
+#pragma unroll
+            for (int j = 0; j < 4; j++) y[t] = fmaf(wt[j], x[t + j], y[t]);
+    } else {
+        for (int j = 0; j < a.taps; j++) {
+            const float wt = rb_ld(w + a.taps - 1 - j);
+#pragma unroll
+            for (int t = 0; t < N; t++) {
+                const T* p = row + t < n_end ? rc_input_row(a, raw0, hist, channels, row + t - j, pos0) : nullptr;
+                if (p) y[t] = fmaf(wt, rb_ld(p + c), y[t]);
+            }
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < N; t++) y[t] = row + t < n_end ? y[t] * rc_fast_sigmoid(y[t]) : 0.f;
+}
+
+template <class T, int DP>
+__global__ void __launch_bounds__(512) rb_delta_chunk_kernel(const kf_rb_delta a, float* __restrict__ chunks, const int32_t* __restrict__ seqs) {
+    constexpr int LD = DP + 4, NB = RC_C / 16, LA = RC_C + 4;
+    extern __shared__ float smem[];
+    const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3];
+    const int h = blockIdx.x, c0 = blockIdx.y * RC_C;
+    if (c0 >= n) return; /* workgroup-uniform */
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, g4 = lane >> 4;
+    float *sk = smem, *sq = sk + RC_C * LD, *sg = sq + RC_C * LD /* logs within the block */, *sB = sg + RC_C * LD /* [4][DP] of whole blocks */, *sA = sB + NB * DP /* [64][LA] minus beta A */,
+          *sT = sA + RC_C * LA /* [4][16][20] */, *s_kn = sT + NB * 16 * 20, *s_qn = s_kn + RC_C, *s_beta = s_qn + RC_C;
+    const int dim = a.dim, vdim = a.vdim, Vp = rc_up(vdim, 16), qd = a.n_kv * dim, channels = 2 * qd + a.n_head * vdim, kvh = h / (a.n_head / a.n_kv);
+    const T* raw0 = reinterpret_cast<const T*>(a.raw) + (size_t)row0 * a.ldraw;
+    const T* hist = reinterpret_cast<const T*>(a.hist) + (size_t)slot * a.hist_slot;
+    float* out = chunks + ((size_t)(rc_chunk_index(row0, blockIdx.z) + blockIdx.y) * a.n_head + h) * rc_chunk_floats(DP, Vp);
+    float *oW = out, *oQ = oW + RC_C * DP, *oK = oQ + RC_C * DP, *oP = oK + RC_C * DP, *oU = oP + RC_C * RC_C, *oG = oU + RC_C * Vp;
+    // q and k of the head, eight tokens of a channel at a time
+    for (int i = tid; i < 2 * DP * (RC_C / 8); i += 512) {
+        const int c = i % DP, which = (i / DP) & 1, t0 = i / (2 * DP) * 8;
+        float y[8];
+        if (c < dim) rc_conv_run<T, 8>(a, raw0, hist, channels, which * qd + kvh * dim + c, c0 + t0, n, pos0, y);
+        float* dst = (which ? sk : sq) + t0 * LD + c;
+#pragma unroll
+        for (int t = 0; t < 8; t++) dst[t * LD] = c < dim ? y[t] : 0.f;
+    }
+    // decays: a thread a block of a channel
+    const float rate = expf(rb_ld(reinterpret_cast<const T*>(a.a_log) + h));
+    for (int i = tid; i < DP * NB; i += 512) {
+        const int c = i % DP, b = i / DP;
+        const float bias = c < dim ? rb_ld(reinterpret_cast<const T*>(a.dt_bias) + h * dim + c) : 0.f;
+        float z[16], s = 0.f;
+#pragma unroll
+        for (int t = 0; t < 16; t++) {
+            const int row = c0 + 16 * b + t;
+            z[t] = c < dim && row < n ? a.a_z[(size_t)(row0 + row) * a.ld_az + h * dim + c] : 0.f;
+        }
+#pragma unroll
+        for (int t = 0; t < 16; t++) {
+            if (c < dim && c0 + 16 * b + t < n) s -= rate * rc_softplus2(z[t] + bias);
+            sg[(16 * b + t) * LD + c] = s;
+        }
+        sB[b * DP + c] = s;
+    }
+    if (tid < RC_C) s_beta[tid] = c0 + tid < n ? rb_sigmoid(rb_ld(raw0 + (size_t)(c0 + tid) * a.ldraw + a.col_b + h)) : 0.f;
+    __syncthreads();
+    { /* 1 / length: a wave eight tokens of q and of k, four lanes each */
+        const int t = 8 * wid + (lane & 7);
+        const float* x = ((lane & 8) ? sk : sq) + t * LD + g4 * (DP / 4);
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < DP / 4; i += 4) {
+            const f32x4 v = *reinterpret_cast<const f32x4*>(x + i);
+#pragma unroll
+            for (int j = 0; j < 4; j++) ss = fmaf(v[j], v[j], ss);
+        }
+        ss = xsum32(xsum16(ss));
+        if (g4 == 0) {
+            if (lane & 8) s_kn[t] = 1.0f / sqrtf(ss + a.unit_eps);
+            else s_qn[t] = a.q_scale / sqrtf(ss + a.unit_eps);
+        }
+    }
+    __syncthreads();
+    // the 16 x 16 blocks of A on and below the diagonal, with k and with q on the left
+    for (int b = wid; b < NB * (NB + 1) / 2; b += 8) {
+        const int I = b < 4 ? 3 : (b < 7 ? 2 : (b < 9 ? 1 : 0)), J = b < 4 ? b : (b < 7 ? b - 4 : (b < 9 ? b - 7 : 0));
+        const int ti = 16 * I + r16, tj = 16 * J + r16;
+        f32x4 kk = f32x4{0.f, 0.f, 0.f, 0.f}, qk = kk;
+        bool safe = true;
+        if (I == J) {
+            float least = 0.f;
+            for (int d = lane; d < DP; d += 64) least = fminf(least, sB[I * DP + d]);
+            safe = wave_max(-least) < 100.f;
+        }
+        if (safe) {
+#pragma unroll 2
+            for (int kb = 0; kb < DP / 16; kb++) {
+                const int d = 16 * kb + 4 * g4;
+                const f32x4 ki = *reinterpret_cast<const f32x4*>(sk + ti * LD + d), qi = *reinterpret_cast<const f32x4*>(sq + ti * LD + d), gi = *reinterpret_cast<const f32x4*>(sg + ti * LD + d);
+                const f32x4 kj = *reinterpret_cast<const f32x4*>(sk + tj * LD + d), gj = *reinterpret_cast<const f32x4*>(sg + tj * LD + d);
+                f32x4 to = f32x4{0.f, 0.f, 0.f, 0.f}; /* from the end of token j's block to the start of block I ... */
+                if (J < I) {
+                    to = *reinterpret_cast<const f32x4*>(sB + J * DP + d);
+                    for (int m = J + 1; m < I; m++) to += *reinterpret_cast<const f32x4*>(sB + m * DP + d);
+                }
+                f32x4 A, Q, B;
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    const float f = rc_exp2(gi[e]);
+                    A[e] = ki[e] * f, Q[e] = qi[e] * f, B[e] = kj[e] * rc_exp2(to[e] - gj[e]);
+                }
+                kk = rc_mfma(A, B, kk), qk = rc_mfma(Q, B, qk);
+            }
+        } else { /* pair by pair, the layout of a result: rows 4 g4 + e, column r16 */
+            for (int d = 0; d < DP; d++) {
+                const float kj = sk[tj * LD + d], gj = sg[tj * LD + d];
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    const int t = 16 * I + 4 * g4 + e;
+                    const float x = kj * rc_exp2(fminf(sg[t * LD + d] - gj, 0.f));
+                    kk[e] = fmaf(sk[t * LD + d], x, kk[e]), qk[e] = fmaf(sq[t * LD + d], x, qk[e]);
+                }
+            }
+        }
+        const float knj = s_kn[tj];
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int t = 16 * I + 4 * g4 + e;
+            sA[t * LA + tj] = t > tj ? -s_beta[t] * s_kn[t] * knj * kk[e] : 0.f;
+            oP[t * RC_C + tj] = t >= tj ? s_qn[t] * knj * qk[e] : 0.f;
+        }
+    }
+    // q e^G and (k e^(G_end - G))^T for the walk
+    for (int i = tid; i < RC_C * DP / 4; i += 512) {
+        const int t = i / (DP / 4), d = 4 * (i % (DP / 4));
+        f32x4 q = *reinterpret_cast<const f32x4*>(sq + t * LD + d), g = *reinterpret_cast<const f32x4*>(sg + t * LD + d);
+        for (int m = 0; m < t / 16; m++) g += *reinterpret_cast<const f32x4*>(sB + m * DP + d);
+        const float f = s_qn[t];
+#pragma unroll
+        for (int e = 0; e < 4; e++) q[e] *= f * rc_exp2(g[e]);
+        *reinterpret_cast<f32x4*>(oQ + t * DP + d) = q;
+    }
+    for (int i = tid; i < RC_C * DP / 4; i += 512) { /* a thread four tokens of a channel */
+        const int t = 4 * (i % (RC_C / 4)), d = i / (RC_C / 4);
+        float end = 0.f;
+        for (int m = NB - 1; m >= t / 16; m--) end += sB[m * DP + d];
+        f32x4 o;
+#pragma unroll
+        for (int e = 0; e < 4; e++) o[e] = sk[(t + e) * LD + d] * s_kn[t + e] * rc_exp2(end - sg[(t + e) * LD + d]);
+        *reinterpret_cast<f32x4*>(oK + d * RC_C + t) = o;
+    }
+    for (int d = tid; d < DP; d += 512) oG[d] = rc_exp2(sB[d] + sB[DP + d] + sB[2 * DP + d] + sB[3 * DP + d]);
+    __syncthreads();
+    if (wid == 0) { /* the diagonal blocks' inverses: a lane column r16 of block g4 */
+        const float* Lb = sA + (16 * g4) * LA + 16 * g4;
+        float x[16];
+#pragma unroll
+        for (int i = 0; i < 16; i++) {
+            float s = i == r16 ? 1.f : 0.f;
+#pragma unroll
+            for (int j = 0; j < i; j++) s = fmaf(Lb[i * LA + j], x[j], s); /* (the stored sign is minus) */
+            x[i] = s;
+            sT[(g4 * 16 + i) * 20 + r16] = s;
+        }
+    }
+    __syncthreads();
+    // W and U, 16 columns at a time
+    for (int ct = wid; ct < (DP + Vp) / 16; ct += 8) {
+        const bool is_w = ct < DP / 16;
+        const int col = is_w ? 16 * ct + r16 : 16 * ct - DP + r16;
+        f32x4 X[NB];
+        f32x4 ahead = f32x4{0.f, 0.f, 0.f, 0.f}; /* x: the blocks in front, of this lane's channel */
+#pragma unroll
+        for (int I = 0; I < NB; I++) {
+            const int t = 16 * I + 4 * g4;
+            f32x4 acc;
+            if (is_w) {
+#pragma unroll
+                for (int e = 0; e < 4; e++) acc[e] = s_beta[t + e] * s_kn[t + e] * sk[(t + e) * LD + col] * rc_exp2(sg[(t + e) * LD + col] + ahead.x);
+                ahead.x += sB[I * DP + col];
+            } else {
+                float y[4] = {0.f, 0.f, 0.f, 0.f};
+                if (col < vdim) rc_conv_run<T, 4>(a, raw0, hist, channels, 2 * qd + h * vdim + col, c0 + t, n, pos0, y);
+#pragma unroll
+                for (int e = 0; e < 4; e++) acc[e] = s_beta[t + e] * y[e];
+            }
+#pragma unroll
+            for (int J = 0; J < I; J++) acc = rc_mfma(*reinterpret_cast<const f32x4*>(sA + (16 * I + r16) * LA + 16 * J + 4 * g4), X[J], acc);
+            X[I] = rc_mfma(*reinterpret_cast<const f32x4*>(sT + (16 * I + r16) * 20 + 4 * g4), acc, f32x4{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                if (is_w) oW[(t + e) * DP + col] = X[I][e];
+                else oU[(t + e) * Vp + col] = X[I][e];
+            }
+        }
+    }
+}
+
+// the walk: four waves, wave w the chunk's tokens 16 w .. and the state's rows w DP / 4 ..; S^T and u^T pass between them through LDS
+template <int DP>
+__global__ void __launch_bounds__(256) rb_delta_walk_kernel(const kf_rb_delta a, const float* __restrict__ chunks, float* __restrict__ o, const int32_t* __restrict__ seqs) {
+    constexpr int LS = DP + 4, LU = RC_C + 4, NT = DP / 64 /* 16-row tiles of the state per wave */;
+    __shared__ __attribute__((aligned(16))) float sS[16 * LS], sU[16 * LU];
+    const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3];
+    const int h = blockIdx.x, v0 = 16 * blockIdx.y, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, g4 = lane >> 4;
+    const int dim = a.dim, vdim = a.vdim, Vp = rc_up(vdim, 16), vs = rc_up(vdim, 4), col = v0 + r16;
+    const size_t head = (size_t)dim * vs, side = (size_t)a.n_head * head, step = (size_t)a.n_head * rc_chunk_floats(DP, Vp);
+    const float* S0 = a.state + ((size_t)slot * 2 + ((pos0 + 1) & 1)) * side + h * head;
+    float* S1 = a.state + ((size_t)slot * 2 + ((pos0 + n - 1) & 1)) * side + h * head;
+    f32x4 S[NT]; /* rows d0 + 16 t + 4 g4 + e, column r16 */
+    const int d0 = wid * 16 * NT;
+#pragma unroll
+    for (int t = 0; t < NT; t++) {
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int d = d0 + 16 * t + 4 * g4 + e;
+            S[t][e] = pos0 > 0 && d < dim && col < vdim ? S0[(size_t)d * vs + col] : 0.f;
+        }
+        *reinterpret_cast<f32x4*>(sS + r16 * LS + d0 + 16 * t + 4 * g4) = S[t];
+    }
+    const float* c = chunks + ((size_t)rc_chunk_index(row0, blockIdx.z) * a.n_head + h) * rc_chunk_floats(DP, Vp);
+    const int nc = (n + RC_C - 1) / RC_C, tok = 16 * wid + r16;
+    f32x4 w[DP / 16], q[DP / 16];
+    auto fetch = [&](const float* c) {
+#pragma unroll
+        for (int k = 0; k < DP / 16; k++) {
+            w[k] = *reinterpret_cast<const f32x4*>(c + tok * DP + 16 * k + 4 * g4);
+            q[k] = *reinterpret_cast<const f32x4*>(c + RC_C * DP + tok * DP + 16 * k + 4 * g4);
+        }
+    };
+    fetch(c);
+    for (int i = 0; i < nc; i++, c += step) {
+        const float *K = c + 2 * RC_C * DP, *Pq = K + RC_C * DP, *U = Pq + RC_C * RC_C, *G = U + RC_C * Vp;
+        f32x4 p[RC_C / 16], kt[NT][RC_C / 16], u, gt[NT];
+#pragma unroll
+        for (int e = 0; e < 4; e++) u[e] = U[(16 * wid + 4 * g4 + e) * Vp + col];
+#pragma unroll
+        for (int b = 0; b < RC_C / 16; b++) p[b] = *reinterpret_cast<const f32x4*>(Pq + tok * RC_C + 16 * b + 4 * g4); /* (above the diagonal: blocks nobody wrote, not used) */
+#pragma unroll
+        for (int t = 0; t < NT; t++) {
+            gt[t] = *reinterpret_cast<const f32x4*>(G + d0 + 16 * t + 4 * g4);
+#pragma unroll
+            for (int b = 0; b < RC_C / 16; b++) kt[t][b] = *reinterpret_cast<const f32x4*>(K + (d0 + 16 * t + r16) * RC_C + 16 * b + 4 * g4);
+        }
+        __syncthreads(); /* the state of the last chunk is in LDS */
+        f32x4 ws = f32x4{0.f, 0.f, 0.f, 0.f}, y = ws;
+#pragma unroll
+        for (int k = 0; k < DP / 16; k++) {
+            const f32x4 s = *reinterpret_cast<const f32x4*>(sS + r16 * LS + 16 * k + 4 * g4);
+            ws = rc_mfma(w[k], s, ws), y = rc_mfma(q[k], s, y);
+        }
+        u -= ws;
+        *reinterpret_cast<f32x4*>(sU + r16 * LU + 16 * wid + 4 * g4) = u;
+        if (i + 1 < nc) fetch(c + step);
+        __syncthreads();
+#pragma unroll
+        for (int t = 0; t < NT; t++) S[t] *= gt[t];
+#pragma unroll
+        for (int b = 0; b < RC_C / 16; b++) {
+            const f32x4 ub = *reinterpret_cast<const f32x4*>(sU + r16 * LU + 16 * b + 4 * g4);
+#pragma unroll
+            for (int t = 0; t < NT; t++) S[t] = rc_mfma(kt[t][b], ub, S[t]);
+            if (b <= wid) y = rc_mfma(p[b], ub, y); /* wave-uniform */
+        }
+#pragma unroll
+        for (int t = 0; t < NT; t++) *reinterpret_cast<f32x4*>(sS + r16 * LS + d0 + 16 * t + 4 * g4) = S[t];
+        if (col < vdim) {
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int row = RC_C * i + 16 * wid + 4 * g4 + e;
+                if (row < n) o[(size_t)(row0 + row) * a.n_head * vdim + (size_t)h * vdim + col] = y[e];
+            }
+        }
+    }
+    if (col < vs) {
+#pragma unroll
+        for (int t = 0; t < NT; t++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int d = d0 + 16 * t + 4 * g4 + e;
+                if (d < dim) S1[(size_t)d * vs + col] = S[t][e];
+            }
+    }
+}
+static int rc_delta_padded(int dim, int vdim) { return vdim > 256 ? 0 : (dim <= 64 ? 64 : (dim <= 128 ? 128 : 0)); } /* 0: not served in chunks */
+template <class T, int DP>
+static int delta_chunks_go(hipStream_t st, const kf_rb_delta& a, float* chunks, float* o, const int32_t* seqs, int n_seq, int max_n) {
+    constexpr size_t smem = (3 * RC_C * (DP + 4) + 4 * DP + RC_C * (RC_C + 4) + 4 * 16 * 20 + 3 * RC_C) * sizeof(float);
+    static_assert(smem <= 160 * 1024, "LDS");
+    static int done = 0;
+    if (!done) {
+        if (hipFuncSetAttribute((const void*)rb_delta_chunk_kernel<T, DP>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) != hipSuccess) return KF_HIP_CHECK;
+        done = 1;
+    }
+    hipLaunchKernelGGL((rb_delta_chunk_kernel<T, DP>), dim3(a.n_head, (max_n + RC_C - 1) / RC_C, n_seq), dim3(512), smem, st, a, chunks, seqs);
+    hipLaunchKernelGGL((rb_delta_walk_kernel<DP>), dim3(a.n_head, (a.vdim + 15) / 16, n_seq), dim3(256), 0, st, a, chunks, o, seqs);
+    return KF_OK;
+}
+
+// ---- the decayed sum in chunks (prompts, bf16 rows): S_c, the state in front of a chunk of 256 tokens, from one product per chunk and a walk over the chunks; then blocks of 128 queries
+//   o_i = decay^(i - c + 1) S_c^T q_i + sum over the chunk's j <= i of decay^(i - j) (q_i . k_j) v_j
+// on v_mfma_f32_32x32x16_bf16: q, k, v are exact, what has been multiplied by a decay enters as two (weights, S_c where it is read) or three (values on their way into the state) bf16 terms.
+typedef __bf16 rc_bf8 __attribute__((ext_vector_type(8)));
+typedef __bf16 rc_bf4 __attribute__((ext_vector_type(4)));
+typedef float rc_f16 __attribute__((ext_vector_type(16)));
+constexpr int RC_SPAN = 256, RC_QB = 128;
+__device__ __forceinline__ rc_f16 rc_mfma32(u32x4 a, u32x4 b, rc_f16 c) { return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(rc_bf8, a), __builtin_bit_cast(rc_bf8, b), c, 0, 0, 0); }
+// decay^n, n >= 0
+struct RcPower {
+    float l2;
+    bool neg;
+    __device__ __forceinline__ explicit RcPower(float decay) : l2(log2f(fabsf(decay))), neg(decay < 0.f) {}
+    __device__ __forceinline__ float operator()(int n) const {
+        const float p = n == 0 ? 1.f : __builtin_amdgcn_exp2f((float)n * l2); /* decay 0: e^-inf */
+        return neg && (n & 1) ? -p : p;
+    }
+};
+// keys (values) r0 .. of 32 rows staged [32][LDR]: a lane's operand of the 16 keys 16 s .. for column 32 b + lane % 32.  Element e is key 16 s + 4 (lane / 32) + e % 4 + 8 (e / 4)
+template <int LDR>
+__device__ __forceinline__ u32x4 rc_transposed(const uint16_t* rows, int s, int b, int lane) {
+    const uint16_t* p = rows + (16 * s + 4 * (lane >> 5) + ((lane & 15) >> 2)) * LDR + b * 32 + (lane & 16) + 4 * (lane & 3);
+    const rc_bf4 x = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) rc_bf4*)(p));
+    const rc_bf4 y = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) rc_bf4*)(p + 8 * LDR));
+    return __builtin_bit_cast(u32x4, rc_bf8{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]});
+}
+__device__ __forceinline__ int rc_tile_key(int h, int i) { return 4 * h + (i & 3) + 8 * (i >> 2); } /* row of register i of a 32 x 32 result */
+
+// the scratch behind the counters and outputs: per (span, head) the span's own sum [HD v][HD d] fp32, and the state in front of it as two bf16 planes of the same layout
+static __host__ __device__ inline int rc_span_index(int row0, int seq) { return row0 / RC_SPAN + seq; }
+
+template <int HD>
+struct RcStage { /* 32 rows of k and of v: global -> registers -> LDS, 256 threads */
+    static constexpr int KS = HD + 8, VS = HD + 32, CH = HD / 8, CPT = 32 * CH / 256, BYTES = 32 * (KS + VS) * 2;
+    u32x4 kr[CPT], vr[CPT];
+    __device__ __forceinline__ void load(const uint16_t* k, const uint16_t* v, int64_t ld, int dim, int vdim, int r0, int r_end, int tid) {
+#pragma unroll
+        for (int i = 0; i < CPT; i++) {
+            const int c = tid + 256 * i, r = r0 + c / CH, d = c % CH * 8;
+            kr[i] = vr[i] = u32x4{0, 0, 0, 0};
+            if (r < r_end) {
+                if (d < dim) kr[i] = *reinterpret_cast<const u32x4*>(k + (int64_t)r * ld + d);
+                if (d < vdim) vr[i] = *reinterpret_cast<const u32x4*>(v + (int64_t)r * ld + d);
+            }
+        }
+    }
+    __device__ __forceinline__ void store(uint16_t* ks, uint16_t* vs, int tid) const {
+#pragma unroll
+        for (int i = 0; i < CPT; i++) {
+            const int c = tid + 256 * i, r = c / CH, d = c % CH * 8;
+            *reinterpret_cast<u32x4*>(ks + r * KS + d) = kr[i];
+            *reinterpret_cast<u32x4*>(vs + r * VS + d) = vr[i];
+        }
+    }
+};
+
+template <int HD>
+__global__ void __launch_bounds__(256) rb_decay_part_kernel(const kf_rb_decay a, float* __restrict__ sums, const int32_t* __restrict__ seqs) {
+    using Stage = RcStage<HD>;
+    constexpr int DB = HD == 128 ? 4 : 1; /* 32 x 32 tiles of a wave: HD 128: v block w, all d blocks; HD 64: one tile */
+    static_assert(HD == 64 || HD == 128, "tiles dealt to four waves");
+    __shared__ __attribute__((aligned(16))) uint16_t lds[2][32 * (Stage::KS + Stage::VS)];
+    const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], t0 = blockIdx.y * RC_SPAN, h = blockIdx.x;
+    if (t0 >= n) return; /* workgroup-uniform */
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, hh = lane >> 5;
+    const int vb = HD == 128 ? wid : wid >> 1, db0 = HD == 128 ? 0 : wid & 1;
+    const uint16_t* k = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw + a.col_q + (size_t)a.n_head * a.dim + (size_t)h * a.dim;
+    const uint16_t* v = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw + a.col_q + (size_t)2 * a.n_head * a.dim + (size_t)h * a.vdim;
+    const int t1 = t0 + RC_SPAN < n ? t0 + RC_SPAN : n, nt = (t1 - t0 + 31) / 32;
+    const RcPower pw(a.decay[h]);
+    rc_f16 acc[DB];
+#pragma unroll
+    for (int d = 0; d < DB; d++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) acc[d][i] = 0.f;
+    Stage st;
+    st.load(k, v, a.ldraw, a.dim, a.vdim, t0, t1, tid);
+    st.store(lds[0], lds[0] + 32 * Stage::KS, tid);
+    __syncthreads();
+    for (int t = 0; t < nt; t++) {
+        const int k0 = t0 + 32 * t, m = t1 - k0 < 32 ? t1 - k0 : 32; /* the tile's keys */
+        if (t + 1 < nt) st.load(k, v, a.ldraw, a.dim, a.vdim, k0 + 32, t1, tid);
+        const uint16_t *ks = lds[t & 1], *vs = ks + 32 * Stage::KS;
+        const float f = pw(m);
+#pragma unroll
+        for (int d = 0; d < DB; d++)
+#pragma unroll
+            for (int i = 0; i < 16; i++) acc[d][i] *= f;
+#pragma unroll
+        for (int s = 0; s < 2; s++) {
+            const u32x4 raw = rc_transposed<Stage::VS>(vs, s, vb, lane);
+            u32x4 p0, p1, p2; /* decay^(m - 1 - key) v as three bf16 terms */
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                const int e = 2 * j, key = 16 * s + 4 * hh + (e & 3) + 8 * (e >> 2);
+                const float x = key < m ? bf_lo(raw[j]) * pw(m - 1 - key) : 0.f, y = key + 1 < m ? bf_hi(raw[j]) * pw(m - 2 - key) : 0.f;
+                p0[j] = pack_bf16x2(x, y);
+                const float x1 = x - bf_lo(p0[j]), y1 = y - bf_hi(p0[j]);
+                p1[j] = pack_bf16x2(x1, y1);
+                p2[j] = pack_bf16x2(x1 - bf_lo(p1[j]), y1 - bf_hi(p1[j]));
+            }
+#pragma unroll
+            for (int d = 0; d < DB; d++) {
+                const u32x4 B = rc_transposed<Stage::KS>(ks, s, db0 + d, lane);
+                acc[d] = rc_mfma32(p0, B, acc[d]), acc[d] = rc_mfma32(p1, B, acc[d]), acc[d] = rc_mfma32(p2, B, acc[d]);
+            }
+        }
+        if (t + 1 < nt) st.store(lds[(t + 1) & 1], lds[(t + 1) & 1] + 32 * Stage::KS, tid);
+        __syncthreads();
+    }
+    float* out = sums + ((size_t)(rc_span_index(row0, blockIdx.z) + blockIdx.y) * a.n_head + h) * HD * HD;
+#pragma unroll
+    for (int d = 0; d < DB; d++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) out[(32 * vb + rc_tile_key(hh, i)) * HD + 32 * (db0 + d) + r] = acc[d][i];
+}
+// a thread four neighbouring d of a v row: the state in front of every span, and the state after the batch
+template <int HD>
+__global__ void __launch_bounds__(256) rb_decay_states_kernel(const kf_rb_decay a, const float* __restrict__ sums, uint16_t* __restrict__ planes, const int32_t* __restrict__ seqs) {
+    const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3], h = blockIdx.x;
+    const int at = 4 * (blockIdx.y * 256 + threadIdx.x), v = at / HD, d = at % HD;
+    const int dim = a.dim, vs = rc_up(a.vdim, 4), ns = (n + RC_SPAN - 1) / RC_SPAN;
+    const size_t head = (size_t)dim * vs, side = (size_t)a.n_head * head;
+    const float* S0 = a.state + ((size_t)slot * 2 + ((pos0 + 1) & 1)) * side + h * head;
+    float* S1 = a.state + ((size_t)slot * 2 + ((pos0 + n - 1) & 1)) * side + h * head;
+    const RcPower pw(a.decay[h]);
+    f32x4 S = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; j++)
+        if (pos0 > 0 && v < a.vdim && d + j < dim) S[j] = S0[(size_t)(d + j) * vs + v];
+    const size_t step = (size_t)a.n_head * HD * HD, first = ((size_t)rc_span_index(row0, blockIdx.z) * a.n_head + h) * HD * HD + at;
+    const float* x = sums + first;
+    f32x4 next = *reinterpret_cast<const f32x4*>(x);
+    for (int c = 0; c < ns; c++) {
+        const f32x4 add = next;
+        if (c + 1 < ns) next = *reinterpret_cast<const f32x4*>(x + (c + 1) * step);
+        uint16_t* hi = planes + 2 * ((size_t)(rc_span_index(row0, blockIdx.z) + c) * a.n_head + h) * HD * HD + at;
+        const u32x2 p = u32x2{pack_bf16x2(S.x, S.y), pack_bf16x2(S.z, S.w)};
+        *reinterpret_cast<u32x2*>(hi) = p;
+        *reinterpret_cast<u32x2*>(hi + HD * HD) = u32x2{pack_bf16x2(S.x - bf_lo(p.x), S.y - bf_hi(p.x)), pack_bf16x2(S.z - bf_lo(p.y), S.w - bf_hi(p.y))};
+        const float f = pw(n - c * RC_SPAN < RC_SPAN ? n - c * RC_SPAN : RC_SPAN);
+#pragma unroll
+        for (int j = 0; j < 4; j++) S[j] = fmaf(f, S[j], add[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; j++)
+        if (v < vs && d + j < dim) S1[(size_t)(d + j) * vs + v] = S[j];
+}
+// 128 queries of a head: a wave 32 of them, one per lane pair
+template <int HD>
+__global__ void __launch_bounds__(256) rb_decay_out_kernel(const kf_rb_decay a, const uint16_t* __restrict__ planes, float* __restrict__ o, const int32_t* __restrict__ seqs) {
+    using Stage = RcStage<HD>;
+    constexpr int NS = HD / 16, NB = HD / 32;
+    __shared__ __attribute__((aligned(16))) uint16_t lds[2][32 * (Stage::KS + Stage::VS)];
+    const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], h = blockIdx.x, q0 = blockIdx.y * RC_QB;
+    if (q0 >= n) return; /* workgroup-uniform */
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, hh = lane >> 5;
+    const uint16_t* q = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw + a.col_q + (size_t)h * a.dim;
+    const uint16_t* k = q + (size_t)a.n_head * a.dim;
+    const uint16_t* v = reinterpret_cast<const uint16_t*>(a.raw) + (size_t)row0 * a.ldraw + a.col_q + (size_t)2 * a.n_head * a.dim + (size_t)h * a.vdim;
+    const int tok = q0 + 32 * wid + r, row = tok < n ? tok : n - 1, c0 = q0 / RC_SPAN * RC_SPAN; /* queries past the end repeat the last one and are not stored */
+    const int last = q0 + RC_QB < n ? q0 + RC_QB : n, nt = (last - c0 + 31) / 32;
+    Stage st;
+    st.load(k, v, a.ldraw, a.dim, a.vdim, c0, last, tid);
+    u32x4 qf[NS];
+#pragma unroll
+    for (int s = 0; s < NS; s++) {
+        qf[s] = u32x4{0, 0, 0, 0};
+        if (16 * s + 8 * hh < a.dim) qf[s] = *reinterpret_cast<const u32x4*>(q + (int64_t)row * a.ldraw + 16 * s + 8 * hh);
+    }
+    const RcPower pw(a.decay[h]);
+    rc_f16 acc[NB];
+    const uint16_t* S = planes + 2 * ((size_t)(rc_span_index(row0, blockIdx.z) + c0 / RC_SPAN) * a.n_head + h) * HD * HD;
+    st.store(lds[0], lds[0] + 32 * Stage::KS, tid);
+    const float f0 = pw(row - c0 + 1);
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+#pragma unroll
+        for (int i = 0; i < 16; i++) acc[b][i] = 0.f;
+#pragma unroll
+        for (int s = 0; s < NS; s++) {
+            const uint16_t* p = S + (32 * b + r) * HD + 16 * s + 8 * hh;
+            acc[b] = rc_mfma32(*reinterpret_cast<const u32x4*>(p), qf[s], acc[b]);
+            acc[b] = rc_mfma32(*reinterpret_cast<const u32x4*>(p + HD * HD), qf[s], acc[b]);
+        }
+#pragma unroll
+        for (int i = 0; i < 16; i++) acc[b][i] *= f0;
+    }
+    float tail[16]; /* decay^(31 - key) of a tile's keys */
+#pragma unroll
+    for (int i = 0; i < 16; i++) tail[i] = pw(31 - rc_tile_key(hh, i));
+    __syncthreads();
+    for (int t = 0; t < nt; t++) {
+        const int k0 = c0 + 32 * t;
+        if (t + 1 < nt) st.load(k, v, a.ldraw, a.dim, a.vdim, k0 + 32, last, tid);
+        const uint16_t *ks = lds[t & 1], *vs = ks + 32 * Stage::KS;
+        if (k0 <= q0 + 32 * wid + 31) { /* wave-uniform */
+            rc_f16 s;
+#pragma unroll
+            for (int i = 0; i < 16; i++) s[i] = 0.f;
+#pragma unroll
+            for (int j = 0; j < NS; j++) s = rc_mfma32(*reinterpret_cast<const u32x4*>(ks + r * Stage::KS + 16 * j + 8 * hh), qf[j], s);
+            if (k0 + 31 <= q0 + 32 * wid) {
+                const float f = pw((row > k0 + 31 ? row : k0 + 31) - k0 - 31);
+#pragma unroll
+                for (int i = 0; i < 16; i++) s[i] *= f * tail[i];
+            } else {
+#pragma unroll
+                for (int i = 0; i < 16; i++) {
+                    const int age = row - k0 - rc_tile_key(hh, i);
+                    s[i] = age >= 0 ? s[i] * pw(age) : 0.f;
+                }
+            }
+            uint32_t ph[8], pl[8];
+#pragma unroll
+            for (int i = 0; i < 8; i++) {
+                ph[i] = pack_bf16x2(s[2 * i], s[2 * i + 1]);
+                pl[i] = pack_bf16x2(s[2 * i] - bf_lo(ph[i]), s[2 * i + 1] - bf_hi(ph[i]));
+            }
+#pragma unroll
+            for (int s2 = 0; s2 < 2; s2++) {
+                const u32x4 B = u32x4{ph[4 * s2], ph[4 * s2 + 1], ph[4 * s2 + 2], ph[4 * s2 + 3]}, B2 = u32x4{pl[4 * s2], pl[4 * s2 + 1], pl[4 * s2 + 2], pl[4 * s2 + 3]};
+#pragma unroll
+                for (int b = 0; b < NB; b++) {
+                    const u32x4 A = rc_transposed<Stage::VS>(vs, s2, b, lane);
+                    acc[b] = rc_mfma32(A, B, acc[b]), acc[b] = rc_mfma32(A, B2, acc[b]);
+                }
+            }
+        }
+        if (t + 1 < nt) st.store(lds[(t + 1) & 1], lds[(t + 1) & 1] + 32 * Stage::KS, tid);
+        __syncthreads();
+    }
+    if (tok >= n) return;
+    float* out = o + (size_t)(row0 + tok) * a.n_head * a.vdim + (size_t)h * a.vdim;
+#pragma unroll
+    for (int b = 0; b < NB; b++)
+#pragma unroll
+        for (int g = 0; g < 4; g++) {
+            const int c = 32 * b + 8 * g + 4 * hh;
+            if (c < a.vdim) rb_st4(out + c, f32x4{acc[b][4 * g], acc[b][4 * g + 1], acc[b][4 * g + 2], acc[b][4 * g + 3]});
+        }
+}
+static int rc_decay_padded(int type, int dim, int vdim) { /* 0: not served in chunks */
+    const int m = std::max(dim, vdim);
+    return type != KF_BF16 || dim % 8 || vdim % 8 || m > 128 ? 0 : (m <= 64 ? 64 : 128);
+}
+template <int HD>
+static void decay_chunks_go(hipStream_t st, const kf_rb_decay& a, float* sums, uint16_t* planes, float* o, const int32_t* seqs, int n_seq, int max_n) {
+    hipLaunchKernelGGL(rb_decay_part_kernel<HD>, dim3(a.n_head, (max_n + RC_SPAN - 1) / RC_SPAN, n_seq), dim3(256), 0, st, a, sums, seqs);
+    hipLaunchKernelGGL(rb_decay_states_kernel<HD>, dim3(a.n_head, HD * HD / 1024, n_seq), dim3(256), 0, st, a, sums, planes, seqs);
+    hipLaunchKernelGGL(rb_decay_out_kernel<HD>, dim3(a.n_head, (max_n + RC_QB - 1) / RC_QB, n_seq), dim3(256), 0, st, a, planes, o, seqs);
+}
+
 // out = scale * o / sqrt(mean(o^2) + eps) * w * sigmoid(gate), the mean over groups of `size` columns; w: of one group (shared) or of all
 struct RcGate {
     const float* o;
@@ -448,27 +1046,101 @@ __global__ void __launch_bounds__(256) rb_gate_kernel(const RcGate a) {
     }
 }
 
+// the same, four columns of a thread in registers; a group is a power-of-two run of at most 64 threads, or the row (GROUPED: false)
+template <class T, int VPT, bool GROUPED>
+__global__ void __launch_bounds__(256) rb_gate_vec_kernel(const RcGate a) {
+    __shared__ float red[4];
+    const int r = blockIdx.x, tid = threadIdx.x, cols = a.groups * a.size;
+    const float* o = a.o + (size_t)r * a.ldo;
+    const T* gate = reinterpret_cast<const T*>(a.gate) + (size_t)r * a.ldg;
+    T* out = reinterpret_cast<T*>(a.out) + (size_t)r * a.ldout;
+    f32x4 v[VPT];
+    float ss[VPT], all = 0.f;
+#pragma unroll
+    for (int i = 0; i < VPT; i++) {
+        const int c = 4 * (tid + 256 * i);
+        v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (c < cols) v[i] = rb_ld4(o + c);
+        ss[i] = 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; j++) ss[i] = fmaf(v[i][j], v[i][j], ss[i]);
+        if (GROUPED)
+            for (int w = 1; w < a.size / 4; w <<= 1) ss[i] += __shfl_xor(ss[i], w, 64);
+        else all += ss[i];
+    }
+    if (!GROUPED) {
+        all = wave_sum(all);
+        if ((tid & 63) == 0) red[tid >> 6] = all;
+        __syncthreads();
+        all = red[0] + red[1] + red[2] + red[3];
+    }
+#pragma unroll
+    for (int i = 0; i < VPT; i++) {
+        const int c = 4 * (tid + 256 * i);
+        if (c >= cols) continue;
+        const float rs = a.scale / sqrtf((GROUPED ? ss[i] : all) / (float)a.size + a.eps);
+        const f32x4 w = rb_ld4(reinterpret_cast<const T*>(a.w) + (GROUPED ? c % a.size : c)), g = rb_ld4(gate + c);
+        f32x4 y;
+#pragma unroll
+        for (int j = 0; j < 4; j++) y[j] = v[i][j] * rs * w[j] * rb_sigmoid(g[j]);
+        rb_st4(out + c, y);
+    }
+}
+template <class T, int VPT>
+static void gate_vec(hipStream_t st, const RcGate& a, int n) {
+    if (a.groups > 1) hipLaunchKernelGGL((rb_gate_vec_kernel<T, VPT, true>), dim3(n), dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((rb_gate_vec_kernel<T, VPT, false>), dim3(n), dim3(256), 0, st, a);
+}
 template <class T>
-static int delta_prefill_go(hipStream_t st, const kf_rb_delta& a, const int32_t* meta, int n, const int32_t* seqs, int n_seq) {
-    const RcPrep p = rc_prep_at(a.scratch, n, a.n_head, a.n_kv, a.dim, a.vdim);
-    hipLaunchKernelGGL(rb_delta_prep_kernel<T>, dim3(n, (2 * a.n_kv + 2 * a.n_head + 3) / 4), dim3(256), 0, st, a, p, meta);
-    const int64_t ldq = 2 * (int64_t)a.n_kv * a.dim, ldv = (int64_t)a.n_head * a.vdim;
-    const RcScan<float> s{p.qk, p.qk + (size_t)a.n_kv * a.dim, p.v, p.g, p.beta, nullptr, p.v, a.state, ldq, ldv, ldv, a.n_head, a.n_head / a.n_kv, a.dim, a.vdim};
-    if (scan_go<float, true>(st, s, seqs, n_seq)) return 1;
+static void gate_go(hipStream_t st, const RcGate& a, int n) {
+    const int cols = a.groups * a.size, quads = a.size / 4, vpt = (cols + 1023) / 1024;
+    const bool aligned = a.size % 4 == 0 && a.ldo % 4 == 0 && a.ldg % 4 == 0 && a.ldout % 4 == 0 && (uintptr_t)a.gate % 16 == 0 && (uintptr_t)a.out % 16 == 0 && (uintptr_t)a.w % 16 == 0 && (uintptr_t)a.o % 16 == 0;
+    const bool grouped = a.groups > 1;
+    if (!aligned || vpt > 8 || (grouped && (quads > 64 || (quads & (quads - 1))))) {
+        hipLaunchKernelGGL(rb_gate_kernel<T>, dim3(n), dim3(256), 0, st, a);
+        return;
+    }
+    if (vpt <= 1) gate_vec<T, 1>(st, a, n);
+    else if (vpt <= 2) gate_vec<T, 2>(st, a, n);
+    else if (vpt <= 4) gate_vec<T, 4>(st, a, n);
+    else gate_vec<T, 8>(st, a, n);
+}
+constexpr int RC_MIN_CHUNKED = 16; /* rows of the longest sequence from which the chunked forms are taken */
+template <class T>
+static int delta_prefill_go(hipStream_t st, const kf_rb_delta& a, const int32_t* meta, int n, const int32_t* seqs, int n_seq, int max_n) {
+    const int64_t ldv = (int64_t)a.n_head * a.vdim;
+    float* o = a.scratch; /* [n][n_head vdim] */
+    const int DP = max_n >= RC_MIN_CHUNKED ? rc_delta_padded(a.dim, a.vdim) : 0;
+    if (DP) {
+        float* chunks = o + ((size_t)n * ldv + 3) / 4 * 4;
+        const int rc = DP == 64 ? delta_chunks_go<T, 64>(st, a, chunks, o, seqs, n_seq, max_n) : delta_chunks_go<T, 128>(st, a, chunks, o, seqs, n_seq, max_n);
+        if (rc) return rc;
+    } else {
+        const RcPrep p = rc_prep_at(a.scratch, n, a.n_head, a.n_kv, a.dim, a.vdim);
+        hipLaunchKernelGGL(rb_delta_prep_kernel<T>, dim3(n, (2 * a.n_kv + 2 * a.n_head + 3) / 4), dim3(256), 0, st, a, p, meta);
+        const int64_t ldq = 2 * (int64_t)a.n_kv * a.dim;
+        const RcScan<float> s{p.qk, p.qk + (size_t)a.n_kv * a.dim, p.v, p.g, p.beta, nullptr, p.v, a.state, ldq, ldv, ldv, a.n_head, a.n_head / a.n_kv, a.dim, a.vdim};
+        if (scan_go<float, true>(st, s, seqs, n_seq)) return 1;
+    }
     hipLaunchKernelGGL(rb_hist_kernel<T>, dim3(n), dim3(256), 0, st, a, meta);
-    const RcGate g{p.v, a.norm_w, a.g_z, a.out, ldv, a.ld_gz, a.ldout, a.n_head, a.vdim, 1.f, a.eps};
-    hipLaunchKernelGGL(rb_gate_kernel<T>, dim3(n), dim3(256), 0, st, g);
+    gate_go<T>(st, RcGate{o, a.norm_w, a.g_z, a.out, ldv, a.ld_gz, a.ldout, a.n_head, a.vdim, 1.f, a.eps}, n);
     return KF_OK;
 }
 template <class T>
-static int decay_prefill_go(hipStream_t st, const kf_rb_decay& a, int n, const int32_t* seqs, int n_seq) {
+static int decay_prefill_go(hipStream_t st, const kf_rb_decay& a, int n, const int32_t* seqs, int n_seq, int max_n) {
     const int64_t ldo = (int64_t)a.n_head * a.vdim;
     float* o = a.scratch + (size_t)RC_CNT_STRIDE * n;
-    const T* q = reinterpret_cast<const T*>(a.raw) + a.col_q;
-    const RcScan<T> s{q, q + (size_t)a.n_head * a.dim, q + (size_t)2 * a.n_head * a.dim, nullptr, nullptr, a.decay, o, a.state, a.ldraw, a.ldraw, ldo, a.n_head, 1, a.dim, a.vdim};
-    if (scan_go<T, false>(st, s, seqs, n_seq)) return 1;
-    const RcGate g{o, a.norm_w, reinterpret_cast<const T*>(a.raw) + a.col_g, a.out, ldo, a.ldraw, a.ldout, 1, a.n_head * a.vdim, a.out_scale, a.eps};
-    hipLaunchKernelGGL(rb_gate_kernel<T>, dim3(n), dim3(256), 0, st, g);
+    const int HD = max_n >= RC_MIN_CHUNKED && a.col_q % 8 == 0 && a.ldraw % 8 == 0 ? rc_decay_padded(a.type, a.dim, a.vdim) : 0;
+    if (HD) {
+        float* sums = o + ((size_t)n * ldo + 3) / 4 * 4;
+        uint16_t* planes = reinterpret_cast<uint16_t*>(sums + (size_t)(n / RC_SPAN + n_seq) * a.n_head * HD * HD);
+        HD == 64 ? decay_chunks_go<64>(st, a, sums, planes, o, seqs, n_seq, max_n) : decay_chunks_go<128>(st, a, sums, planes, o, seqs, n_seq, max_n);
+    } else {
+        const T* q = reinterpret_cast<const T*>(a.raw) + a.col_q;
+        const RcScan<T> s{q, q + (size_t)a.n_head * a.dim, q + (size_t)2 * a.n_head * a.dim, nullptr, nullptr, a.decay, o, a.state, a.ldraw, a.ldraw, ldo, a.n_head, 1, a.dim, a.vdim};
+        if (scan_go<T, false>(st, s, seqs, n_seq)) return 1;
+    }
+    gate_go<T>(st, RcGate{o, a.norm_w, reinterpret_cast<const T*>(a.raw) + a.col_g, a.out, ldo, a.ldraw, a.ldout, 1, a.n_head * a.vdim, a.out_scale, a.eps}, n);
     return KF_OK;
 }
 // threads of a decode workgroup: at most RC_RPT rows of four columns each where the state allows it
@@ -520,7 +1192,7 @@ static int check_decay(const kf_rb_decay* a, const int32_t* meta, int n, const c
     if (a->dim > RC_MAX_DIM || a->vdim > RC_MAX_DIM) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: head sizes %d / %d (served: up to %d)", who, a->dim, a->vdim, RC_MAX_DIM);
     const int64_t qk = 2 * (int64_t)a->n_head * a->dim, all = (int64_t)a->n_head * a->vdim;
     if (a->col_q < 0 || a->col_g < 0 || a->ldraw < a->col_q + qk + all || a->ldraw < a->col_g + all || a->ldout < all) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
-    if (!al16(a->state) || !al16(a->scratch)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
+    if (!al16(a->state) || !al16(a->scratch) || !al16(a->raw)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
     return KF_OK;
 }
 static int launched(int rc, const char* who) {
@@ -531,12 +1203,17 @@ static int launched(int rc, const char* who) {
 extern "C" {
 
 size_t kf_rb_delta_scratch(int type, int n_rows, int n_seq, int n_head, int n_kv, int dim, int vdim) {
-    if (n_rows < 1 || n_seq < 1) return 0;
-    return ((size_t)n_rows * (2 * (size_t)n_kv * dim + (size_t)n_head * (dim + vdim + 1)) + 16) * 4;
+    if (n_rows < 1 || n_seq < 1 || n_head < 1 || n_kv < 1 || dim < 1 || vdim < 1) return 0;
+    const size_t o = (size_t)n_rows * n_head * vdim + 4, rows = (size_t)n_rows * (2 * (size_t)n_kv * dim + (size_t)n_head * (dim + 1));
+    const int DP = rc_delta_padded(dim, vdim);
+    const size_t chunks = DP ? (size_t)(n_rows / RC_C + n_seq) * n_head * rc_chunk_floats(DP, rc_up(vdim, 16)) : 0;
+    return (o + std::max(rows, chunks) + 16) * 4;
 }
 size_t kf_rb_decay_scratch(int type, int n_rows, int n_seq, int n_head, int dim, int vdim) {
-    if (n_rows < 1) return 0;
-    return ((size_t)n_rows * (RC_CNT_STRIDE + (size_t)n_head * vdim) + 16) * 4;
+    if (n_rows < 1 || n_seq < 1 || n_head < 1 || dim < 1 || vdim < 1) return 0;
+    const int HD = rc_decay_padded(type, dim, vdim);
+    const size_t spans = HD ? (size_t)(n_rows / RC_SPAN + n_seq) * n_head * HD * HD * 2 : 0; /* a sum and two half-width planes */
+    return ((size_t)n_rows * (RC_CNT_STRIDE + (size_t)n_head * vdim) + 4 + spans + 16) * 4;
 }
 int kf_rb_delta_prefill(kf_ctx* c, const kf_rb_delta* a, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n) {
     CHKCTX(c);
@@ -544,7 +1221,7 @@ int kf_rb_delta_prefill(kf_ctx* c, const kf_rb_delta* a, const int32_t* meta, in
     if (rc) return rc;
     if (!seqs || n_seq < 1 || max_n < 1 || max_n > n_rows || !a->a_z || !a->g_z || !a->scratch || !al16(a->scratch) || a->ld_az < (int64_t)a->n_head * a->dim || a->ld_gz < (int64_t)a->n_head * a->vdim)
         return abi_fail(KF_INVALID_ARGS, "kf_rb_delta_prefill: bad arguments");
-    return launched(a->type == KF_BF16 ? delta_prefill_go<uint16_t>(c->stream, *a, meta, n_rows, seqs, n_seq) : delta_prefill_go<float>(c->stream, *a, meta, n_rows, seqs, n_seq), "kf_rb_delta_prefill");
+    return launched(a->type == KF_BF16 ? delta_prefill_go<uint16_t>(c->stream, *a, meta, n_rows, seqs, n_seq, max_n) : delta_prefill_go<float>(c->stream, *a, meta, n_rows, seqs, n_seq, max_n), "kf_rb_delta_prefill");
 }
 int kf_rb_delta_decode(kf_ctx* c, const kf_rb_delta* a, const int32_t* meta, int n_rows) {
     CHKCTX(c);
@@ -562,7 +1239,7 @@ int kf_rb_decay_prefill(kf_ctx* c, const kf_rb_decay* a, const int32_t* meta, in
     const int rc = check_decay(a, meta, n_rows, "kf_rb_decay_prefill");
     if (rc) return rc;
     if (!seqs || n_seq < 1 || max_n < 1 || max_n > n_rows) return abi_fail(KF_INVALID_ARGS, "kf_rb_decay_prefill: bad arguments");
-    return launched(a->type == KF_BF16 ? decay_prefill_go<uint16_t>(c->stream, *a, n_rows, seqs, n_seq) : decay_prefill_go<float>(c->stream, *a, n_rows, seqs, n_seq), "kf_rb_decay_prefill");
+    return launched(a->type == KF_BF16 ? decay_prefill_go<uint16_t>(c->stream, *a, n_rows, seqs, n_seq, max_n) : decay_prefill_go<float>(c->stream, *a, n_rows, seqs, n_seq, max_n), "kf_rb_decay_prefill");
 }
 int kf_rb_decay_decode(kf_ctx* c, const kf_rb_decay* a, const int32_t* meta, int n_rows) {
     CHKCTX(c);

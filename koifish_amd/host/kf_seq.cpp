@@ -488,10 +488,11 @@ int SeqFish::Ensure(RowWork& w, int rows, int n_seq, int head_rows, bool decode)
         ok = ok && t;
     };
     if (rows > w.rows || n_seq > w.n_seq || head_rows > w.head_rows) KF_TRY(kf_sync(ctx));
-    if (rows > w.rows) {
+    if (rows > w.rows || n_seq > w.n_seq) {
+        rows = std::max(rows, w.rows);
         size_t act = 0, y = 0, rl = 0, pairs = 0, list = 0, tiles = 0;
         RowNeed need;
-        for (const auto& a : mixers) a->Need(need, rows, rows, decode); /* (as many sequences as rows: no more) */
+        for (const auto& a : mixers) a->Need(need, rows, decode ? rows : std::max(n_seq, w.n_seq), decode);
         for (const auto& f : ffs) {
             if (f->c.kind == FF_CARD::NONE) continue;
             const bool moe = f->c.kind == FF_CARD::MOE;
