@@ -22,6 +22,12 @@ __device__ __forceinline__ float row16_sum(float v) { /* over the 16 lanes of a 
 __device__ __forceinline__ float rc_silu(float z) { return z * rb_sigmoid(z); }
 __device__ __forceinline__ void rc_st_sc1(float* p, float v) { __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
 __device__ __forceinline__ float rc_ld_sc1(const float* p) { return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
+// a barrier for what passes through LDS only: loads and stores of global memory stay in flight over it
+__device__ __forceinline__ void rc_lds_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
 constexpr int RC_CNT_STRIDE = 16; /* words between arrival counters */
 static __host__ __device__ inline int rc_up(int n, int m) { return (n + m - 1) / m * m; }
 
@@ -315,15 +321,13 @@ __global__ void __launch_bounds__(256) rb_delta_prep_kernel(const kf_rb_delta a,
         out.g[((size_t)r * a.n_head + u) * dim + c] = expf(-rate * rb_softplus(a.a_z[(size_t)r * a.ld_az + u * dim + c] + rb_ld(reinterpret_cast<const T*>(a.dt_bias) + u * dim + c)));
     if (lane == 0) out.beta[(size_t)r * a.n_head + u] = rb_sigmoid(rb_ld(raw + a.col_b + u));
 }
-// the batch's last `taps` rows of every sequence into its slot's ring
+// the batch's last `taps` rows of every sequence into its slot's ring: grid (column blocks, taps, sequences)
 template <class T>
-__global__ void __launch_bounds__(256) rb_hist_kernel(const kf_rb_delta a, const int32_t* __restrict__ meta) {
-    const int r = blockIdx.x, pos = meta[KF_RB_META * r], last = meta[KF_RB_META * r + 3];
-    if (pos < 0 || pos <= last - a.taps) return;
-    const int channels = 2 * a.n_kv * a.dim + a.n_head * a.vdim;
-    const T* raw = reinterpret_cast<const T*>(a.raw) + (size_t)r * a.ldraw;
-    T* hist = reinterpret_cast<T*>(a.hist) + (size_t)meta[KF_RB_META * r + 1] * a.hist_slot + (size_t)(pos % a.taps) * channels;
-    for (int i = threadIdx.x; i < channels; i += 256) hist[i] = raw[i];
+__global__ void __launch_bounds__(256) rb_hist_kernel(const kf_rb_delta a, const int32_t* __restrict__ seqs) {
+    const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3];
+    const int channels = 2 * a.n_kv * a.dim + a.n_head * a.vdim, t = n - 1 - (int)blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
+    if (t < 0 || c >= channels) return;
+    reinterpret_cast<T*>(a.hist)[(size_t)slot * a.hist_slot + (size_t)((pos0 + t) % a.taps) * channels + c] = reinterpret_cast<const T*>(a.raw)[(size_t)(row0 + t) * a.ldraw + c];
 }
 
 // token by token: a wave owns four columns of a head's state, its 16-lane rows share the key channels (rg, rg + 16, ...); the next token's rows are on their way while one is done
@@ -434,8 +438,12 @@ __device__ __forceinline__ float rc_softplus2(float z) {
     const float l = d == 0.f ? e * RC_LOG2E : __builtin_amdgcn_logf(u) * (e * __builtin_amdgcn_rcpf(d));
     return fmaxf(z, 0.f) * RC_LOG2E + l;
 }
-// what a chunk leaves for the walk, floats: W [64][DP], q e^G [64][DP], (k e^(G_end - G))^T [DP][64], q-k products [64][64], U [64][Vp], e^(G_end) [DP]
+// what a chunk leaves for the walk, floats: W [64][DP], q e^G [64][DP], (k e^(G_end - G))^T [DP][64], q-k products [64][64], U [64][Vp], e^(G_end) [DP].  The matrices lie in 16 x 16
+// tiles, row of tiles after row of tiles, 64 x 4 floats each in the order of a left operand (lane 16 g + r: row r, columns 4 g ..; U: of a result, rows 4 g .., column r): a wave reads a
+// tile as one contiguous kilobyte
 static __host__ __device__ inline size_t rc_chunk_floats(int DP, int Vp) { return (size_t)RC_C * (3 * DP + RC_C + Vp) + DP; }
+// where element (row, col) of such a matrix lies
+__device__ __forceinline__ int rc_tiled(int row, int col, int tiles) { return ((row / 16 * tiles + col / 16) * 64 + col % 16 / 4 * 16 + row % 16) * 4 + col % 4; }
 static __host__ __device__ inline int rc_chunk_index(int row0, int seq) { return row0 / RC_C + seq; } /* of a sequence's first chunk: the sequences' chunks never meet */
 
 template <class T>
@@ -445,83 +453,144 @@ __device__ __forceinline__ const T* rc_input_row(const kf_rb_delta& a, const T* 
     const int p = pos0 + row;
     return p < 0 ? nullptr : hist + (size_t)(p % a.taps) * channels;
 }
-// silu(conv) of channel c at N consecutive rows from `row`; rows at or past n_end give 0
-template <class T, int N>
-__device__ __forceinline__ void rc_conv_run(const kf_rb_delta& a, const T* raw0, const T* hist, int channels, int c, int row, int n_end, int pos0, float (&y)[N]) {
-    const T* w = reinterpret_cast<const T*>(a.conv) + (size_t)c * a.taps;
+// two neighbouring channels of a row (the second may not exist), as they lie in memory: one load where they share one
+__device__ __forceinline__ uint32_t rc_ld_pair(const uint16_t* p, bool paired, bool second) {
+    if (paired) return *reinterpret_cast<const uint32_t*>(p);
+    return p[0] | (second ? (uint32_t)p[1] << 16 : 0u);
+}
+__device__ __forceinline__ float2 rc_ld_pair(const float* p, bool paired, bool second) {
+    if (paired) return *reinterpret_cast<const float2*>(p);
+    return make_float2(p[0], second ? p[1] : 0.f);
+}
+__device__ __forceinline__ float2 rc_pair(uint32_t v) { return make_float2(bf_lo(v), bf_hi(v)); }
+__device__ __forceinline__ float2 rc_pair(float2 v) { return v; }
+template <class T>
+struct RcPairOf {
+    typedef uint32_t type;
+};
+template <>
+struct RcPairOf<float> {
+    typedef float2 type;
+};
+// the convolution and SiLU of channels c and c + 1 at 16 rows from `row` (a multiple of 16): the rows on their way (load), the results into dst [16][LD] (finish).  Rows at or past n_end give 0
+template <class T>
+struct RcConv {
+    typename RcPairOf<T>::type x[19]; /* four taps; other numbers of taps load where they multiply */
+    __device__ __forceinline__ void load(const kf_rb_delta& a, const T* raw0, const T* hist, int channels, int c, bool paired, bool second, int row, int n_end, int pos0) {
+        if (a.taps != 4) return;
+        const uint32_t ld = (uint32_t)a.ldraw;
 #pragma unroll
-    for (int t = 0; t < N; t++) y[t] = 0.f;
-    if (a.taps == 4) {
-        float wt[4], x[N + 3];
-#pragma unroll
-        for (int j = 0; j < 4; j++) wt[j] = rb_ld(w + j);
-#pragma unroll
-        for (int t = 0; t < N + 3; t++) {
-            const T* p = row + t - 3 < n_end ? rc_input_row(a, raw0, hist, channels, row + t - 3, pos0) : nullptr;
-            x[t] = p ? rb_ld(p + c) : 0.f;
+        for (int t = 3; t < 19; t++) {
+            const int r = row + t - 3;
+            x[t] = rc_ld_pair(raw0 + ((uint32_t)(r < n_end ? r : n_end - 1) * ld + c), paired, second);
         }
+        if (row >= 3) {
 #pragma unroll
-        for (int t = 0; t < N; t++)
+            for (int t = 0; t < 3; t++) x[t] = rc_ld_pair(raw0 + ((uint32_t)(row + t - 3 < n_end ? row + t - 3 : n_end - 1) * ld + c), paired, second);
+        } else { /* the batch's first rows */
 #pragma unroll
-            for (int j = 0; j < 4; j++) y[t] = fmaf(wt[j], x[t + j], y[t]);
-    } else {
-        for (int j = 0; j < a.taps; j++) {
-            const float wt = rb_ld(w + a.taps - 1 - j);
-#pragma unroll
-            for (int t = 0; t < N; t++) {
-                const T* p = row + t < n_end ? rc_input_row(a, raw0, hist, channels, row + t - j, pos0) : nullptr;
-                if (p) y[t] = fmaf(wt, rb_ld(p + c), y[t]);
+            for (int t = 0; t < 3; t++) {
+                const T* p = rc_input_row(a, raw0, hist, channels, row + t - 3, pos0);
+                x[t] = typename RcPairOf<T>::type{};
+                if (p) x[t] = rc_ld_pair(p + c, paired, second);
             }
         }
     }
+    template <int LD>
+    __device__ __forceinline__ void finish(const kf_rb_delta& a, const T* raw0, const T* hist, int channels, int c, bool paired, bool second, int row, int n_end, int pos0, float* dst) const {
+        const T* w = reinterpret_cast<const T*>(a.conv) + (size_t)c * a.taps;
+        float2 y[16];
 #pragma unroll
-    for (int t = 0; t < N; t++) y[t] = row + t < n_end ? y[t] * rc_fast_sigmoid(y[t]) : 0.f;
-}
+        for (int t = 0; t < 16; t++) y[t] = make_float2(0.f, 0.f);
+        if (a.taps == 4) {
+            float2 wt[4];
+#pragma unroll
+            for (int j = 0; j < 4; j++) wt[j] = make_float2(rb_ld(w + j), second ? rb_ld(w + 4 + j) : 0.f);
+#pragma unroll
+            for (int t = 0; t < 19; t++) {
+                const float2 v = rc_pair(x[t]);
+#pragma unroll
+                for (int j = 0; j < 4; j++)
+                    if (t - j >= 0 && t - j < 16) y[t - j].x = fmaf(wt[j].x, v.x, y[t - j].x), y[t - j].y = fmaf(wt[j].y, v.y, y[t - j].y);
+            }
+        } else {
+            for (int j = 0; j < a.taps; j++) {
+                const float w0 = rb_ld(w + a.taps - 1 - j), w1 = second ? rb_ld(w + 2 * a.taps - 1 - j) : 0.f;
+#pragma unroll
+                for (int t = 0; t < 16; t++) {
+                    const T* p = row + t < n_end ? rc_input_row(a, raw0, hist, channels, row + t - j, pos0) : nullptr;
+                    if (!p) continue;
+                    const float2 v = rc_pair(rc_ld_pair(p + c, paired, second));
+                    y[t].x = fmaf(w0, v.x, y[t].x), y[t].y = fmaf(w1, v.y, y[t].y);
+                }
+            }
+        }
+#pragma unroll
+        for (int t = 0; t < 16; t++) {
+            const bool on = row + t < n_end;
+            *reinterpret_cast<float2*>(dst + t * LD) = make_float2(on ? y[t].x * rc_fast_sigmoid(y[t].x) : 0.f, on ? y[t].y * rc_fast_sigmoid(y[t].y) : 0.f);
+        }
+    }
+};
 
+// sB[J] + ... + sB[I - 1] of channels d .. d + 3
+template <int DP>
+__device__ __forceinline__ f32x4 rc_between(const float* sB, int J, int I, int d) {
+    f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int m = J; m < I; m++) s += *reinterpret_cast<const f32x4*>(sB + m * DP + d);
+    return s;
+}
 template <class T, int DP>
 __global__ void __launch_bounds__(512) rb_delta_chunk_kernel(const kf_rb_delta a, float* __restrict__ chunks, const int32_t* __restrict__ seqs) {
-    constexpr int LD = DP + 4, NB = RC_C / 16, LA = RC_C + 4;
+    constexpr int LD = DP + 4, NB = RC_C / 16, LA = RC_C + 4, NE = NB * (NB + 1) / 2;
     extern __shared__ float smem[];
     const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3];
     const int h = blockIdx.x, c0 = blockIdx.y * RC_C;
     if (c0 >= n) return; /* workgroup-uniform */
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r16 = lane & 15, g4 = lane >> 4;
-    float *sk = smem, *sq = sk + RC_C * LD, *sg = sq + RC_C * LD /* logs within the block */, *sB = sg + RC_C * LD /* [4][DP] of whole blocks */, *sA = sB + NB * DP /* [64][LA] minus beta A */,
-          *sT = sA + RC_C * LA /* [4][16][20] */, *s_kn = sT + NB * 16 * 20, *s_qn = s_kn + RC_C, *s_beta = s_qn + RC_C;
+    // three arrays of rows: k, q, logs of the decays within the block; then k e^g, q e^g, k e^(block's end - g); the second becomes v
+    float *sk = smem, *sq = sk + RC_C * LD, *sg = sq + RC_C * LD, *sB = sg + RC_C * LD /* [4][DP] logs of whole blocks */, *sE = sB + NB * DP /* [10][DP] factors of a block pair */,
+          *sA = sE + NE * DP /* [64][LA] minus beta A */, *sT = sA + RC_C * LA /* [4][16][20] */, *s_kn = sT + NB * 16 * 20, *s_qn = s_kn + RC_C, *s_beta = s_qn + RC_C;
     const int dim = a.dim, vdim = a.vdim, Vp = rc_up(vdim, 16), qd = a.n_kv * dim, channels = 2 * qd + a.n_head * vdim, kvh = h / (a.n_head / a.n_kv);
     const T* raw0 = reinterpret_cast<const T*>(a.raw) + (size_t)row0 * a.ldraw;
     const T* hist = reinterpret_cast<const T*>(a.hist) + (size_t)slot * a.hist_slot;
     float* out = chunks + ((size_t)(rc_chunk_index(row0, blockIdx.z) + blockIdx.y) * a.n_head + h) * rc_chunk_floats(DP, Vp);
     float *oW = out, *oQ = oW + RC_C * DP, *oK = oQ + RC_C * DP, *oP = oK + RC_C * DP, *oU = oP + RC_C * RC_C, *oG = oU + RC_C * Vp;
-    // q and k of the head, eight tokens of a channel at a time
-    for (int i = tid; i < 2 * DP * (RC_C / 8); i += 512) {
-        const int c = i % DP, which = (i / DP) & 1, t0 = i / (2 * DP) * 8;
-        float y[8];
-        if (c < dim) rc_conv_run<T, 8>(a, raw0, hist, channels, which * qd + kvh * dim + c, c0 + t0, n, pos0, y);
-        float* dst = (which ? sk : sq) + t0 * LD + c;
+    const bool paired = dim % 2 == 0 && vdim % 2 == 0 && a.ldraw % 2 == 0 && a.hist_slot % 2 == 0;
+    auto zero16 = [&](float* dst) {
 #pragma unroll
-        for (int t = 0; t < 8; t++) dst[t * LD] = c < dim ? y[t] : 0.f;
+        for (int t = 0; t < 16; t++) *reinterpret_cast<float2*>(dst + t * LD) = make_float2(0.f, 0.f);
+    };
+    // everything this thread reads of the rows sets out together: a pair of q's or k's channels, the logs' inputs of a channel, a pair of v's
+    constexpr int QK = DP * NB; /* work items of q and k (half of them each), of the decays; v: half as many.  At most one of each kind per thread */
+    static_assert(QK <= 512, "an item per thread");
+    const int qc = 2 * (tid % (DP / 2)), qw = tid / (DP / 2) & 1, qb = tid / DP, dc = tid % DP, db = tid / DP, vb = tid / (DP / 2);
+    const bool q_on = tid < QK && qc < dim, d_on = tid < QK && dc < dim, v_on = tid < QK / 2 && qc < vdim;
+    RcConv<T> cq, cv;
+    if (q_on) cq.load(a, raw0, hist, channels, qw * qd + kvh * dim + qc, paired, qc + 1 < dim, c0 + 16 * qb, n, pos0);
+    float z[16];
+    if (d_on) {
+        const float* zp = a.a_z + (size_t)(row0 + c0) * a.ld_az + h * dim + dc;
+#pragma unroll
+        for (int t = 0; t < 16; t++) z[t] = zp[(uint32_t)(c0 + 16 * db + t < n ? 16 * db + t : n - 1 - c0) * (uint32_t)a.ld_az];
     }
-    // decays: a thread a block of a channel
-    const float rate = expf(rb_ld(reinterpret_cast<const T*>(a.a_log) + h));
-    for (int i = tid; i < DP * NB; i += 512) {
-        const int c = i % DP, b = i / DP;
-        const float bias = c < dim ? rb_ld(reinterpret_cast<const T*>(a.dt_bias) + h * dim + c) : 0.f;
-        float z[16], s = 0.f;
+    if (v_on) cv.load(a, raw0, hist, channels, 2 * qd + h * vdim + qc, paired, qc + 1 < vdim, c0 + 16 * vb, n, pos0);
+    if (tid < QK) {
+        float* dst = (qw ? sk : sq) + 16 * qb * LD + qc;
+        if (q_on) cq.template finish<LD>(a, raw0, hist, channels, qw * qd + kvh * dim + qc, paired, qc + 1 < dim, c0 + 16 * qb, n, pos0, dst);
+        else zero16(dst);
+        // decays: a thread a block of a channel
+        const float rate = expf(rb_ld(reinterpret_cast<const T*>(a.a_log) + h)), bias = d_on ? rb_ld(reinterpret_cast<const T*>(a.dt_bias) + h * dim + dc) : 0.f;
+        float l = 0.f;
 #pragma unroll
         for (int t = 0; t < 16; t++) {
-            const int row = c0 + 16 * b + t;
-            z[t] = c < dim && row < n ? a.a_z[(size_t)(row0 + row) * a.ld_az + h * dim + c] : 0.f;
+            if (d_on && c0 + 16 * db + t < n) l -= rate * rc_softplus2(z[t] + bias);
+            sg[(16 * db + t) * LD + dc] = l;
         }
-#pragma unroll
-        for (int t = 0; t < 16; t++) {
-            if (c < dim && c0 + 16 * b + t < n) s -= rate * rc_softplus2(z[t] + bias);
-            sg[(16 * b + t) * LD + c] = s;
-        }
-        sB[b * DP + c] = s;
+        sB[db * DP + dc] = l;
     }
     if (tid < RC_C) s_beta[tid] = c0 + tid < n ? rb_sigmoid(rb_ld(raw0 + (size_t)(c0 + tid) * a.ldraw + a.col_b + h)) : 0.f;
-    __syncthreads();
+    rc_lds_barrier();
     { /* 1 / length: a wave eight tokens of q and of k, four lanes each */
         const int t = 8 * wid + (lane & 7);
         const float* x = ((lane & 8) ? sk : sq) + t * LD + g4 * (DP / 4);
@@ -538,78 +607,100 @@ __global__ void __launch_bounds__(512) rb_delta_chunk_kernel(const kf_rb_delta a
             else s_qn[t] = a.q_scale / sqrtf(ss + a.unit_eps);
         }
     }
-    __syncthreads();
-    // the 16 x 16 blocks of A on and below the diagonal, with k and with q on the left
-    for (int b = wid; b < NB * (NB + 1) / 2; b += 8) {
-        const int I = b < 4 ? 3 : (b < 7 ? 2 : (b < 9 ? 1 : 0)), J = b < 4 ? b : (b < 7 ? b - 4 : (b < 9 ? b - 7 : 0));
-        const int ti = 16 * I + r16, tj = 16 * J + r16;
-        f32x4 kk = f32x4{0.f, 0.f, 0.f, 0.f}, qk = kk;
-        bool safe = true;
-        if (I == J) {
-            float least = 0.f;
-            for (int d = lane; d < DP; d += 64) least = fminf(least, sB[I * DP + d]);
-            safe = wave_max(-least) < 100.f;
-        }
-        if (safe) {
-#pragma unroll 2
-            for (int kb = 0; kb < DP / 16; kb++) {
-                const int d = 16 * kb + 4 * g4;
-                const f32x4 ki = *reinterpret_cast<const f32x4*>(sk + ti * LD + d), qi = *reinterpret_cast<const f32x4*>(sq + ti * LD + d), gi = *reinterpret_cast<const f32x4*>(sg + ti * LD + d);
-                const f32x4 kj = *reinterpret_cast<const f32x4*>(sk + tj * LD + d), gj = *reinterpret_cast<const f32x4*>(sg + tj * LD + d);
-                f32x4 to = f32x4{0.f, 0.f, 0.f, 0.f}; /* from the end of token j's block to the start of block I ... */
-                if (J < I) {
-                    to = *reinterpret_cast<const f32x4*>(sB + J * DP + d);
-                    for (int m = J + 1; m < I; m++) to += *reinterpret_cast<const f32x4*>(sB + m * DP + d);
-                }
-                f32x4 A, Q, B;
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    const float f = rc_exp2(gi[e]);
-                    A[e] = ki[e] * f, Q[e] = qi[e] * f, B[e] = kj[e] * rc_exp2(to[e] - gj[e]);
-                }
-                kk = rc_mfma(A, B, kk), qk = rc_mfma(Q, B, qk);
-            }
-        } else { /* pair by pair, the layout of a result: rows 4 g4 + e, column r16 */
-            for (int d = 0; d < DP; d++) {
-                const float kj = sk[tj * LD + d], gj = sg[tj * LD + d];
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    const int t = 16 * I + 4 * g4 + e;
-                    const float x = kj * rc_exp2(fminf(sg[t * LD + d] - gj, 0.f));
-                    kk[e] = fmaf(sk[t * LD + d], x, kk[e]), qk[e] = fmaf(sq[t * LD + d], x, qk[e]);
-                }
-            }
-        }
+    // the 16 x 16 blocks of A on and below the diagonal, with k and with q on the left: block (I, J) is number I (I + 1) / 2 + J
+    auto finish = [&](int I, int J, f32x4 kk, f32x4 qk) {
+        const int tj = 16 * J + r16;
         const float knj = s_kn[tj];
 #pragma unroll
         for (int e = 0; e < 4; e++) {
             const int t = 16 * I + 4 * g4 + e;
             sA[t * LA + tj] = t > tj ? -s_beta[t] * s_kn[t] * knj * kk[e] : 0.f;
-            oP[t * RC_C + tj] = t >= tj ? s_qn[t] * knj * qk[e] : 0.f;
+            oP[rc_tiled(t, tj, NB)] = t >= tj ? s_qn[t] * knj * qk[e] : 0.f;
         }
+    };
+    // a diagonal block whose decays multiply to next to nothing: pair by pair, while q, k and the logs are there.  Waves I and I + 4 see to block I: one tells, one sums
+    bool by_pairs;
+    {
+        float least = 0.f;
+        for (int d = lane; d < DP; d += 64) least = fminf(least, sB[(wid & 3) * DP + d]);
+        by_pairs = wave_max(-least) >= 100.f;
     }
-    // q e^G and (k e^(G_end - G))^T for the walk
+    rc_lds_barrier(); /* (the lengths) */
+    if (by_pairs && wid < NB) { /* the layout of a result: rows 4 g4 + e, column r16 */
+        f32x4 kk = f32x4{0.f, 0.f, 0.f, 0.f}, qk = kk;
+        const int tj = 16 * wid + r16;
+        for (int d = 0; d < DP; d++) {
+            const float kj = sk[tj * LD + d], gj = sg[tj * LD + d];
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int t = 16 * wid + 4 * g4 + e;
+                const float x = kj * rc_exp2(fminf(sg[t * LD + d] - gj, 0.f));
+                kk[e] = fmaf(sk[t * LD + d], x, kk[e]), qk[e] = fmaf(sq[t * LD + d], x, qk[e]);
+            }
+        }
+        finish(wid, wid, kk, qk);
+    }
+    rc_lds_barrier();
     for (int i = tid; i < RC_C * DP / 4; i += 512) {
-        const int t = i / (DP / 4), d = 4 * (i % (DP / 4));
-        f32x4 q = *reinterpret_cast<const f32x4*>(sq + t * LD + d), g = *reinterpret_cast<const f32x4*>(sg + t * LD + d);
-        for (int m = 0; m < t / 16; m++) g += *reinterpret_cast<const f32x4*>(sB + m * DP + d);
+        const int at = i / (DP / 4) * LD + 4 * (i % (DP / 4));
+        f32x4 k = *reinterpret_cast<const f32x4*>(sk + at), q = *reinterpret_cast<const f32x4*>(sq + at), g = *reinterpret_cast<const f32x4*>(sg + at);
+        const f32x4 B = *reinterpret_cast<const f32x4*>(sB + i / (DP / 4) / 16 * DP + 4 * (i % (DP / 4)));
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const float f = rc_exp2(g[e]);
+            g[e] = k[e] * rc_exp2(B[e] - g[e]), k[e] *= f, q[e] *= f;
+        }
+        *reinterpret_cast<f32x4*>(sk + at) = k, *reinterpret_cast<f32x4*>(sq + at) = q, *reinterpret_cast<f32x4*>(sg + at) = g;
+    }
+    for (int i = tid; i < NE * DP / 4; i += 512) { /* from the end of block J to the start of block I; J = I: from its end back to its start */
+        const int b = i / (DP / 4), d = 4 * (i % (DP / 4)), I = b < 1 ? 0 : (b < 3 ? 1 : (b < 6 ? 2 : 3)), J = b - I * (I + 1) / 2;
+        f32x4 x = J < I ? rc_between<DP>(sB, J + 1, I, d) : -*reinterpret_cast<const f32x4*>(sB + I * DP + d);
+#pragma unroll
+        for (int e = 0; e < 4; e++) x[e] = rc_exp2(fminf(x[e], 100.f));
+        *reinterpret_cast<f32x4*>(sE + b * DP + d) = x;
+    }
+    rc_lds_barrier();
+    for (int b = wid; b < NE; b += 8) {
+        const int I = b < 1 ? 0 : (b < 3 ? 1 : (b < 6 ? 2 : 3)), J = b - I * (I + 1) / 2;
+        if (I == J) { /* (block I is this wave's or its partner's: 0, 2, 5 and 9 go to waves 0, 2, 5 and 1) */
+            float least = 0.f;
+            for (int d = lane; d < DP; d += 64) least = fminf(least, sB[I * DP + d]);
+            if (wave_max(-least) >= 100.f) continue;
+        }
+        const float *pk = sk + (16 * I + r16) * LD + 4 * g4, *pq = sq + (16 * I + r16) * LD + 4 * g4, *pj = sg + (16 * J + r16) * LD + 4 * g4, *pe = sE + b * DP + 4 * g4;
+        f32x4 kk[2], qk[2]; /* two chains each */
+#pragma unroll
+        for (int j = 0; j < 2; j++) kk[j] = qk[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+        for (int kb = 0; kb < DP / 16; kb++) {
+            const f32x4 B = *reinterpret_cast<const f32x4*>(pj + 16 * kb) * *reinterpret_cast<const f32x4*>(pe + 16 * kb);
+            kk[kb & 1] = rc_mfma(*reinterpret_cast<const f32x4*>(pk + 16 * kb), B, kk[kb & 1]), qk[kb & 1] = rc_mfma(*reinterpret_cast<const f32x4*>(pq + 16 * kb), B, qk[kb & 1]);
+        }
+        finish(I, J, kk[0] + kk[1], qk[0] + qk[1]);
+    }
+    // q e^G and (k e^(G_end - G))^T for the walk, in tiles
+    for (int i = tid; i < RC_C * DP / 4; i += 512) {
+        const int tile = i / 64, t = tile / (DP / 16) * 16 + r16, d = tile % (DP / 16) * 16 + 4 * g4;
+        f32x4 q = *reinterpret_cast<const f32x4*>(sq + t * LD + d);
+        const f32x4 x = rc_between<DP>(sB, 0, t / 16, d);
         const float f = s_qn[t];
 #pragma unroll
-        for (int e = 0; e < 4; e++) q[e] *= f * rc_exp2(g[e]);
-        *reinterpret_cast<f32x4*>(oQ + t * DP + d) = q;
+        for (int e = 0; e < 4; e++) q[e] *= f * rc_exp2(x[e]);
+        *reinterpret_cast<f32x4*>(oQ + 4 * i) = q;
     }
-    for (int i = tid; i < RC_C * DP / 4; i += 512) { /* a thread four tokens of a channel */
-        const int t = 4 * (i % (RC_C / 4)), d = i / (RC_C / 4);
-        float end = 0.f;
-        for (int m = NB - 1; m >= t / 16; m--) end += sB[m * DP + d];
+    for (int i = tid; i < RC_C * DP / 4; i += 512) {
+        const int tile = i / 64, d = tile / NB * 16 + r16, t = tile % NB * 16 + 4 * g4;
+        float x = 0.f;
+        for (int m = t / 16 + 1; m < NB; m++) x += sB[m * DP + d];
+        x = rc_exp2(x);
         f32x4 o;
 #pragma unroll
-        for (int e = 0; e < 4; e++) o[e] = sk[(t + e) * LD + d] * s_kn[t + e] * rc_exp2(end - sg[(t + e) * LD + d]);
-        *reinterpret_cast<f32x4*>(oK + d * RC_C + t) = o;
+        for (int e = 0; e < 4; e++) o[e] = sg[(t + e) * LD + d] * s_kn[t + e] * x;
+        *reinterpret_cast<f32x4*>(oK + 4 * i) = o;
     }
     for (int d = tid; d < DP; d += 512) oG[d] = rc_exp2(sB[d] + sB[DP + d] + sB[2 * DP + d] + sB[3 * DP + d]);
-    __syncthreads();
-    if (wid == 0) { /* the diagonal blocks' inverses: a lane column r16 of block g4 */
+    rc_lds_barrier();
+    if (wid == 7) { /* the diagonal blocks' inverses: a lane column r16 of block g4 */
         const float* Lb = sA + (16 * g4) * LA + 16 * g4;
         float x[16];
 #pragma unroll
@@ -621,42 +712,49 @@ __global__ void __launch_bounds__(512) rb_delta_chunk_kernel(const kf_rb_delta a
             sT[(g4 * 16 + i) * 20 + r16] = s;
         }
     }
-    __syncthreads();
-    // W and U, 16 columns at a time
-    for (int ct = wid; ct < (DP + Vp) / 16; ct += 8) {
-        const bool is_w = ct < DP / 16;
-        const int col = is_w ? 16 * ct + r16 : 16 * ct - DP + r16;
-        f32x4 X[NB];
-        f32x4 ahead = f32x4{0.f, 0.f, 0.f, 0.f}; /* x: the blocks in front, of this lane's channel */
+    // W, and U as many columns at a time as one array of rows holds
+    for (int v0 = 0; v0 < Vp; v0 += DP) {
+        if (tid < QK / 2) {
+            const int c = v0 + qc;
+            float* dst = sq + 16 * vb * LD + qc;
+            if (v0 && c < vdim) cv.load(a, raw0, hist, channels, 2 * qd + h * vdim + c, paired, c + 1 < vdim, c0 + 16 * vb, n, pos0);
+            if (c < vdim) cv.template finish<LD>(a, raw0, hist, channels, 2 * qd + h * vdim + c, paired, c + 1 < vdim, c0 + 16 * vb, n, pos0, dst);
+            else zero16(dst);
+        }
+        rc_lds_barrier();
+        const int first = v0 ? DP / 16 : 0, cols = Vp - v0 < DP ? Vp - v0 : DP;
+        for (int ct = first + wid; ct < (DP + cols) / 16; ct += 8) { /* 16 columns: of W, of U */
+            const bool is_w = ct < DP / 16;
+            const int col = is_w ? 16 * ct + r16 : 16 * ct - DP + r16;
+            f32x4 X[NB];
+            float ahead = 0.f; /* the logs of the blocks in front, of this lane's channel */
 #pragma unroll
-        for (int I = 0; I < NB; I++) {
-            const int t = 16 * I + 4 * g4;
-            f32x4 acc;
-            if (is_w) {
+            for (int I = 0; I < NB; I++) {
+                const int t = 16 * I + 4 * g4;
+                f32x4 acc;
+                const float f = is_w ? rc_exp2(ahead) : 1.f;
+                const float* src = (is_w ? sk : sq) + t * LD + col;
 #pragma unroll
-                for (int e = 0; e < 4; e++) acc[e] = s_beta[t + e] * s_kn[t + e] * sk[(t + e) * LD + col] * rc_exp2(sg[(t + e) * LD + col] + ahead.x);
-                ahead.x += sB[I * DP + col];
-            } else {
-                float y[4] = {0.f, 0.f, 0.f, 0.f};
-                if (col < vdim) rc_conv_run<T, 4>(a, raw0, hist, channels, 2 * qd + h * vdim + col, c0 + t, n, pos0, y);
+                for (int e = 0; e < 4; e++) acc[e] = s_beta[t + e] * (is_w ? s_kn[t + e] * f : 1.f) * src[e * LD];
+                if (is_w) ahead += sB[I * DP + col];
 #pragma unroll
-                for (int e = 0; e < 4; e++) acc[e] = s_beta[t + e] * y[e];
-            }
+                for (int J = 0; J < I; J++) acc = rc_mfma(*reinterpret_cast<const f32x4*>(sA + (16 * I + r16) * LA + 16 * J + 4 * g4), X[J], acc);
+                X[I] = rc_mfma(*reinterpret_cast<const f32x4*>(sT + (16 * I + r16) * 20 + 4 * g4), acc, f32x4{0.f, 0.f, 0.f, 0.f});
+                if (is_w) {
 #pragma unroll
-            for (int J = 0; J < I; J++) acc = rc_mfma(*reinterpret_cast<const f32x4*>(sA + (16 * I + r16) * LA + 16 * J + 4 * g4), X[J], acc);
-            X[I] = rc_mfma(*reinterpret_cast<const f32x4*>(sT + (16 * I + r16) * 20 + 4 * g4), acc, f32x4{0.f, 0.f, 0.f, 0.f});
-#pragma unroll
-            for (int e = 0; e < 4; e++) {
-                if (is_w) oW[(t + e) * DP + col] = X[I][e];
-                else oU[(t + e) * Vp + col] = X[I][e];
+                    for (int e = 0; e < 4; e++) oW[rc_tiled(t + e, col, DP / 16)] = X[I][e];
+                } else {
+                    *reinterpret_cast<f32x4*>(oU + ((I * (Vp / 16) + (v0 + col) / 16) * 64 + lane) * 4) = X[I];
+                }
             }
         }
+        rc_lds_barrier();
     }
 }
 
 // the walk: four waves, wave w the chunk's tokens 16 w .. and the state's rows w DP / 4 ..; S^T and u^T pass between them through LDS
 template <int DP>
-__global__ void __launch_bounds__(256) rb_delta_walk_kernel(const kf_rb_delta a, const float* __restrict__ chunks, float* __restrict__ o, const int32_t* __restrict__ seqs) {
+__global__ void __launch_bounds__(256, 1) rb_delta_walk_kernel(const kf_rb_delta a, const float* __restrict__ chunks, float* __restrict__ o, const int32_t* __restrict__ seqs) {
     constexpr int LS = DP + 4, LU = RC_C + 4, NT = DP / 64 /* 16-row tiles of the state per wave */;
     __shared__ __attribute__((aligned(16))) float sS[16 * LS], sU[16 * LU];
     const int row0 = seqs[4 * blockIdx.z], n = seqs[4 * blockIdx.z + 1], pos0 = seqs[4 * blockIdx.z + 2], slot = seqs[4 * blockIdx.z + 3];
@@ -677,48 +775,48 @@ __global__ void __launch_bounds__(256) rb_delta_walk_kernel(const kf_rb_delta a,
         *reinterpret_cast<f32x4*>(sS + r16 * LS + d0 + 16 * t + 4 * g4) = S[t];
     }
     const float* c = chunks + ((size_t)rc_chunk_index(row0, blockIdx.z) * a.n_head + h) * rc_chunk_floats(DP, Vp);
-    const int nc = (n + RC_C - 1) / RC_C, tok = 16 * wid + r16;
-    f32x4 w[DP / 16], q[DP / 16];
-    auto fetch = [&](const float* c) {
+    const int nc = (n + RC_C - 1) / RC_C;
+    struct Rows { /* what a wave reads of a chunk: one chunk ahead of its use */
+        f32x4 w[DP / 16], q[DP / 16], p[RC_C / 16], kt[NT][RC_C / 16], u, gt[NT];
+    } rows[2];
+    auto fetch = [&](Rows& x, const float* c) {
+        const float *K = c + 2 * RC_C * DP, *Pq = K + RC_C * DP, *U = Pq + RC_C * RC_C, *G = U + RC_C * Vp;
 #pragma unroll
         for (int k = 0; k < DP / 16; k++) {
-            w[k] = *reinterpret_cast<const f32x4*>(c + tok * DP + 16 * k + 4 * g4);
-            q[k] = *reinterpret_cast<const f32x4*>(c + RC_C * DP + tok * DP + 16 * k + 4 * g4);
+            x.w[k] = *reinterpret_cast<const f32x4*>(c + ((wid * (DP / 16) + k) * 64 + lane) * 4);
+            x.q[k] = *reinterpret_cast<const f32x4*>(c + RC_C * DP + ((wid * (DP / 16) + k) * 64 + lane) * 4);
         }
-    };
-    fetch(c);
-    for (int i = 0; i < nc; i++, c += step) {
-        const float *K = c + 2 * RC_C * DP, *Pq = K + RC_C * DP, *U = Pq + RC_C * RC_C, *G = U + RC_C * Vp;
-        f32x4 p[RC_C / 16], kt[NT][RC_C / 16], u, gt[NT];
-#pragma unroll
-        for (int e = 0; e < 4; e++) u[e] = U[(16 * wid + 4 * g4 + e) * Vp + col];
-#pragma unroll
-        for (int b = 0; b < RC_C / 16; b++) p[b] = *reinterpret_cast<const f32x4*>(Pq + tok * RC_C + 16 * b + 4 * g4); /* (above the diagonal: blocks nobody wrote, not used) */
+        x.u = *reinterpret_cast<const f32x4*>(U + ((wid * (Vp / 16) + v0 / 16) * 64 + lane) * 4);
 #pragma unroll
         for (int t = 0; t < NT; t++) {
-            gt[t] = *reinterpret_cast<const f32x4*>(G + d0 + 16 * t + 4 * g4);
+            x.gt[t] = *reinterpret_cast<const f32x4*>(G + d0 + 16 * t + 4 * g4);
 #pragma unroll
-            for (int b = 0; b < RC_C / 16; b++) kt[t][b] = *reinterpret_cast<const f32x4*>(K + (d0 + 16 * t + r16) * RC_C + 16 * b + 4 * g4);
+            for (int b = 0; b < RC_C / 16; b++) x.kt[t][b] = *reinterpret_cast<const f32x4*>(K + (((wid * NT + t) * (RC_C / 16) + b) * 64 + lane) * 4);
         }
-        __syncthreads(); /* the state of the last chunk is in LDS */
-        f32x4 ws = f32x4{0.f, 0.f, 0.f, 0.f}, y = ws;
+#pragma unroll
+        for (int b = 0; b < RC_C / 16; b++) x.p[b] = *reinterpret_cast<const f32x4*>(Pq + ((wid * (RC_C / 16) + b) * 64 + lane) * 4); /* (above the diagonal: tiles nobody wrote, not used) */
+    };
+    auto chunk = [&](Rows& x, Rows& ahead, int i) {
+        if (i + 1 < nc) fetch(ahead, c + (size_t)(i + 1) * step);
+        rc_lds_barrier(); /* the state of the last chunk is in LDS */
+        f32x4 ws[2], y[2]; /* two chains each */
+#pragma unroll
+        for (int j = 0; j < 2; j++) ws[j] = y[j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int k = 0; k < DP / 16; k++) {
             const f32x4 s = *reinterpret_cast<const f32x4*>(sS + r16 * LS + 16 * k + 4 * g4);
-            ws = rc_mfma(w[k], s, ws), y = rc_mfma(q[k], s, y);
+            ws[k & 1] = rc_mfma(x.w[k], s, ws[k & 1]), y[k & 1] = rc_mfma(x.q[k], s, y[k & 1]);
         }
-        u -= ws;
-        *reinterpret_cast<f32x4*>(sU + r16 * LU + 16 * wid + 4 * g4) = u;
-        if (i + 1 < nc) fetch(c + step);
-        __syncthreads();
+        *reinterpret_cast<f32x4*>(sU + r16 * LU + 16 * wid + 4 * g4) = x.u - (ws[0] + ws[1]);
+        rc_lds_barrier();
 #pragma unroll
-        for (int t = 0; t < NT; t++) S[t] *= gt[t];
+        for (int t = 0; t < NT; t++) S[t] *= x.gt[t];
 #pragma unroll
         for (int b = 0; b < RC_C / 16; b++) {
             const f32x4 ub = *reinterpret_cast<const f32x4*>(sU + r16 * LU + 16 * b + 4 * g4);
 #pragma unroll
-            for (int t = 0; t < NT; t++) S[t] = rc_mfma(kt[t][b], ub, S[t]);
-            if (b <= wid) y = rc_mfma(p[b], ub, y); /* wave-uniform */
+            for (int t = 0; t < NT; t++) S[t] = rc_mfma(x.kt[t][b], ub, S[t]);
+            if (b <= wid) y[b & 1] = rc_mfma(x.p[b], ub, y[b & 1]); /* wave-uniform */
         }
 #pragma unroll
         for (int t = 0; t < NT; t++) *reinterpret_cast<f32x4*>(sS + r16 * LS + d0 + 16 * t + 4 * g4) = S[t];
@@ -726,9 +824,14 @@ __global__ void __launch_bounds__(256) rb_delta_walk_kernel(const kf_rb_delta a,
 #pragma unroll
             for (int e = 0; e < 4; e++) {
                 const int row = RC_C * i + 16 * wid + 4 * g4 + e;
-                if (row < n) o[(size_t)(row0 + row) * a.n_head * vdim + (size_t)h * vdim + col] = y[e];
+                if (row < n) o[(size_t)(row0 + row) * a.n_head * vdim + (size_t)h * vdim + col] = y[0][e] + y[1][e];
             }
         }
+    };
+    fetch(rows[0], c);
+    for (int i = 0; i < nc; i += 2) {
+        chunk(rows[0], rows[1], i);
+        if (i + 1 < nc) chunk(rows[1], rows[0], i + 1);
     }
     if (col < vs) {
 #pragma unroll
@@ -743,7 +846,7 @@ __global__ void __launch_bounds__(256) rb_delta_walk_kernel(const kf_rb_delta a,
 static int rc_delta_padded(int dim, int vdim) { return vdim > 256 ? 0 : (dim <= 64 ? 64 : (dim <= 128 ? 128 : 0)); } /* 0: not served in chunks */
 template <class T, int DP>
 static int delta_chunks_go(hipStream_t st, const kf_rb_delta& a, float* chunks, float* o, const int32_t* seqs, int n_seq, int max_n) {
-    constexpr size_t smem = (3 * RC_C * (DP + 4) + 4 * DP + RC_C * (RC_C + 4) + 4 * 16 * 20 + 3 * RC_C) * sizeof(float);
+    constexpr size_t smem = (3 * RC_C * (DP + 4) + 14 * DP + RC_C * (RC_C + 4) + 4 * 16 * 20 + 3 * RC_C) * sizeof(float);
     static_assert(smem <= 160 * 1024, "LDS");
     static int done = 0;
     if (!done) {
@@ -833,7 +936,7 @@ __global__ void __launch_bounds__(256) rb_decay_part_kernel(const kf_rb_decay a,
     Stage st;
     st.load(k, v, a.ldraw, a.dim, a.vdim, t0, t1, tid);
     st.store(lds[0], lds[0] + 32 * Stage::KS, tid);
-    __syncthreads();
+    rc_lds_barrier();
     for (int t = 0; t < nt; t++) {
         const int k0 = t0 + 32 * t, m = t1 - k0 < 32 ? t1 - k0 : 32; /* the tile's keys */
         if (t + 1 < nt) st.load(k, v, a.ldraw, a.dim, a.vdim, k0 + 32, t1, tid);
@@ -863,7 +966,7 @@ __global__ void __launch_bounds__(256) rb_decay_part_kernel(const kf_rb_decay a,
             }
         }
         if (t + 1 < nt) st.store(lds[(t + 1) & 1], lds[(t + 1) & 1] + 32 * Stage::KS, tid);
-        __syncthreads();
+        rc_lds_barrier();
     }
     float* out = sums + ((size_t)(rc_span_index(row0, blockIdx.z) + blockIdx.y) * a.n_head + h) * HD * HD;
 #pragma unroll
@@ -946,7 +1049,7 @@ __global__ void __launch_bounds__(256) rb_decay_out_kernel(const kf_rb_decay a, 
     float tail[16]; /* decay^(31 - key) of a tile's keys */
 #pragma unroll
     for (int i = 0; i < 16; i++) tail[i] = pw(31 - rc_tile_key(hh, i));
-    __syncthreads();
+    rc_lds_barrier();
     for (int t = 0; t < nt; t++) {
         const int k0 = c0 + 32 * t;
         if (t + 1 < nt) st.load(k, v, a.ldraw, a.dim, a.vdim, k0 + 32, last, tid);
@@ -985,7 +1088,7 @@ __global__ void __launch_bounds__(256) rb_decay_out_kernel(const kf_rb_decay a, 
             }
         }
         if (t + 1 < nt) st.store(lds[(t + 1) & 1], lds[(t + 1) & 1] + 32 * Stage::KS, tid);
-        __syncthreads();
+        rc_lds_barrier();
     }
     if (tok >= n) return;
     float* out = o + (size_t)(row0 + tok) * a.n_head * a.vdim + (size_t)h * a.vdim;
@@ -1110,7 +1213,8 @@ template <class T>
 static int delta_prefill_go(hipStream_t st, const kf_rb_delta& a, const int32_t* meta, int n, const int32_t* seqs, int n_seq, int max_n) {
     const int64_t ldv = (int64_t)a.n_head * a.vdim;
     float* o = a.scratch; /* [n][n_head vdim] */
-    const int DP = max_n >= RC_MIN_CHUNKED ? rc_delta_padded(a.dim, a.vdim) : 0;
+    const bool offsets = (int64_t)n * std::max(a.ldraw, a.ld_az) < ((int64_t)1 << 30); /* of a row inside the batch: 32 bits */
+    const int DP = max_n >= RC_MIN_CHUNKED && offsets ? rc_delta_padded(a.dim, a.vdim) : 0;
     if (DP) {
         float* chunks = o + ((size_t)n * ldv + 3) / 4 * 4;
         const int rc = DP == 64 ? delta_chunks_go<T, 64>(st, a, chunks, o, seqs, n_seq, max_n) : delta_chunks_go<T, 128>(st, a, chunks, o, seqs, n_seq, max_n);
@@ -1122,7 +1226,7 @@ static int delta_prefill_go(hipStream_t st, const kf_rb_delta& a, const int32_t*
         const RcScan<float> s{p.qk, p.qk + (size_t)a.n_kv * a.dim, p.v, p.g, p.beta, nullptr, p.v, a.state, ldq, ldv, ldv, a.n_head, a.n_head / a.n_kv, a.dim, a.vdim};
         if (scan_go<float, true>(st, s, seqs, n_seq)) return 1;
     }
-    hipLaunchKernelGGL(rb_hist_kernel<T>, dim3(n), dim3(256), 0, st, a, meta);
+    hipLaunchKernelGGL(rb_hist_kernel<T>, dim3((2 * a.n_kv * a.dim + a.n_head * a.vdim + 255) / 256, a.taps, n_seq), dim3(256), 0, st, a, seqs);
     gate_go<T>(st, RcGate{o, a.norm_w, a.g_z, a.out, ldv, a.ld_gz, a.ldout, a.n_head, a.vdim, 1.f, a.eps}, n);
     return KF_OK;
 }
