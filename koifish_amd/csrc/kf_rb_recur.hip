@@ -674,7 +674,12 @@ __global__ void __launch_bounds__(512) rb_delta_chunk_kernel(const kf_rb_delta a
 #pragma unroll 4
         for (int kb = 0; kb < DP / 16; kb++) {
             const f32x4 B = *reinterpret_cast<const f32x4*>(pj + 16 * kb) * *reinterpret_cast<const f32x4*>(pe + 16 * kb);
-            kk[kb & 1] = rc_mfma(*reinterpret_cast<const f32x4*>(pk + 16 * kb), B, kk[kb & 1]), qk[kb & 1] = rc_mfma(*reinterpret_cast<const f32x4*>(pq + 16 * kb), B, qk[kb & 1]);
+            const f32x4 k = *reinterpret_cast<const f32x4*>(pk + 16 * kb), q = *reinterpret_cast<const f32x4*>(pq + 16 * kb);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                kk[kb & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(k[e], B[e], kk[kb & 1], 0, 0, 0);
+                qk[kb & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[e], B[e], qk[kb & 1], 0, 0, 0);
+            }
         }
         finish(I, J, kk[0] + kk[1], qk[0] + qk[1]);
     }
@@ -776,63 +781,86 @@ __global__ void __launch_bounds__(256, 1) rb_delta_walk_kernel(const kf_rb_delta
     }
     const float* c = chunks + ((size_t)rc_chunk_index(row0, blockIdx.z) * a.n_head + h) * rc_chunk_floats(DP, Vp);
     const int nc = (n + RC_C - 1) / RC_C;
-    struct Rows { /* what a wave reads of a chunk: one chunk ahead of its use */
-        f32x4 w[DP / 16], q[DP / 16], p[RC_C / 16], kt[NT][RC_C / 16], u, gt[NT];
-    } rows[2];
-    auto fetch = [&](Rows& x, const float* c) {
-        const float *K = c + 2 * RC_C * DP, *Pq = K + RC_C * DP, *U = Pq + RC_C * RC_C, *G = U + RC_C * Vp;
+    // what a wave reads of a chunk.  A register is loaded for the next chunk as soon as this one has used it, a load or two between the products: a CU takes in 64 bytes a cycle, and a
+    // wave that issued a chunk's loads in one go would wait for that instead of multiplying
+    f32x4 w[DP / 16], q[DP / 16], p[RC_C / 16], kt[NT][RC_C / 16], u, gt[NT];
+    auto ld_w = [&](const float* c, int k) { w[k] = *reinterpret_cast<const f32x4*>(c + ((wid * (DP / 16) + k) * 64 + lane) * 4); };
+    auto ld_q = [&](const float* c, int k) { q[k] = *reinterpret_cast<const f32x4*>(c + RC_C * DP + ((wid * (DP / 16) + k) * 64 + lane) * 4); };
+    auto ld_k = [&](const float* c, int t, int b) { kt[t][b] = *reinterpret_cast<const f32x4*>(c + 2 * RC_C * DP + (((wid * NT + t) * (RC_C / 16) + b) * 64 + lane) * 4); };
+    auto ld_p = [&](const float* c, int b) { p[b] = *reinterpret_cast<const f32x4*>(c + 3 * RC_C * DP + ((wid * (RC_C / 16) + b) * 64 + lane) * 4); }; /* (above the diagonal: tiles nobody wrote, not used) */
+    auto ld_u = [&](const float* c) { u = *reinterpret_cast<const f32x4*>(c + RC_C * (3 * DP + RC_C) + ((wid * (Vp / 16) + v0 / 16) * 64 + lane) * 4); };
+    auto ld_g = [&](const float* c, int t) { gt[t] = *reinterpret_cast<const f32x4*>(c + RC_C * (3 * DP + RC_C + Vp) + d0 + 16 * t + 4 * g4); };
 #pragma unroll
-        for (int k = 0; k < DP / 16; k++) {
-            x.w[k] = *reinterpret_cast<const f32x4*>(c + ((wid * (DP / 16) + k) * 64 + lane) * 4);
-            x.q[k] = *reinterpret_cast<const f32x4*>(c + RC_C * DP + ((wid * (DP / 16) + k) * 64 + lane) * 4);
-        }
-        x.u = *reinterpret_cast<const f32x4*>(U + ((wid * (Vp / 16) + v0 / 16) * 64 + lane) * 4);
+    for (int k = 0; k < DP / 16; k++) ld_w(c, k), ld_q(c, k);
+    ld_u(c);
 #pragma unroll
-        for (int t = 0; t < NT; t++) {
-            x.gt[t] = *reinterpret_cast<const f32x4*>(G + d0 + 16 * t + 4 * g4);
+    for (int t = 0; t < NT; t++) {
+        ld_g(c, t);
 #pragma unroll
-            for (int b = 0; b < RC_C / 16; b++) x.kt[t][b] = *reinterpret_cast<const f32x4*>(K + (((wid * NT + t) * (RC_C / 16) + b) * 64 + lane) * 4);
-        }
+        for (int b = 0; b < RC_C / 16; b++) ld_k(c, t, b);
+    }
 #pragma unroll
-        for (int b = 0; b < RC_C / 16; b++) x.p[b] = *reinterpret_cast<const f32x4*>(Pq + ((wid * (RC_C / 16) + b) * 64 + lane) * 4); /* (above the diagonal: tiles nobody wrote, not used) */
-    };
-    auto chunk = [&](Rows& x, Rows& ahead, int i) {
-        if (i + 1 < nc) fetch(ahead, c + (size_t)(i + 1) * step);
-        rc_lds_barrier(); /* the state of the last chunk is in LDS */
-        f32x4 ws[2], y[2]; /* two chains each */
-#pragma unroll
-        for (int j = 0; j < 2; j++) ws[j] = y[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int k = 0; k < DP / 16; k++) {
-            const f32x4 s = *reinterpret_cast<const f32x4*>(sS + r16 * LS + 16 * k + 4 * g4);
-            ws[k & 1] = rc_mfma(x.w[k], s, ws[k & 1]), y[k & 1] = rc_mfma(x.q[k], s, y[k & 1]);
-        }
-        *reinterpret_cast<f32x4*>(sU + r16 * LU + 16 * wid + 4 * g4) = x.u - (ws[0] + ws[1]);
-        rc_lds_barrier();
-#pragma unroll
-        for (int t = 0; t < NT; t++) S[t] *= x.gt[t];
-#pragma unroll
-        for (int b = 0; b < RC_C / 16; b++) {
-            const f32x4 ub = *reinterpret_cast<const f32x4*>(sU + r16 * LU + 16 * b + 4 * g4);
-#pragma unroll
-            for (int t = 0; t < NT; t++) S[t] = rc_mfma(x.kt[t][b], ub, S[t]);
-            if (b <= wid) y[b & 1] = rc_mfma(x.p[b], ub, y[b & 1]); /* wave-uniform */
-        }
-#pragma unroll
-        for (int t = 0; t < NT; t++) *reinterpret_cast<f32x4*>(sS + r16 * LS + d0 + 16 * t + 4 * g4) = S[t];
+    for (int b = 0; b < RC_C / 16; b++) ld_p(c, b);
+    f32x4 done = f32x4{0.f, 0.f, 0.f, 0.f}; /* the last chunk's outputs: stored while this one multiplies, a chunk's time before the next wait for memory */
+    auto store = [&](int i) {
         if (col < vdim) {
 #pragma unroll
             for (int e = 0; e < 4; e++) {
                 const int row = RC_C * i + 16 * wid + 4 * g4 + e;
-                if (row < n) o[(size_t)(row0 + row) * a.n_head * vdim + (size_t)h * vdim + col] = y[0][e] + y[1][e];
+                if (row < n) o[(size_t)(row0 + row) * a.n_head * vdim + (size_t)h * vdim + col] = done[e];
             }
         }
     };
-    fetch(rows[0], c);
-    for (int i = 0; i < nc; i += 2) {
-        chunk(rows[0], rows[1], i);
-        if (i + 1 < nc) chunk(rows[1], rows[0], i + 1);
+    for (int i = 0; i < nc; i++) {
+        const float* next = i + 1 < nc ? c + step : c; /* (the last chunk again: not used) */
+        rc_lds_barrier(); /* the state of the last chunk is in LDS */
+        f32x4 ws[2], y[2]; /* two chains each */
+#pragma unroll
+        for (int j = 0; j < 2; j++) ws[j] = y[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        f32x4 s = *reinterpret_cast<const f32x4*>(sS + r16 * LS + 4 * g4);
+#pragma unroll
+        for (int k = 0; k < DP / 16; k++) {
+            f32x4 s1 = s;
+            if (k + 1 < DP / 16) s1 = *reinterpret_cast<const f32x4*>(sS + r16 * LS + 16 * (k + 1) + 4 * g4);
+            ws[k & 1] = rc_mfma(w[k], s, ws[k & 1]);
+            if (k > 0) ld_q(next, k - 1);
+            __builtin_amdgcn_sched_barrier(0);
+            y[k & 1] = rc_mfma(q[k], s, y[k & 1]);
+            ld_w(next, k);
+            s = s1;
+            __builtin_amdgcn_sched_barrier(0);
+            if (k == 0 && i > 0) store(i - 1);
+        }
+        *reinterpret_cast<f32x4*>(sU + r16 * LU + 16 * wid + 4 * g4) = u - (ws[0] + ws[1]);
+        ld_q(next, DP / 16 - 1), ld_u(next);
+        rc_lds_barrier();
+        f32x4 ub = *reinterpret_cast<const f32x4*>(sU + r16 * LU + 4 * g4);
+#pragma unroll
+        for (int t = 0; t < NT; t++) {
+            S[t] *= gt[t];
+            ld_g(next, t);
+        }
+#pragma unroll
+        for (int b = 0; b < RC_C / 16; b++) {
+            f32x4 u1 = ub;
+            if (b + 1 < RC_C / 16) u1 = *reinterpret_cast<const f32x4*>(sU + r16 * LU + 16 * (b + 1) + 4 * g4);
+#pragma unroll
+            for (int t = 0; t < NT; t++) {
+                S[t] = rc_mfma(kt[t][b], ub, S[t]);
+                ld_k(next, t, b);
+                __builtin_amdgcn_sched_barrier(0);
+            }
+            if (b <= wid) y[b & 1] = rc_mfma(p[b], ub, y[b & 1]); /* wave-uniform */
+            ld_p(next, b);
+            ub = u1;
+            __builtin_amdgcn_sched_barrier(0);
+        }
+#pragma unroll
+        for (int t = 0; t < NT; t++) *reinterpret_cast<f32x4*>(sS + r16 * LS + d0 + 16 * t + 4 * g4) = S[t];
+        done = y[0] + y[1];
+        c = next;
     }
+    store(nc - 1);
     if (col < vs) {
 #pragma unroll
         for (int t = 0; t < NT; t++)
