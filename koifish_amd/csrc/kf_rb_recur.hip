@@ -9,45 +9,10 @@
 #include <algorithm>
 
 #include "kf_ctx.h"
-#include "kf_rb_common.h"
+#include "kf_rb_recur.h"
 
 namespace kf {
 
-__device__ __forceinline__ float row16_sum(float v) { /* over the 16 lanes of a row, in all of them */
-    v += dpp_f<0xB1>(v);
-    v += dpp_f<0x4E>(v);
-    v += dpp_f<0x141>(v);
-    return v + dpp_f<0x140>(v);
-}
-__device__ __forceinline__ float rc_silu(float z) { return z * rb_sigmoid(z); }
-__device__ __forceinline__ void rc_st_sc1(float* p, float v) { __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
-__device__ __forceinline__ float rc_ld_sc1(const float* p) { return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }
-// a barrier for what passes through LDS only: loads and stores of global memory stay in flight over it
-__device__ __forceinline__ void rc_lds_barrier() {
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    __builtin_amdgcn_s_barrier();
-    asm volatile("" ::: "memory");
-}
-constexpr int RC_CNT_STRIDE = 16; /* words between arrival counters */
-static __host__ __device__ inline int rc_up(int n, int m) { return (n + m - 1) / m * m; }
-
-// row r of a product's weight (ld columns) times a[0 .. rank), a in LDS padded with zeros to a multiple of 8
-__device__ __forceinline__ float rc_weight_dot(const uint16_t* __restrict__ w, int ld, int r, const float* a, int rank) {
-    const uint16_t* tile = w + (size_t)(r / 16) * (ld / 32) * 512 + (r & 15) * 8;
-    float s = 0.f;
-    for (int o = 0; o < (rank + 7) / 8; o++) {
-        const u32x4 v = *reinterpret_cast<const u32x4*>(tile + (o >> 2) * 512 + (o & 3) * 128);
-        const float* x = a + 8 * o;
-        s = fmaf(bf_lo(v.x), x[0], s), s = fmaf(bf_hi(v.x), x[1], s), s = fmaf(bf_lo(v.y), x[2], s), s = fmaf(bf_hi(v.y), x[3], s);
-        s = fmaf(bf_lo(v.z), x[4], s), s = fmaf(bf_hi(v.z), x[5], s), s = fmaf(bf_lo(v.w), x[6], s), s = fmaf(bf_hi(v.w), x[7], s);
-    }
-    return s;
-}
-__device__ __forceinline__ float rc_weight_dot(const float* __restrict__ w, int ld, int r, const float* a, int rank) {
-    float s = 0.f;
-    for (int i = 0; i < rank; i++) s = fmaf(w[(size_t)r * ld + i], a[i], s);
-    return s;
-}
 // channel c of the convolution at position pos, batch row r (the batch holds the sequence's positions from pos0 on), before the activation
 template <class T>
 __device__ __forceinline__ float rc_conv(const kf_rb_delta& a, const T* raw_r, const T* hist, int channels, int c, int pos, int pos0) {
@@ -62,217 +27,159 @@ __device__ __forceinline__ float rc_conv(const kf_rb_delta& a, const T* raw_r, c
     return s;
 }
 
-// ---- decode.  NT threads: groups of vs / 4 threads side by side, each group the rows rg, rg + RG, ...; RPT rows of a thread stay in registers (KEEP), otherwise they are read twice
-constexpr int RC_RPT = 16;
-template <class T, int NT, bool KEEP>
+// ---- decode
+// eight consecutive columns of row r of a product's weight (ld columns), octet o, and their product with eight floats of LDS
+__device__ __forceinline__ u32x4 rc_octet(const uint16_t* __restrict__ w, int ld, int r, int o) { return *reinterpret_cast<const u32x4*>(w + ((size_t)(r / 16) * (ld / 32) + (o >> 2)) * 512 + (r & 15) * 8 + (o & 3) * 128); }
+__device__ __forceinline__ float rc_octet_dot(u32x4 v, const float* x, float s) {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(x), b = *reinterpret_cast<const f32x4*>(x + 4);
+    s = fmaf(bf_lo(v.x), a.x, s), s = fmaf(bf_hi(v.x), a.y, s), s = fmaf(bf_lo(v.y), a.z, s), s = fmaf(bf_hi(v.y), a.w, s);
+    return fmaf(bf_hi(v.w), b.w, fmaf(bf_lo(v.w), b.z, fmaf(bf_hi(v.z), b.y, fmaf(bf_lo(v.z), b.x, s))));
+}
+struct RcOctet32 {
+    f32x4 a, b;
+};
+__device__ __forceinline__ RcOctet32 rc_octet(const float* __restrict__ w, int ld, int r, int o) {
+    const float* p = w + (size_t)r * ld + 8 * o;
+    return RcOctet32{*reinterpret_cast<const f32x4*>(p), *reinterpret_cast<const f32x4*>(p + 4)};
+}
+__device__ __forceinline__ float rc_octet_dot(const RcOctet32& v, const float* x, float s) {
+#pragma unroll
+    for (int j = 0; j < 4; j++) s = fmaf(v.b[j], x[4 + j], fmaf(v.a[j], x[j], s));
+    return s;
+}
+// One workgroup per (head, row).  What it reads sets out at once, in the order of its use: the channels' last inputs, the low-rank rows, the state (barriers wait for LDS only)
+template <class T, int NT, int RPT>
 __global__ void __launch_bounds__(NT) rb_delta_step_kernel(const kf_rb_delta a, const int32_t* __restrict__ meta) {
     extern __shared__ float smem[];
+    constexpr int NW = NT / 64, PF = NT > 512 || sizeof(T) == 4 ? 4 : 8; /* octets in flight per lane */
     const int h = blockIdx.x, rr = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const int pos = meta[KF_RB_META * rr], slot = meta[KF_RB_META * rr + 1];
     if (pos < 0) return; /* workgroup-uniform */
-    const int dim = a.dim, vdim = a.vdim, vs = rc_up(vdim, 4), c4 = vs / 4, RG = NT / c4, rg = tid / c4, col = 4 * (tid - rg * c4);
-    const int kvh = h / (a.n_head / a.n_kv), qd = a.n_kv * dim, channels = 2 * qd + a.n_head * vdim;
-    const int ra8 = rc_up(a.rank_a, 8), rg8 = rc_up(a.rank_g, 8), d4 = rc_up(dim, 4);
-    float *s_q = smem, *s_k = s_q + d4, *s_g = s_k + d4, *s_v = s_g + d4, *s_z = s_v + vs, *s_a = s_z + vs, *s_gl = s_a + ra8, *s_red = s_gl + rg8 /* [2][RG][vs] */, *s_one = s_red + 2 * NT * 4;
+    const int dim = a.dim, vdim = a.vdim, kvh = h / (a.n_head / a.n_kv), qd = a.n_kv * dim, channels = 2 * qd + a.n_head * vdim, n_ch = 2 * dim + vdim;
+    const int ra8 = rc_up(a.rank_a, 8), rg8 = rc_up(a.rank_g, 8), d4 = rc_up(dim, 4), vs = rc_up(vdim, 4);
+    float *s_a = smem, *s_gl = s_a + ra8, *s_q = s_gl + rg8, *s_k = s_q + d4, *s_g = s_k + d4, *s_v = s_g + d4, *s_z = s_v + vs, *s_red = s_z + vs /* [2][parts][vs] */, *s_one = s_red + 8 * NT;
+    const T* raw = reinterpret_cast<const T*>(a.raw) + (size_t)rr * a.ldraw;
+    T* hist = reinterpret_cast<T*>(a.hist) + (size_t)slot * a.hist_slot;
+    auto channel = [&](int i) { return i < dim ? kvh * dim + i : (i < 2 * dim ? qd + kvh * dim + (i - dim) : 2 * qd + h * vdim + (i - 2 * dim)); };
+    T x0[4], w0[4]; /* four taps: this thread's first channel */
+    const bool four = a.taps == 4, ch_on = tid < n_ch;
+    if (four && ch_on) {
+        const int c = channel(tid);
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            x0[j] = j == 3 ? raw[c] : hist[(size_t)((pos + 1 + j) & 3) * channels + c]; /* row (pos - 3 + j) % 4 */
+            w0[j] = reinterpret_cast<const T*>(a.conv)[(size_t)c * 4 + j];
+        }
+    }
+    T lr0 = T();
+    auto low_rank_input = [&](int i) { return i < ra8 ? (i < a.rank_a ? raw[a.col_a + i] : T()) : (i - ra8 < a.rank_g ? raw[a.col_g + i - ra8] : T()); };
+    if (tid < ra8 + rg8) lr0 = low_rank_input(tid);
+    // rows of the two factors: 32 of them per wave and turn, two lanes (16 apart) share a row's octets
+    const T *wa = reinterpret_cast<const T*>(a.w_a2), *wg = reinterpret_cast<const T*>(a.w_g2);
+    const int half = lane >> 4 & 1, n_row = dim + vdim;
+    decltype(rc_octet(wa, 0, 0, 0)) pre[PF];
+    {
+        const int i = 32 * wid + (lane & 15) + 16 * (lane >> 5);
+        const bool is_a = i < dim;
+        const int no = (is_a ? ra8 : rg8) / 8;
+#pragma unroll
+        for (int j = 0; j < PF; j++) {
+            pre[j] = decltype(rc_octet(wa, 0, 0, 0)){};
+            if (i < n_row && half + 2 * j < no) pre[j] = is_a ? rc_octet(wa, a.ld_a, h * dim + i, half + 2 * j) : rc_octet(wg, a.ld_g, h * vdim + i - dim, half + 2 * j);
+        }
+    }
+    RcStep<NT, RPT> st(dim, vdim, tid);
     const size_t head = (size_t)dim * vs, side = (size_t)a.n_head * head;
     const float* S0 = a.state + ((size_t)slot * 2 + ((pos + 1) & 1)) * side + h * head;
     float* S1 = a.state + ((size_t)slot * 2 + (pos & 1)) * side + h * head;
-    const bool on = rg < RG, old = pos > 0;
-    f32x4 S[KEEP ? RC_RPT : 1];
-    if constexpr (KEEP) {
+    st.load(S0, pos > 0);
+    for (int i = tid; i < ra8 + rg8; i += NT) s_a[i] = rb_ld1(i == tid ? lr0 : low_rank_input(i));
+    const bool first = h == kvh * (a.n_head / a.n_kv);
+    for (int i = tid; i < n_ch; i += NT) { /* the head's channels: q, k, v */
+        const int c = channel(i);
+        float y;
+        if (four && i == tid) {
+            y = 0.f;
 #pragma unroll
-        for (int i = 0; i < RC_RPT; i++) {
-            const int r = rg + i * RG;
-            S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-            if (on && old && r < dim) S[i] = *reinterpret_cast<const f32x4*>(S0 + (size_t)r * vs + col);
+            for (int j = 0; j < 4; j++)
+                if (pos - 3 + j >= 0) y = fmaf(rb_ld1(w0[j]), rb_ld1(x0[j]), y);
+        } else {
+            y = rc_conv(a, raw, hist, channels, c, pos, pos);
         }
-    }
-    const T* raw = reinterpret_cast<const T*>(a.raw) + (size_t)rr * a.ldraw;
-    T* hist = reinterpret_cast<T*>(a.hist) + (size_t)slot * a.hist_slot;
-    for (int i = tid; i < ra8 + rg8; i += NT) {
-        const bool g = i >= ra8;
-        const int j = g ? i - ra8 : i;
-        s_a[i] = j < (g ? a.rank_g : a.rank_a) ? rb_ld(raw + (g ? a.col_g : a.col_a) + j) : 0.f;
-    }
-    for (int i = tid; i < 2 * dim + vdim; i += NT) { /* the head's channels: q, k, v */
-        const int c = i < dim ? kvh * dim + i : (i < 2 * dim ? qd + kvh * dim + (i - dim) : 2 * qd + h * vdim + (i - 2 * dim));
-        const float y = rc_silu(rc_conv(a, raw, hist, channels, c, pos, pos));
+        y *= rc_fast_sigmoid(y);
         (i < dim ? s_q[i] : (i < 2 * dim ? s_k[i - dim] : s_v[i - 2 * dim])) = y;
-        if (i >= 2 * dim || h == kvh * (a.n_head / a.n_kv)) hist[(size_t)(pos % a.taps) * channels + c] = raw[c];
+        if (i >= 2 * dim || first) hist[(size_t)(pos % a.taps) * channels + c] = raw[c];
     }
     for (int i = vdim + tid; i < vs; i += NT) s_v[i] = 0.f;
-    __syncthreads();
-    for (int w = wid; w < 2; w += NT / 64) { /* 1 / length of q and of k, and q . k between them below */
-        float ss = 0.f;
-        const float* x = w ? s_k : s_q;
-        for (int i = lane; i < dim; i += 64) ss = fmaf(x[i], x[i], ss);
-        ss = wave_sum(ss);
-        if (lane == 0) s_one[w] = 1.0f / sqrtf(ss + a.unit_eps);
+    const float rate = expf(rb_ld(reinterpret_cast<const T*>(a.a_log) + h)), beta = rb_sigmoid(rb_ld(raw + a.col_b + h));
+    rc_lds_barrier();
+    for (int g = wid; 32 * g < n_row; g += NW) {
+        const int i = 32 * g + (lane & 15) + 16 * (lane >> 5);
+        const bool is_a = i < dim, in = i < n_row;
+        const int no = in ? (is_a ? ra8 : rg8) / 8 : 0, r = is_a ? h * dim + i : h * vdim + i - dim;
+        const float* x = is_a ? s_a : s_gl;
+        float z = 0.f;
+#pragma unroll
+        for (int j = 0; j < PF; j++) {
+            const int o = half + 2 * j;
+            if (o < no) z = rc_octet_dot(g == wid ? pre[j] : (is_a ? rc_octet(wa, a.ld_a, r, o) : rc_octet(wg, a.ld_g, r, o)), x + 8 * o, z);
+        }
+        for (int o = half + 2 * PF; o < no; o += 2) z = rc_octet_dot(is_a ? rc_octet(wa, a.ld_a, r, o) : rc_octet(wg, a.ld_g, r, o), x + 8 * o, z);
+        z = xsum16(z);
+        if (in && half == 0) {
+            if (is_a) s_g[i] = rc_exp2(-rate * rc_softplus2(z + rb_ld(reinterpret_cast<const T*>(a.dt_bias) + r)));
+            else s_z[i - dim] = rb_sigmoid(z);
+        }
     }
-    const T *wa = reinterpret_cast<const T*>(a.w_a2), *wg = reinterpret_cast<const T*>(a.w_g2);
-    const float rate = expf(rb_ld(reinterpret_cast<const T*>(a.a_log) + h));
-    for (int i = tid; i < dim; i += NT) {
-        const float z = rc_weight_dot(wa, a.ld_a, h * dim + i, s_a, a.rank_a) + rb_ld(reinterpret_cast<const T*>(a.dt_bias) + h * dim + i);
-        s_g[i] = expf(-rate * rb_softplus(z));
-    }
-    for (int i = tid; i < vdim; i += NT) s_z[i] = rb_sigmoid(rc_weight_dot(wg, a.ld_g, h * vdim + i, s_gl, a.rank_g));
-    __syncthreads();
-    const float qn = s_one[0] * a.q_scale, kn = s_one[1];
-    if (wid == 0) {
+    for (int w = NW - 1 - wid; w < 3; w += NW) { /* squares of q, of k, and q . k */
+        const float *x = w == 1 ? s_k : s_q, *y = w ? s_k : s_q;
         float d = 0.f;
-        for (int i = lane; i < dim; i += 64) d = fmaf(s_q[i], s_k[i], d);
+        for (int i = lane; i < dim; i += 64) d = fmaf(x[i], y[i], d);
         d = wave_sum(d);
-        if (lane == 0) s_one[2] = d * qn * kn;
+        if (lane == 0) s_one[w] = d;
     }
+    rc_lds_barrier();
+    const float qn = a.q_scale / sqrtf(s_one[0] + a.unit_eps), kn = 1.0f / sqrtf(s_one[1] + a.unit_eps), qk = s_one[2] * qn * kn;
     f32x4 p = f32x4{0.f, 0.f, 0.f, 0.f}, o = p;
-    auto walk = [&](int r, f32x4 s) {
+    st.each(S0, pos > 0, [&](int r, f32x4 s) {
         const float g = s_g[r], kk = g * (s_k[r] * kn), qq = g * (s_q[r] * qn);
 #pragma unroll
         for (int j = 0; j < 4; j++) p[j] = fmaf(kk, s[j], p[j]), o[j] = fmaf(qq, s[j], o[j]);
-    };
-    if (on && old) {
-        if constexpr (KEEP) {
-#pragma unroll
-            for (int i = 0; i < RC_RPT; i++)
-                if (rg + i * RG < dim) walk(rg + i * RG, S[i]);
-        } else {
-            for (int r = rg; r < dim; r += RG) walk(r, *reinterpret_cast<const f32x4*>(S0 + (size_t)r * vs + col));
-        }
-    }
-    if (on) {
-        *reinterpret_cast<f32x4*>(s_red + (size_t)rg * vs + col) = p;
-        *reinterpret_cast<f32x4*>(s_red + (size_t)(RG + rg) * vs + col) = o;
-    }
-    __syncthreads();
-    const float beta = rb_sigmoid(rb_ld(raw + a.col_b + h)), qk = s_one[2];
+    });
+    const int parts = st.parts();
+    st.partial(p, s_red), st.partial(o, s_red + (size_t)parts * vs);
+    rc_lds_barrier();
     float ss = 0.f;
     for (int i = tid; i < vs; i += NT) {
         float sp = 0.f, so = 0.f;
-        for (int g = 0; g < RG; g++) sp += s_red[(size_t)g * vs + i], so += s_red[(size_t)(RG + g) * vs + i];
+        for (int g = 0; g < parts; g++) sp += s_red[(size_t)g * vs + i], so += s_red[(size_t)(parts + g) * vs + i];
         const float u = beta * (s_v[i] - sp), y = fmaf(qk, u, so);
         s_v[i] = i < vdim ? u : 0.f;
-        s_red[i] = y; /* this thread's column of the first group: nobody else's */
+        s_red[i] = y; /* this thread's column of the first part: nobody else's */
         if (i < vdim) ss = fmaf(y, y, ss);
     }
     ss = wave_sum(ss);
     if (lane == 0) s_one[4 + wid] = ss;
-    __syncthreads();
+    rc_lds_barrier();
     ss = 0.f;
 #pragma unroll
-    for (int w = 0; w < NT / 64; w++) ss += s_one[4 + w];
+    for (int w = 0; w < NW; w++) ss += s_one[4 + w];
     const float rs = 1.0f / sqrtf(ss / (float)vdim + a.eps);
     T* out = reinterpret_cast<T*>(a.out) + (size_t)rr * a.ldout + (size_t)h * vdim;
     for (int i = tid; i < vdim; i += NT) rb_st(out + i, s_red[i] * rs * rb_ld(reinterpret_cast<const T*>(a.norm_w) + i) * s_z[i]);
-    if (on) {
-        const f32x4 u = *reinterpret_cast<const f32x4*>(s_v + col);
-        auto write = [&](int r, f32x4 s) {
-            const float g = s_g[r], kk = s_k[r] * kn;
-            f32x4 n;
-#pragma unroll
-            for (int j = 0; j < 4; j++) n[j] = fmaf(kk, u[j], g * s[j]);
-            *reinterpret_cast<f32x4*>(S1 + (size_t)r * vs + col) = n;
-        };
-        if constexpr (KEEP) {
-#pragma unroll
-            for (int i = 0; i < RC_RPT; i++)
-                if (rg + i * RG < dim) write(rg + i * RG, S[i]);
-        } else {
-            for (int r = rg; r < dim; r += RG) {
-                f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
-                if (old) s = *reinterpret_cast<const f32x4*>(S0 + (size_t)r * vs + col);
-                write(r, s);
-            }
-        }
-    }
-}
-template <class T, int NT, bool KEEP>
-__global__ void __launch_bounds__(NT) rb_decay_step_kernel(const kf_rb_decay a, const int32_t* __restrict__ meta) {
-    extern __shared__ float smem[];
-    const int h = blockIdx.x, rr = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
-    const int pos = meta[KF_RB_META * rr], slot = meta[KF_RB_META * rr + 1];
-    if (pos < 0) return; /* workgroup-uniform */
-    const int dim = a.dim, vdim = a.vdim, vs = rc_up(vdim, 4), c4 = vs / 4, RG = NT / c4, rg = tid / c4, col = 4 * (tid - rg * c4);
-    float *s_q = smem, *s_k = s_q + rc_up(dim, 4), *s_v = s_k + rc_up(dim, 4), *s_red = s_v + vs /* [RG][vs] */, *s_one = s_red + NT * 4;
-    __shared__ int s_last;
-    const size_t head = (size_t)dim * vs, side = (size_t)a.n_head * head;
-    const float* S0 = a.state + ((size_t)slot * 2 + ((pos + 1) & 1)) * side + h * head;
-    float* S1 = a.state + ((size_t)slot * 2 + (pos & 1)) * side + h * head;
-    const bool on = rg < RG, old = pos > 0;
-    const float lam = a.decay[h];
-    f32x4 S[KEEP ? RC_RPT : 1];
-    if constexpr (KEEP) {
-#pragma unroll
-        for (int i = 0; i < RC_RPT; i++) {
-            const int r = rg + i * RG;
-            S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-            if (on && old && r < dim) S[i] = *reinterpret_cast<const f32x4*>(S0 + (size_t)r * vs + col);
-        }
-    }
-    const T* raw = reinterpret_cast<const T*>(a.raw) + (size_t)rr * a.ldraw;
-    const T* q = raw + a.col_q + (size_t)h * dim;
-    const T* v = raw + a.col_q + (size_t)2 * a.n_head * dim + (size_t)h * vdim;
-    for (int i = tid; i < dim; i += NT) s_q[i] = rb_ld(q + i), s_k[i] = rb_ld(q + (size_t)a.n_head * dim + i);
-    for (int i = tid; i < vs; i += NT) s_v[i] = i < vdim ? rb_ld(v + i) : 0.f;
-    __syncthreads();
-    if (wid == 0) {
-        float d = 0.f;
-        for (int i = lane; i < dim; i += 64) d = fmaf(s_q[i], s_k[i], d);
-        d = wave_sum(d);
-        if (lane == 0) s_one[0] = d;
-    }
-    f32x4 o = f32x4{0.f, 0.f, 0.f, 0.f}, u = o;
-    if (on) u = *reinterpret_cast<const f32x4*>(s_v + col);
-    auto step = [&](int r, f32x4 s) {
-        const float qq = s_q[r], kk = s_k[r];
+    const f32x4 u = *reinterpret_cast<const f32x4*>(s_v + st.col);
+    st.each(S0, pos > 0, [&](int r, f32x4 s) {
+        const float g = s_g[r], kk = s_k[r] * kn;
         f32x4 n;
 #pragma unroll
-        for (int j = 0; j < 4; j++) o[j] = fmaf(qq, s[j], o[j]), n[j] = fmaf(kk, u[j], lam * s[j]);
-        *reinterpret_cast<f32x4*>(S1 + (size_t)r * vs + col) = n;
-    };
-    if (on) {
-        if constexpr (KEEP) {
-#pragma unroll
-            for (int i = 0; i < RC_RPT; i++)
-                if (rg + i * RG < dim) step(rg + i * RG, S[i]);
-        } else {
-            for (int r = rg; r < dim; r += RG) {
-                f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
-                if (old) s = *reinterpret_cast<const f32x4*>(S0 + (size_t)r * vs + col);
-                step(r, s);
-            }
-        }
-        *reinterpret_cast<f32x4*>(s_red + (size_t)rg * vs + col) = o;
-    }
-    __syncthreads();
-    const int all = a.n_head * vdim;
-    float* parts = a.scratch + (size_t)RC_CNT_STRIDE * gridDim.y + (size_t)rr * all; /* behind the arrival counters: the row's heads */
-    for (int i = tid; i < vdim; i += NT) {
-        float so = 0.f;
-        for (int g = 0; g < RG; g++) so += s_red[(size_t)g * vs + i];
-        rc_st_sc1(parts + h * vdim + i, fmaf(s_one[0], s_v[i], lam * so));
-    }
-    // the heads' outputs leave with write-through stores; every wave has their acknowledgements before one lane counts the workgroup in; the last one in norms and gates the row
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();
-    int* counter = reinterpret_cast<int*>(a.scratch) + RC_CNT_STRIDE * (size_t)rr;
-    if (tid == 0) s_last = __hip_atomic_fetch_add(counter, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (int)gridDim.x - 1;
-    __syncthreads();
-    if (!s_last) return;
-    if (tid == 0) __hip_atomic_store(counter, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    float ss = 0.f;
-    for (int i = tid; i < all; i += NT) {
-        const float y = rc_ld_sc1(parts + i);
-        ss = fmaf(y, y, ss);
-    }
-    ss = wave_sum(ss);
-    if (lane == 0) s_one[4 + wid] = ss;
-    __syncthreads();
-    ss = 0.f;
-#pragma unroll
-    for (int w = 0; w < NT / 64; w++) ss += s_one[4 + w];
-    const float rs = a.out_scale / sqrtf(ss / (float)all + a.eps);
-    T* out = reinterpret_cast<T*>(a.out) + (size_t)rr * a.ldout;
-    for (int i = tid; i < all; i += NT) rb_st(out + i, rc_ld_sc1(parts + i) * rs * rb_ld(reinterpret_cast<const T*>(a.norm_w) + i) * rb_sigmoid(rb_ld(raw + a.col_g + i)));
+        for (int j = 0; j < 4; j++) n[j] = fmaf(kk, u[j], g * s[j]);
+        *reinterpret_cast<f32x4*>(S1 + (size_t)r * vs + st.col) = n;
+    });
+}
+template <class T, int NT, int RPT>
+__global__ void __launch_bounds__(NT) rb_decay_step_kernel(const kf_rb_decay a, const int32_t* __restrict__ meta) {
+    extern __shared__ float smem[];
+    rc_decay_step<T, NT, RPT>(a, meta, blockIdx.x, blockIdx.y, gridDim.y, smem);
 }
 
 // ---- prompts
@@ -428,15 +335,6 @@ __device__ __forceinline__ f32x4 rc_mfma(f32x4 a, f32x4 b, f32x4 c) { /* 16 x 16
 #pragma unroll
     for (int i = 0; i < 4; i++) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
     return c;
-}
-__device__ __forceinline__ float rc_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
-constexpr float RC_LOG2E = 1.44269502162933349609375f;
-__device__ __forceinline__ float rc_fast_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + rc_exp2(-RC_LOG2E * z)); }
-// softplus in units of ln 2: log2(1 + e^z); the correction factor keeps the small ones exact to rounding
-__device__ __forceinline__ float rc_softplus2(float z) {
-    const float e = rc_exp2(-RC_LOG2E * fabsf(z)), u = 1.0f + e, d = u - 1.0f;
-    const float l = d == 0.f ? e * RC_LOG2E : __builtin_amdgcn_logf(u) * (e * __builtin_amdgcn_rcpf(d));
-    return fmaxf(z, 0.f) * RC_LOG2E + l;
 }
 // what a chunk leaves for the walk, floats: W [64][DP], q e^G [64][DP], (k e^(G_end - G))^T [DP][64], q-k products [64][64], U [64][Vp], e^(G_end) [DP].  The matrices lie in 16 x 16
 // tiles, row of tiles after row of tiles, 64 x 4 floats each in the order of a left operand (lane 16 g + r: row r, columns 4 g ..; U: of a result, rows 4 g .., column r): a wave reads a
@@ -1275,32 +1173,25 @@ static int decay_prefill_go(hipStream_t st, const kf_rb_decay& a, int n, const i
     gate_go<T>(st, RcGate{o, a.norm_w, reinterpret_cast<const T*>(a.raw) + a.col_g, a.out, ldo, a.ldraw, a.ldout, 1, a.n_head * a.vdim, a.out_scale, a.eps}, n);
     return KF_OK;
 }
-// threads of a decode workgroup: at most RC_RPT rows of four columns each where the state allows it
-static int step_threads(int dim, int vdim) {
-    const int vs = rc_up(vdim, 4);
-    for (int nt : {256, 512, 1024})
-        if (vs / 4 <= nt && (dim + nt / (vs / 4) - 1) / (nt / (vs / 4)) <= RC_RPT) return nt;
-    return 0; /* 1024 threads that read the state twice */
-}
 template <class T>
 static void delta_step_go(hipStream_t st, const kf_rb_delta& a, const int32_t* meta, int n) {
-    const int nt = step_threads(a.dim, a.vdim);
+    const int nt = rc_step_threads(a.dim, a.vdim);
     const size_t smem = (3 * (size_t)rc_up(a.dim, 4) + 2 * rc_up(a.vdim, 4) + rc_up(a.rank_a, 8) + rc_up(a.rank_g, 8) + 8 * (size_t)(nt ? nt : 1024) + 32) * 4;
     const dim3 grid(a.n_head, n);
-    if (nt == 256) hipLaunchKernelGGL((rb_delta_step_kernel<T, 256, true>), grid, dim3(256), smem, st, a, meta);
-    else if (nt == 512) hipLaunchKernelGGL((rb_delta_step_kernel<T, 512, true>), grid, dim3(512), smem, st, a, meta);
-    else if (nt == 1024) hipLaunchKernelGGL((rb_delta_step_kernel<T, 1024, true>), grid, dim3(1024), smem, st, a, meta);
-    else hipLaunchKernelGGL((rb_delta_step_kernel<T, 1024, false>), grid, dim3(1024), smem, st, a, meta);
+    if (nt == 256) hipLaunchKernelGGL((rb_delta_step_kernel<T, 256, 8>), grid, dim3(256), smem, st, a, meta);
+    else if (nt == 512) hipLaunchKernelGGL((rb_delta_step_kernel<T, 512, 8>), grid, dim3(512), smem, st, a, meta);
+    else if (nt == 1024) hipLaunchKernelGGL((rb_delta_step_kernel<T, 1024, 16>), grid, dim3(1024), smem, st, a, meta);
+    else hipLaunchKernelGGL((rb_delta_step_kernel<T, 1024, 0>), grid, dim3(1024), smem, st, a, meta);
 }
 template <class T>
 static void decay_step_go(hipStream_t st, const kf_rb_decay& a, const int32_t* meta, int n) {
-    const int nt = step_threads(a.dim, a.vdim);
-    const size_t smem = (2 * (size_t)rc_up(a.dim, 4) + rc_up(a.vdim, 4) + 4 * (size_t)(nt ? nt : 1024) + 32) * 4;
+    const int nt = rc_step_threads(a.dim, a.vdim);
+    const size_t smem = rc_decay_step_lds(a.dim, a.vdim, nt ? nt : 1024);
     const dim3 grid(a.n_head, n);
-    if (nt == 256) hipLaunchKernelGGL((rb_decay_step_kernel<T, 256, true>), grid, dim3(256), smem, st, a, meta);
-    else if (nt == 512) hipLaunchKernelGGL((rb_decay_step_kernel<T, 512, true>), grid, dim3(512), smem, st, a, meta);
-    else if (nt == 1024) hipLaunchKernelGGL((rb_decay_step_kernel<T, 1024, true>), grid, dim3(1024), smem, st, a, meta);
-    else hipLaunchKernelGGL((rb_decay_step_kernel<T, 1024, false>), grid, dim3(1024), smem, st, a, meta);
+    if (nt == 256) hipLaunchKernelGGL((rb_decay_step_kernel<T, 256, 8>), grid, dim3(256), smem, st, a, meta);
+    else if (nt == 512) hipLaunchKernelGGL((rb_decay_step_kernel<T, 512, 8>), grid, dim3(512), smem, st, a, meta);
+    else if (nt == 1024) hipLaunchKernelGGL((rb_decay_step_kernel<T, 1024, 16>), grid, dim3(1024), smem, st, a, meta);
+    else hipLaunchKernelGGL((rb_decay_step_kernel<T, 1024, 0>), grid, dim3(1024), smem, st, a, meta);
 }
 
 }  // namespace kf
