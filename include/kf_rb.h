@@ -205,6 +205,8 @@ typedef struct kf_rb_decay {
 } kf_rb_decay;
 int kf_rb_decay_prefill(kf_ctx* ctx, const kf_rb_decay* a, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n);
 int kf_rb_decay_decode(kf_ctx* ctx, const kf_rb_decay* a, const int32_t* meta, int n_rows);
+/* a layer's attention and its decayed sum of the same rows: kf_rb_attention_decode and kf_rb_decay_decode, in one launch where the rows are few */
+int kf_rb_attention_decay_decode(kf_ctx* ctx, const kf_rb_attention* a, const kf_rb_decay* d, const int32_t* meta, int n_rows, int max_pos);
 size_t kf_rb_decay_scratch(int type, int n_rows, int n_seq, int n_head, int dim, int vdim);
 
 /* router: logits fp32 [n][ld] (+ bias [n_expert] in the batch's storage, may be NULL) -> the `top` largest of every row (ties: the lower expert) and the softmax over them;

@@ -12,7 +12,7 @@
 #include <algorithm>
 
 #include "kf_ctx.h"
-#include "kf_rb_common.h"
+#include "kf_rb_recur.h"
 
 namespace kf {
 
@@ -431,15 +431,14 @@ __global__ void __launch_bounds__(256 * KH, HD <= 128 ? 2 : 1) rb_attn_prefill_k
 // decode: grid (n_kv * column blocks of 32 query heads, key ranges of `span` keys, rows).  raw is not prepared: q and the new key are normed and rotated here while the first
 // tiles are on their way; the workgroup whose range holds the row's position patches the new key and value into its tile and puts them into the ring.
 template <int HD>
-__global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta, int span, int n_range) {
+__device__ __forceinline__ void rb_attn_decode(const kf_rb_attention& a, const int32_t* __restrict__ meta, int span, int n_range, int block, int range, int rr, int n_rows, unsigned char* smem_raw) {
     using Tile = RbTile<HD>;
-    extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
     constexpr int KS = Tile::KS, VS = Tile::VS, CH = HD / 8, WAVE_EL = 32 * (KS + VS), NREG = Tile::NDB * 16;
-    const int rr = blockIdx.z, pos = meta[KF_RB_META * rr], slot = meta[KF_RB_META * rr + 1];
+    const int pos = meta[KF_RB_META * rr], slot = meta[KF_RB_META * rr + 1];
     if (pos < 0) return; /* workgroup-uniform, like the next */
-    const int first = rb_first_key(pos, a), k_lo = first + (int)blockIdx.y * span, k_hi = k_lo + span - 1 < pos ? k_lo + span - 1 : pos;
+    const int first = rb_first_key(pos, a), k_lo = first + range * span, k_hi = k_lo + span - 1 < pos ? k_lo + span - 1 : pos;
     if (k_lo > pos) return;
-    const int GQ = a.n_head / a.n_kv, ncb = (GQ + 31) / 32, g = blockIdx.x / ncb, cb = blockIdx.x % ncb, col0 = cb * 32, ncol = GQ - col0 < 32 ? GQ - col0 : 32;
+    const int GQ = a.n_head / a.n_kv, ncb = (GQ + 31) / 32, g = block / ncb, cb = block % ncb, col0 = cb * 32, ncol = GQ - col0 < 32 ? GQ - col0 : 32;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, r = lane & 31, h = lane >> 5;
     uint16_t* s_new = reinterpret_cast<uint16_t*>(smem_raw);             /* the new key, the new value: [2][HD] */
     uint16_t* s_kv = s_new + 2 * HD;                                     /* [4 waves] [32][KS] + [32][VS]; before the walk: */
@@ -531,8 +530,8 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     const int head = g * GQ + col0 + (r < ncol ? r : 0);
     const uint16_t* gate = raw + a.gate_col + (size_t)head * a.vdim;
     uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)rr * a.ldout + (size_t)head * a.vdim;
-    float* parts = reinterpret_cast<float*>(a.scratch) + RB_CNT_STRIDE * (size_t)gridDim.z * a.n_head; /* behind the arrival counters: [row][head][range][vdim + 2] */
-    float* part = parts + (((size_t)rr * a.n_head + head) * n_range + blockIdx.y) * (a.vdim + 2);
+    float* parts = reinterpret_cast<float*>(a.scratch) + RB_CNT_STRIDE * (size_t)n_rows * a.n_head; /* behind the arrival counters: [row][head][range][vdim + 2] */
+    float* part = parts + (((size_t)rr * a.n_head + head) * n_range + range) * (a.vdim + 2);
     const float inv = a.out_scale * rb_softmax_factor(M, L, a.sink);
     for (int q = wid; q < Tile::NDB * 4 && r < ncol; q += 4) { /* a quad of registers = four consecutive d */
         const int d = 8 * q + 4 * h;
@@ -558,7 +557,7 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
     if (wid == 0 && h == 0 && r < ncol) rb_st_sc1(part, M), rb_st_sc1(part + 1, L);
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
-    int* counter = reinterpret_cast<int*>(a.scratch) + RB_CNT_STRIDE * ((size_t)rr * a.n_head + blockIdx.x);
+    int* counter = reinterpret_cast<int*>(a.scratch) + RB_CNT_STRIDE * ((size_t)rr * a.n_head + block);
     if (tid == 0) s_last = __hip_atomic_fetch_add(counter, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == n_used - 1;
     __syncthreads();
     if (!s_last) return;
@@ -595,6 +594,19 @@ __global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attenti
         }
     }
 }
+template <int HD>
+__global__ void __launch_bounds__(256) rb_attn_decode_kernel(const kf_rb_attention a, const int32_t* __restrict__ meta, int span, int n_range) {
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+    rb_attn_decode<HD>(a, meta, span, n_range, blockIdx.x, blockIdx.y, blockIdx.z, gridDim.z, smem_raw);
+}
+// a layer's decayed sum (its heads first) and its attention in one launch: neither waits for the other
+template <int HD>
+__global__ void __launch_bounds__(256) rb_attn_decay_decode_kernel(const kf_rb_attention a, const kf_rb_decay d, const int32_t* __restrict__ meta, int span, int n_range) {
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+    const int block = (int)blockIdx.x - d.n_head, blocks = ((int)gridDim.x - d.n_head) / n_range;
+    if (block < 0) rc_decay_step<uint16_t, 256, 16>(d, meta, blockIdx.x, blockIdx.y, gridDim.y, reinterpret_cast<float*>(smem_raw));
+    else rb_attn_decode<HD>(a, meta, span, n_range, block % blocks, block / blocks, blockIdx.y, gridDim.y, smem_raw);
+}
 constexpr int RB_MAX_RANGES = 32;
 static void decode_ranges(int n_rows, int n_kv, int keys, int& span, int& n_range) {
     n_range = (keys + 255) / 256; /* a range is at least two tiles per wave */
@@ -629,15 +641,24 @@ static int prefill_go(hipStream_t st, const kf_rb_attention& a, const int32_t* s
     return prefill_kh<HD, 1>(st, a, seqs, grid);
 }
 template <int HD>
-static int decode_go(hipStream_t st, const kf_rb_attention& a, const int32_t* meta, int n_rows, int span, int n_range) {
+static int decode_go(hipStream_t st, const kf_rb_attention& a, const kf_rb_decay* d, const int32_t* meta, int n_rows, int span, int n_range) {
     constexpr size_t tiles = 4 * 2 * 32 * (size_t)(RbTile<HD>::KS + RbTile<HD>::VS), merge = 4 * (size_t)(RbTile<HD>::NDB * 16 + 2) * 256;
     constexpr size_t smem = 4 * HD + (tiles > merge ? tiles : merge);
     static_assert(32 * RbTile<HD>::KS * 2 + 16 * HD <= tiles, "queries in the tiles' place");
     static_assert(smem <= 160 * 1024, "LDS");
+    const int blocks = a.n_kv * ((a.n_head / a.n_kv + 31) / 32);
+    if (d) {
+        static int done = 0;
+        const size_t both = std::max(smem, rc_decay_step_lds(d->dim, d->vdim, 256));
+        if (both > 150 * 1024) return 1;
+        if (!done && hipFuncSetAttribute((const void*)rb_attn_decay_decode_kernel<HD>, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024) != hipSuccess) return KF_HIP_CHECK;
+        done = 1;
+        hipLaunchKernelGGL(rb_attn_decay_decode_kernel<HD>, dim3(d->n_head + blocks * n_range, n_rows), dim3(256), both, st, a, *d, meta, span, n_range);
+        return KF_OK;
+    }
     static int done = 0;
     if (big_lds(rb_attn_decode_kernel<HD>, smem, done)) return KF_HIP_CHECK;
-    const int ncb = (a.n_head / a.n_kv + 31) / 32;
-    hipLaunchKernelGGL(rb_attn_decode_kernel<HD>, dim3(a.n_kv * ncb, n_range, n_rows), dim3(256), smem, st, a, meta, span, n_range);
+    hipLaunchKernelGGL(rb_attn_decode_kernel<HD>, dim3(blocks, n_range, n_rows), dim3(256), smem, st, a, meta, span, n_range);
     return KF_OK;
 }
 static bool mfma_served(const kf_rb_attention& a, int n_rows) {
@@ -703,6 +724,36 @@ static int check_attention(const kf_rb_attention* a, const int32_t* meta, int n,
     if (!al16(a->raw) || !al16(a->out) || !al16(a->k_cache) || !al16(a->v_cache)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
     return KF_OK;
 }
+constexpr int RB_BESIDE_ROWS = 16; /* rows up to which a decayed sum goes into the attention's launch */
+static int attention_decode(kf_ctx* c, const kf_rb_attention* ap, const kf_rb_decay* d, const int32_t* meta, int n_rows, int max_pos, const char* who) {
+    CHKCTX(c);
+    if (!ap) return abi_fail(KF_INVALID_ARGS, "%s: null pointer", who);
+    const kf_rb_attention a = whole_form(*ap);
+    const int rc = check_attention(&a, meta, n_rows, who);
+    if (rc) return rc;
+    if (max_pos < 0) return abi_fail(KF_INVALID_ARGS, "%s: max_pos %d", who, max_pos);
+    hipStream_t st = c->stream;
+    int r = KF_OK;
+    if (mfma_served(a, n_rows)) {
+        int keys = max_pos + 1, span, n_range;
+        const int seen = a.window > 0 ? a.window : a.chunk;
+        if (seen > 0 && keys > seen) keys = seen;
+        decode_ranges(n_rows, a.n_kv * ((a.n_head / a.n_kv + 31) / 32), keys, span, n_range);
+        if (n_range > 1 && !a.scratch) return abi_fail(KF_INVALID_ARGS, "%s: null scratch", who);
+#define RB_CALL(HD) decode_go<HD>(st, a, d, meta, n_rows, span, n_range)
+        r = RB_BY_DIM(RB_CALL);
+#undef RB_CALL
+    } else if (a.type == KF_BF16) {
+        prep_go<uint16_t>(st, a, meta, n_rows, true);
+        plain_go<uint16_t>(st, a, meta, n_rows, 1);
+    } else {
+        prep_go<float>(st, a, meta, n_rows, true);
+        plain_go<float>(st, a, meta, n_rows, 1);
+    }
+    if (r == 1) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: these sizes do not share a launch", who);
+    if (r != KF_OK || hipGetLastError() != hipSuccess) return abi_fail(KF_HIP_CHECK, "%s: launch failed", who);
+    return KF_OK;
+}
 extern "C" {
 
 size_t kf_rb_attention_scratch(int n_rows, int n_head, int dim) { return n_rows < 1 || n_head < 1 || dim < 1 ? 0 : (size_t)n_rows * n_head * (RB_CNT_STRIDE + (size_t)RB_MAX_RANGES * (dim + 2)) * sizeof(float); }
@@ -734,33 +785,17 @@ int kf_rb_attention_prefill(kf_ctx* c, const kf_rb_attention* ap, const int32_t*
     if (r != KF_OK || hipGetLastError() != hipSuccess) return abi_fail(KF_HIP_CHECK, "kf_rb_attention_prefill: launch failed");
     return KF_OK;
 }
-int kf_rb_attention_decode(kf_ctx* c, const kf_rb_attention* ap, const int32_t* meta, int n_rows, int max_pos) {
+int kf_rb_attention_decode(kf_ctx* c, const kf_rb_attention* ap, const int32_t* meta, int n_rows, int max_pos) { return attention_decode(c, ap, nullptr, meta, n_rows, max_pos, "kf_rb_attention_decode"); }
+int kf_rb_attention_decay_decode(kf_ctx* c, const kf_rb_attention* ap, const kf_rb_decay* d, const int32_t* meta, int n_rows, int max_pos) {
     CHKCTX(c);
-    if (!ap) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: null pointer");
-    const kf_rb_attention a = whole_form(*ap);
-    const int rc = check_attention(&a, meta, n_rows, "kf_rb_attention_decode");
+    int rc = rc_check_decay(d, meta, n_rows, "kf_rb_attention_decay_decode");
     if (rc) return rc;
-    if (max_pos < 0) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: max_pos %d", max_pos);
-    hipStream_t st = c->stream;
-    int r = KF_OK;
-    if (mfma_served(a, n_rows)) {
-        int keys = max_pos + 1, span, n_range;
-        const int seen = a.window > 0 ? a.window : a.chunk;
-        if (seen > 0 && keys > seen) keys = seen;
-        decode_ranges(n_rows, a.n_kv * ((a.n_head / a.n_kv + 31) / 32), keys, span, n_range);
-        if (n_range > 1 && !a.scratch) return abi_fail(KF_INVALID_ARGS, "kf_rb_attention_decode: null scratch");
-#define RB_CALL(HD) decode_go<HD>(st, a, meta, n_rows, span, n_range)
-        r = RB_BY_DIM(RB_CALL);
-#undef RB_CALL
-    } else if (a.type == KF_BF16) {
-        prep_go<uint16_t>(st, a, meta, n_rows, true);
-        plain_go<uint16_t>(st, a, meta, n_rows, 1);
-    } else {
-        prep_go<float>(st, a, meta, n_rows, true);
-        plain_go<float>(st, a, meta, n_rows, 1);
-    }
-    if (r != KF_OK || hipGetLastError() != hipSuccess) return abi_fail(KF_HIP_CHECK, "kf_rb_attention_decode: launch failed");
-    return KF_OK;
+    // one launch where a head's state fits the registers of an attention workgroup and the rows are few (more of them fill the chip either way)
+    const int c4 = (d->vdim + 3) / 4;
+    const bool fits = d->type == KF_BF16 && c4 <= 256 && (d->dim + 256 / c4 - 1) / (256 / c4) <= 16 && n_rows <= RB_BESIDE_ROWS;
+    if (fits && ap && mfma_served(whole_form(*ap), n_rows)) return attention_decode(c, ap, d, meta, n_rows, max_pos, "kf_rb_attention_decay_decode");
+    rc = kf_rb_attention_decode(c, ap, meta, n_rows, max_pos);
+    return rc ? rc : kf_rb_decay_decode(c, d, meta, n_rows);
 }
 
 }  // extern "C"

@@ -3,6 +3,7 @@
 #pragma once
 #include <math.h>
 
+#include "kf_ctx.h"
 #include "kf_rb_common.h"
 
 namespace kf {
@@ -92,6 +93,7 @@ static inline int rc_step_threads(int dim, int vdim) {
 }
 static inline size_t rc_decay_step_lds(int dim, int vdim, int nt) { return (2 * (size_t)rc_up(dim, 4) + rc_up(vdim, 4) + 4 * (size_t)nt + 40) * 4; }
 
+int rc_check_decay(const kf_rb_decay* a, const int32_t* meta, int n, const char* who); // kf_rb_recur.hip
 // head h of row rr (of n_rows): o = decay S^T q + (q . k) v, S' = decay S + k v^T; the row's last head norms and gates all of them
 template <class T, int NT, int RPT>
 __device__ __forceinline__ void rc_decay_step(const kf_rb_decay& a, const int32_t* __restrict__ meta, int h, int rr, int n_rows, float* smem) {

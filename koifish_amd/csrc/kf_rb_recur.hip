@@ -49,7 +49,7 @@ __device__ __forceinline__ float rc_octet_dot(const RcOctet32& v, const float* x
 }
 // One workgroup per (head, row).  What it reads sets out at once, in the order of its use: the channels' last inputs, the low-rank rows, the state (barriers wait for LDS only)
 template <class T, int NT, int RPT>
-__global__ void __launch_bounds__(NT) rb_delta_step_kernel(const kf_rb_delta a, const int32_t* __restrict__ meta) {
+__global__ void __launch_bounds__(NT, 4) rb_delta_step_kernel(const kf_rb_delta a, const int32_t* __restrict__ meta) {
     extern __shared__ float smem[];
     constexpr int NW = NT / 64, PF = NT > 512 || sizeof(T) == 4 ? 4 : 8; /* octets in flight per lane */
     const int h = blockIdx.x, rr = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
@@ -1194,10 +1194,21 @@ static void decay_step_go(hipStream_t st, const kf_rb_decay& a, const int32_t* m
     else hipLaunchKernelGGL((rb_decay_step_kernel<T, 1024, 0>), grid, dim3(1024), smem, st, a, meta);
 }
 
+constexpr int RC_MAX_DIM = 512;
+int rc_check_decay(const kf_rb_decay* a, const int32_t* meta, int n, const char* who) {
+    if (!a || !meta || n < 1 || !a->raw || !a->out || !a->norm_w || !a->decay || !a->state || !a->scratch) return abi_fail(KF_INVALID_ARGS, "%s: null pointer", who);
+    if (a->type != KF_BF16 && a->type != KF_F32) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: storage %d", who, a->type);
+    if (a->n_head < 1 || a->dim < 1 || a->vdim < 1) return abi_fail(KF_INVALID_ARGS, "%s: %d heads of %d / %d", who, a->n_head, a->dim, a->vdim);
+    if (a->dim > RC_MAX_DIM || a->vdim > RC_MAX_DIM) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: head sizes %d / %d (served: up to %d)", who, a->dim, a->vdim, RC_MAX_DIM);
+    const int64_t qk = 2 * (int64_t)a->n_head * a->dim, all = (int64_t)a->n_head * a->vdim;
+    if (a->col_q < 0 || a->col_g < 0 || a->ldraw < a->col_q + qk + all || a->ldraw < a->col_g + all || a->ldout < all) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
+    if (!al16(a->state) || !al16(a->scratch) || !al16(a->raw)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
+    return KF_OK;
+}
+
 }  // namespace kf
 
 using namespace kf;
-constexpr int RC_MAX_DIM = 512;
 static int check_delta(const kf_rb_delta* a, const int32_t* meta, int n, const char* who) {
     if (!a || !meta || n < 1 || !a->raw || !a->out || !a->conv || !a->a_log || !a->dt_bias || !a->norm_w || !a->state || !a->hist) return abi_fail(KF_INVALID_ARGS, "%s: null pointer", who);
     if (a->type != KF_BF16 && a->type != KF_F32) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: storage %d", who, a->type);
@@ -1206,16 +1217,6 @@ static int check_delta(const kf_rb_delta* a, const int32_t* meta, int n, const c
     const int64_t channels = 2 * (int64_t)a->n_kv * a->dim + (int64_t)a->n_head * a->vdim;
     if (a->hist_slot < channels * a->taps || a->ldout < (int64_t)a->n_head * a->vdim || a->col_b < channels || a->ldraw < a->col_b + a->n_head) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
     if (!al16(a->state) || !al16(a->raw) || !al16(a->out)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
-    return KF_OK;
-}
-static int check_decay(const kf_rb_decay* a, const int32_t* meta, int n, const char* who) {
-    if (!a || !meta || n < 1 || !a->raw || !a->out || !a->norm_w || !a->decay || !a->state || !a->scratch) return abi_fail(KF_INVALID_ARGS, "%s: null pointer", who);
-    if (a->type != KF_BF16 && a->type != KF_F32) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: storage %d", who, a->type);
-    if (a->n_head < 1 || a->dim < 1 || a->vdim < 1) return abi_fail(KF_INVALID_ARGS, "%s: %d heads of %d / %d", who, a->n_head, a->dim, a->vdim);
-    if (a->dim > RC_MAX_DIM || a->vdim > RC_MAX_DIM) return abi_fail(KF_UNSUPPORTED_DATATYPE, "%s: head sizes %d / %d (served: up to %d)", who, a->dim, a->vdim, RC_MAX_DIM);
-    const int64_t qk = 2 * (int64_t)a->n_head * a->dim, all = (int64_t)a->n_head * a->vdim;
-    if (a->col_q < 0 || a->col_g < 0 || a->ldraw < a->col_q + qk + all || a->ldraw < a->col_g + all || a->ldout < all) return abi_fail(KF_INVALID_ARGS, "%s: strides", who);
-    if (!al16(a->state) || !al16(a->scratch) || !al16(a->raw)) return abi_fail(KF_BLAS_UNALIGN, "%s: unaligned pointer", who);
     return KF_OK;
 }
 static int launched(int rc, const char* who) {
@@ -1259,14 +1260,14 @@ int kf_rb_delta_decode(kf_ctx* c, const kf_rb_delta* a, const int32_t* meta, int
 }
 int kf_rb_decay_prefill(kf_ctx* c, const kf_rb_decay* a, const int32_t* meta, int n_rows, const int32_t* seqs, int n_seq, int max_n) {
     CHKCTX(c);
-    const int rc = check_decay(a, meta, n_rows, "kf_rb_decay_prefill");
+    const int rc = rc_check_decay(a, meta, n_rows, "kf_rb_decay_prefill");
     if (rc) return rc;
     if (!seqs || n_seq < 1 || max_n < 1 || max_n > n_rows) return abi_fail(KF_INVALID_ARGS, "kf_rb_decay_prefill: bad arguments");
     return launched(a->type == KF_BF16 ? decay_prefill_go<uint16_t>(c->stream, *a, n_rows, seqs, n_seq, max_n) : decay_prefill_go<float>(c->stream, *a, n_rows, seqs, n_seq, max_n), "kf_rb_decay_prefill");
 }
 int kf_rb_decay_decode(kf_ctx* c, const kf_rb_decay* a, const int32_t* meta, int n_rows) {
     CHKCTX(c);
-    const int rc = check_decay(a, meta, n_rows, "kf_rb_decay_decode");
+    const int rc = rc_check_decay(a, meta, n_rows, "kf_rb_decay_decode");
     if (rc) return rc;
     if (a->type == KF_BF16) decay_step_go<uint16_t>(c->stream, *a, meta, n_rows);
     else decay_step_go<float>(c->stream, *a, meta, n_rows);

@@ -77,7 +77,7 @@ int RowMixer::Forw(RowWork& w, const KVCache& kv, const RowBatch& b, bool defer)
 void RowMixer::Need(RowNeed& need, int rows, int, bool) const {
     need.raw = std::max(need.raw, (size_t)rows * ldraw), need.ao = std::max(need.ao, (size_t)rows * ldout);
 }
-int RowAttention::Mix(RowWork& w, const KVCache& kv, const RowBatch& b) {
+kf_rb_attention RowAttention::Args(const RowWork& w, const KVCache& kv) const {
     const SEQ_CARD& card = hFish->Seq()->card;
     const KVCache::Ring& ring = kv.rings[layid - 1];
     kf_rb_attention a;
@@ -89,6 +89,10 @@ int RowAttention::Mix(RowWork& w, const KVCache& kv, const RowBatch& b) {
     a.scale = c.scale, a.eps = card.eps;
     a.v_col = v_col, a.vdim = c.vdim, a.unit = c.qk_unit, a.window = c.window, a.sink = c.sink;
     if (c.kind == MIXER_CARD::PARALLEL) a.scaled = 1, a.out_scale = c.left_scale;
+    return a;
+}
+int RowAttention::Mix(RowWork& w, const KVCache& kv, const RowBatch& b) {
+    const kf_rb_attention a = Args(w, kv);
     if (b.n_seq) return kf_rb_attention_prefill(hFish->ctx, &a, I(w.meta), b.n, I(w.seqs), b.n_seq, b.max_n);
     return kf_rb_attention_decode(hFish->ctx, &a, I(w.meta), b.n, b.max_pos);
 }
@@ -121,14 +125,17 @@ void ChannelDelta::Need(RowNeed& need, int rows, int n_seq, bool decode) const {
 }
 int ParallelMixer::Mix(RowWork& w, const KVCache& kv, const RowBatch& b) {
     SeqFish* f = hFish->Seq();
+    kf_rb_decay d;
+    std::memset(&d, 0, sizeof(d));
+    d.raw = P(w.raw), d.out = reinterpret_cast<uint8_t*>(P(w.ao)) + out_sum * f->Elem(), d.norm_w = P(sum_norm), d.decay = F(decay), d.state = kv.State0(layid - 1), d.scratch = F(w.recur);
+    d.ldraw = ldraw, d.ldout = ldout, d.type = f->card.type, d.n_head = c.sum_heads, d.dim = c.sum_dim, d.vdim = c.sum_vdim, d.col_q = col_sum, d.col_g = col_gate;
+    d.out_scale = c.right_scale, d.eps = f->card.eps;
+    if (!b.n_seq) {
+        const kf_rb_attention a = Args(w, kv);
+        return kf_rb_attention_decay_decode(f->ctx, &a, &d, I(w.meta), b.n, b.max_pos);
+    }
     KF_TRY(RowAttention::Mix(w, kv, b));
-    kf_rb_decay a;
-    std::memset(&a, 0, sizeof(a));
-    a.raw = P(w.raw), a.out = reinterpret_cast<uint8_t*>(P(w.ao)) + out_sum * f->Elem(), a.norm_w = P(sum_norm), a.decay = F(decay), a.state = kv.State0(layid - 1), a.scratch = F(w.recur);
-    a.ldraw = ldraw, a.ldout = ldout, a.type = f->card.type, a.n_head = c.sum_heads, a.dim = c.sum_dim, a.vdim = c.sum_vdim, a.col_q = col_sum, a.col_g = col_gate;
-    a.out_scale = c.right_scale, a.eps = f->card.eps;
-    if (b.n_seq) return kf_rb_decay_prefill(f->ctx, &a, I(w.meta), b.n, I(w.seqs), b.n_seq, b.max_n);
-    return kf_rb_decay_decode(f->ctx, &a, I(w.meta), b.n);
+    return kf_rb_decay_prefill(f->ctx, &d, I(w.meta), b.n, I(w.seqs), b.n_seq, b.max_n);
 }
 void ParallelMixer::Need(RowNeed& need, int rows, int n_seq, bool decode) const {
     RowAttention::Need(need, rows, n_seq, decode);

@@ -125,6 +125,7 @@ struct RowAttention : RowMixer {
     hGTensor qn, kn;
     const float* rope = nullptr;
     int v_col = 0;
+    kf_rb_attention Args(const RowWork& w, const KVCache& kv) const;
     int Mix(RowWork& w, const KVCache& kv, const RowBatch& b) override;
     void Need(RowNeed& need, int rows, int n_seq, bool decode) const override;
 };

@@ -25,7 +25,7 @@ ABI_SYMBOLS = [
     "kf_xengine_workspace_bytes", "kf_xengine_create", "kf_xengine_served", "kf_xengine_set_embedding", "kf_xengine_set_head", "kf_xengine_steps", "kf_xengine_check", "kf_xengine_reset", "kf_xengine_destroy", "kf_xengine_workspace_bytes_tp", "kf_xengine_create_tp", "kf_xengine_set_head_tp",
     "kf_rb_linear", "kf_rb_linear_norms", "kf_rb_pack", "kf_rb_embed", "kf_rb_embed_state", "kf_rb_norm", "kf_rb_attention_prefill", "kf_rb_attention_decode", "kf_rb_attention_scratch", "kf_rb_rope_table_host",
     "kf_rb_route", "kf_rb_list_tiles", "kf_rb_pick", "kf_rb_pick_scratch", "kf_rb_to_bf16", "kf_rb_norm_rows", "kf_rb_sinusoid_tables_host",
-    "kf_rb_delta_prefill", "kf_rb_delta_decode", "kf_rb_delta_scratch", "kf_rb_decay_prefill", "kf_rb_decay_decode", "kf_rb_decay_scratch",
+    "kf_rb_delta_prefill", "kf_rb_delta_decode", "kf_rb_delta_scratch", "kf_rb_decay_prefill", "kf_rb_decay_decode", "kf_rb_decay_scratch", "kf_rb_attention_decay_decode",
     "kf_tp_recv_bytes", "kf_tp_push_bytes", "kf_tp_commit", "kf_tp_alloc", "kf_tp_ipc_export", "kf_tp_ipc_open", "kf_tp_ipc_close", "kf_linear_f32_push", "kf_tp_reduce_recv", "kf_tp_lm_head", "kf_tp_pick",
 ]
 
@@ -329,6 +329,7 @@ def load():
         hip.kf_rb_delta_scratch.argtypes, hip.kf_rb_delta_scratch.restype = [C.c_int] * 7, C.c_size_t
         hip.kf_rb_decay_prefill.argtypes = [C.c_void_p, C.POINTER(RbDecay), C.c_void_p, C.c_int, C.c_void_p, C.c_int, C.c_int]
         hip.kf_rb_decay_decode.argtypes = [C.c_void_p, C.POINTER(RbDecay), C.c_void_p, C.c_int]
+        hip.kf_rb_attention_decay_decode.argtypes = [C.c_void_p, C.POINTER(RbAttention), C.POINTER(RbDecay), C.c_void_p, C.c_int, C.c_int]
         hip.kf_rb_decay_scratch.argtypes, hip.kf_rb_decay_scratch.restype = [C.c_int] * 6, C.c_size_t
         hip.kf_rb_to_bf16.argtypes = [C.c_void_p, C.c_void_p, C.c_void_p, C.c_size_t]
         host.kfh_arch.restype, host.kfh_arch.argtypes = C.c_char_p, [C.c_void_p]

@@ -84,8 +84,8 @@ class Layer:
     def rows(self, n):
         return store_type(self.rng.normal(size=(n, self.cols)), self.dt)
 
-    def feed(self, parts, decode=False):
-        """parts: {slot: raw rows}; returns {slot: (got, reference)} for the fed rows"""
+    def batch(self, parts, decode):
+        """the fed rows as launch()'s arguments"""
         order = list(parts) if not decode else list(range(self.n_slots))
         raw, meta, seqs, r0 = [], [], [], {}
         for s in order:
@@ -102,14 +102,23 @@ class Layer:
         n, seqs = len(meta), np.array(seqs)
         raw = pad(dev(np.concatenate(raw), self.dt), n, self.ldraw)
         out = torch.full((n, up(self.out_cols)), 7.0, dtype=self.dt, device="cuda")
-        self.launch(raw, out, dev(np.array(meta), torch.int32), n, None if decode else dev(seqs, torch.int32), len(seqs), int(seqs[:, 1].max()), max(len(self.hist[s]) for s in parts) - 1)
-        got = f64(out)
+        self.r0 = r0
+        return raw, out, dev(np.array(meta), torch.int32), n, None if decode else dev(seqs, torch.int32), len(seqs), int(seqs[:, 1].max()), max(len(self.hist[s]) for s in parts) - 1
+
+    def feed(self, parts, decode=False):
+        """parts: {slot: raw rows}; returns {slot: (got, reference)} for the fed rows"""
+        args = self.batch(parts, decode)
+        self.launch(*args)
+        return self.compare(parts, args[1])
+
+    def compare(self, parts, out):
+        got, r0 = f64(out), self.r0
         assert (got[:, self.out_cols:] == 7.0).all()
         return {s: (got[r0[s]:r0[s] + len(x), :self.out_cols], self.reference(s)[-len(x):]) for s, x in parts.items()}
 
-    def check(self, parts, decode=False):
+    def check(self, parts, decode=False, results=None):
         tol = 5e-5 if self.typ == L.F32 else 0.04
-        for s, (a, b) in self.feed(parts, decode).items():
+        for s, (a, b) in (results or self.feed(parts, decode)).items():
             err = np.abs(a - b).max(axis=1)
             assert err.max() < tol * max(1.0, np.abs(b).max()), (s, int(err.argmax()), err.max(), decode)
 
@@ -421,3 +430,24 @@ def test_window_edges(ctx, kind, window, how):
         d = np.abs(a.reference(0) - r).max(1)
         hi = min(at + window, len(d))
         assert (d[at:hi] > 0.5).all() and (d[at + window:] < 1e-12).all()
+
+
+@pytest.mark.parametrize("sizes", [(3, (4, 2, 64, 64, 300, 0.1), (4, 64, 128, (0.1, 0.6, 0.98, 0.9995))), (3, (16, 2, 128, 128, 90, 0.08), (2, 128, 128, (0.95, 0.998))), (3, (2, 1, 64, 48, 24, 0.2), (1, 264, 300, (0.97,))),
+                                   (24, (4, 1, 32, 64, 50, 0.1), (2, 64, 64, (0.8, 0.97)))], ids=["wide", "heads", "apart", "many"])
+def test_attention_and_decayed_sum_in_one_launch(ctx, kind, sizes):
+    n, w, d = sizes
+    a, b = Window(ctx, kind, *w, n_slots=n), Decay(ctx, kind, *d, n_slots=n)
+    for s in range(n):
+        a.new(s), b.new(s)
+    lens = {s: 5 + 7 * s for s in range(n) if s != 1}
+    a.check({s: a.rows(k) for s, k in lens.items()}), b.check({s: b.rows(k) for s, k in lens.items()})
+    for i in range(6):
+        on = [s for s in range(n) if (s + i) % 3]
+        pa, pb = {s: a.rows(1) for s in on}, {s: b.rows(1) for s in on}
+        ra, rb = a.batch(pa, True), b.batch(pb, True)
+        sc = torch.zeros(ctx.hip.kf_rb_attention_scratch(n, w[0], w[3]) // 4, device="cuda")
+        a.a.raw, a.a.out, a.a.scratch = ra[0].data_ptr(), ra[1].data_ptr(), sc.data_ptr()
+        b.a.raw, b.a.out, b.a.scratch = rb[0].data_ptr(), rb[1].data_ptr(), b.step_scratch.data_ptr()
+        L.check(ctx.hip.kf_rb_attention_decay_decode(ctx.h, C.byref(a.a), C.byref(b.a), ra[2].data_ptr(), n, ra[7]))
+        ctx.sync()
+        a.check(pa, results=a.compare(pa, ra[1])), b.check(pb, results=b.compare(pb, rb[1]))
